@@ -10,7 +10,10 @@ import os
 import threading
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
-LIB_PATH = os.path.join(_HERE, "libbased_hip.so")  # the in-tree build is the only library ever loaded
+LIB_PATH = os.path.join(_HERE, "libbased_hip.so")  # the in-tree build of every kernel
+# Builds of some of the sources (based_amd.build.build_part) lie beside it; `use_part` selects one
+# where the whole library has not been built.
+_part_path = None
 
 BASED_BF16 = 0
 BASED_F32 = 1
@@ -95,6 +98,27 @@ SIGNATURES = {
     "based_swiglu": (C.c_int, [_P, _P] + [_I64] * 4 + [C.c_int, _P]),
     "based_decode_linear": (C.c_int, [_P, _I64, _P, _I64, _P, _I64, _P, _P, _I64, _I64, _I64, _I64, C.c_int,
                                       _P, _I64, _P, _I64, _P, C.c_float, C.c_int, _P, C.c_int, _P, _P, C.c_int, _P]),
+    "based_add_norm": (C.c_int, [_P] * 5 + [_I64] * 6 + [C.c_float, C.c_int, C.c_float, C.c_int, _P]),
+    "based_stream_conv": (C.c_int, [_P] * 6 + [_I64] * 4 + [C.c_int] + [_I64] * 5 + [C.c_int] * 3 + [_P]),
+    "based_window_attn_prefill": (
+        C.c_int,
+        [_P] * 5 + [_I64] * 19 + [C.c_float, C.c_int, C.c_float, C.c_float, _P, _P, _I64, _I64, C.c_int, C.c_int, _P],
+    ),
+    "based_window_attn_step": (
+        C.c_int,
+        [_P] * 6 + [_I64] * 14 + [C.c_float, C.c_int, C.c_float, C.c_float, _P, _P, _I64, _I64, C.c_int, C.c_int, _P],
+    ),
+    "based_gated_delta_scan": (C.c_int, [_P] * 9 + [_I64] * 11 + [C.c_int, C.c_int, _P]),
+    "based_gated_rms_norm": (C.c_int, [_P] * 4 + [_I64] * 8 + [C.c_float, C.c_float, C.c_int, _P]),
+    "based_gated_delta_step": (
+        C.c_int, [_P] * 12 + [_I64] * 8 + [C.c_int] + [_I64] * 7 + [C.c_float, C.c_float, C.c_int, _P]),
+    "based_rglru_prefill": (C.c_int, [_P] * 12 + [_I64] * 10 + [C.c_float, C.c_int, C.c_int, _P]),
+    "based_rglru_step": (C.c_int, [_P] * 13 + [_I64] * 4 + [C.c_int] + [_I64] * 4 + [C.c_float, C.c_int, _P]),
+    "based_decode_linear_stream": (
+        C.c_int,
+        [_P, _I64, _P, _I64, _P, _I64, _P, _P] + [_I64] * 4 + [_P, _I64, _P, _I64, C.c_float, C.c_int, _P, C.c_float,
+                                                              _P, _P, _I64, C.c_int, _P, _I64, C.c_int, _P],
+    ),
     "based_swa_step": (
         C.c_int,
         [_P, _P, _P, _P, _P, _P, _P, _I64] + [_I64] * 3 + [_I64] * 8 + [_I64] * 3
@@ -110,23 +134,54 @@ class BasedHipError(RuntimeError):
     """Raised when the native library is missing or a launch is refused by the runtime."""
 
 
+def part_path(part: str) -> str:
+    """Where the build of one named part of the sources lies."""
+    return os.path.join(_HERE, f"libbased_hip_{part}.so")
+
+
+def use_part(part: str) -> None:
+    """Lets a process that needs only the kernels of `part` run from that part's build where the
+    whole library does not exist.  Entry points the part does not hold raise when they are called."""
+    global _part_path
+    _part_path = part_path(part)
+
+
+def _absent(name):
+    def refuse(*args):
+        raise BasedHipError(f"{name} is not in {_part_path}: build the whole library with `python -m based_amd.build`")
+
+    return refuse
+
+
+class _Entries:
+    """The typed entry points of a loaded library."""
+
+    def __init__(self, handle, partial: bool):
+        for name, (res, args) in SIGNATURES.items():
+            if partial and not hasattr(handle, name):
+                setattr(self, name, _absent(name))
+                continue
+            fn = getattr(handle, name)
+            fn.restype = res
+            fn.argtypes = args
+            setattr(self, name, fn)
+
+
 def lib():
     """Returns the loaded library, loading and typing it on first use."""
     global _lib
     if _lib is None:
         with _lock:
             if _lib is None:
-                if not os.path.exists(LIB_PATH):
+                path = LIB_PATH
+                if not os.path.exists(path) and _part_path is not None:
+                    path = _part_path
+                if not os.path.exists(path):
                     raise BasedHipError(
-                        f"{LIB_PATH} not found: build it with `python -m based_amd.build` "
+                        f"{path} not found: build it with `python -m based_amd.build` "
                         "(there is no non-HIP fallback)"
                     )
-                handle = C.CDLL(LIB_PATH)
-                for name, (res, args) in SIGNATURES.items():
-                    fn = getattr(handle, name)
-                    fn.restype = res
-                    fn.argtypes = args
-                _lib = handle
+                _lib = _Entries(C.CDLL(path), partial=path != LIB_PATH)
     return _lib
 
 

@@ -1,0 +1,112 @@
+"""Sozilix: a decoder-only stack of two kinds of layers on an fp32 residual stream.
+
+    x <- x + m * mixer(h),  h = n + conv(n),  n = layer_norm(x)        (bias-free norm, causal convolution)
+    x <- x + m * swiglu_mlp(layer_norm(x))                             (layers with a feed-forward)
+
+"parallel" layers run grouped sliding-window attention (interleaved rotary positions on leading
+channels, normalised values) and the gated delta rule on the same input; "rglru" layers are the
+recurrent block with a real-gated linear recurrent unit.  Embedding and head are separate matrices.
+"""
+from __future__ import annotations
+
+import torch
+
+from ..mixers.streaming import round_up
+
+RGLRU_DECAY_SCALE = 8.0
+
+
+def _mixer_spec(layer: dict, eps: float) -> dict:
+    m = layer["mixer"]
+    if layer["type"] == "rglru":
+        return {"_target_": "based_amd.mixers.rglru.RGLRU", "width": m["width"], "blocks": m["blocks"], "conv_taps": m["conv"],
+                "decay_scale": RGLRU_DECAY_SCALE}
+    if layer["type"] == "parallel":
+        left, right = m["left"], m["right"]
+        return {
+            "_target_": "based_amd.mixers.side_by_side.SideBySide",
+            "cores": [
+                {"_target_": "based_amd.mixers.window_attention.WindowAttention", "heads": left["heads"], "kv_heads": left["kv_heads"],
+                 "dim": left["dim"], "vdim": left["vdim"], "window": left["mask"]["size"], "scale": left["scale"],
+                 "rotary_dim": left["rot"]["dims"], "rotary_base": left["rot"]["base"], "rotary_interleaved": True,
+                 "value_norm_eps": eps},
+                {"_target_": "based_amd.mixers.gated_delta.GatedDeltaRule", "heads": right["heads"], "kv_heads": right["kv_heads"],
+                 "dim": right["dim"], "vdim": right["vdim"], "conv_taps": right["conv"], "norm_eps": eps},
+            ],
+            "scales": [m["left_scale"], m["right_scale"]],
+        }
+    raise NotImplementedError(f"layer type {layer['type']!r}")
+
+
+def _mlp_spec(layer: dict):
+    mlp = layer["mlp"]
+    if mlp is None:
+        return None
+    if mlp["kind"] != "dense":
+        raise NotImplementedError(f"feed-forward kind {mlp['kind']!r}")
+    return {"hidden": mlp["ff"]}
+
+
+def stack_config(raw: dict) -> dict:
+    """Keywords of StackConfig for a Sozilix config.json."""
+    eps = raw["norm"]["eps"]
+    return dict(
+        n_embd=raw["width"], n_layer=len(raw["layers"]), vocab_size=raw["vocab"], pad_vocab_size_multiple=1,
+        layer_norm_epsilon=eps, stream_norm="layer", residual_in_fp32=True, residual_mult=raw["residual_mult"],
+        input_conv_taps=raw["canon"]["taps"], tie_word_embeddings=False, max_position_embeddings=0,
+        layer_specs=[{"mixer": _mixer_spec(layer, eps), "mlp": _mlp_spec(layer)} for layer in raw["layers"]],
+    )
+
+
+def _stack(parts, to: int = 8):
+    """Matrices or vectors one below the other, each starting on a multiple of `to` rows (zeros between)."""
+    rows = []
+    for p in parts:
+        rows.append(p)
+        gap = round_up(p.shape[0], to) - p.shape[0]
+        if gap:
+            rows.append(p.new_zeros(gap, *p.shape[1:]))
+    return torch.cat(rows)
+
+
+def _beside(parts, to: int = 8):
+    return _stack([p.T for p in parts], to).T.contiguous()
+
+
+def convert_state(raw: dict, w: dict) -> dict:
+    """The stack's state dict from the design's tensors.  Projections that read the same input are
+    stacked, convolution weights turned to (taps, channels)."""
+    out = {
+        "transformer.embeddings.word_embeddings.weight": w["embed"],
+        "transformer.ln_f.weight": w["final.norm"],
+        "lm_head.weight": w["head"],
+    }
+    for i, layer in enumerate(raw["layers"]):
+        src, dst = f"l{i}", f"transformer.layers.{i}"
+        mix = f"{dst}.mixer"
+        out[f"{dst}.norm1.weight"] = w[f"{src}.norm1"]
+        out[f"{dst}.input_conv.weight"] = w[f"{src}.canon1"].T.contiguous()
+        if layer["type"] == "rglru":
+            t = lambda name: w[f"{src}.mix.{name}"]
+            out[f"{mix}.in_proj.weight"] = _stack([t("y"), t("x")])
+            out[f"{mix}.in_proj.bias"] = _stack([t("y.b"), t("x.b")])
+            out[f"{mix}.conv.weight"] = t("conv").T.contiguous()
+            out[f"{mix}.conv.bias"] = t("conv.b")
+            out[f"{mix}.gate_r"], out[f"{mix}.bias_r"] = t("ra"), t("ra.b").reshape(-1)
+            out[f"{mix}.gate_i"], out[f"{mix}.bias_i"] = t("ri"), t("ri.b").reshape(-1)
+            out[f"{mix}.lam"] = t("lam")
+            out[f"{mix}.out_proj.weight"] = _beside([t("o")])
+        else:
+            l = lambda name: w[f"{src}.mix.left.{name}"]
+            r = lambda name: w[f"{src}.mix.right.{name}"]
+            out[f"{mix}.in_proj.weight"] = _stack([l("q"), l("k"), l("v"), r("q"), r("k"), r("v"), r("g"), r("b"), r("a")])
+            out[f"{mix}.out_proj.weight"] = _beside([l("o"), r("o")])
+            delta = f"{mix}.cores.1"
+            out[f"{delta}.conv.weight"] = _stack([r("q.conv"), r("k.conv"), r("v.conv")]).T.contiguous()
+            out[f"{delta}.A_log"], out[f"{delta}.dt_bias"], out[f"{delta}.norm_weight"] = r("A_log"), r("dt_bias"), r("norm")
+        if layer["mlp"] is not None:
+            out[f"{dst}.norm2.weight"] = w[f"{src}.norm2"]
+            # the gate kernels take (value, gate): value * silu(gate)
+            out[f"{dst}.mlp.fc1.weight"] = _stack([w[f"{src}.mlp.up"], w[f"{src}.mlp.gate"]])
+            out[f"{dst}.mlp.fc2.weight"] = _beside([w[f"{src}.mlp.down"]])
+    return out

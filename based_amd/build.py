@@ -67,6 +67,35 @@ def _compile(src: str):
     return obj, usage
 
 
+# Sources a group of models needs, for a machine that serves nothing else: `build_part`.
+PARTS = {
+    "streaming": ("capi", "decode_linear", "gated_conv", "gated_delta", "greedy", "rglru", "stream_norm_conv", "window_attn"),
+}
+
+
+def _link(objs, out: str) -> None:
+    # linked beside its final place and moved there, so that a library that exists is whole
+    tmp = f"{out}.{os.getpid()}.tmp"
+    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", tmp]
+    r = subprocess.run(cmd, capture_output=True, text=True)
+    if r.returncode != 0:
+        raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
+    os.replace(tmp, out)
+
+
+def build_part(part: str) -> str:
+    """Compiles the sources of one part into a library of its own (based_amd/_lib.py: use_part)."""
+    from ._lib import part_path
+
+    os.makedirs(OBJDIR, exist_ok=True)
+    srcs = [os.path.join(CSRC, f"{name}.hip") for name in PARTS[part]]
+    with cf.ThreadPoolExecutor(max_workers=min(8, len(srcs))) as ex:
+        objs = [o for o, _ in ex.map(_compile, srcs)]
+    out = part_path(part)
+    _link(objs, out)
+    return out
+
+
 def build(verbose: bool = False) -> str:
     os.makedirs(OBJDIR, exist_ok=True)
     srcs = sorted(glob.glob(os.path.join(CSRC, "*.hip")))
@@ -85,10 +114,7 @@ def build(verbose: bool = False) -> str:
         for name, u in kernels.items():
             if u.get("VGPRs Spill", 0) > 0:
                 sys.stderr.write(f"note: {src}: {name} spills {u['VGPRs Spill']} vector registers\n")
-    cmd = [HIPCC, "--offload-arch=gfx950", "-shared", "-fPIC", *objs, "-o", LIB]
-    r = subprocess.run(cmd, capture_output=True, text=True)
-    if r.returncode != 0:
-        raise RuntimeError(f"link failed:\n{r.stdout}\n{r.stderr}")
+    _link(objs, LIB)
     if verbose:
         print(f"built {LIB} from {len(srcs)} sources")
     return LIB

@@ -18,7 +18,11 @@
 //     workgroup forms r = x + residual and its norm; workgroup 0 writes r out for the next block;
 //     the rows of x can be gathered through an index (the token embedding lookup of the first
 //     block);
-//   * the SwiGLU gate between fc1 and fc2 (mlp.py:147-151).
+//   * the SwiGLU gate between fc1 and fc2 (mlp.py:147-151);
+//   * the streamed-input prologue (based_decode_linear_stream): residual + mult * x in fp32, layer or
+//     RMS norm of that sum, and h + causal convolution of h on a ring of past norm outputs.  Every
+//     workgroup reads the ring; workgroup 0 writes the current row into the slot of its position,
+//     which no reader of the same step looks at.
 // What FOLLOWS a projection whose output is consumed in (value, gate) pairs runs in its tail: a
 // wavefront then takes R/2 rows of the value half of the weight and the R/2 matching rows of the
 // gate half, so that after the sums one lane holds both numbers of an output element, and
@@ -28,6 +32,8 @@
 //     one owner here,
 // is applied to the bf16-rounded pair before anything is stored.
 // All of them use the arithmetic (and the roundings to bf16) of the stand-alone kernels.
+#include <initializer_list>
+
 #include "common.hpp"
 
 namespace based {
@@ -55,6 +61,17 @@ struct DecodeLinearArgs {
   const __bf16* conv_w;
   const __bf16* conv_b;
   int conv_k, conv_state_f32, m0;
+  // streamed-input prologue: residual + mult * x, layer or RMS norm of the fp32 sum, and the causal
+  // convolution on the ring of past norm outputs (ic_taps = 0: none); rows of pos / ic_ring are
+  // counted from the first row of the whole call
+  float mult;
+  int norm_kind;
+  const __bf16* ic_w;  // (taps, K)
+  __bf16* ic_ring;     // (rows, taps, K)
+  long ic_ring_sr;
+  int ic_taps;
+  const int32_t* pos;
+  int pos_host;
 };
 
 typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
@@ -126,7 +143,8 @@ __device__ __forceinline__ float wave_sum_dpp(float x) {
 
 __device__ __forceinline__ float silu_f(float a) { return a / (1.0f + __expf(-a)); }
 
-enum { kProNone = BASED_PROLOGUE_NONE, kProNorm = BASED_PROLOGUE_ADD_RMS_NORM, kProSwiglu = BASED_PROLOGUE_SWIGLU };
+enum { kProNone = BASED_PROLOGUE_NONE, kProNorm = BASED_PROLOGUE_ADD_RMS_NORM, kProSwiglu = BASED_PROLOGUE_SWIGLU,
+       kProStream = 3 };
 enum { kEpiNone = BASED_EPILOGUE_NONE, kEpiSwiglu = BASED_EPILOGUE_SWIGLU, kEpiConv = BASED_EPILOGUE_GATED_CONV_STEP };
 
 __device__ __forceinline__ void lds_barrier() {
@@ -264,6 +282,88 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
         float o[8];
 #pragma unroll
         for (int i = 0; i < 8; ++i) o[i] = v[c][i] * rstd * to_f32(nw[c][i]);
+        xs[m][c][lane] = u32x4{pack_bf16(o[0], o[1]), pack_bf16(o[2], o[3]), pack_bf16(o[4], o[5]), pack_bf16(o[6], o[7])};
+      }
+    }
+  } else if constexpr (PRO == kProStream) {
+#pragma unroll
+    for (int m = wave; m < MT; m += WV)
+    if (m < a.M) {
+      bool poison;
+      const __bf16* xrow = x_row(m, poison);
+      const bool has_res = a.res_in != nullptr;
+      const float mult = has_res ? a.mult : 1.0f;
+      const int pos = a.ic_taps > 0 ? (a.pos != nullptr ? a.pos[a.m0 + m] : a.pos_host) : 0;
+      float v[C][8], nw[C][8];
+      float sum = 0.f;
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        const bf16x8 h = *reinterpret_cast<const bf16x8*>(live[c] ? xrow + e0[c] : zeros);
+        const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.norm_w + e0[c] : zeros);
+        const float* rp = has_res && live[c] ? a.res_in + (long)m * a.ri_sr + e0[c] : reinterpret_cast<const float*>(kZeroPage);
+        const f32x4 r0 = reinterpret_cast<const f32x4*>(rp)[0], r1 = reinterpret_cast<const f32x4*>(rp)[1];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          nw[c][i] = to_f32(w8[i]);
+          v[c][i] = __builtin_fmaf(mult, to_f32(h[i]), i < 4 ? r0[i & 3] : r1[i & 3]);
+          sum += v[c][i];
+        }
+      }
+      // the ring rows of the past inputs, in flight during the reductions
+      constexpr int kMaxPast = BASED_STREAM_MAX_TAPS - 1;
+      float past[C][8];
+#pragma unroll
+      for (int c = 0; c < C; ++c)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) past[c][i] = 0.f;
+      const __bf16* ring = a.ic_ring + (long)(a.m0 + m) * a.ic_ring_sr;
+#pragma unroll 1
+      for (int j = 0; j < kMaxPast; ++j) {
+        const int p = pos - (a.ic_taps - 1) + j;
+        if (j >= a.ic_taps - 1) break;
+        if (p < 0) continue;
+#pragma unroll
+        for (int c = 0; c < C; ++c) {
+          const bf16x8 x8 = *reinterpret_cast<const bf16x8*>(live[c] ? ring + (long)(p % a.ic_taps) * a.K + e0[c] : zeros);
+          const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.ic_w + (long)j * a.K + e0[c] : zeros);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) past[c][i] = __builtin_fmaf(to_f32(w8[i]), to_f32(x8[i]), past[c][i]);
+        }
+      }
+      const float mean = a.norm_kind == BASED_NORM_LAYER ? wave_sum_dpp(sum) / (float)a.K : 0.f;
+      float ss = 0.f;
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        if (a.res_out != nullptr && wg == 0 && live[c]) {
+          float* op = a.res_out + (long)m * a.ro_sr + e0[c];
+          reinterpret_cast<f32x4*>(op)[0] = f32x4{v[c][0], v[c][1], v[c][2], v[c][3]};
+          reinterpret_cast<f32x4*>(op)[1] = f32x4{v[c][4], v[c][5], v[c][6], v[c][7]};
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+          v[c][i] = live[c] ? v[c][i] - mean : 0.f;
+          ss = __builtin_fmaf(v[c][i], v[c][i], ss);
+        }
+      }
+      ss = wave_sum_dpp(ss);
+      float rstd = 1.0f / sqrtf(ss / (float)a.K + a.eps);
+      if (poison) rstd = __builtin_nanf("");
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        bf16x8 h;
+        float o[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) h[i] = from_f32<__bf16>(v[c][i] * rstd * nw[c][i]);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) o[i] = to_f32(h[i]);
+        if (a.ic_taps > 0) {
+          const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.ic_w + (long)(a.ic_taps - 1) * a.K + e0[c] : zeros);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) o[i] += __builtin_fmaf(to_f32(w8[i]), o[i], past[c][i]);
+          // a slot that no reader of this step looks at
+          if (wg == 0 && live[c] && pos >= 0)
+            *reinterpret_cast<bf16x8*>(a.ic_ring + (long)(a.m0 + m) * a.ic_ring_sr + (long)(pos % a.ic_taps) * a.K + e0[c]) = h;
+        }
         xs[m][c][lane] = u32x4{pack_bf16(o[0], o[1]), pack_bf16(o[2], o[3]), pack_bf16(o[4], o[5]), pack_bf16(o[6], o[7])};
       }
     }
@@ -440,6 +540,8 @@ void launch_decode_linear_pro(const DecodeLinearArgs& a, int prologue, hipStream
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProNone, EPI>), grid, block, 0, s, a);
   } else if (prologue == kProNorm) {
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProNorm, EPI>), grid, block, 0, s, a);
+  } else if (prologue == kProStream) {
+    if constexpr (EPI != kEpiConv) hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProStream, EPI>), grid, block, 0, s, a);
   } else if constexpr (EPI == kEpiNone) {
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProSwiglu, EPI>), grid, block, 0, s, a);
   }
@@ -477,6 +579,24 @@ static bool ranges_overlap(const void* a, int64_t na, const void* b, int64_t nb)
   if (a == nullptr || b == nullptr || na <= 0 || nb <= 0) return false;
   const uintptr_t a0 = reinterpret_cast<uintptr_t>(a), b0 = reinterpret_cast<uintptr_t>(b);
   return a0 < b0 + (uintptr_t)nb && b0 < a0 + (uintptr_t)na;
+}
+
+static bool aligned16_all(std::initializer_list<const void*> ps) {
+  uintptr_t bits = 0;
+  for (const void* p : ps) bits |= reinterpret_cast<uintptr_t>(p);
+  return (bits & 15) == 0;
+}
+
+static void launch_decode_linear_chunks(const DecodeLinearArgs& a, int prologue, int epilogue, hipStream_t s) {
+  const int chunks = (a.K + 511) / 512;
+  if (chunks <= 1)
+    launch_decode_linear<1>(a, prologue, epilogue, s);
+  else if (chunks <= 2)
+    launch_decode_linear<2>(a, prologue, epilogue, s);
+  else if (chunks <= 4)
+    launch_decode_linear<4>(a, prologue, epilogue, s);
+  else
+    launch_decode_linear<8>(a, prologue, epilogue, s);
 }
 
 }  // namespace based
@@ -548,7 +668,7 @@ extern "C" BASED_API int based_decode_linear(const void* x, int64_t x_row_stride
                   BASED_ERR_ARG, "decode_linear: an output (y, residual_out) overlaps an input or the other output");
   }
 
-  DecodeLinearArgs a;
+  DecodeLinearArgs a = {};
   a.x_sr = x_row_stride;
   a.x_index_rows = x_index_rows;
   a.w = static_cast<const __bf16*>(weight);
@@ -568,7 +688,6 @@ extern "C" BASED_API int based_decode_linear(const void* x, int64_t x_row_stride
   a.conv_k = conv_k;
   a.conv_state_f32 = conv_state_dtype == BASED_F32;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const int chunks = (int)((K + 511) / 512);
   a.M = (int)M;
   a.m0 = 0;
   a.x = static_cast<const __bf16*>(x);
@@ -576,13 +695,76 @@ extern "C" BASED_API int based_decode_linear(const void* x, int64_t x_row_stride
   a.y = static_cast<__bf16*>(y);
   a.res_in = residual_in;
   a.res_out = residual_out;
-  if (chunks <= 1)
-    launch_decode_linear<1>(a, prologue, epilogue, s);
-  else if (chunks <= 2)
-    launch_decode_linear<2>(a, prologue, epilogue, s);
-  else if (chunks <= 4)
-    launch_decode_linear<4>(a, prologue, epilogue, s);
-  else
-    launch_decode_linear<8>(a, prologue, epilogue, s);
+  launch_decode_linear_chunks(a, prologue, epilogue, s);
   return check_launch("decode_linear");
+}
+
+extern "C" BASED_API int based_decode_linear_stream(const void* x, int64_t x_row_stride, const int64_t* x_row_index, int64_t x_index_rows,
+                                                    const void* weight, int64_t w_row_stride, const void* bias, void* y,
+                                                    int64_t y_row_stride, int64_t M, int64_t N, int64_t K, const float* residual_in,
+                                                    int64_t ri_row_stride, float* residual_out, int64_t ro_row_stride, float mult,
+                                                    int norm_kind, const void* norm_weight, float eps, const void* conv_weight,
+                                                    void* conv_ring, int64_t conv_ring_row_stride, int taps, const int32_t* pos,
+                                                    int64_t pos_host, int epilogue, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x && weight && y && norm_weight, BASED_ERR_ARG, "decode_linear_stream: null pointer argument");
+  BASED_REQUIRE(M >= 0 && N > 0 && K > 0 && pos_host >= 0 && pos_host < (1ll << 31), BASED_ERR_ARG, "decode_linear_stream: bad sizes");
+  BASED_REQUIRE(M <= BASED_DECODE_LINEAR_MAX_ROWS, BASED_ERR_SHAPE, "decode_linear_stream: %ld activation rows, at most %d", (long)M,
+                BASED_DECODE_LINEAR_MAX_ROWS);
+  BASED_REQUIRE(K % 8 == 0 && K <= 4096, BASED_ERR_SHAPE,
+                "decode_linear_stream: contraction length %ld unsupported (multiple of 8, at most 4096)", (long)K);
+  BASED_REQUIRE(N < (1ll << 30), BASED_ERR_SHAPE, "decode_linear_stream: too many output features");
+  BASED_REQUIRE(norm_kind == BASED_NORM_RMS || norm_kind == BASED_NORM_LAYER, BASED_ERR_ARG, "decode_linear_stream: unknown norm %d", norm_kind);
+  BASED_REQUIRE(epilogue == kEpiNone || epilogue == kEpiSwiglu, BASED_ERR_ARG, "decode_linear_stream: unknown epilogue %d", epilogue);
+  BASED_REQUIRE(epilogue == kEpiNone || (N % 2 == 0 && K <= 2048), BASED_ERR_SHAPE,
+                "decode_linear_stream: the paired epilogue takes an even number of rows of up to 2048 elements");
+  BASED_REQUIRE(taps >= 0 && taps <= BASED_STREAM_MAX_TAPS, BASED_ERR_SHAPE, "decode_linear_stream: %d taps (0 to %d)", taps,
+                BASED_STREAM_MAX_TAPS);
+  BASED_REQUIRE(taps == 0 || (conv_weight && conv_ring), BASED_ERR_ARG, "decode_linear_stream: the convolution needs weight and ring");
+  BASED_REQUIRE(x_row_index == nullptr || x_index_rows > 0, BASED_ERR_ARG,
+                "decode_linear_stream: a row index needs the number of rows it may address");
+  BASED_REQUIRE(x_row_stride % 8 == 0 && w_row_stride % 8 == 0 && ri_row_stride % 4 == 0 && ro_row_stride % 4 == 0 &&
+                    conv_ring_row_stride % 8 == 0,
+                BASED_ERR_ALIGN, "decode_linear_stream: rows must be whole 16-byte pieces");
+  BASED_REQUIRE(aligned16_all({x, weight, residual_in, residual_out, norm_weight, conv_weight, conv_ring}), BASED_ERR_ALIGN,
+                "decode_linear_stream: tensors must be 16-byte aligned");
+  if (M == 0) return BASED_OK;
+  {
+    const int64_t x_bytes = (((x_row_index ? x_index_rows : M) - 1) * x_row_stride + K) * 2;
+    const int64_t ri_bytes = ((M - 1) * ri_row_stride + K) * 4, ro_bytes = ((M - 1) * ro_row_stride + K) * 4;
+    const int64_t y_bytes = ((M - 1) * y_row_stride + (epilogue == kEpiNone ? N : N / 2)) * 2;
+    BASED_REQUIRE(!ranges_overlap(residual_out, ro_bytes, residual_in, ri_bytes) && !ranges_overlap(residual_out, ro_bytes, x, x_bytes) &&
+                      !ranges_overlap(y, y_bytes, x, x_bytes) && !ranges_overlap(y, y_bytes, residual_in, ri_bytes) &&
+                      !ranges_overlap(y, y_bytes, residual_out, ro_bytes),
+                  BASED_ERR_ARG, "decode_linear_stream: an output (y, residual_out) overlaps an input or the other output");
+  }
+  DecodeLinearArgs a = {};
+  a.x = static_cast<const __bf16*>(x);
+  a.x_sr = x_row_stride;
+  a.x_index = x_row_index;
+  a.x_index_rows = x_index_rows;
+  a.w = static_cast<const __bf16*>(weight);
+  a.w_sr = w_row_stride;
+  a.bias = static_cast<const __bf16*>(bias);
+  a.y = static_cast<__bf16*>(y);
+  a.y_sr = y_row_stride;
+  a.M = (int)M;
+  a.N = (int)N;
+  a.K = (int)K;
+  a.res_in = residual_in;
+  a.ri_sr = ri_row_stride;
+  a.res_out = residual_out;
+  a.ro_sr = ro_row_stride;
+  a.norm_w = static_cast<const __bf16*>(norm_weight);
+  a.eps = eps;
+  a.mult = mult;
+  a.norm_kind = norm_kind;
+  a.ic_w = static_cast<const __bf16*>(conv_weight);
+  a.ic_ring = static_cast<__bf16*>(conv_ring);
+  a.ic_ring_sr = conv_ring_row_stride;
+  a.ic_taps = taps;
+  a.pos = pos;
+  a.pos_host = (int)pos_host;
+  launch_decode_linear_chunks(a, kProStream, epilogue, static_cast<hipStream_t>(stream));
+  return check_launch("decode_linear_stream");
 }

@@ -1,0 +1,664 @@
+// Causal softmax attention over a sliding window of any size with grouped heads, for gfx950:
+// position i attends j with 0 <= i - j < window; query head h reads key/value head h / (H / G);
+// key and value sizes may differ.  In the same launches: rotary positions on the leading
+// rotary_dim channels of q and k (interleaved pairs (2i, 2i + 1), or half-split pairs
+// (i, i + rotary_dim / 2)) and the value norm v / sqrt(mean(v^2) + eps).
+//
+// The cache holds one row per token and key/value head: dim key channels (rotated), then vdim
+// value channels (normalised), (B, S, G, dim + vdim).
+//
+//   window_kv_write      a portion's keys and values into the cache
+//   window_prefill_mfma  bf16: 128 (token, head) rows per workgroup, 32 per wavefront.  The heads of
+//                        a group are rows of the same tile, so that a key tile is fetched once for
+//                        all of them and a tile of tokens is short against the window.  Scores are
+//                        formed transposed (keys x queries), which leaves the weights in the lanes
+//                        that the product with the values wants them in.
+//   window_prefill_any   any element type and size: one wavefront per query
+//   window_step          one token per sequence: rotation, value norm, cache write and attention,
+//                        one workgroup per (sequence, key/value head)
+#include "stream_common.hpp"
+
+namespace based {
+
+struct WindowArgs {
+  const void* q;
+  const void* k;
+  const void* v;
+  void* kv;
+  void* o;
+  const float* cos_t;  // (n_pos, rot / 2) or null
+  const float* sin_t;
+  const int32_t* pos;
+  int pos_host, n_pos;
+  int B, L, H, G, d, dv, S;
+  long q_sb, q_sl, k_sb, k_sl, v_sb, v_sl, o_sb, o_sl;  // heads are contiguous blocks of d / dv
+  long kv_sb, kv_st;
+  int rot, half_split, window, norm_v;
+  float scale, eps, out_scale;
+};
+
+// partner and sign of channel c in the rotation: x'_c = x_c cos + sgn * x_partner sin
+__device__ __forceinline__ void rope_pair(int c, int rot, int half_split, int& pair, int& partner, float& sgn) {
+  if (half_split) {
+    const int h = rot / 2;
+    pair = c < h ? c : c - h;
+    partner = c < h ? c + h : c - h;
+    sgn = c < h ? -1.f : 1.f;
+  } else {
+    pair = c >> 1;
+    partner = c ^ 1;
+    sgn = (c & 1) ? 1.f : -1.f;
+  }
+}
+
+template <typename T>
+__device__ __forceinline__ float rotated(const T* row, int c, int pos, const WindowArgs& a) {
+  const float x = to_f32(row[c]);
+  if (c >= a.rot) return x;
+  int pair, partner;
+  float sgn;
+  rope_pair(c, a.rot, a.half_split, pair, partner, sgn);
+  const long t = (long)pos * (a.rot / 2) + pair;
+  return x * a.cos_t[t] + sgn * to_f32(row[partner]) * a.sin_t[t];
+}
+
+// One wavefront per (token, key/value head).
+template <typename T>
+__global__ __launch_bounds__(256) void window_kv_write_kernel(const WindowArgs a) {
+  const long item = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (item >= (long)a.B * a.L * a.G) return;
+  const int lane = threadIdx.x & 63;
+  const int g = (int)(item % a.G);
+  const long bl = item / a.G;
+  const int l = (int)(bl % a.L), b = (int)(bl / a.L);
+  const int pos = a.pos_host + l;
+  const T* k = static_cast<const T*>(a.k) + b * a.k_sb + l * a.k_sl + (long)g * a.d;
+  const T* v = static_cast<const T*>(a.v) + b * a.v_sb + l * a.v_sl + (long)g * a.dv;
+  T* out = static_cast<T*>(a.kv) + b * a.kv_sb + pos * a.kv_st + (long)g * (a.d + a.dv);
+  float ss = 0.f;
+  for (int c = lane; c < a.dv; c += 64) ss = __builtin_fmaf(to_f32(v[c]), to_f32(v[c]), ss);
+  const float r = a.norm_v ? 1.0f / sqrtf(wave_sum(ss) / (float)a.dv + a.eps) : 1.0f;
+  for (int c = lane; c < a.d; c += 64) out[c] = from_f32<T>(rotated(k, c, pos, a));
+  for (int c = lane; c < a.dv; c += 64) out[a.d + c] = from_f32<T>(to_f32(v[c]) * r);
+}
+
+// The same with 16-byte pieces: 16 lanes per (token, key/value head), interleaved pairs or none.
+// d, dv and every stride multiples of 8, pointers 16-byte aligned; d, dv <= 256.
+__global__ __launch_bounds__(256) void window_kv_write_vec_kernel(const WindowArgs a) {
+  const long item0 = (long)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const long n_items = (long)a.B * a.L * a.G;
+  const bool live = item0 < n_items;
+  const long item = live ? item0 : n_items - 1;
+  const int lane = threadIdx.x & 15;
+  const int g = (int)(item % a.G);
+  const long bl = item / a.G;
+  const int l = (int)(bl % a.L), b = (int)(bl / a.L);
+  const int pos = a.pos_host + l;
+  const __bf16* k = static_cast<const __bf16*>(a.k) + b * a.k_sb + l * a.k_sl + (long)g * a.d;
+  const __bf16* v = static_cast<const __bf16*>(a.v) + b * a.v_sb + l * a.v_sl + (long)g * a.dv;
+  __bf16* out = static_cast<__bf16*>(a.kv) + b * a.kv_sb + pos * a.kv_st + (long)g * (a.d + a.dv);
+  float x[2][8], y[2][8];
+  float ss = 0.f;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int c = (i * 16 + lane) * 8;
+    load_vec<__bf16, 8>(k + (c < a.d ? c : 0), x[i]);
+    load_vec<__bf16, 8>(v + (c < a.dv ? c : 0), y[i]);
+    if (c < a.dv) {
+#pragma unroll
+      for (int j = 0; j < 8; ++j) ss = __builtin_fmaf(y[i][j], y[i][j], ss);
+    }
+  }
+  const float r = a.norm_v ? 1.0f / sqrtf(sum16(ss) / (float)a.dv + a.eps) : 1.0f;
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int c = (i * 16 + lane) * 8;
+#pragma unroll
+    for (int j = 0; j < 8; j += 2) {
+      if (c + j < a.rot) {
+        const long t = (long)pos * (a.rot / 2) + (c + j) / 2;
+        const float cs = a.cos_t[t], sn = a.sin_t[t], u0 = x[i][j], u1 = x[i][j + 1];
+        x[i][j] = u0 * cs - u1 * sn;
+        x[i][j + 1] = u1 * cs + u0 * sn;
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < 8; ++j) y[i][j] *= r;
+    if (live && c < a.d) store_vec<__bf16, 8>(out + c, x[i]);
+    if (live && c < a.dv) store_vec<__bf16, 8>(out + a.d + c, y[i]);
+  }
+}
+
+// ---- prefill, bf16, MFMA ----
+// KC: 32-channel pieces of the key size; VC: 32-channel pieces of the value size (both rounded up;
+// channels past the real sizes are zeros).
+constexpr int kTileKeys = 64;
+constexpr int kTileRows = 128;  // (token, head) rows per workgroup
+
+__device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) {
+  return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
+}
+
+template <int KC, int VC>
+__global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowArgs a) {
+  constexpr int D = KC * 32, DV = VC * 32;
+  constexpr int KS = D + 8, VS = kTileKeys + 8;  // LDS row strides: 16-lane reads of 16 bytes meet every bank once
+  __shared__ __attribute__((aligned(16))) __bf16 lds_k[kTileKeys * KS];
+  __shared__ __attribute__((aligned(16))) __bf16 lds_v[DV * VS];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int bg = blockIdx.y, b = bg / a.G, g = bg % a.G;
+  const int qpk = a.H / a.G;
+  const int n_rows = a.L * qpk;
+  const int r0 = blockIdx.x * kTileRows;
+  const int r_end = r0 + kTileRows < n_rows ? r0 + kTileRows : n_rows;
+  const int row_w = r0 + wave * 32;  // first row of this wavefront
+  const __bf16* kv = static_cast<const __bf16*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
+
+  // queries: lane holds channels quad*8 + 32 c .. of row l16 (+16): the MFMA's second operand
+  bf16x8 qf[2][KC];
+  int qpos[2], qtok[2], qhead[2];
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    const int row = row_w + t * 16 + l16;
+    const int rr = row < n_rows ? row : n_rows - 1;
+    qtok[t] = rr / qpk;
+    qhead[t] = g * qpk + rr % qpk;
+    qpos[t] = a.pos_host + qtok[t];
+    const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + qtok[t] * a.q_sl + (long)qhead[t] * a.d;
+#pragma unroll
+    for (int c = 0; c < KC; ++c) {
+      const int e = c * 32 + quad * 8;
+      float x[8];
+      load_vec<__bf16, 8>(qp + (e < a.d ? e : 0), x);
+      if (a.half_split && e < a.rot) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = rotated(qp, e + j, qpos[t], a);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 8; j += 2)
+          if (e + j < a.rot) {
+            const long ti = (long)qpos[t] * (a.rot / 2) + (e + j) / 2;
+            const float cs = a.cos_t[ti], sn = a.sin_t[ti], u0 = x[j], u1 = x[j + 1];
+            x[j] = u0 * cs - u1 * sn;
+            x[j + 1] = u1 * cs + u0 * sn;
+          }
+      }
+#pragma unroll
+      for (int j = 0; j < 8; ++j) qf[t][c][j] = (__bf16)(e < a.d ? x[j] : 0.f);
+    }
+  }
+  const int wave_lo_tok = a.pos_host + (row_w < n_rows ? row_w : n_rows - 1) / qpk;
+  const int wave_hi_row = row_w + 31 < n_rows ? row_w + 31 : n_rows - 1;
+  const int wave_hi_tok = a.pos_host + wave_hi_row / qpk;
+
+  f32x4 acc[2][2 * VC];
+#pragma unroll
+  for (int t = 0; t < 2; ++t)
+#pragma unroll
+    for (int i = 0; i < 2 * VC; ++i) acc[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
+  float m_run[2] = {-INFINITY, -INFINITY}, l_run[2] = {0.f, 0.f};
+
+  const int first_pos = a.pos_host + r0 / qpk, last_pos = a.pos_host + (r_end - 1) / qpk;
+  const int lo = first_pos - a.window + 1 > 0 ? first_pos - a.window + 1 : 0;
+
+  // staging: keys as 16-byte pieces of rows; values as 4 keys x 8 channels, turned on the way
+  constexpr int KP = kTileKeys * (D / 8) / 256;  // pieces per thread
+  constexpr int VP = 16 * (DV / 8) / 256 > 0 ? 16 * (DV / 8) / 256 : 1;
+  typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
+  u32x4 kbuf[KP];
+  u32x4 vbuf[VP][4];
+  const u32x4 zero4 = {0u, 0u, 0u, 0u};
+  auto fetch = [&](int k0) {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
+      const bool ok = k0 + key <= last_pos && e < a.d;
+      const u32x4 x = *reinterpret_cast<const u32x4*>(kv + (long)(ok ? k0 + key : lo) * a.kv_st + (ok ? e : 0));
+      kbuf[i] = ok ? x : zero4;
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int p = i * 256 + tid, k4 = p & 15, e = (p >> 4) * 8;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const int key = k0 + k4 * 4 + r;
+        const bool ok = key <= last_pos && e < a.dv;
+        const u32x4 x = *reinterpret_cast<const u32x4*>(kv + (long)(ok ? key : lo) * a.kv_st + a.d + (ok ? e : 0));
+        vbuf[i][r] = ok ? x : zero4;
+      }
+    }
+  };
+  auto stage = [&]() {
+#pragma unroll
+    for (int i = 0; i < KP; ++i) {
+      const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
+      *reinterpret_cast<u32x4*>(&lds_k[key * KS + e]) = kbuf[i];
+    }
+#pragma unroll
+    for (int i = 0; i < VP; ++i) {
+      const int p = i * 256 + tid, k4 = p & 15, e = (p >> 4) * 8;
+      if (e < DV) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) {
+          bf16x4 col;
+#pragma unroll
+          for (int r = 0; r < 4; ++r) col[r] = __builtin_bit_cast(bf16x8, vbuf[i][r])[j];
+          *reinterpret_cast<bf16x4*>(&lds_v[(e + j) * VS + k4 * 4]) = col;
+        }
+      }
+    }
+  };
+
+  fetch(lo);
+  for (int k0 = lo; k0 <= last_pos; k0 += kTileKeys) {
+    __syncthreads();  // every wavefront is done with the tile before
+    stage();
+    __syncthreads();
+    if (k0 + kTileKeys <= last_pos) fetch(k0 + kTileKeys);
+    // does any row of this wavefront see a key of this tile?
+    if (k0 > wave_hi_tok || k0 + kTileKeys - 1 <= wave_lo_tok - a.window) continue;
+    f32x4 s[2][4];
+#pragma unroll
+    for (int kt = 0; kt < 4; ++kt) {
+#pragma unroll
+      for (int t = 0; t < 2; ++t) s[t][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int c = 0; c < KC; ++c) {
+        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(&lds_k[(kt * 16 + l16) * KS + c * 32 + quad * 8]);
+#pragma unroll
+        for (int t = 0; t < 2; ++t) s[t][kt] = mfma_bf16(kf, qf[t][c], s[t][kt]);
+      }
+    }
+    bf16x8 pf[2][2];
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+      float mx = -INFINITY;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int dist = qpos[t] - (k0 + kt * 16 + quad * 4 + i);
+          const float sc = dist >= 0 && dist < a.window ? s[t][kt][i] * a.scale : -INFINITY;
+          s[t][kt][i] = sc;
+          mx = fmaxf(mx, sc);
+        }
+      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+      const float m_new = fmaxf(m_run[t], mx);
+      const float m_use = m_new == -INFINITY ? 0.f : m_new;  // no key seen yet: every weight is exp(-inf) = 0
+      const float alpha = __expf(m_run[t] - m_use);
+      m_run[t] = m_new;
+      float sum = 0.f;
+#pragma unroll
+      for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const float p = __expf(s[t][kt][i] - m_use);
+          sum += p;
+          pf[t][kt >> 1][(kt & 1) * 4 + i] = (__bf16)p;
+        }
+      l_run[t] = l_run[t] * alpha + sum;  // this lane's keys; the four lane groups are added at the end
+#pragma unroll
+      for (int i = 0; i < 2 * VC; ++i) acc[t][i] *= alpha;
+    }
+#pragma unroll
+    for (int i = 0; i < 2 * VC; ++i)
+#pragma unroll
+      for (int h = 0; h < 2; ++h) {
+        const __bf16* vp = &lds_v[(i * 16 + l16) * VS + h * 32 + quad * 4];
+        const bf16x4 v0 = *reinterpret_cast<const bf16x4*>(vp), v1 = *reinterpret_cast<const bf16x4*>(vp + 16);
+        const bf16x8 vf = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
+#pragma unroll
+        for (int t = 0; t < 2; ++t) acc[t][i] = mfma_bf16(vf, pf[t][h], acc[t][i]);
+      }
+  }
+#pragma unroll
+  for (int t = 0; t < 2; ++t) {
+    float l = l_run[t];
+    l += __shfl_xor(l, 16, 64);
+    l += __shfl_xor(l, 32, 64);
+    const float inv = a.out_scale / l;
+    if (row_w + t * 16 + l16 < n_rows) {
+      __bf16* op = static_cast<__bf16*>(a.o) + b * a.o_sb + qtok[t] * a.o_sl + (long)qhead[t] * a.dv;
+#pragma unroll
+      for (int i = 0; i < 2 * VC; ++i) {
+        const int e = i * 16 + quad * 4;
+        if (e < a.dv) {
+          bf16x4 o;
+#pragma unroll
+          for (int j = 0; j < 4; ++j) o[j] = (__bf16)(acc[t][i][j] * inv);
+          *reinterpret_cast<bf16x4*>(op + e) = o;
+        }
+      }
+    }
+  }
+}
+
+// ---- prefill, any element type and any sizes: one wavefront per (token, query head) ----
+constexpr int kAnyMaxDim = 512;  // largest key / value size
+
+template <typename T>
+__global__ __launch_bounds__(64) void window_prefill_any_kernel(const WindowArgs a) {
+  __shared__ float qs[kAnyMaxDim];
+  __shared__ float ps[64];
+  const int lane = threadIdx.x, l = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int g = h / (a.H / a.G), pos = a.pos_host + l;
+  const T* q = static_cast<const T*>(a.q) + b * a.q_sb + l * a.q_sl + (long)h * a.d;
+  const T* kv = static_cast<const T*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
+  for (int c = lane; c < a.d; c += 64) qs[c] = round_to<T>(rotated(q, c, pos, a));
+  float acc[kAnyMaxDim / 64];
+#pragma unroll
+  for (int i = 0; i < kAnyMaxDim / 64; ++i) acc[i] = 0.f;
+  float m_run = -INFINITY, l_run = 0.f;
+  const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  __syncthreads();
+  for (int k0 = lo; k0 <= pos; k0 += 64) {
+    const int key = k0 + lane;
+    float s = -INFINITY;
+    if (key <= pos) {
+      const T* kr = kv + (long)key * a.kv_st;
+      float dot = 0.f;
+      for (int c = 0; c < a.d; ++c) dot = __builtin_fmaf(qs[c], to_f32(kr[c]), dot);
+      s = dot * a.scale;
+    }
+    float mx = s;
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) mx = fmaxf(mx, __shfl_xor(mx, m, 64));
+    const float m_new = fmaxf(m_run, mx);
+    const float alpha = expf(m_run - m_new), p = expf(s - m_new);
+    m_run = m_new;
+    l_run = l_run * alpha + wave_sum(p);
+    __syncthreads();
+    ps[lane] = p;
+    __syncthreads();
+    const int n = pos - k0 + 1 < 64 ? pos - k0 + 1 : 64;
+#pragma unroll
+    for (int i = 0; i < kAnyMaxDim / 64; ++i) {
+      const int c = i * 64 + lane;
+      if (c < a.dv) {
+        float v = acc[i] * alpha;
+        for (int j = 0; j < n; ++j) v = __builtin_fmaf(ps[j], to_f32(kv[(long)(k0 + j) * a.kv_st + a.d + c]), v);
+        acc[i] = v;
+      }
+    }
+  }
+  T* o = static_cast<T*>(a.o) + b * a.o_sb + l * a.o_sl + (long)h * a.dv;
+  const float inv = a.out_scale / l_run;
+#pragma unroll
+  for (int i = 0; i < kAnyMaxDim / 64; ++i) {
+    const int c = i * 64 + lane;
+    if (c < a.dv) o[c] = from_f32<T>(acc[i] * inv);
+  }
+}
+
+// ---- one token per sequence ----
+constexpr int kStepThreads = 256;
+constexpr int kStepKeys = 256;  // keys per round of the running softmax
+
+// QT: query heads of the group served together (the group is walked QT heads at a time).
+// VEC: 16-byte pieces of the rows (sizes and strides multiples of the piece); otherwise element by element.
+template <typename T, int QT, bool VEC>
+__global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowArgs a) {
+  constexpr int N = VEC ? Pack<T>::kN : 1;
+  extern __shared__ float smem[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int b = blockIdx.x / a.G, g = blockIdx.x % a.G;
+  const int qpk = a.H / a.G;
+  const int pos = row_pos(a.pos, a.pos_host, b);
+  if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;  // a position the cache does not hold
+  float* qs = smem;                        // [QT][d]
+  float* sc = qs + QT * a.d;               // [QT][kStepKeys]
+  float* stat = sc + QT * kStepKeys;       // [3][QT]: running maximum, running sum, rescale of this round
+  float* part = stat + 3 * QT;             // [kStepThreads][N], reduction of the output (16-byte aligned: see the launch)
+  part += (4 - ((QT * a.d + QT * kStepKeys + 3 * QT) & 3)) & 3;
+  const T* k = static_cast<const T*>(a.k) + b * a.k_sb + (long)g * a.d;
+  const T* v = static_cast<const T*>(a.v) + b * a.v_sb + (long)g * a.dv;
+  T* kv = static_cast<T*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
+  {
+    T* out = kv + (long)pos * a.kv_st;
+    if (wave == 0) {
+      float ss = 0.f;
+      for (int c = lane; c < a.dv; c += 64) ss = __builtin_fmaf(to_f32(v[c]), to_f32(v[c]), ss);
+      const float r = a.norm_v ? 1.0f / sqrtf(wave_sum(ss) / (float)a.dv + a.eps) : 1.0f;
+      for (int c = lane; c < a.dv; c += 64) out[a.d + c] = from_f32<T>(to_f32(v[c]) * r);
+    } else {
+      for (int c = tid - 64; c < a.d; c += kStepThreads - 64) out[c] = from_f32<T>(rotated(k, c, pos, a));
+    }
+  }
+  const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  // lanes per key: the smallest power of two that covers the row in N-element pieces, 64 at most
+  const int pieces = (a.d + N - 1) / N;
+  int lpk = 1;
+  while (lpk < pieces && lpk < 64) lpk <<= 1;
+  const int keys_at_once = kStepThreads / lpk, my_key = tid / lpk, my_piece = tid % lpk;
+  const int v_pieces = (a.dv + N - 1) / N;                       // <= kStepThreads
+  const int v_groups = kStepThreads / v_pieces, my_vp = tid % v_pieces, my_vg = tid / v_pieces;
+
+  for (int h0 = 0; h0 < qpk; h0 += QT) {
+    __syncthreads();  // the new row is visible; the round before is done with LDS
+    for (int i = tid; i < QT * a.d; i += kStepThreads) {
+      const int hh = i / a.d, c = i % a.d;
+      const int h = g * qpk + (h0 + hh < qpk ? h0 + hh : h0);
+      const T* q = static_cast<const T*>(a.q) + b * a.q_sb + (long)h * a.d;
+      qs[i] = round_to<T>(rotated(q, c, pos, a));
+    }
+    if (tid < QT) {
+      stat[tid] = -INFINITY;
+      stat[QT + tid] = 0.f;
+    }
+    float acc[QT][N];
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+      for (int i = 0; i < N; ++i) acc[hh][i] = 0.f;
+    for (int k0 = lo; k0 <= pos; k0 += kStepKeys) {
+      const int n = pos - k0 + 1 < kStepKeys ? pos - k0 + 1 : kStepKeys;
+      __syncthreads();
+      for (int j0 = 0; j0 < n; j0 += keys_at_once) {
+        const int j = j0 + my_key;
+        float dot[QT];
+#pragma unroll
+        for (int hh = 0; hh < QT; ++hh) dot[hh] = 0.f;
+        const T* kr = kv + (long)(k0 + (j < n ? j : 0)) * a.kv_st;
+        for (int p = my_piece; p < pieces; p += lpk) {
+          float x[N];
+          if constexpr (VEC)
+            load_vec<T, N>(kr + p * N, x);
+          else
+            x[0] = to_f32(kr[p]);
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+            for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(x[i], qs[hh * a.d + p * N + i], dot[hh]);
+        }
+#pragma unroll
+        for (int hh = 0; hh < QT; ++hh) {
+          for (int m = 1; m < lpk; m <<= 1) dot[hh] += __shfl_xor(dot[hh], m, 64);
+          if (my_piece == 0 && j < n) sc[hh * kStepKeys + j] = dot[hh] * a.scale;
+        }
+      }
+      __syncthreads();
+      for (int hh = wave; hh < QT; hh += kStepThreads / 64) {
+        float mx = -INFINITY;
+        for (int j = lane; j < n; j += 64) mx = fmaxf(mx, sc[hh * kStepKeys + j]);
+#pragma unroll
+        for (int m = 32; m >= 1; m >>= 1) mx = fmaxf(mx, __shfl_xor(mx, m, 64));
+        const float m_old = stat[hh], m_new = fmaxf(m_old, mx);
+        float sum = 0.f;
+        for (int j = lane; j < n; j += 64) {
+          const float p = expf(sc[hh * kStepKeys + j] - m_new);
+          sc[hh * kStepKeys + j] = p;
+          sum += p;
+        }
+        sum = wave_sum(sum);
+        const float alpha = expf(m_old - m_new);
+        if (lane == 0) {
+          stat[hh] = m_new;
+          stat[QT + hh] = stat[QT + hh] * alpha + sum;
+          stat[2 * QT + hh] = alpha;
+        }
+      }
+      __syncthreads();
+      if (my_vg < v_groups) {
+#pragma unroll
+        for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+          for (int i = 0; i < N; ++i) acc[hh][i] *= stat[2 * QT + hh];
+#pragma unroll 4
+        for (int j = my_vg; j < n; j += v_groups) {
+          const T* vr = kv + (long)(k0 + j) * a.kv_st + a.d;
+          float x[N];
+          if constexpr (VEC)
+            load_vec<T, N>(vr + my_vp * N, x);
+          else
+            x[0] = to_f32(vr[my_vp]);
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+            for (int i = 0; i < N; ++i) acc[hh][i] = __builtin_fmaf(sc[hh * kStepKeys + j], x[i], acc[hh][i]);
+        }
+      }
+    }
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      __syncthreads();
+#pragma unroll
+      for (int i = 0; i < N; ++i) part[tid * N + i] = acc[hh][i];
+      __syncthreads();
+      if (h0 + hh < qpk) {
+        T* o = static_cast<T*>(a.o) + b * a.o_sb + (long)(g * qpk + h0 + hh) * a.dv;
+        const float inv = a.out_scale / stat[QT + hh];
+        for (int c = tid; c < a.dv; c += kStepThreads) {
+          float s = 0.f;
+          for (int vg = 0; vg < v_groups; ++vg) s += part[(vg * v_pieces + c / N) * N + c % N];
+          o[c] = from_f32<T>(s * inv);
+        }
+      }
+    }
+  }
+}
+
+template <typename T, bool VEC> void launch_window_step(const WindowArgs& a, hipStream_t s) {
+  const int qpk = a.H / a.G;
+  const dim3 grid((unsigned)(a.B * a.G)), block(kStepThreads);
+  auto bytes = [&](int qt) {
+    return (size_t)(qt * a.d + qt * kStepKeys + 3 * qt + 4 + kStepThreads * (VEC ? Pack<T>::kN : 1)) * sizeof(float);
+  };
+  if (qpk == 1)
+    hipLaunchKernelGGL((window_step_kernel<T, 1, VEC>), grid, block, bytes(1), s, a);
+  else if (qpk == 2)
+    hipLaunchKernelGGL((window_step_kernel<T, 2, VEC>), grid, block, bytes(2), s, a);
+  else if (qpk <= 4)
+    hipLaunchKernelGGL((window_step_kernel<T, 4, VEC>), grid, block, bytes(4), s, a);
+  else
+    hipLaunchKernelGGL((window_step_kernel<T, 8, VEC>), grid, block, bytes(8), s, a);
+}
+
+template <int KC> void launch_window_mfma(const WindowArgs& a, dim3 grid, hipStream_t s) {
+  const int vc = (a.dv + 31) / 32;
+  if (vc <= 1)
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 1>), grid, dim3(256), 0, s, a);
+  else if (vc <= 2)
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 2>), grid, dim3(256), 0, s, a);
+  else if (vc <= 4)
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 4>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 8>), grid, dim3(256), 0, s, a);
+}
+
+static int window_check(const char* who, const WindowArgs& a, int64_t n_rope, int io_dtype, int64_t last) {
+  BASED_REQUIRE(a.q && a.k && a.v && a.kv && a.o, BASED_ERR_ARG, "%s: null pointer argument", who);
+  BASED_REQUIRE(a.B >= 0 && a.L >= 0 && a.H > 0 && a.G > 0 && a.d > 0 && a.dv > 0 && a.S > 0, BASED_ERR_ARG, "%s: bad sizes", who);
+  BASED_REQUIRE(a.H % a.G == 0, BASED_ERR_SHAPE, "%s: %d query heads do not divide into %d key/value heads", who, a.H, a.G);
+  BASED_REQUIRE(a.d <= kAnyMaxDim && a.dv <= kAnyMaxDim, BASED_ERR_SHAPE, "%s: head sizes %d / %d (at most %d)", who, a.d, a.dv,
+                kAnyMaxDim);
+  BASED_REQUIRE(a.window > 0, BASED_ERR_ARG, "%s: window %d", who, a.window);
+  BASED_REQUIRE(a.rot >= 0 && a.rot <= a.d && a.rot % 2 == 0, BASED_ERR_SHAPE, "%s: rotary size %d of %d channels", who, a.rot, a.d);
+  BASED_REQUIRE(a.rot == 0 || (a.cos_t && a.sin_t), BASED_ERR_ARG, "%s: rotary tables missing", who);
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "%s: bad dtype", who);
+  BASED_REQUIRE(last < a.S, BASED_ERR_SHAPE, "%s: position %ld does not fit a cache of %d rows", who, (long)last, a.S);
+  BASED_REQUIRE(a.rot == 0 || last < n_rope, BASED_ERR_SHAPE, "%s: rotary tables end before position %ld", who, (long)last);
+  return BASED_OK;
+}
+
+static bool window_vec(const WindowArgs& a, int n) {
+  return a.d % n == 0 && a.dv % n == 0 && a.q_sb % n == 0 && a.q_sl % n == 0 && a.k_sb % n == 0 && a.k_sl % n == 0 &&
+         a.v_sb % n == 0 && a.v_sl % n == 0 && a.o_sb % n == 0 && a.o_sl % n == 0 && a.kv_sb % n == 0 && a.kv_st % n == 0 &&
+         aligned_to(a.q, 16) && aligned_to(a.k, 16) && aligned_to(a.v, 16) && aligned_to(a.kv, 16) && aligned_to(a.o, 16);
+}
+
+}  // namespace based
+
+extern "C" BASED_API int based_window_attn_prefill(
+    const void* q, const void* k, const void* v, void* kv_cache, void* o, int64_t start, int64_t B, int64_t L, int64_t H, int64_t G,
+    int64_t D, int64_t DV, int64_t S, int64_t q_sb, int64_t q_sl, int64_t k_sb, int64_t k_sl, int64_t v_sb, int64_t v_sl,
+    int64_t o_sb, int64_t o_sl, int64_t kv_sb, int64_t kv_st, int64_t window, float scale, int norm_v, float eps, float out_scale,
+    const float* rope_cos, const float* rope_sin, int64_t rope_len, int64_t rotary_dim, int half_split, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(start >= 0 && start + L < (1ll << 31) && window < (1ll << 31) && L * H < (1ll << 31), BASED_ERR_SHAPE,
+                "window_attn_prefill: sequence too long");
+  const WindowArgs a{q,       k,       v,      kv_cache, o,        rope_cos, rope_sin, nullptr, (int)start, (int)rope_len,
+                     (int)B,  (int)L,  (int)H, (int)G,   (int)D,   (int)DV,  (int)S,   q_sb,    q_sl,       k_sb,
+                     k_sl,    v_sb,    v_sl,   o_sb,     o_sl,     kv_sb,    kv_st,    (int)rotary_dim, half_split, (int)window,
+                     norm_v,  scale,   eps,    out_scale};
+  const int rc = window_check("window_attn_prefill", a, rope_len, io_dtype, start + L - 1);
+  if (rc != BASED_OK) return rc;
+  BASED_REQUIRE(B * G < 65536 && B < 65536 && H < 65536, BASED_ERR_SHAPE, "window_attn_prefill: grid too large");
+  if (B == 0 || L == 0) return BASED_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const bool vec = io_dtype == BASED_BF16 && D <= 256 && DV <= 256 && window_vec(a, 8);
+  const int64_t items = B * L * G;
+  BASED_REQUIRE((items + 3) / 4 < (1ll << 31), BASED_ERR_SHAPE, "window_attn_prefill: grid too large");
+  if (vec && !half_split)
+    hipLaunchKernelGGL(window_kv_write_vec_kernel, dim3((unsigned)((items + 15) / 16)), dim3(256), 0, s, a);
+  else if (io_dtype == BASED_BF16)
+    hipLaunchKernelGGL(window_kv_write_kernel<__bf16>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL(window_kv_write_kernel<float>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
+  if (vec) {
+    const dim3 grid((unsigned)((L * (H / G) + kTileRows - 1) / kTileRows), (unsigned)(B * G));
+    const int kc = (int)((D + 31) / 32);
+    if (kc <= 1)
+      launch_window_mfma<1>(a, grid, s);
+    else if (kc <= 2)
+      launch_window_mfma<2>(a, grid, s);
+    else if (kc <= 4)
+      launch_window_mfma<4>(a, grid, s);
+    else
+      launch_window_mfma<8>(a, grid, s);
+  } else {
+    const dim3 grid((unsigned)L, (unsigned)H, (unsigned)B);
+    if (io_dtype == BASED_BF16)
+      hipLaunchKernelGGL(window_prefill_any_kernel<__bf16>, grid, dim3(64), 0, s, a);
+    else
+      hipLaunchKernelGGL(window_prefill_any_kernel<float>, grid, dim3(64), 0, s, a);
+  }
+  return check_launch("window_attn_prefill");
+}
+
+extern "C" BASED_API int based_window_attn_step(
+    const void* q, const void* k, const void* v, void* kv_cache, void* o, const int32_t* pos, int64_t pos_host, int64_t B, int64_t H,
+    int64_t G, int64_t D, int64_t DV, int64_t S, int64_t q_sb, int64_t k_sb, int64_t v_sb, int64_t o_sb, int64_t kv_sb,
+    int64_t kv_st, int64_t window, float scale, int norm_v, float eps, float out_scale, const float* rope_cos,
+    const float* rope_sin, int64_t rope_len, int64_t rotary_dim, int half_split, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(pos_host >= 0 && pos_host < (1ll << 31) && window < (1ll << 31), BASED_ERR_SHAPE, "window_attn_step: bad position");
+  const WindowArgs a{q,      k,      v,      kv_cache, o,       rope_cos, rope_sin, pos,  (int)pos_host, (int)rope_len,
+                     (int)B, 1,      (int)H, (int)G,   (int)D,  (int)DV,  (int)S,   q_sb, 0,             k_sb,
+                     0,      v_sb,   0,      o_sb,     0,       kv_sb,    kv_st,    (int)rotary_dim, half_split, (int)window,
+                     norm_v, scale,  eps,    out_scale};
+  const int rc = window_check("window_attn_step", a, rope_len, io_dtype, pos != nullptr ? 0 : pos_host);
+  if (rc != BASED_OK) return rc;
+  BASED_REQUIRE(B * G < (1ll << 31), BASED_ERR_SHAPE, "window_attn_step: grid too large");
+  const int n = io_dtype == BASED_BF16 ? 8 : 4;
+  const bool vec = window_vec(a, n);
+  BASED_REQUIRE(vec || DV <= kStepThreads, BASED_ERR_SHAPE, "window_attn_step: value size %ld with unaligned rows (at most %d)",
+                (long)DV, kStepThreads);
+  if (B == 0) return BASED_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16)
+    vec ? launch_window_step<__bf16, true>(a, s) : launch_window_step<__bf16, false>(a, s);
+  else
+    vec ? launch_window_step<float, true>(a, s) : launch_window_step<float, false>(a, s);
+  return check_launch("window_attn_step");
+}

@@ -580,7 +580,7 @@ def greedy_step(logits, next_ids, lengths, sequences=None, position_ids=None, vo
 
 
 DECODE_LINEAR_MAX_ROWS = 32  # BASED_DECODE_LINEAR_MAX_ROWS of include/based_hip.h
-PROLOGUE_NONE, PROLOGUE_ADD_RMS_NORM, PROLOGUE_SWIGLU = 0, 1, 2
+PROLOGUE_NONE, PROLOGUE_ADD_RMS_NORM, PROLOGUE_SWIGLU, PROLOGUE_STREAM = 0, 1, 2, 3
 EPILOGUE_NONE, EPILOGUE_SWIGLU, EPILOGUE_GATED_CONV_STEP = 0, 1, 2
 
 
@@ -593,8 +593,8 @@ def decode_linear_weight_ok(weight: torch.Tensor) -> bool:
 
 def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residual_in=None, residual_out=None,
                   norm_weight=None, eps: float = 1e-5, row_index=None, epilogue: int = EPILOGUE_NONE,
-                  conv_state=None, conv_weight=None, conv_bias=None, out: Optional[torch.Tensor] = None
-                  ) -> torch.Tensor:
+                  conv_state=None, conv_weight=None, conv_bias=None, out: Optional[torch.Tensor] = None,
+                  mult: float = 1.0, norm_kind: int = 0, input_conv=None) -> torch.Tensor:
     """y = epi(pro(x) @ weight.T (+ bias)) for the few rows of a single-token step, one launch.
 
     x: (M, K) bf16 rows (M <= 32; any leading shape is flattened), or for PROLOGUE_SWIGLU (M, 2K):
@@ -605,7 +605,17 @@ def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residu
     EPILOGUE_SWIGLU: weight is (2F, K), y[:, f] = p[:, f] * silu(p[:, F + f]).
     EPILOGUE_GATED_CONV_STEP: weight is (2F, K); the gated short-convolution step on p with
     conv_state (M, F, k) rolled in place, conv_weight the (F, 1, k) or (F, k) Conv1d weight,
-    conv_bias None or (F).  Returns y (M, N) or (M, F), written into `out` when given."""
+    conv_bias None or (F).  Returns y (M, N) or (M, F), written into `out` when given.
+
+    PROLOGUE_STREAM: r = residual_in + mult * x in fp32 (written to residual_out), then the norm
+    `norm_kind` of that sum times norm_weight, rounded to bf16, and with input_conv =
+    (weight (taps, K), ring (M, taps, K), pos) that row plus its causal convolution; epilogues NONE and
+    SWIGLU."""
+    if prologue == PROLOGUE_STREAM:
+        if conv_state is not None or conv_weight is not None or conv_bias is not None:
+            raise ValueError("the streamed-input prologue has no convolution epilogue")
+        return _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult,
+                                     norm_kind, input_conv, out)
     N, K = weight.shape
     x2 = x if x.dim() == 2 else x.reshape(-1, x.shape[-1])
     M = x2.shape[0] if row_index is None else row_index.numel()
@@ -691,4 +701,325 @@ def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residu
             conv_weight.data_ptr() if conv else None,
             conv_bias.data_ptr() if conv and conv_bias is not None else None,
             conv_weight.shape[-1] if conv else 0, _stream_ptr(x2)))
+    return y
+
+
+# --------------------------------------------------------------------------------------------------
+# Streaming layers: portions of any length on caches, rings of past inputs and fp32 states
+# --------------------------------------------------------------------------------------------------
+NORM_RMS, NORM_LAYER = 0, 1
+ACT_NONE, ACT_SILU = 0, 1
+STREAM_MAX_TAPS = 8  # BASED_STREAM_MAX_TAPS
+RGLRU_SEGMENT = 64   # tokens per segment of based_rglru_prefill
+
+
+def _ptr(t):
+    return None if t is None else t.data_ptr()
+
+
+def _check_rows(*ts) -> None:
+    _require_cuda(*ts)
+    for t in ts:
+        if t.stride(-1) != 1:
+            raise ValueError("innermost dimension must be contiguous")
+
+
+def _check_same_dtype(x, *ts) -> None:
+    for t in ts:
+        if t is not None and t.dtype != x.dtype:
+            raise ValueError(f"expected {x.dtype}, got {t.dtype}")
+
+
+def _pos_args(pos, rows: int):
+    """pos: an int for every row, or a contiguous int32 device vector of at least `rows` positions."""
+    if isinstance(pos, torch.Tensor):
+        if pos.dtype != torch.int32 or not pos.is_cuda or pos.dim() != 1 or pos.numel() < rows or not pos.is_contiguous():
+            raise ValueError(f"positions must be a contiguous int32 device vector with {rows} entries")
+        return pos.data_ptr(), 0
+    return None, int(pos)
+
+
+def _check_ring(ring, rows: int, taps: int, channels: int, like) -> None:
+    if (ring.dim() != 3 or tuple(ring.shape) != (rows, taps, channels) or ring.stride(2) != 1 or ring.stride(1) != channels
+            or ring.dtype != like.dtype or ring.device != like.device):
+        raise ValueError(f"ring must be ({rows}, {taps}, {channels}) {like.dtype} with contiguous slots, got {tuple(ring.shape)} {ring.dtype}")
+
+
+def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: float = 1.0, want_residual: bool = True):
+    """r = residual + mult * x in fp32 (r = x without a residual); y = norm(r) * weight in x's dtype.
+    x: (..., D); residual fp32 of the same shape or None.  Returns (y, r), r None if not wanted."""
+    D = x.shape[-1]
+    _require_cuda(x, weight)
+    _check_same_dtype(x, weight)
+    if tuple(weight.shape) != (D,) or not weight.is_contiguous():
+        raise ValueError(f"weight must be a contiguous ({D},), got {tuple(weight.shape)}")
+    x2 = x.reshape(-1, D)
+    if x2.stride(1) != 1:
+        x2 = x2.contiguous()
+    r2 = None
+    if residual is not None:
+        _require_cuda(x, residual)
+        if residual.shape != x.shape or residual.dtype != torch.float32:
+            raise ValueError(f"residual must be float32 {tuple(x.shape)}, got {residual.dtype} {tuple(residual.shape)}")
+        r2 = residual.reshape(-1, D)
+        if r2.stride(1) != 1:
+            r2 = r2.contiguous()
+    rows = x2.shape[0]
+    y = torch.empty(rows, D, dtype=x.dtype, device=x.device)
+    out = torch.empty(rows, D, dtype=torch.float32, device=x.device) if want_residual else None
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_add_norm(x2.data_ptr(), _ptr(r2), weight.data_ptr(), y.data_ptr(), _ptr(out), rows, D,
+                                             x2.stride(0), 0 if r2 is None else r2.stride(0), D, D, float(eps), int(kind),
+                                             float(mult), _dtype_code(x), _stream_ptr(x)))
+    return y.view(x.shape), None if out is None else out.view(x.shape)
+
+
+def stream_conv(x, weight, bias=None, ring=None, pos=0, activation: int = ACT_NONE, add_input: bool = False) -> torch.Tensor:
+    """y_t = [x_t +] act(bias + sum_j weight[j] * x_{t - taps + 1 + j}) on each channel of x (B, L, D), the
+    portion of a sequence that starts at `pos`.  weight (taps, D); ring (B, taps, D) or None (nothing
+    before the portion): read for the inputs before it, left with its last ones."""
+    B, L, D = x.shape
+    taps = weight.shape[0]
+    _check_rows(x, weight)
+    _check_same_dtype(x, weight, bias)
+    if tuple(weight.shape) != (taps, D) or not weight.is_contiguous() or not 1 <= taps <= STREAM_MAX_TAPS:
+        raise ValueError(f"weight must be a contiguous (taps, {D}) with 1 to {STREAM_MAX_TAPS} taps, got {tuple(weight.shape)}")
+    if bias is not None and (tuple(bias.shape) != (D,) or not bias.is_contiguous() or not bias.is_cuda):
+        raise ValueError(f"bias must be a contiguous ({D},) on the device")
+    if ring is not None:
+        _check_ring(ring, B, taps, D, x)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    y = torch.empty(B, L, D, dtype=x.dtype, device=x.device)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_stream_conv(
+            x.data_ptr(), weight.data_ptr(), _ptr(bias), y.data_ptr(), _ptr(ring), pos_ptr, pos_host, B, L, D, taps, x.stride(0),
+            x.stride(1), y.stride(0), y.stride(1), 0 if ring is None else ring.stride(0), int(activation), int(add_input),
+            _dtype_code(x), _stream_ptr(x)))
+    return y
+
+
+def _window_shapes(q, k, v, kv_cache, heads: int, kv_heads: int, out):
+    """q (..., H * d), k (..., G * d), v (..., G * dv), cache (B, S, G, d + dv): the sizes, checked."""
+    _check_rows(q, k, v, kv_cache, out)
+    _check_same_dtype(q, k, v, kv_cache, out)
+    d, dv = q.shape[-1] // heads, v.shape[-1] // kv_heads
+    if q.shape[-1] != heads * d or k.shape[-1] != kv_heads * d or v.shape[-1] != kv_heads * dv or out.shape[-1] != heads * dv:
+        raise ValueError(f"bad head sizes q{tuple(q.shape)} k{tuple(k.shape)} v{tuple(v.shape)} out{tuple(out.shape)}")
+    if not (q.shape[:-1] == k.shape[:-1] == v.shape[:-1] == out.shape[:-1]):
+        raise ValueError("q, k, v and out must agree in batch and length")
+    if (kv_cache.dim() != 4 or kv_cache.shape[0] != q.shape[0] or tuple(kv_cache.shape[2:]) != (kv_heads, d + dv)
+            or kv_cache.stride(2) != d + dv):
+        raise ValueError(f"cache must be ({q.shape[0]}, S, {kv_heads}, {d + dv}), got {tuple(kv_cache.shape)}")
+    return d, dv
+
+
+def _stream_rope(rope, device):
+    """(cos, sin, interleaved) tables or None -> (cos_ptr, sin_ptr, n_pos, rotary_dim, half_split)."""
+    if rope is None:
+        return None, None, 0, 0, 0
+    cos, sin, interleaved = rope
+    for t in (cos, sin):
+        if t.device != device or t.dtype != torch.float32 or t.dim() != 2 or not t.is_contiguous() or t.shape != cos.shape:
+            raise ValueError("rotary tables must be contiguous fp32 (n_pos, rotary_dim / 2) tensors on the device of q")
+    return cos.data_ptr(), sin.data_ptr(), cos.shape[0], 2 * cos.shape[1], int(not interleaved)
+
+
+def window_attn_prefill(q, k, v, kv_cache, heads: int, kv_heads: int, window: int, scale: float, start: int = 0, rope=None,
+                        value_norm_eps: Optional[float] = None, out_scale: float = 1.0, *, out):
+    """Causal attention of a portion at positions start .. start + L - 1 over the last `window` keys (itself
+    included).  q (B, L, H * d), k (B, L, G * d), v (B, L, G * dv); kv_cache (B, S, G, d + dv) receives the
+    portion's rotated keys and (normalised, when value_norm_eps is given) values and is attended.
+    Written, times out_scale, into out (B, L, H * dv)."""
+    d, dv = _window_shapes(q, k, v, kv_cache, heads, kv_heads, out)
+    cos_ptr, sin_ptr, n_pos, rot, half = _stream_rope(rope, q.device)
+    B, L = q.shape[:2]
+    with _on_device(q.device):
+        _lib.check(_lib.lib().based_window_attn_prefill(
+            q.data_ptr(), k.data_ptr(), v.data_ptr(), kv_cache.data_ptr(), out.data_ptr(), int(start), B, L, heads, kv_heads, d, dv,
+            kv_cache.shape[1], q.stride(0), q.stride(1), k.stride(0), k.stride(1), v.stride(0), v.stride(1), out.stride(0),
+            out.stride(1), kv_cache.stride(0), kv_cache.stride(1), int(window), float(scale), int(value_norm_eps is not None),
+            float(value_norm_eps or 0.0), float(out_scale), cos_ptr, sin_ptr, n_pos, rot, half, _dtype_code(q), _stream_ptr(q)))
+    return out
+
+
+def window_attn_step(q, k, v, kv_cache, heads: int, kv_heads: int, window: int, scale: float, pos, rope=None,
+                     value_norm_eps: Optional[float] = None, out_scale: float = 1.0, *, out):
+    """One token per sequence: q (B, H * d), k (B, G * d), v (B, G * dv), out (B, H * dv); `pos` an int or an
+    int32 device vector.  Otherwise as window_attn_prefill."""
+    d, dv = _window_shapes(q, k, v, kv_cache, heads, kv_heads, out)
+    cos_ptr, sin_ptr, n_pos, rot, half = _stream_rope(rope, q.device)
+    B = q.shape[0]
+    pos_ptr, pos_host = _pos_args(pos, B)
+    with _on_device(q.device):
+        _lib.check(_lib.lib().based_window_attn_step(
+            q.data_ptr(), k.data_ptr(), v.data_ptr(), kv_cache.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B, heads, kv_heads, d,
+            dv, kv_cache.shape[1], q.stride(0), k.stride(0), v.stride(0), out.stride(0), kv_cache.stride(0), kv_cache.stride(1),
+            int(window), float(scale), int(value_norm_eps is not None), float(value_norm_eps or 0.0), float(out_scale), cos_ptr,
+            sin_ptr, n_pos, rot, half, _dtype_code(q), _stream_ptr(q)))
+    return out
+
+
+def _check_delta(state, rows: int, heads: int, d: int, dv: int) -> None:
+    if (state.dim() != 4 or tuple(state.shape[:3]) != (rows, heads, d) or state.shape[3] < dv or state.shape[3] % 4 != 0
+            or state.dtype != torch.float32 or not state.is_contiguous() or not state.is_cuda):
+        raise ValueError(f"state must be a contiguous float32 ({rows}, {heads}, {d}, {dv} rounded up to 4), got {tuple(state.shape)}")
+
+
+def gated_delta_scan(q, k, v, a_gate, b_gate, a_log, dt_bias, state, heads: int, kv_heads: int, fresh: bool) -> torch.Tensor:
+    """The gated delta recurrence over a portion.  q, k (B, L, G * d) and v (B, L, H * dv) share their strides
+    (slices of one tensor); a_gate, b_gate (B, L, H); state (B, H, d, dv rounded up to 4) fp32, updated in
+    place, taken as zero when `fresh`.  Returns o (B, L, H, dv) fp32."""
+    _check_rows(q, k, v, a_gate, b_gate)
+    _check_same_dtype(q, k, v, a_gate, b_gate, a_log, dt_bias)
+    B, L = q.shape[:2]
+    d, dv = q.shape[-1] // kv_heads, v.shape[-1] // heads
+    if q.shape != k.shape or tuple(v.shape[:2]) != (B, L) or q.shape[-1] != kv_heads * d or v.shape[-1] != heads * dv:
+        raise ValueError(f"bad shapes q{tuple(q.shape)} k{tuple(k.shape)} v{tuple(v.shape)}")
+    if not (q.stride() == k.stride() == v.stride()) or a_gate.stride() != b_gate.stride():
+        raise ValueError("q, k and v must share their strides, and the two gates theirs")
+    if tuple(a_gate.shape) != (B, L, heads) or b_gate.shape != a_gate.shape:
+        raise ValueError(f"gates must be ({B}, {L}, {heads})")
+    _check_delta(state, B, heads, d, dv)
+    o = torch.empty(B, L, heads, dv, dtype=torch.float32, device=q.device)
+    with _on_device(q.device):
+        _lib.check(_lib.lib().based_gated_delta_scan(
+            q.data_ptr(), k.data_ptr(), v.data_ptr(), a_gate.data_ptr(), b_gate.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),
+            state.data_ptr(), o.data_ptr(), B, L, heads, kv_heads, d, dv, state.shape[3], q.stride(0), q.stride(1),
+            a_gate.stride(0), a_gate.stride(1), int(fresh), _dtype_code(q), _stream_ptr(q)))
+    return o
+
+
+def gated_rms_norm(o, weight, gate, eps: float, scale: float = 1.0, *, out) -> torch.Tensor:
+    """out = o / sqrt(mean(o^2) + eps) * weight * silu(gate) * scale per head; o (B, L, H, dv) fp32, gate and
+    out (B, L, H * dv)."""
+    B, L, H, dv = o.shape
+    _check_rows(gate, out)
+    _check_same_dtype(gate, out, weight)
+    if o.dtype != torch.float32 or not o.is_contiguous() or tuple(gate.shape) != (B, L, H * dv) or out.shape != gate.shape \
+            or tuple(weight.shape) != (dv,):
+        raise ValueError(f"bad shapes o{tuple(o.shape)} gate{tuple(gate.shape)} out{tuple(out.shape)} weight{tuple(weight.shape)}")
+    with _on_device(o.device):
+        _lib.check(_lib.lib().based_gated_rms_norm(o.data_ptr(), weight.data_ptr(), gate.data_ptr(), out.data_ptr(), B, L, H, dv,
+                                                   gate.stride(0), gate.stride(1), out.stride(0), out.stride(1), float(eps),
+                                                   float(scale), _dtype_code(gate), _stream_ptr(gate)))
+    return out
+
+
+def gated_delta_step(x, conv_weight, ring, a_gate, b_gate, gate, a_log, dt_bias, norm_weight, state, heads: int, kv_heads: int,
+                     d: int, dv: int, k_off: int, v_off: int, pos, eps: float, scale: float = 1.0, *, out) -> torch.Tensor:
+    """One token of the delta-rule block between its projections: x (B, C) is what the short convolution
+    reads (queries at channel 0, keys at k_off, values at v_off), conv_weight (taps, C), ring (B, taps, C);
+    a_gate, b_gate (B, H), gate and out (B, H * dv)."""
+    _check_rows(x, a_gate, b_gate, gate, out)
+    _check_same_dtype(x, conv_weight, a_gate, b_gate, gate, a_log, dt_bias, norm_weight, out)
+    B, C = x.shape
+    taps = conv_weight.shape[0]
+    if tuple(conv_weight.shape) != (taps, C) or not conv_weight.is_contiguous():
+        raise ValueError(f"conv_weight must be a contiguous (taps, {C}), got {tuple(conv_weight.shape)}")
+    if tuple(a_gate.shape) != (B, heads) or b_gate.shape != a_gate.shape or a_gate.stride() != b_gate.stride() \
+            or tuple(gate.shape) != (B, heads * dv) or out.shape != gate.shape:
+        raise ValueError("bad gate or output shapes")
+    _check_ring(ring, B, taps, C, x)
+    _check_delta(state, B, heads, d, dv)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_gated_delta_step(
+            x.data_ptr(), conv_weight.data_ptr(), ring.data_ptr(), a_gate.data_ptr(), b_gate.data_ptr(), gate.data_ptr(),
+            a_log.data_ptr(), dt_bias.data_ptr(), norm_weight.data_ptr(), state.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B,
+            heads, kv_heads, d, dv, state.shape[3], C, taps, k_off, v_off, x.stride(0), a_gate.stride(0), gate.stride(0),
+            out.stride(0), ring.stride(0), float(eps), float(scale), _dtype_code(x), _stream_ptr(x)))
+    return out
+
+
+def _check_lru(x, y, ra, rb, ri, ib, lam, state, out, rows: int):
+    _check_rows(x, y, out)
+    _check_same_dtype(x, y, ra, rb, ri, ib, lam, out)
+    W = x.shape[-1]
+    blocks, n = ra.shape[:2]
+    if blocks * n != W or tuple(ra.shape) != (blocks, n, n) or ri.shape != ra.shape or y.shape != x.shape or out.shape != x.shape:
+        raise ValueError(f"bad shapes x{tuple(x.shape)} y{tuple(y.shape)} ra{tuple(ra.shape)} ri{tuple(ri.shape)}")
+    for t in (ra, ri, rb, ib, lam):
+        if not t.is_contiguous() or (t.dim() < 3 and t.numel() != W):
+            raise ValueError("gate parameters must be contiguous, one value per channel")
+    if tuple(state.shape) != (rows, W) or state.dtype != torch.float32 or not state.is_contiguous():
+        raise ValueError(f"state must be a contiguous float32 ({rows}, {W}), got {tuple(state.shape)}")
+    return W, blocks
+
+
+def rglru_prefill(u, y, ra, rb, ri, ib, lam, state, decay_scale: float, fresh: bool, *, out) -> torch.Tensor:
+    """The gated linear recurrence over a portion: u (B, L, W) convolved, y (B, L, W) before its gelu; ra, ri
+    (blocks, n, n) as [out, in], rb, ib, lam (W) values; state (B, W) fp32, updated in place, taken as
+    zero when `fresh`.  out (B, L, W) = S * gelu_tanh(y)."""
+    B, L, _ = u.shape
+    W, blocks = _check_lru(u, y, ra, rb, ri, ib, lam, state, out, B)
+    segs = (L + RGLRU_SEGMENT - 1) // RGLRU_SEGMENT
+    work = torch.empty(2, B, L, W, dtype=torch.float32, device=u.device)
+    agg = torch.empty(B, segs + 1, 2, W, dtype=torch.float32, device=u.device)
+    with _on_device(u.device):
+        _lib.check(_lib.lib().based_rglru_prefill(
+            u.data_ptr(), y.data_ptr(), ra.data_ptr(), rb.data_ptr(), ri.data_ptr(), ib.data_ptr(), lam.data_ptr(),
+            work[0].data_ptr(), work[1].data_ptr(), agg.data_ptr(), state.data_ptr(), out.data_ptr(), B, L, W, blocks, u.stride(0),
+            u.stride(1), y.stride(0), y.stride(1), out.stride(0), out.stride(1), float(decay_scale), int(fresh), _dtype_code(u),
+            _stream_ptr(u)))
+    return out
+
+
+def rglru_step(x, y, conv_weight, conv_bias, ring, ra, rb, ri, ib, lam, state, decay_scale: float, pos, *, out) -> torch.Tensor:
+    """One token of it with the short convolution in front: x, y, out (B, W); conv_weight (taps, W), conv_bias
+    (W) or None, ring (B, taps, W)."""
+    B = x.shape[0]
+    W, blocks = _check_lru(x, y, ra, rb, ri, ib, lam, state, out, B)
+    taps = conv_weight.shape[0]
+    _check_same_dtype(x, conv_weight, conv_bias)
+    if tuple(conv_weight.shape) != (taps, W) or not conv_weight.is_contiguous():
+        raise ValueError(f"conv_weight must be a contiguous (taps, {W}), got {tuple(conv_weight.shape)}")
+    _check_ring(ring, B, taps, W, x)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_rglru_step(
+            x.data_ptr(), y.data_ptr(), conv_weight.data_ptr(), _ptr(conv_bias), ring.data_ptr(), ra.data_ptr(), rb.data_ptr(),
+            ri.data_ptr(), ib.data_ptr(), lam.data_ptr(), state.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B, W, blocks, taps,
+            x.stride(0), y.stride(0), out.stride(0), ring.stride(0), float(decay_scale), _dtype_code(x), _stream_ptr(x)))
+    return out
+
+
+def _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult, norm_kind,
+                          input_conv, out):
+    """`decode_linear` behind PROLOGUE_STREAM."""
+    N, K = weight.shape
+    x2 = x if x.dim() == 2 else x.reshape(-1, x.shape[-1])
+    M = x2.shape[0] if row_index is None else row_index.numel()
+    n_out = N if epilogue == EPILOGUE_NONE else N // 2
+    _require_cuda(x2, weight, norm_weight)
+    if x2.dtype != torch.bfloat16 or weight.dtype != torch.bfloat16 or norm_weight.dtype != torch.bfloat16 or x2.shape[1] != K \
+            or weight.stride(1) != 1 or x2.stride(1) != 1 or tuple(norm_weight.shape) != (K,) or not norm_weight.is_contiguous():
+        raise ValueError("x, weight and norm_weight must be bfloat16 rows of the contraction length")
+    if bias is not None and (tuple(bias.shape) != (N,) or bias.dtype != torch.bfloat16 or not bias.is_contiguous()):
+        raise ValueError(f"bias must be a contiguous bfloat16 ({N},)")
+    for r in (residual_in, residual_out):
+        if r is not None and (r.dtype != torch.float32 or tuple(r.shape) != (M, K) or r.stride(1) != 1 or not r.is_cuda):
+            raise ValueError(f"residuals must be float32 ({M}, {K}) device tensors with contiguous rows")
+    if row_index is not None and (row_index.dtype != torch.int64 or row_index.dim() != 1 or not row_index.is_contiguous()
+                                  or not row_index.is_cuda):
+        raise ValueError("row_index must be a contiguous int64 device vector")
+    conv_w = ring = pos_ptr = None
+    taps = pos_host = ring_stride = 0
+    if input_conv is not None:
+        conv_w, ring, pos = input_conv
+        taps = conv_w.shape[0]
+        if tuple(conv_w.shape) != (taps, K) or not conv_w.is_contiguous() or conv_w.dtype != torch.bfloat16 or not conv_w.is_cuda:
+            raise ValueError(f"the input convolution's weight must be a contiguous bfloat16 (taps, {K})")
+        _check_ring(ring, M, taps, K, x2)
+        ring_stride = ring.stride(0)
+        pos_ptr, pos_host = _pos_args(pos, M)
+    y = torch.empty(M, n_out, dtype=torch.bfloat16, device=x2.device) if out is None else out
+    if tuple(y.shape) != (M, n_out) or y.dtype != torch.bfloat16 or y.stride(1) != 1:
+        raise ValueError(f"out must be a ({M}, {n_out}) bfloat16 tensor with contiguous rows")
+    with _on_device(x2.device):
+        _lib.check(_lib.lib().based_decode_linear_stream(
+            x2.data_ptr(), x2.stride(0), _ptr(row_index), 0 if row_index is None else x2.shape[0], weight.data_ptr(), weight.stride(0),
+            _ptr(bias), y.data_ptr(), y.stride(0), M, N, K, _ptr(residual_in), 0 if residual_in is None else residual_in.stride(0),
+            _ptr(residual_out), 0 if residual_out is None else residual_out.stride(0), float(mult), int(norm_kind),
+            norm_weight.data_ptr(), float(eps), _ptr(conv_w), _ptr(ring), ring_stride, taps, pos_ptr, pos_host, epilogue,
+            _stream_ptr(x2)))
     return y

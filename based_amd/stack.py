@@ -24,8 +24,13 @@ from . import ops
 
 from .generation import GenerationMixin
 from .mixers.convolution import BaseConv, ShortConvolution
+from .mixers.gated_delta import GatedDeltaRule
 from .mixers.linear_attention import LinearAttention, TaylorExp
+from .mixers.rglru import RGLRU
+from .mixers.side_by_side import SideBySide
 from .mixers.slide_attention import SlidingAttention
+from .mixers.streaming import StreamConv, portion_start
+from .mixers.window_attention import WindowAttention
 
 # `_target_` strings accepted in mixer config dicts: the reference's own paths and this package's.
 _TARGETS = {
@@ -39,14 +44,27 @@ _TARGETS = {
     "based_amd.mixers.slide_attention.SlidingAttention": SlidingAttention,
     "based_amd.mixers.convolution.BaseConv": BaseConv,
     "based_amd.mixers.convolution.ShortConvolution": ShortConvolution,
+    "based_amd.mixers.gated_delta.GatedDeltaRule": GatedDeltaRule,
+    "based_amd.mixers.rglru.RGLRU": RGLRU,
+    "based_amd.mixers.side_by_side.SideBySide": SideBySide,
+    "based_amd.mixers.window_attention.WindowAttention": WindowAttention,
 }
 
 
 def _instantiate(spec: dict, *args, **extra):
-    """Tiny stand-in for hydra.utils.instantiate: nested dicts with `_target_` become objects."""
+    """Tiny stand-in for hydra.utils.instantiate: nested dicts with `_target_` become objects; in a list
+    they become constructors, which the mixer that holds the list completes (layer_idx, device, ...)."""
     spec = dict(spec)
     cls = _TARGETS[spec.pop("_target_")]
-    kwargs = {k: (_instantiate(v) if isinstance(v, dict) and "_target_" in v else v) for k, v in spec.items()}
+
+    def value(v):
+        if isinstance(v, dict) and "_target_" in v:
+            return _instantiate(v)
+        if isinstance(v, (list, tuple)) and any(isinstance(x, dict) and "_target_" in x for x in v):
+            return [partial(_TARGETS[x["_target_"]], **{k: y for k, y in x.items() if k != "_target_"}) for x in v]
+        return v
+
+    kwargs = {k: value(v) for k, v in spec.items()}
     kwargs.update(extra)
     return cls(*args, **kwargs)
 
@@ -64,6 +82,11 @@ class StackConfig(SimpleNamespace):
             qkv_proj_bias=False, out_proj_bias=False, rotary_emb_fraction=0.0, rotary_emb_base=10000.0,
             rotary_emb_interleaved=False, scale_attn_weights=True, max_position_embeddings=0,
             mixer=None, alt_mixer=None, alt_mixer_layers=None, alt_mixer_2=None, alt_mixer_2_layers=None,
+            # Streamed designs.  layer_specs: one {"mixer": spec, "mlp": {"hidden": n} or None} per layer
+            # instead of the mixer / alt_mixer routing; stream_norm: "layer" or "rms" without a bias on the
+            # fp32 residual sum; residual_mult: factor of every sublayer's output; input_conv_taps: causal
+            # convolution added to what a mixer reads (0: none).
+            layer_specs=None, stream_norm=None, residual_mult=1.0, input_conv_taps=0,
         )
         defaults.update(kw)
         super().__init__(**defaults)
@@ -144,6 +167,8 @@ def based_360m_released_config(**overrides) -> StackConfig:
 
 def create_mixer_cls(config, layer_idx=None, device=None, dtype=None):
     """Layer -> mixer routing of gpt.py:64-96."""
+    if config.layer_specs is not None:
+        return partial(_instantiate, config.layer_specs[layer_idx]["mixer"], device=device, dtype=dtype, layer_idx=layer_idx)
     value = config.mixer
     if config.alt_mixer_2_layers is not None and layer_idx in config.alt_mixer_2_layers:
         value = config.alt_mixer_2
@@ -199,11 +224,40 @@ class RMSNorm(nn.Module):
         return (x * rstd * self.weight).to(x.dtype)
 
 
+class StreamNorm(nn.Module):
+    """Layer norm without a bias ("layer") or RMS norm ("rms") of the fp32 residual sum
+    residual + mult * x, in one launch with that sum (`ops.add_norm`)."""
+
+    KINDS = {"layer": ops.NORM_LAYER, "rms": ops.NORM_RMS}
+
+    def __init__(self, hidden_size, eps=1e-5, kind="layer", mult=1.0, device=None, dtype=None):
+        super().__init__()
+        self.eps, self.kind, self.mult = eps, self.KINDS[kind], mult
+        self.weight = nn.Parameter(torch.ones(hidden_size, device=device, dtype=dtype))
+
+    def forward(self, x):
+        return ops.add_norm(x, None, self.weight, self.eps, self.kind, want_residual=False)[0]
+
+
+def norm_prologue(norm, residual_in, residual_out=None):
+    """Arguments of `ops.decode_linear` that put residual add + `norm` in front of a projection."""
+    common = dict(residual_in=residual_in, residual_out=residual_out, norm_weight=norm.weight, eps=norm.eps)
+    if isinstance(norm, StreamNorm):
+        return dict(prologue=ops.PROLOGUE_STREAM, mult=norm.mult, norm_kind=norm.kind, **common)
+    return dict(prologue=ops.PROLOGUE_ADD_RMS_NORM, **common)
+
+
+def norm_fuses(norm) -> bool:
+    return isinstance(norm, (RMSNorm, StreamNorm)) and norm.weight.dtype == torch.bfloat16
+
+
 def add_norm(norm, hidden_states, residual, residual_in_fp32: bool, want_residual: bool = True):
     """residual + hidden, the norm of the sum, and the sum itself for the next block
     (block.py:134-139; gpt.py:676-694 for the closing norm).  RMSNorm on tensors the kernel takes
     is one launch; nn.LayerNorm (`rms_norm: False`, the reference's default) and everything the
     kernel refuses run the reference's own torch statement."""
+    if isinstance(norm, StreamNorm):
+        return ops.add_norm(hidden_states, residual, norm.weight, norm.eps, norm.kind, norm.mult, want_residual)
     if isinstance(norm, RMSNorm) and _norm_kernel_takes(hidden_states, residual, norm.weight):
         if residual is None:
             return ops.add_rms_norm(hidden_states, None, norm.weight, norm.eps, residual_in_fp32, want_residual)
@@ -259,19 +313,24 @@ class GatedMlp(nn.Module):
 
 class Block(nn.Module):
     """Prenorm block: add -> norm1 -> mixer -> add -> norm2 -> mlp, returning (hidden, residual)
-    (block.py:134-163, dropout-free)."""
+    (block.py:134-163, dropout-free).  mlp_cls None: the mixer alone.  input_conv_cls: a causal
+    convolution between norm1 and the mixer whose output is added to its input."""
 
-    def __init__(self, dim, mixer_cls, mlp_cls, norm_cls, residual_in_fp32=True, layer_idx=None):
+    def __init__(self, dim, mixer_cls, mlp_cls, norm_cls, residual_in_fp32=True, layer_idx=None, input_conv_cls=None):
         super().__init__()
         self.residual_in_fp32 = residual_in_fp32
         self.layer_idx = layer_idx
         self.mixer = mixer_cls(dim)
         self.norm1 = norm_cls(dim)
-        self.mlp = mlp_cls(dim)
-        self.norm2 = norm_cls(dim)
+        self.input_conv = None if input_conv_cls is None else input_conv_cls(dim, layer_idx=layer_idx)
+        self.mlp = None if mlp_cls is None else mlp_cls(dim)
+        self.norm2 = None if mlp_cls is None else norm_cls(dim)
 
     def allocate_inference_cache(self, batch_size, max_seqlen, dtype=None, **kwargs):
-        return self.mixer.allocate_inference_cache(batch_size, max_seqlen, dtype=dtype, **kwargs)
+        cache = self.mixer.allocate_inference_cache(batch_size, max_seqlen, dtype=dtype, **kwargs)
+        if self.input_conv is not None:
+            cache[self.input_conv.name] = self.input_conv.allocate_ring(batch_size)
+        return cache
 
     def _add_norm(self, norm, hidden_states, residual):
         """residual + hidden, the norm of the sum, and the sum kept for the next block
@@ -281,10 +340,10 @@ class Block(nn.Module):
     def supports_decode_step(self) -> bool:
         mlp = self.mlp
         return (getattr(self.mixer, "supports_decode_step", lambda: False)()
-                and mlp.mlp_type == "base" and mlp.activation == "swiglu"
-                and ops.decode_linear_weight_ok(mlp.fc1.weight) and ops.decode_linear_weight_ok(mlp.fc2.weight)
-                and isinstance(self.norm1, RMSNorm) and isinstance(self.norm2, RMSNorm)
-                and self.norm1.weight.dtype == torch.bfloat16 and self.residual_in_fp32)
+                and (mlp is None or (mlp.mlp_type == "base" and mlp.activation == "swiglu"
+                                     and ops.decode_linear_weight_ok(mlp.fc1.weight)
+                                     and ops.decode_linear_weight_ok(mlp.fc2.weight) and norm_fuses(self.norm2)))
+                and norm_fuses(self.norm1) and self.residual_in_fp32)
 
     def decode_step(self, hidden_states, residual, spare, inference_params, row_index=None):
         """The block for one token per sequence in four to five launches: both norms run inside the
@@ -296,13 +355,17 @@ class Block(nn.Module):
             residual_in, mid, last = None, spare[0], spare[1]
         else:
             residual_in, mid, last = residual, spare, residual
-        norm = dict(prologue=ops.PROLOGUE_ADD_RMS_NORM, residual_in=residual_in, residual_out=mid,
-                    norm_weight=self.norm1.weight, eps=self.norm1.eps)
+        norm = norm_prologue(self.norm1, residual_in, mid)
         if row_index is not None:
             norm["row_index"] = row_index
+        if self.input_conv is not None:
+            rows = mid.shape[0]
+            pos, _ = portion_start(inference_params, rows, 1)
+            norm["input_conv"] = (self.input_conv.weight, self.input_conv.ring(inference_params, rows), pos)
         hidden_states = self.mixer.decode_step(hidden_states, inference_params, **norm)
-        norm = dict(prologue=ops.PROLOGUE_ADD_RMS_NORM, residual_in=mid, residual_out=last,
-                    norm_weight=self.norm2.weight, eps=self.norm2.eps)
+        if self.mlp is None:
+            return hidden_states, mid, last
+        norm = norm_prologue(self.norm2, mid, last)
         fc1, fc2 = self.mlp.fc1, self.mlp.fc2
         if fc1.weight.shape[1] <= 2048:
             # the gate in the tail of fc1
@@ -317,10 +380,14 @@ class Block(nn.Module):
     def forward(self, hidden_states, residual=None, mixer_kwargs=None, position_ids=None, decay=None):
         hidden_states, residual = self._add_norm(self.norm1, hidden_states, residual)
         mixer_kwargs = mixer_kwargs or {}
+        if self.input_conv is not None:
+            hidden_states = self.input_conv(hidden_states, mixer_kwargs.get("inference_params"))
         if position_ids is not None or decay is not None:
             hidden_states = self.mixer(hidden_states, position_ids=position_ids, decay=decay, **mixer_kwargs)
         else:
             hidden_states = self.mixer(hidden_states, **mixer_kwargs)
+        if self.mlp is None:
+            return hidden_states, residual
         hidden_states, residual = self._add_norm(self.norm2, hidden_states, residual)
         return self.mlp(hidden_states), residual
 
@@ -349,13 +416,29 @@ class GPTModel(nn.Module):
         if config.max_position_embeddings > 0:
             self.embeddings.position_embeddings = nn.Embedding(config.max_position_embeddings, config.hidden_size, **fk)
         # rms_norm absent from a reference config means nn.LayerNorm (gpt.py:352,537)
-        norm_cls = partial(RMSNorm if config.rms_norm else nn.LayerNorm, eps=config.layer_norm_epsilon, **fk)
+        if config.stream_norm is not None:
+            norm_cls = partial(StreamNorm, eps=config.layer_norm_epsilon, kind=config.stream_norm, mult=config.residual_mult, **fk)
+        else:
+            if config.residual_mult != 1.0:
+                raise NotImplementedError("residual_mult needs stream_norm")
+            norm_cls = partial(RMSNorm if config.rms_norm else nn.LayerNorm, eps=config.layer_norm_epsilon, **fk)
+        input_conv_cls = None
+        if config.input_conv_taps > 0:
+            input_conv_cls = partial(StreamConv, taps=config.input_conv_taps, add_input=True, name="input_conv", **fk)
         mlp_cls = partial(GatedMlp, hidden_features=config.n_inner, activation=config.activation_function,
                           bias1=config.mlp_fc1_bias, bias2=config.mlp_fc2_bias, mlp_type=config.mlp_type,
                           ff_mult=config.ff_mult, **fk)
+
+        def layer_mlp(i):
+            if config.layer_specs is None:
+                return mlp_cls
+            spec = config.layer_specs[i]["mlp"]
+            # hidden sizes are rounded up to the 16-byte pieces of the gate kernel; the extra ones carry zero weights
+            return None if spec is None else partial(mlp_cls, hidden_features=spec["hidden"], multiple_of=8)
+
         self.layers = nn.ModuleList([
-            Block(config.hidden_size, create_mixer_cls(config, layer_idx=i, **fk), mlp_cls, norm_cls,
-                  residual_in_fp32=config.residual_in_fp32, layer_idx=i)
+            Block(config.hidden_size, create_mixer_cls(config, layer_idx=i, **fk), layer_mlp(i), norm_cls,
+                  residual_in_fp32=config.residual_in_fp32, layer_idx=i, input_conv_cls=input_conv_cls)
             for i in range(config.num_hidden_layers)
         ])
         self.ln_f = norm_cls(config.hidden_size)
@@ -382,8 +465,7 @@ class GPTModel(nn.Module):
         table = self.embeddings.word_embeddings.weight
         cached = self.__dict__.get("_decode_layers_supported")
         if cached is None or cached[0] != (table.dtype, table.device):
-            ok = (ops.decode_linear_weight_ok(table) and isinstance(self.ln_f, RMSNorm)
-                  and self.ln_f.weight.dtype == torch.bfloat16
+            ok = (ops.decode_linear_weight_ok(table) and norm_fuses(self.ln_f)
                   and all(layer.supports_decode_step() for layer in self.layers))
             cached = ((table.dtype, table.device), ok)
             self.__dict__["_decode_layers_supported"] = cached
@@ -446,13 +528,18 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
         `config.json` (the GPT2Config dictionary) and `pytorch_model.bin` or `model.safetensors`.
         Counterpart of from_pretrained_hf (gpt.py:446-459) without the hub: same key clean-up
         (leading "model." stripped, training-metric entries dropped).  The weights file is read
-        with a loader that executes nothing from it."""
+        with a loader that executes nothing from it.  A config.json that names an `architecture` of
+        `based_amd.architectures` has its own keys and tensor names, which that module translates."""
         import json
         import os
         import re
 
+        from . import architectures
+
         with open(os.path.join(directory, "config.json")) as f:
-            config = StackConfig.from_reference_dict(json.load(f))
+            raw = json.load(f)
+        design = architectures.find(raw)
+        config = StackConfig(**design.stack_config(raw)) if design else StackConfig.from_reference_dict(raw)
         model = cls(config, device=device, dtype=dtype)
         st_path = os.path.join(directory, "model.safetensors")
         if os.path.exists(st_path):
@@ -461,6 +548,9 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             state = load_file(st_path, device="cpu")
         else:
             state = torch.load(os.path.join(directory, "pytorch_model.bin"), map_location="cpu", weights_only=True)
+        if design:
+            model.load_state_dict(design.convert_state(raw, state), strict=strict)
+            return model
         state = {re.sub(r"^model\.", "", k): v for k, v in state.items() if "metrics" not in k}
         if config.tie_word_embeddings and "lm_head.weight" not in state:
             state["lm_head.weight"] = state["transformer.embeddings.word_embeddings.weight"]
@@ -489,7 +579,9 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             move("transformer.ln_0", "transformer.layers.0.norm1")
         return super().load_state_dict(state_dict, strict=strict, **kwargs)
 
-    def forward(self, input_ids, position_ids=None, inference_params=None, num_last_tokens=0, stream=None, **kwargs):
+    def forward(self, input_ids, position_ids=None, inference_params=None, num_last_tokens=0, stream=None,
+                logits_at=None, **kwargs):
+        """logits_at: None, or the places within the portion whose logits are wanted."""
         assert input_ids.ndim == 2, f"Expected `input_ids` to have shape [b, slen], but got shape {input_ids.shape}"
         CausalLMOutput = namedtuple("CausalLMOutput", ["logits"])
         if (self.transformer.decode_layers_ok(input_ids, inference_params)
@@ -497,12 +589,12 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             # closing add + norm inside the LM head's projection
             hidden_states, residual = self.transformer.decode_layers(input_ids, inference_params)
             ln_f = self.transformer.ln_f
-            logits = ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias,
-                                       prologue=ops.PROLOGUE_ADD_RMS_NORM, residual_in=residual,
-                                       norm_weight=ln_f.weight, eps=ln_f.eps)
+            logits = ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias, **norm_prologue(ln_f, residual))
             return CausalLMOutput(logits=logits.unsqueeze(1))
         hidden_states = self.transformer(input_ids, position_ids=position_ids, inference_params=inference_params,
                                          stream=stream)
         if num_last_tokens > 0:
             hidden_states = hidden_states[:, -num_last_tokens:]
+        if logits_at is not None:
+            hidden_states = hidden_states[:, logits_at]
         return CausalLMOutput(logits=self.lm_head(hidden_states))

@@ -461,6 +461,107 @@ BASED_API int based_greedy_step(const void* logits, int64_t B, int64_t V, int64_
                                 int64_t seq_stride, int64_t seq_len, int32_t* lengths,
                                 int64_t* position_ids, int64_t pos_stride, int io_dtype, void* stream);
 
+/* ------------------------------------------------------------------------------------------------
+ * Streaming layers: no counterpart in the reference.  Sequences arrive in portions of any length;
+ * what a portion needs of the ones before it is a cache of keys and values, fp32 recurrent states, and
+ * rings of past convolution inputs (rows, taps, channels) in which slot p % taps holds the input at
+ * position p.  Nothing has to be cleared when a sequence starts: inputs before position 0 count as
+ * zeros, and `fresh` (or position 0 in a single-token step) starts a recurrence at zero.
+ * Single-token entry points take their positions from `pos` (int32, one per row) or, when it is
+ * NULL, from pos_host.  Element type BASED_BF16 or BASED_F32 throughout; what enters a norm, a softmax
+ * or a recurrence is evaluated in fp32.
+ */
+
+enum { BASED_NORM_RMS = 0, BASED_NORM_LAYER = 1 };
+enum { BASED_ACT_NONE = 0, BASED_ACT_SILU = 1 };
+#define BASED_STREAM_MAX_TAPS 8
+
+/* r = residual_in + mult * x in fp32 (r = x when residual_in is NULL), written to residual_out when
+ * given; y = norm(r) * weight, norm = r / sqrt(mean(r^2) + eps) or (r - mean) / sqrt(var + eps). */
+BASED_API int based_add_norm(const void* x, const float* residual_in, const void* weight, void* y,
+                             float* residual_out, int64_t rows, int64_t D, int64_t x_sr, int64_t ri_sr,
+                             int64_t y_sr, int64_t ro_sr, float eps, int kind, float mult, int io_dtype,
+                             void* stream);
+
+/* y_t = [x_t +] act(bias + sum_j weight[j] x_{t - taps + 1 + j}) per channel; x, y (B, L, D);
+ * weight (taps, D); bias (D) or NULL; ring (B, taps, D) or NULL, read for the inputs before the portion
+ * and updated with its last ones.  The portion starts at pos[b] / pos_host. */
+BASED_API int based_stream_conv(const void* x, const void* weight, const void* bias, void* y, void* ring,
+                                const int32_t* pos, int64_t pos_host, int64_t B, int64_t L, int64_t D,
+                                int taps, int64_t x_sb, int64_t x_sl, int64_t y_sb, int64_t y_sl,
+                                int64_t ring_sb, int activation, int add_input, int io_dtype, void* stream);
+
+/* Sliding-window attention with grouped heads: position i attends j, 0 <= i - j < window; query head h
+ * reads key/value head h / (H / G).  q (B, L, H, D), k (B, L, G, D), v (B, L, G, DV), heads contiguous;
+ * kv_cache (B, S, G, D + DV): key channels (rotated), then value channels.  Rows start .. start + L - 1
+ * are written before they are attended.  Rotation of the first rotary_dim channels by tables
+ * (rope_len, rotary_dim / 2), interleaved pairs or, half_split, pairs (i, i + rotary_dim / 2); norm_v
+ * divides each value by sqrt(mean(v^2) + eps); the output is multiplied by out_scale. */
+BASED_API int based_window_attn_prefill(const void* q, const void* k, const void* v, void* kv_cache, void* o, int64_t start,
+                                        int64_t B, int64_t L, int64_t H, int64_t G, int64_t D, int64_t DV, int64_t S,
+                                        int64_t q_sb, int64_t q_sl, int64_t k_sb, int64_t k_sl, int64_t v_sb, int64_t v_sl,
+                                        int64_t o_sb, int64_t o_sl, int64_t kv_sb, int64_t kv_st, int64_t window,
+                                        float scale, int norm_v, float eps, float out_scale, const float* rope_cos,
+                                        const float* rope_sin, int64_t rope_len, int64_t rotary_dim, int half_split,
+                                        int io_dtype, void* stream);
+BASED_API int based_window_attn_step(const void* q, const void* k, const void* v, void* kv_cache, void* o, const int32_t* pos,
+                                     int64_t pos_host, int64_t B, int64_t H, int64_t G, int64_t D, int64_t DV, int64_t S,
+                                     int64_t q_sb, int64_t k_sb, int64_t v_sb, int64_t o_sb, int64_t kv_sb, int64_t kv_st,
+                                     int64_t window, float scale, int norm_v, float eps, float out_scale,
+                                     const float* rope_cos, const float* rope_sin, int64_t rope_len, int64_t rotary_dim,
+                                     int half_split, int io_dtype, void* stream);
+
+/* Gated delta rule over a portion.  q, k (B, L, G, D) and v (B, L, H, DV) convolved and activated, one
+ * pair of strides for the three; a_gate, b_gate (B, L, H) projections; a_log, dt_bias (H).
+ * g = exp(-exp(a_log) softplus(a + dt_bias)), beta = sigmoid(b); q and k made unit vectors, q times
+ * D^(-1/2); S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
+ * state (B, H, D, state_row) fp32, o (B, L, H, DV) fp32. */
+BASED_API int based_gated_delta_scan(const void* q, const void* k, const void* v, const void* a_gate, const void* b_gate,
+                                     const void* a_log, const void* dt_bias, float* state, float* o, int64_t B, int64_t L,
+                                     int64_t H, int64_t G, int64_t D, int64_t DV, int64_t state_row, int64_t x_sb,
+                                     int64_t x_sl, int64_t g_sb, int64_t g_sl, int fresh, int io_dtype, void* stream);
+
+/* y = o / sqrt(mean(o^2) + eps) * weight * silu(gate) * scale per (token, head); o (B, L, H, DV) fp32. */
+BASED_API int based_gated_rms_norm(const float* o, const void* weight, const void* gate, void* y, int64_t B, int64_t L,
+                                   int64_t H, int64_t DV, int64_t g_sb, int64_t g_sl, int64_t y_sb, int64_t y_sl, float eps,
+                                   float scale, int io_dtype, void* stream);
+
+/* One token of the whole block between its projections: convolution + silu of x (B, C) (queries at
+ * channel 0, keys at k_off, values at v_off), the delta rule, the output norm and gate. */
+BASED_API int based_gated_delta_step(const void* x, const void* conv_w, void* ring, const void* a_gate, const void* b_gate,
+                                     const void* out_gate, const void* a_log, const void* dt_bias, const void* norm_w,
+                                     float* state, void* y, const int32_t* pos, int64_t pos_host, int64_t B, int64_t H,
+                                     int64_t G, int64_t D, int64_t DV, int64_t state_row, int64_t C, int taps, int64_t k_off,
+                                     int64_t v_off, int64_t x_sb, int64_t g_sb, int64_t gate_sb, int64_t y_sb,
+                                     int64_t ring_sb, float eps, float scale, int io_dtype, void* stream);
+
+/* Real-gated linear recurrent unit over a portion.  u (B, L, W) convolved; ra, ri (blocks, W / blocks,
+ * W / blocks) as [out, in]; rb, ib, lam (W).  r = sigmoid(ra u + rb), i = sigmoid(ri u + ib),
+ * a = exp(-c r softplus(lam)), S <- a S + sqrt(1 - a^2) i u, out = S * gelu_tanh(y).
+ * work_a, work_x: fp32 (B, L, W); work_agg: fp32 (B, ceil(L / 64) + 1, 2, W); state (B, W) fp32. */
+BASED_API int based_rglru_prefill(const void* u, const void* y, const void* ra, const void* rb, const void* ri, const void* ib,
+                                  const void* lam, float* work_a, float* work_x, float* work_agg, float* state, void* out,
+                                  int64_t B, int64_t L, int64_t W, int64_t blocks, int64_t u_sb, int64_t u_sl, int64_t y_sb,
+                                  int64_t y_sl, int64_t o_sb, int64_t o_sl, float c, int fresh, int io_dtype, void* stream);
+
+/* One token of it, with the convolution (weight (taps, W), bias (W) or NULL) in front. */
+BASED_API int based_rglru_step(const void* x, const void* y, const void* conv_w, const void* conv_b, void* ring, const void* ra,
+                               const void* rb, const void* ri, const void* ib, const void* lam, float* state, void* out,
+                               const int32_t* pos, int64_t pos_host, int64_t B, int64_t W, int64_t blocks, int taps,
+                               int64_t x_sb, int64_t y_sb, int64_t o_sb, int64_t ring_sb, float c, int io_dtype,
+                               void* stream);
+
+/* based_decode_linear (bf16) behind the streamed-input prologue: r = residual_in + mult * x in fp32,
+ * h = norm(r) * norm_weight rounded to bf16 and, with taps > 0, h + sum_j conv_weight[j] h_{t-taps+1+j} on
+ * a ring (M, taps, K), projected.  epilogue: BASED_EPILOGUE_NONE or BASED_EPILOGUE_SWIGLU. */
+BASED_API int based_decode_linear_stream(const void* x, int64_t x_row_stride, const int64_t* x_row_index, int64_t x_index_rows,
+                                         const void* weight, int64_t w_row_stride, const void* bias, void* y,
+                                         int64_t y_row_stride, int64_t M, int64_t N, int64_t K, const float* residual_in,
+                                         int64_t ri_row_stride, float* residual_out, int64_t ro_row_stride, float mult,
+                                         int norm_kind, const void* norm_weight, float eps, const void* conv_weight,
+                                         void* conv_ring, int64_t conv_ring_row_stride, int taps, const int32_t* pos,
+                                         int64_t pos_host, int epilogue, void* stream);
+
 #ifdef __cplusplus
 }
 #endif
