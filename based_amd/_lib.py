@@ -108,7 +108,7 @@ SIGNATURES = {
         C.c_int,
         [_P] * 6 + [_I64] * 14 + [C.c_float, C.c_int, C.c_float, C.c_float, _P, _P, _I64, _I64, C.c_int, C.c_int, _P],
     ),
-    "based_gated_delta_scan": (C.c_int, [_P] * 9 + [_I64] * 11 + [C.c_int, C.c_int, _P]),
+    "based_gated_delta_scan": (C.c_int, [_P] * 10 + [_I64] * 11 + [C.c_int, C.c_int, _P]),
     "based_gated_rms_norm": (C.c_int, [_P] * 4 + [_I64] * 8 + [C.c_float, C.c_float, C.c_int, _P]),
     "based_gated_delta_step": (
         C.c_int, [_P] * 12 + [_I64] * 8 + [C.c_int] + [_I64] * 7 + [C.c_float, C.c_float, C.c_int, _P]),

@@ -310,24 +310,34 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
         }
       }
       // the ring rows of the past inputs, in flight during the reductions
-      constexpr int kMaxPast = BASED_STREAM_MAX_TAPS - 1;
       float past[C][8];
 #pragma unroll
       for (int c = 0; c < C; ++c)
 #pragma unroll
         for (int i = 0; i < 8; ++i) past[c][i] = 0.f;
-      const __bf16* ring = a.ic_ring + (long)(a.m0 + m) * a.ic_ring_sr;
-#pragma unroll 1
-      for (int j = 0; j < kMaxPast; ++j) {
-        const int p = pos - (a.ic_taps - 1) + j;
-        if (j >= a.ic_taps - 1) break;
-        if (p < 0) continue;
+      if (a.ic_taps > 1) {
+        const __bf16* ring = a.ic_ring + (long)(a.m0 + m) * a.ic_ring_sr;
+        // a few inputs at a time; those that do not exist are fetched as zeros
+        constexpr int PB = C >= 8 ? 1 : 3;
+        for (int j0 = 0; j0 < a.ic_taps - 1; j0 += PB) {
+          bf16x8 x8[PB][C], w8[PB][C];
 #pragma unroll
-        for (int c = 0; c < C; ++c) {
-          const bf16x8 x8 = *reinterpret_cast<const bf16x8*>(live[c] ? ring + (long)(p % a.ic_taps) * a.K + e0[c] : zeros);
-          const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.ic_w + (long)j * a.K + e0[c] : zeros);
+          for (int j = 0; j < PB; ++j) {
+            const int p = pos - (a.ic_taps - 1) + j0 + j;
+            const bool ok = j0 + j < a.ic_taps - 1 && p >= 0;
+            const long slot = (long)((ok ? p : 0) % a.ic_taps) * a.K, tap = (long)(ok ? j0 + j : 0) * a.K;
 #pragma unroll
-          for (int i = 0; i < 8; ++i) past[c][i] = __builtin_fmaf(to_f32(w8[i]), to_f32(x8[i]), past[c][i]);
+            for (int c = 0; c < C; ++c) {
+              x8[j][c] = *reinterpret_cast<const bf16x8*>(ok && live[c] ? ring + slot + e0[c] : zeros);
+              w8[j][c] = *reinterpret_cast<const bf16x8*>(ok && live[c] ? a.ic_w + tap + e0[c] : zeros);
+            }
+          }
+#pragma unroll
+          for (int j = 0; j < PB; ++j)
+#pragma unroll
+            for (int c = 0; c < C; ++c)
+#pragma unroll
+              for (int i = 0; i < 8; ++i) past[c][i] = __builtin_fmaf(to_f32(w8[j][c][i]), to_f32(x8[j][c][i]), past[c][i]);
         }
       }
       const float mean = a.norm_kind == BASED_NORM_LAYER ? wave_sum_dpp(sum) / (float)a.K : 0.f;

@@ -12,25 +12,31 @@
 //                       output norm and the output gate.
 //   gated_rms_norm      o / rms(o) * w * silu(gate) * scale, behind the scan.
 //
-// The scan walks tokens rather than blocks of tokens: 32-bit products are required, fp32 MFMA has
-// the rate of the vector unit, and the blocked form needs about twice the products of the
-// recurrence.  How a prompt is cut then cannot change more than the rounding of the carried state.
-// Three products per state element and token:
-//   * S^T k and S^T q are taken in one pass over the state BEFORE the update,
-//     o = g S0^T q + (k . q) u, so that one reduction per token is on the dependent path;
-//   * the decay is not multiplied into the state: the state is kept divided by the running product
-//     of decays G, S = G Z, Z += k (u / G)^T, and Z is brought back to G = 1 when G gets small.
-// A wavefront holds 8 CPL columns: lane = 8 column groups x 8 row groups, RPL rows x CPL columns in
-// registers; the sums over rows are three DPP additions within 8 lanes.  Queries, keys and values
-// of 16 tokens at a time are normalised and laid out in LDS in fp32 (two buffers), the raw ones of
-// the tile after that being on their way in registers.
+// The scan takes 16 tokens at a time, all of it in fp32 (fp32 MFMA, which has twice the rate of the
+// vector unit).  With the decays multiplied up inside the block, G_t = g_1 .. g_t:
+//   u_t = beta_t (v_t - G_t S0^T k_t) - sum_{s<t} A_ts u_s,   A_ts = beta_t (k_t . k_s) G_t / G_s
+//   o_t = G_t S0^T q_t + sum_{s<=t} P_ts u_s,                 P_ts = (q_t . k_s) G_t / G_s
+//   S16 = G_16 S0 + sum_s k_s (G_16 / G_s) u_s^T
+// so with T = (I + A)^-1, U = T R.  At 16 tokens the products inside a block are a seventh of those
+// with the state for 128 channels.  The quotients of decays are exponentials of differences of log
+// decays: none of them overflows, and a decay of zero is zero.
+//   gated_delta_prepare  T, P, the decays and the norm factors of every block, all blocks at once, one
+//                        wavefront each; T by forward substitution (a power series in A would lose
+//                        digits to cancellation)
+//   gated_delta_scan     walks the blocks with the state in MFMA accumulators.  The accumulator layout
+//                        (column = lane % 16, rows 4 (lane / 16) + i) is the second operand of
+//                        instruction i as it stands when the contraction runs over rows {i, 4 + i,
+//                        8 + i, 12 + i}, so neither the state nor U is ever moved between lanes.
 #include "stream_common.hpp"
 
 namespace based {
 
 constexpr float kUnitEps = 1e-6f;
-constexpr int kDeltaTile = 16;               // tokens staged together
-constexpr float kRescaleBelow = 1e-9f;       // running decay at which the stored state is brought back to scale 1
+constexpr int kBlk = 16;            // tokens per block
+// what gated_delta_prepare leaves per (sequence, head, block): T and P row-major, then 16 each of G_t,
+// G_16 / G_t, beta_t, the factor of q_t and of k_t
+constexpr int kPrepT = 0, kPrepP = 256, kPrepG = 512, kPrepTail = 528, kPrepBeta = 544, kPrepFq = 560, kPrepFk = 576;
+constexpr int kPrepFloats = BASED_DELTA_PREP_FLOATS;
 
 struct DeltaArgs {
   const void* q;
@@ -42,215 +48,280 @@ struct DeltaArgs {
   const void* dt_bias;
   float* state;  // (B, H, d, dvp)
   float* o;      // (B, L, H, dv)
-  int B, L, H, G, d, dv, dvp;
+  float* prep;   // (B, H, blocks, kPrepFloats)
+  int B, L, H, G, d, dv, dvp, blocks;
   long x_sb, x_sl;  // strides of q, k, v
   long g_sb, g_sl;  // strides of a, bt
-  int fresh;
+  int fresh, vec;
 };
 
-template <typename T> __device__ __forceinline__ float decay_of(float a, const void* a_log, const void* dt_bias, int h) {
+template <typename T> __device__ __forceinline__ float log_decay_of(float a, const void* a_log, const void* dt_bias, int h) {
   const float dt = softplus_f(a + to_f32(static_cast<const T*>(dt_bias)[h]));
-  return expf(-expf(to_f32(static_cast<const T*>(a_log)[h])) * dt);
+  return -expf(to_f32(static_cast<const T*>(a_log)[h])) * dt;
 }
 
-// E consecutive elements as they lie in memory; VEC: aligned to their size (16 bytes at most)
-template <typename T, int E> struct Raw {
-  static constexpr int kPer = E * (int)sizeof(T) > 16 ? 16 / (int)sizeof(T) : E;
-  typedef __attribute__((ext_vector_type(kPer))) T piece_t;
-  piece_t p[E / kPer];
-  __device__ __forceinline__ float get(int i) const { return to_f32(p[i / kPer][i % kPer]); }
-  template <bool VEC> __device__ __forceinline__ void load(const T* src, int valid) {
+__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
+
+// 4 consecutive channels of a row of d, zeros past its end
+template <typename T> __device__ __forceinline__ f32x4 load4(const T* row, int e, int d, int vec) {
+  f32x4 x = {0.f, 0.f, 0.f, 0.f};
+  if (vec) {
+    typedef __attribute__((ext_vector_type(4))) T t4;
+    if (e < d) {
+      const t4 r = *reinterpret_cast<const t4*>(row + e);
 #pragma unroll
-    for (int i = 0; i < E / kPer; ++i) {
-      if constexpr (VEC) {
-        // whole pieces are inside the row or outside of it
-        const piece_t x = *reinterpret_cast<const piece_t*>(src + (i * kPer < valid ? i * kPer : 0));
+      for (int i = 0; i < 4; ++i) x[i] = to_f32(r[i]);
+    }
+  } else {
 #pragma unroll
-        for (int j = 0; j < kPer; ++j) p[i][j] = i * kPer < valid ? x[j] : (T)0.0f;
-      } else {
+    for (int i = 0; i < 4; ++i)
+      if (e + i < d) x[i] = to_f32(row[e + i]);
+  }
+  return x;
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArgs a) {
+  __shared__ __attribute__((aligned(16))) float s_a[4][kBlk][kBlk + 4];
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, quad = lane >> 4;
+  const long n_items = (long)a.B * a.H * a.blocks;
+  const long item0 = (long)blockIdx.x * 4 + wave;
+  const bool live = item0 < n_items;
+  const long item = live ? item0 : n_items - 1;
+  const int blk = (int)(item % a.blocks);
+  const int h = (int)(item / a.blocks % a.H), b = (int)(item / a.blocks / a.H), hk = h / (a.H / a.G);
+  const int t0 = blk * kBlk, tok = t0 + l16;
+  const bool in = tok < a.L;
+  const long row = in ? tok : a.L - 1;
+  const T* q = static_cast<const T*>(a.q) + b * a.x_sb + row * a.x_sl + (long)hk * a.d;
+  const T* k = static_cast<const T*>(a.k) + b * a.x_sb + row * a.x_sl + (long)hk * a.d;
+  const long gate = b * a.g_sb + row * a.g_sl + h;
+  // token l16's gates, in every lane of that number
+  const float beta = in ? sigmoid_f(to_f32(static_cast<const T*>(a.bt)[gate])) : 0.f;
+  float lg = in ? log_decay_of<T>(to_f32(static_cast<const T*>(a.a)[gate]), a.a_log, a.dt_bias, h) : 0.f;
+  lg = fmaxf(lg, -200.f);  // exp(-200) is zero in fp32
+  f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
+  float sq = 0.f, sk = 0.f;
+  for (int e = quad * 4; e < a.d + quad * 4; e += 16) {
+    const f32x4 x = load4(q, e, a.d, a.vec), y = load4(k, e, a.d, a.vec);
 #pragma unroll
-        for (int j = 0; j < kPer; ++j) {
-          const T x = src[i * kPer + j < valid ? i * kPer + j : 0];
-          p[i][j] = i * kPer + j < valid ? x : (T)0.0f;
-        }
-      }
+    for (int i = 0; i < 4; ++i) {
+      sq = __builtin_fmaf(x[i], x[i], sq);
+      sk = __builtin_fmaf(y[i], y[i], sk);
+      kk = mfma_f32(y[i], y[i], kk);
+      qk = mfma_f32(x[i], y[i], qk);
     }
   }
-};
+  sq += __shfl_xor(sq, 16, 64), sk += __shfl_xor(sk, 16, 64);
+  sq += __shfl_xor(sq, 32, 64), sk += __shfl_xor(sk, 32, 64);
+  const float fq = in ? 1.0f / (sqrtf((float)a.d) * sqrtf(sq + kUnitEps)) : 0.f, fk = in ? 1.0f / sqrtf(sk + kUnitEps) : 0.f;
+  // log G of token l16, in 64 bits: behind a token that forgets nearly everything the differences of
+  // these sums still have to carry the ordinary decays
+  double lc = lg;
+#pragma unroll
+  for (int m = 1; m < 16; m <<= 1) {
+    const double up = __shfl_up(lc, m, 16);
+    if (l16 >= m) lc += up;
+  }
+  const double lc_end = __shfl(lc, 15, 64);
+  float* out = a.prep + item * kPrepFloats;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int t = quad * 4 + i;  // row; l16 is the column s
+    const double lc_t = __shfl(lc, t, 64);
+    const float beta_t = __shfl(beta, t, 64), fq_t = __shfl(fq, t, 64), fk_t = __shfl(fk, t, 64);
+    const float ratio = l16 <= t ? expf(fminf((float)(lc_t - lc), 0.f)) : 0.f;
+    s_a[wave][t][l16] = l16 < t ? beta_t * kk[i] * fk_t * fk * ratio : 0.f;
+    if (live) out[kPrepP + t * kBlk + l16] = qk[i] * fq_t * fk * ratio;
+  }
+  if (live && quad == 0) {
+    out[kPrepG + l16] = expf((float)lc);
+    out[kPrepTail + l16] = expf(fminf((float)(lc_end - lc), 0.f));
+    out[kPrepBeta + l16] = beta;
+    out[kPrepFq + l16] = fq;
+    out[kPrepFk + l16] = fk;
+  }
+  __syncthreads();
+  // column l16 of T: x_t = [t = l16] - sum_{s<t} A_ts x_s
+  float x[kBlk];
+#pragma unroll
+  for (int t = 0; t < kBlk; ++t) {
+    float acc = t == l16 ? 1.f : 0.f;
+#pragma unroll
+    for (int s4 = 0; s4 < t; s4 += 4) {
+      const f32x4 r = *reinterpret_cast<const f32x4*>(&s_a[wave][t][s4]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (s4 + j < t) acc = __builtin_fmaf(-r[j], x[s4 + j], acc);
+    }
+    x[t] = acc;
+  }
+  if (live && quad == 0) {
+#pragma unroll
+    for (int t = 0; t < kBlk; ++t) out[kPrepT + t * kBlk + l16] = x[t];
+  }
+}
 
-template <typename T, int RPL, int CPL, int NW, bool VEC>
-__global__ __launch_bounds__(64 * NW) void gated_delta_scan_kernel(const DeltaArgs a) {
-  constexpr int D = RPL * 8;            // rows held (d <= D)
-  constexpr int COLS = NW * 8 * CPL;    // columns of the workgroup
-  constexpr int E = RPL / 2;            // channels of q and of k a staging thread brings: 16 threads per token
-  constexpr int PASSES = 4 / NW;        // tokens per pass: 4 NW
-  constexpr int EV = 2 * CPL;           // value channels a staging thread brings
-  __shared__ __attribute__((aligned(16))) float s_k[2][kDeltaTile][D];
-  __shared__ __attribute__((aligned(16))) float s_q[2][kDeltaTile][D];
-  __shared__ __attribute__((aligned(16))) float s_v[2][kDeltaTile][COLS];
-  __shared__ __attribute__((aligned(16))) float s_g[2][kDeltaTile][4];  // decay, beta, k . q
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, rg = lane & 7, cg = lane >> 3;
+// RB: 16-row blocks of the state; RS: wavefronts that share a 16-column tile, RB / RS row blocks each
+// (their partial products with the state are added up through LDS).  Four wavefronts per workgroup.
+template <typename T, int RB, int RS>
+__global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a) {
+  static_assert(RB % RS == 0 && 4 % RS == 0, "row blocks divide among the wavefronts of a tile");
+  constexpr int D = RB * 16, CT = 4 / RS, RBW = RB / RS;
+  constexpr int KS = D + 4, TS = kBlk + 4;           // LDS row strides in floats: 16 lanes of 16 bytes meet every bank once
+  constexpr int PIECES = kBlk * (D / 8);             // 8 channels of a token, of q and of k
+  constexpr int PP = (PIECES + 255) / 256;           // per thread
+  __shared__ __attribute__((aligned(16))) float s_k[2][kBlk * KS], s_q[2][kBlk * KS], s_kt[2][D * TS];
+  __shared__ __attribute__((aligned(16))) float s_part[RS > 1 ? CT * RS * 2 * 256 : 4];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int ct = wave / RS, rs = wave % RS;
   const int b = blockIdx.x / a.H, h = blockIdx.x % a.H, hk = h / (a.H / a.G);
-  const int col_wg = blockIdx.y * COLS, my_col = wave * 8 * CPL + cg * CPL;  // within the workgroup
+  const int col = (blockIdx.y * CT + ct) * 16 + l16;
+  const bool col_in = col < a.dv;
   const T* q = static_cast<const T*>(a.q) + b * a.x_sb + (long)hk * a.d;
   const T* k = static_cast<const T*>(a.k) + b * a.x_sb + (long)hk * a.d;
-  const T* v = static_cast<const T*>(a.v) + b * a.x_sb + (long)h * a.dv;
-  const T* ga = static_cast<const T*>(a.a) + b * a.g_sb + h;
-  const T* gb = static_cast<const T*>(a.bt) + b * a.g_sb + h;
+  const T* v = static_cast<const T*>(a.v) + b * a.x_sb + (long)h * a.dv + (col_in ? col : 0);
+  const float* prep = a.prep + ((long)b * a.H + h) * a.blocks * kPrepFloats;
+  float* st = a.state + ((long)b * a.H + h) * a.d * a.dvp + (col_in ? col : 0);
+  float* o = a.o + ((long)b * a.L * a.H + h) * a.dv + (col_in ? col : 0);
 
-  float S[RPL][CPL];
-  float* st = a.state + ((long)b * a.H + h) * a.d * a.dvp + col_wg + my_col;
+  f32x4 S[RBW];
 #pragma unroll
-  for (int i = 0; i < RPL; ++i) {
-    const int row = (i >> 2) * 32 + rg * 4 + (i & 3);
+  for (int r = 0; r < RBW; ++r)
 #pragma unroll
-    for (int c = 0; c < CPL; ++c) {
-      const bool in = !a.fresh && row < a.d && col_wg + my_col + c < a.dv;
-      S[i][c] = in ? st[(long)row * a.dvp + c] : 0.f;
+    for (int i = 0; i < 4; ++i) {
+      const int row = (rs * RBW + r) * 16 + quad * 4 + i;
+      const bool in = !a.fresh && col_in && row < a.d;
+      S[r][i] = in ? st[(long)row * a.dvp] : 0.f;
     }
-  }
 
-  // staging roles
-  const int part = tid & 15, tok0 = tid >> 4;               // q, k: channels part * E ..
-  const int vtok = tid / (4 * NW), vch = (tid % (4 * NW)) * EV;
-  Raw<T, E> rq[PASSES], rk[PASSES];
-  Raw<T, EV> rv;
-  T ra[PASSES], rb[PASSES];
-  auto fetch = [&](int l0) {
+  // what a block needs from memory is asked for one block ahead
+  f32x4 rk[PP][2], rq[PP][2];
+  float fk[PP], fq[PP];
+  f32x4 tn, pn, gn, tailn, betan;
+  T vn[4];
+  float lastn = 1.f;
+  auto fetch = [&](int blk) {
+    const float* pr = prep + (long)blk * kPrepFloats;
+    tn = *reinterpret_cast<const f32x4*>(pr + kPrepT + l16 * kBlk + quad * 4);
+    pn = *reinterpret_cast<const f32x4*>(pr + kPrepP + l16 * kBlk + quad * 4);
+    gn = *reinterpret_cast<const f32x4*>(pr + kPrepG + quad * 4);
+    tailn = *reinterpret_cast<const f32x4*>(pr + kPrepTail + quad * 4);
+    betan = *reinterpret_cast<const f32x4*>(pr + kPrepBeta + quad * 4);
+    lastn = pr[kPrepG + kBlk - 1];
 #pragma unroll
-    for (int p = 0; p < PASSES; ++p) {
-      const int l = l0 + p * 4 * NW + tok0;
-      const long row = l < a.L ? l : a.L - 1;
-      const int left = a.d - part * E;
-      rq[p].template load<VEC>(q + row * a.x_sl + (left > 0 ? part * E : 0), left);
-      rk[p].template load<VEC>(k + row * a.x_sl + (left > 0 ? part * E : 0), left);
-      ra[p] = ga[row * a.g_sl];
-      rb[p] = gb[row * a.g_sl];
+    for (int i = 0; i < 4; ++i) {
+      const int t = blk * kBlk + quad * 4 + i;
+      vn[i] = v[(long)(t < a.L ? t : a.L - 1) * a.x_sl];
     }
-    const int l = l0 + vtok;
-    const long row = l < a.L ? l : a.L - 1;
-    const int left = a.dv - col_wg - vch;
-    rv.template load<VEC>(v + row * a.x_sl + (left > 0 ? col_wg + vch : 0), left);
   };
-  const float q_scale = 1.0f / sqrtf((float)a.d);
+  auto fetch_qk = [&](int blk) {
+    const float* pr = prep + (long)blk * kPrepFloats;
+#pragma unroll
+    for (int p = 0; p < PP; ++p) {
+      const int piece = p * 256 + tid, t = piece & 15, e = (piece >> 4) * 8;
+      const long row = blk * kBlk + t < a.L ? blk * kBlk + t : a.L - 1;
+#pragma unroll
+      for (int j = 0; j < 2; ++j) {
+        rk[p][j] = load4(k + row * a.x_sl, e + 4 * j, a.d, a.vec);
+        rq[p][j] = load4(q + row * a.x_sl, e + 4 * j, a.d, a.vec);
+      }
+      fk[p] = pr[kPrepFk + t];
+      fq[p] = pr[kPrepFq + t];
+    }
+  };
   auto stage = [&](int buf) {
 #pragma unroll
-    for (int p = 0; p < PASSES; ++p) {
-      const int t = p * 4 * NW + tok0;
-      float qq = 0.f, kk = 0.f, qk = 0.f;
+    for (int p = 0; p < PP; ++p) {
+      const int piece = p * 256 + tid, t = piece & 15, e = (piece >> 4) * 8;
+      if (PIECES % 256 == 0 || piece < PIECES) {
 #pragma unroll
-      for (int i = 0; i < E; ++i) {
-        const float x = rq[p].get(i), y = rk[p].get(i);
-        qq = __builtin_fmaf(x, x, qq);
-        kk = __builtin_fmaf(y, y, kk);
-        qk = __builtin_fmaf(x, y, qk);
-      }
-      qq = sum16(qq), kk = sum16(kk), qk = sum16(qk);
-      const float fq = q_scale / sqrtf(qq + kUnitEps), fk = 1.0f / sqrtf(kk + kUnitEps);
+        for (int j = 0; j < 2; ++j) {
+          const f32x4 y = rk[p][j] * fk[p];
+          *reinterpret_cast<f32x4*>(&s_k[buf][t * KS + e + 4 * j]) = y;
+          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j] * fq[p];
 #pragma unroll
-      for (int i = 0; i < E; ++i) {
-        s_q[buf][t][part * E + i] = rq[p].get(i) * fq;
-        s_k[buf][t][part * E + i] = rk[p].get(i) * fk;
-      }
-      if (part == 0) {
-        s_g[buf][t][0] = decay_of<T>(to_f32(ra[p]), a.a_log, a.dt_bias, h);
-        s_g[buf][t][1] = sigmoid_f(to_f32(rb[p]));
-        s_g[buf][t][2] = qk * fq * fk;
+          for (int i = 0; i < 4; ++i) s_kt[buf][(e + 4 * j + i) * TS + t] = y[i];
+        }
       }
     }
-#pragma unroll
-    for (int i = 0; i < EV; ++i) s_v[buf][vtok][vch + i] = rv.get(i);
   };
 
+  fetch_qk(0);
   fetch(0);
   stage(0);
-  float G = 1.0f;
-  int buf = 0;
-  const bool writer = rg == 0;
-  float* op = a.o + ((long)b * a.L * a.H + h) * a.dv + col_wg + my_col;
-  const int cols_left = a.dv - col_wg - my_col;
-  for (int l0 = 0; l0 < a.L; l0 += kDeltaTile, buf ^= 1) {
-    __syncthreads();  // this tile is laid out; everyone is done with the other buffer
-    const bool more = l0 + kDeltaTile < a.L;
-    if (more) fetch(l0 + kDeltaTile);
-    const int n = a.L - l0 < kDeltaTile ? a.L - l0 : kDeltaTile;
-    f32x4 kn[RPL / 4], qn[RPL / 4], gn;
-    float vn[CPL];
-    auto load_token = [&](int t) {
+  for (int blk = 0, buf = 0; blk < a.blocks; ++blk, buf ^= 1) {
+    __syncthreads();  // this block is laid out; everyone is done with the other buffer
+    const f32x4 tm = tn, pm = pn, gm = gn, tail = tailn, beta = betan;
+    const float last = lastn;
+    float vv[4];
 #pragma unroll
-      for (int i = 0; i < RPL / 4; ++i) {
-        kn[i] = *reinterpret_cast<const f32x4*>(&s_k[buf][t][i * 32 + rg * 4]);
-        qn[i] = *reinterpret_cast<const f32x4*>(&s_q[buf][t][i * 32 + rg * 4]);
+    for (int i = 0; i < 4; ++i) vv[i] = to_f32(vn[i]);
+    const bool more = blk + 1 < a.blocks;
+    fetch_qk(more ? blk + 1 : blk);
+    fetch(more ? blk + 1 : blk);
+    f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
+#pragma unroll
+    for (int r = 0; r < RBW; ++r) {
+      const int e = (rs * RBW + r) * 16 + quad * 4;
+      const f32x4 kf = *reinterpret_cast<const f32x4*>(&s_k[buf][l16 * KS + e]);
+      const f32x4 qf = *reinterpret_cast<const f32x4*>(&s_q[buf][l16 * KS + e]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        ks = mfma_f32(kf[i], S[r][i], ks);
+        qs = mfma_f32(qf[i], S[r][i], qs);
       }
-      gn = *reinterpret_cast<const f32x4*>(&s_g[buf][t][0]);
+    }
+    if constexpr (RS > 1) {
+      f32x4* part = reinterpret_cast<f32x4*>(s_part) + ct * RS * 2 * 64;
+      part[(rs * 2 + 0) * 64 + lane] = ks;
+      part[(rs * 2 + 1) * 64 + lane] = qs;
+      __syncthreads();
+      ks = part[lane];
+      qs = part[64 + lane];
 #pragma unroll
-      for (int c = 0; c < CPL; ++c) vn[c] = s_v[buf][t][my_col + c];
-    };
-    load_token(0);
-    for (int t = 0; t < n; ++t) {
-      f32x4 kc[RPL / 4], qc[RPL / 4];
-      float vc[CPL];
-#pragma unroll
-      for (int i = 0; i < RPL / 4; ++i) kc[i] = kn[i], qc[i] = qn[i];
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) vc[c] = vn[c];
-      const float g = gn[0], beta = gn[1], kq = gn[2];
-      load_token(t + 1 < n ? t + 1 : t);
-      float sk[CPL], sq[CPL];
-#pragma unroll
-      for (int c = 0; c < CPL; ++c) {
-        float k0 = 0.f, k1 = 0.f, q0 = 0.f, q1 = 0.f;
-#pragma unroll
-        for (int i = 0; i < RPL; i += 2) {
-          k0 = __builtin_fmaf(S[i][c], kc[i >> 2][i & 3], k0);
-          q0 = __builtin_fmaf(S[i][c], qc[i >> 2][i & 3], q0);
-          k1 = __builtin_fmaf(S[i + 1][c], kc[i >> 2][(i & 3) + 1], k1);
-          q1 = __builtin_fmaf(S[i + 1][c], qc[i >> 2][(i & 3) + 1], q1);
-        }
-        sk[c] = sum8(k0 + k1);
-        sq[c] = sum8(q0 + q1);
+      for (int r = 1; r < RS; ++r) {
+        ks += part[(r * 2 + 0) * 64 + lane];
+        qs += part[(r * 2 + 1) * 64 + lane];
       }
-      G *= g;  // the same in every lane
-      float o[CPL], u[CPL];
+    }
+    f32x4 u = {0.f, 0.f, 0.f, 0.f}, oo;
+    float r4[4];
 #pragma unroll
-      for (int c = 0; c < CPL; ++c) {
-        u[c] = beta * (vc[c] - G * sk[c]);
-        o[c] = __builtin_fmaf(kq, u[c], G * sq[c]);
-      }
-      if (G < kRescaleBelow) {
+    for (int i = 0; i < 4; ++i) r4[i] = beta[i] * (vv[i] - gm[i] * ks[i]);
 #pragma unroll
-        for (int i = 0; i < RPL; ++i)
+    for (int i = 0; i < 4; ++i) u = mfma_f32(tm[i], r4[i], u);
 #pragma unroll
-          for (int c = 0; c < CPL; ++c) S[i][c] *= G;
-        G = 1.0f;
-      }
-      const float inv = __builtin_amdgcn_rcpf(G);
+    for (int i = 0; i < 4; ++i) oo[i] = gm[i] * qs[i];
 #pragma unroll
-      for (int c = 0; c < CPL; ++c) {
-        const float uz = u[c] * inv;
+    for (int r = 0; r < RBW; ++r) S[r] *= last;
 #pragma unroll
-        for (int i = 0; i < RPL; ++i) S[i][c] = __builtin_fmaf(kc[i >> 2][i & 3], uz, S[i][c]);
-      }
-      if (writer) {
-        float* dst = op + (long)(l0 + t) * a.H * a.dv;
-        if (CPL == 4 && (a.dv & 3) == 0) {
-          if (cols_left > 0) *reinterpret_cast<f32x4*>(dst) = f32x4{o[0], o[1 % CPL], o[2 % CPL], o[3 % CPL]};
-        } else {
+    for (int i = 0; i < 4; ++i) oo = mfma_f32(pm[i], u[i], oo);
+    float ut[4];
 #pragma unroll
-          for (int c = 0; c < CPL; ++c)
-            if (c < cols_left) dst[c] = o[c];
-        }
+    for (int i = 0; i < 4; ++i) ut[i] = u[i] * tail[i];
+#pragma unroll
+    for (int r = 0; r < RBW; ++r) {
+      const f32x4 kt = *reinterpret_cast<const f32x4*>(&s_kt[buf][((rs * RBW + r) * 16 + l16) * TS + quad * 4]);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) S[r] = mfma_f32(kt[i], ut[i], S[r]);
+    }
+    if (rs == 0 && col_in) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = blk * kBlk + quad * 4 + i;
+        if (t < a.L) o[(long)t * a.H * a.dv] = oo[i];
       }
     }
     if (more) stage(buf ^ 1);
   }
 #pragma unroll
-  for (int i = 0; i < RPL; ++i) {
-    const int row = (i >> 2) * 32 + rg * 4 + (i & 3);
+  for (int r = 0; r < RBW; ++r)
 #pragma unroll
-    for (int c = 0; c < CPL; ++c)
-      if (row < a.d && c < cols_left) st[(long)row * a.dvp + c] = S[i][c] * G;
-  }
+    for (int i = 0; i < 4; ++i) {
+      const int row = (rs * RBW + r) * 16 + quad * 4 + i;
+      if (col_in && row < a.d) st[(long)row * a.dvp] = S[r][i];
+    }
 }
 
 // ---- o / rms(o) * w * silu(gate) * scale: 16 lanes per (token, head) ----
@@ -331,16 +402,15 @@ struct DeltaStepArgs {
   float eps, scale;
 };
 
-constexpr int kDeltaStepThreads = 512;
-
-template <typename T, int RPT>
-__global__ __launch_bounds__(kDeltaStepThreads) void gated_delta_step_kernel(const DeltaStepArgs a) {
+// NT threads, RPT rows of the state per thread.
+template <typename T, int NT, int RPT>
+__global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaStepArgs a) {
   extern __shared__ float smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int b = blockIdx.x / a.H, h = blockIdx.x % a.H, share = a.H / a.G, hk = h / share;
   const int pos = row_pos(a.pos, a.pos_host, b);
   if (pos < 0) return;
-  const int cq_n = a.dvp / 4, rg_n = kDeltaStepThreads / cq_n;
+  const int cq_n = a.dvp / 4, rg_n = NT / cq_n;
   float* sq = smem;                 // [d]
   float* sk = sq + a.d;             // [d]
   float* sv = sk + a.d;             // [dvp]
@@ -368,7 +438,7 @@ __global__ __launch_bounds__(kDeltaStepThreads) void gated_delta_step_kernel(con
   const T* x = static_cast<const T*>(a.x) + b * a.x_sb;
   const T* cw = static_cast<const T*>(a.conv_w);
   T* ring = static_cast<T*>(a.ring) + b * a.ring_sb;
-  for (int i = tid; i < 2 * a.d + a.dv; i += kDeltaStepThreads) {
+  for (int i = tid; i < 2 * a.d + a.dv; i += NT) {
     const int ch = i < a.d ? hk * a.d + i : (i < 2 * a.d ? a.k_off + hk * a.d + i - a.d : a.v_off + h * a.dv + i - 2 * a.d);
     const T now = x[ch];
     float acc = 0.f;
@@ -383,7 +453,7 @@ __global__ __launch_bounds__(kDeltaStepThreads) void gated_delta_step_kernel(con
     if (i >= 2 * a.d || h % share == 0) ring[(long)(pos % a.taps) * a.C + ch] = now;
   }
   if (tid == 0) {
-    sc[3] = decay_of<T>(to_f32(static_cast<const T*>(a.a)[b * a.g_sb + h]), a.a_log, a.dt_bias, h);
+    sc[3] = expf(log_decay_of<T>(to_f32(static_cast<const T*>(a.a)[b * a.g_sb + h]), a.a_log, a.dt_bias, h));
     sc[4] = sigmoid_f(to_f32(static_cast<const T*>(a.bt)[b * a.g_sb + h]));
   }
   __syncthreads();
@@ -418,7 +488,7 @@ __global__ __launch_bounds__(kDeltaStepThreads) void gated_delta_step_kernel(con
   __syncthreads();
   const float fq = 1.0f / (sqrtf((float)a.d) * sqrtf(sc[0] + kUnitEps)), fk = 1.0f / sqrtf(sc[1] + kUnitEps);
   const float g = sc[3], beta = sc[4], kq = sc[2] * fq * fk;
-  for (int c = tid; c < a.dvp; c += kDeltaStepThreads) {
+  for (int c = tid; c < a.dvp; c += NT) {
     float tk = 0.f, tq = 0.f;
     for (int r = 0; r < rg_n; ++r) {
       tk += pk[r * a.dvp + c];
@@ -450,44 +520,88 @@ __global__ __launch_bounds__(kDeltaStepThreads) void gated_delta_step_kernel(con
   const float r = 1.0f / sqrtf(wave_sum(ss) / (float)a.dv + a.eps);
   T* y = static_cast<T*>(a.y) + b * a.y_sb + (long)h * a.dv;
   const T* gate = static_cast<const T*>(a.gate) + b * a.gate_sb + (long)h * a.dv;
-  for (int c = tid; c < a.dv; c += kDeltaStepThreads)
+  for (int c = tid; c < a.dv; c += NT)
     y[c] = from_f32<T>(so[c] * r * to_f32(static_cast<const T*>(a.norm_w)[c]) * silu_exact(to_f32(gate[c])) * a.scale);
 }
 
-template <typename T, int RPL, int CPL, int NW> void launch_delta_scan_vec(const DeltaArgs& a, bool vec, hipStream_t s) {
-  const dim3 grid((unsigned)(a.B * a.H), (unsigned)((a.dv + NW * 8 * CPL - 1) / (NW * 8 * CPL))), block(64 * NW);
-  if (vec)
-    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RPL, CPL, NW, true>), grid, block, 0, s, a);
-  else
-    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RPL, CPL, NW, false>), grid, block, 0, s, a);
+template <typename T, int RB, int RS> void launch_delta_scan_split(const DeltaArgs& a, hipStream_t s) {
+  const int cols = 16 * (4 / RS);
+  hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS>), dim3((unsigned)(a.B * a.H), (unsigned)((a.dv + cols - 1) / cols)), dim3(256), 0, s, a);
 }
 
-// More columns per lane spend fewer instructions per state element, fewer columns make more
-// wavefronts: enough of them for two per SIMD are wanted first.
-template <typename T, int RPL> void launch_delta_scan(const DeltaArgs& a, bool vec, hipStream_t s) {
-  const long cols = (long)a.B * a.H * a.dv;
-  if (cols >= 32l * 2048 && a.dv > 64)
-    launch_delta_scan_vec<T, RPL, 4, 4>(a, vec, s);
-  else if (cols >= 16l * 2048 && a.dv > 32)
-    launch_delta_scan_vec<T, RPL, 2, 4>(a, vec, s);
-  else
-    launch_delta_scan_vec<T, RPL, 1, 4>(a, vec, s);
+// Tiles are shared by as many wavefronts as it takes to give every compute unit a workgroup.
+template <typename T, int RB> void launch_delta_scan(const DeltaArgs& a, hipStream_t s) {
+  const long tiles = (long)a.B * a.H * ((a.dv + 15) / 16);
+  if constexpr (RB % 4 == 0) {
+    if (tiles < 512) {
+      launch_delta_scan_split<T, RB, 4>(a, s);
+      return;
+    }
+  }
+  if constexpr (RB % 2 == 0) {
+    if (tiles < 1024) {
+      launch_delta_scan_split<T, RB, 2>(a, s);
+      return;
+    }
+  }
+  launch_delta_scan_split<T, RB, 1>(a, s);
 }
 
-template <typename T, int RPT> void launch_delta_step(const DeltaStepArgs& a, hipStream_t s) {
-  const int rg_n = kDeltaStepThreads / (a.dvp / 4);
+template <typename T> void launch_delta(const DeltaArgs& a, hipStream_t s) {
+  const long items = (long)a.B * a.H * a.blocks;
+  hipLaunchKernelGGL(gated_delta_prepare_kernel<T>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
+  const int rb = (a.d + 15) / 16;
+  if (rb <= 1)
+    launch_delta_scan<T, 1>(a, s);
+  else if (rb <= 2)
+    launch_delta_scan<T, 2>(a, s);
+  else if (rb <= 3)
+    launch_delta_scan<T, 3>(a, s);
+  else if (rb <= 4)
+    launch_delta_scan<T, 4>(a, s);
+  else if (rb <= 6)
+    launch_delta_scan<T, 6>(a, s);
+  else if (rb <= 8)
+    launch_delta_scan<T, 8>(a, s);
+  else if (rb <= 12)
+    launch_delta_scan<T, 12>(a, s);
+  else
+    launch_delta_scan<T, 16>(a, s);
+}
+
+template <typename T, int NT, int RPT> void launch_delta_step_rows(const DeltaStepArgs& a, hipStream_t s) {
+  const int rg_n = NT / (a.dvp / 4);
   const size_t bytes = (size_t)(2 * a.d + 3 * a.dvp + 8 + 2 * rg_n * a.dvp) * sizeof(float);
-  hipLaunchKernelGGL((gated_delta_step_kernel<T, RPT>), dim3((unsigned)(a.B * a.H)), dim3(kDeltaStepThreads), bytes, s, a);
+  hipLaunchKernelGGL((gated_delta_step_kernel<T, NT, RPT>), dim3((unsigned)(a.B * a.H)), dim3(NT), bytes, s, a);
+}
+
+constexpr int kDeltaStepMaxThreads = 512, kDeltaStepMaxRows = 32;
+
+// About eight 16-byte pieces of the state per thread: enough in flight, and a small state does not pay
+// for the barriers of many wavefronts.
+template <typename T> void launch_delta_step(const DeltaStepArgs& a, hipStream_t s) {
+  const int cq_n = a.dvp / 4;
+  auto rows = [&](int nt) { return (a.d + nt / cq_n - 1) / (nt / cq_n); };
+  if (cq_n <= 128 && rows(128) <= 8)
+    launch_delta_step_rows<T, 128, 8>(a, s);
+  else if (rows(256) <= 8)
+    launch_delta_step_rows<T, 256, 8>(a, s);
+  else if (rows(512) <= 8)
+    launch_delta_step_rows<T, 512, 8>(a, s);
+  else if (rows(512) <= 16)
+    launch_delta_step_rows<T, 512, 16>(a, s);
+  else
+    launch_delta_step_rows<T, 512, 32>(a, s);
 }
 
 }  // namespace based
 
 extern "C" BASED_API int based_gated_delta_scan(const void* q, const void* k, const void* v, const void* a_gate, const void* b_gate,
-                                                const void* a_log, const void* dt_bias, float* state, float* o, int64_t B, int64_t L,
-                                                int64_t H, int64_t G, int64_t D, int64_t DV, int64_t state_row, int64_t x_sb,
+                                                const void* a_log, const void* dt_bias, float* state, float* work, float* o,
+                                                int64_t B, int64_t L, int64_t H, int64_t G, int64_t D, int64_t DV, int64_t state_row, int64_t x_sb,
                                                 int64_t x_sl, int64_t g_sb, int64_t g_sl, int fresh, int io_dtype, void* stream) {
   using namespace based;
-  BASED_REQUIRE(q && k && v && a_gate && b_gate && a_log && dt_bias && state && o, BASED_ERR_ARG, "gated_delta_scan: null pointer argument");
+  BASED_REQUIRE(q && k && v && a_gate && b_gate && a_log && dt_bias && state && work && o, BASED_ERR_ARG, "gated_delta_scan: null pointer argument");
   BASED_REQUIRE(B >= 0 && L >= 0 && H > 0 && G > 0 && D > 0 && DV > 0, BASED_ERR_ARG, "gated_delta_scan: bad sizes");
   BASED_REQUIRE(H % G == 0, BASED_ERR_SHAPE, "gated_delta_scan: %ld heads do not divide into %ld query/key heads", (long)H, (long)G);
   BASED_REQUIRE(D <= 256, BASED_ERR_SHAPE, "gated_delta_scan: query/key size %ld (at most 256)", (long)D);
@@ -495,26 +609,18 @@ extern "C" BASED_API int based_gated_delta_scan(const void* q, const void* k, co
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "gated_delta_scan: bad dtype");
   BASED_REQUIRE(B * H < (1ll << 31) && L < (1ll << 31) && DV < (1ll << 20), BASED_ERR_SHAPE, "gated_delta_scan: grid too large");
   if (B == 0 || L == 0) return BASED_OK;
-  const DeltaArgs a{q,      k,      v,      a_gate,  b_gate, a_log,          dt_bias, state, o,    (int)B, (int)L,
-                    (int)H, (int)G, (int)D, (int)DV, (int)state_row, x_sb, x_sl,  g_sb,  g_sl, fresh};
+  const int64_t blocks = (L + kBlk - 1) / kBlk;
+  BASED_REQUIRE(B * H * blocks < (1ll << 32), BASED_ERR_SHAPE, "gated_delta_scan: grid too large");
+  BASED_REQUIRE(aligned_to(work, 16), BASED_ERR_ALIGN, "gated_delta_scan: the work space must be 16-byte aligned");
+  // groups of four channels as one load
+  const int vec = D % 4 == 0 && x_sb % 4 == 0 && x_sl % 4 == 0 && aligned_to(q, 16) && aligned_to(k, 16);
+  const DeltaArgs a{q,      k,      v,      a_gate, b_gate,  a_log,          dt_bias,     state, o,    work, (int)B, (int)L,
+                    (int)H, (int)G, (int)D, (int)DV, (int)state_row, (int)blocks, x_sb,  x_sl, g_sb, g_sl,   fresh, vec};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  // staging pieces: half a lane's rows (16 bytes at most) of q and k, 2 .. 8 elements of v
-  const bool vec = D % 16 == 0 && DV % 8 == 0 && x_sb % 8 == 0 && x_sl % 8 == 0 && aligned_to(q, 16) && aligned_to(k, 16) && aligned_to(v, 16);
-#define BASED_DELTA_ROWS(T)                              \
-  if (D <= 32)                                           \
-    launch_delta_scan<T, 4>(a, vec, s);                  \
-  else if (D <= 64)                                      \
-    launch_delta_scan<T, 8>(a, vec, s);                  \
-  else if (D <= 128)                                     \
-    launch_delta_scan<T, 16>(a, vec, s);                 \
-  else                                                   \
-    launch_delta_scan<T, 32>(a, vec, s);
-  if (io_dtype == BASED_BF16) {
-    BASED_DELTA_ROWS(__bf16)
-  } else {
-    BASED_DELTA_ROWS(float)
-  }
-#undef BASED_DELTA_ROWS
+  if (io_dtype == BASED_BF16)
+    launch_delta<__bf16>(a, s);
+  else
+    launch_delta<float>(a, s);
   return check_launch("gated_delta_scan");
 }
 
@@ -572,22 +678,12 @@ extern "C" BASED_API int based_gated_delta_step(const void* x, const void* conv_
                         pos,    (int)pos_host, (int)B, (int)H,  (int)G, (int)D,   (int)DV, (int)state_row, (int)C, taps, (int)k_off,
                         (int)v_off, x_sb, g_sb, gate_sb, y_sb, ring_sb, eps, scale};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const int rg_n = kDeltaStepThreads / ((int)state_row / 4), rows = ((int)D + rg_n - 1) / rg_n;
-#define BASED_DELTA_STEP(T)                 \
-  if (rows <= 4)                            \
-    launch_delta_step<T, 4>(a, s);          \
-  else if (rows <= 8)                       \
-    launch_delta_step<T, 8>(a, s);          \
-  else if (rows <= 16)                      \
-    launch_delta_step<T, 16>(a, s);         \
-  else                                      \
-    launch_delta_step<T, 32>(a, s);
-  BASED_REQUIRE(rows <= 32, BASED_ERR_SHAPE, "gated_delta_step: a state of %ld x %ld per head is too large", (long)D, (long)state_row);
-  if (io_dtype == BASED_BF16) {
-    BASED_DELTA_STEP(__bf16)
-  } else {
-    BASED_DELTA_STEP(float)
-  }
-#undef BASED_DELTA_STEP
+  const int rg_n = kDeltaStepMaxThreads / ((int)state_row / 4);
+  BASED_REQUIRE((D + rg_n - 1) / rg_n <= kDeltaStepMaxRows, BASED_ERR_SHAPE, "gated_delta_step: a state of %ld x %ld per head is too large",
+                (long)D, (long)state_row);
+  if (io_dtype == BASED_BF16)
+    launch_delta_step<__bf16>(a, s);
+  else
+    launch_delta_step<float>(a, s);
   return check_launch("gated_delta_step");
 }

@@ -250,12 +250,12 @@ constexpr int kLruRows = 8;  // sequences held at a time
 template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) {
   constexpr int N = VEC ? Pack<T>::kN : 1;
-  extern __shared__ float s_u[];  // [kLruRows][n rounded up to 8 N]
+  extern __shared__ __attribute__((aligned(16))) float s_u[];  // [kLruRows][n rounded up to 4]
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int tiles = (a.n + 31) / 32;
   const int blk = blockIdx.x / tiles, tile = blockIdx.x % tiles, m0 = blockIdx.y * kLruRows;
   const int rows = a.B - m0 < kLruRows ? a.B - m0 : kLruRows;
-  const int ns = a.n;
+  const int ns = (a.n + 3) & ~3;  // rows of whole 16-byte pieces
   for (int i = tid; i < kLruRows * a.n; i += 256) {
     const int m = i / a.n, k = i % a.n, ch = blk * a.n + k;
     float val = 0.f;
@@ -295,13 +295,18 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) 
       r[0] = to_f32(wr[k]), q[0] = to_f32(wi[k]);
     }
 #pragma unroll
-    for (int m = 0; m < kLruRows; ++m)
+    for (int m = 0; m < kLruRows; ++m) {
+      float uv[N];
+      if constexpr (VEC)
+        load_vec<float, N>(&s_u[m * ns + k], uv);
+      else
+        uv[0] = s_u[m * ns + k];
 #pragma unroll
       for (int j = 0; j < N; ++j) {
-        const float uv = s_u[m * ns + k + j];
-        zr[m] = __builtin_fmaf(r[j], uv, zr[m]);
-        zi[m] = __builtin_fmaf(q[j], uv, zi[m]);
+        zr[m] = __builtin_fmaf(r[j], uv[j], zr[m]);
+        zi[m] = __builtin_fmaf(q[j], uv[j], zi[m]);
       }
+    }
   }
   float my_r = 0.f, my_i = 0.f;
 #pragma unroll
@@ -374,7 +379,7 @@ extern "C" BASED_API int based_rglru_step(const void* x, const void* y, const vo
   const int v = io_dtype == BASED_BF16 ? 8 : 4;
   const bool vec = n % v == 0 && aligned_to(ra, 16) && aligned_to(ri, 16);
   const dim3 grid((unsigned)tiles, (unsigned)mt), block(256);
-  const size_t bytes = (size_t)kLruRows * n * sizeof(float);
+  const size_t bytes = (size_t)kLruRows * ((n + 3) & ~3) * sizeof(float);
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (io_dtype == BASED_BF16) {
     if (vec)

@@ -62,6 +62,30 @@ __device__ __forceinline__ float rotated(const T* row, int c, int pos, const Win
   return x * a.cos_t[t] + sgn * to_f32(row[partner]) * a.sin_t[t];
 }
 
+// 8 channels from c on (a multiple of 8) of interleaved pairs, in registers.
+__device__ __forceinline__ void rotate8(float (&x)[8], int c, int pos, const WindowArgs& a) {
+  if (c >= a.rot) return;
+  const long t = (long)pos * (a.rot / 2) + c / 2;
+  float cs[4], sn[4];
+  if ((a.rot & 7) == 0) {
+    load_vec<float, 4>(a.cos_t + t, cs);
+    load_vec<float, 4>(a.sin_t + t, sn);
+  } else {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const bool in = c + 2 * j < a.rot;
+      cs[j] = in ? a.cos_t[t + j] : 1.f;
+      sn[j] = in ? a.sin_t[t + j] : 0.f;
+    }
+  }
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const float u = x[2 * j], v = x[2 * j + 1];
+    x[2 * j] = u * cs[j] - v * sn[j];
+    x[2 * j + 1] = v * cs[j] + u * sn[j];
+  }
+}
+
 // One wavefront per (token, key/value head).
 template <typename T>
 __global__ __launch_bounds__(256) void window_kv_write_kernel(const WindowArgs a) {
@@ -113,15 +137,7 @@ __global__ __launch_bounds__(256) void window_kv_write_vec_kernel(const WindowAr
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
     const int c = (i * 16 + lane) * 8;
-#pragma unroll
-    for (int j = 0; j < 8; j += 2) {
-      if (c + j < a.rot) {
-        const long t = (long)pos * (a.rot / 2) + (c + j) / 2;
-        const float cs = a.cos_t[t], sn = a.sin_t[t], u0 = x[i][j], u1 = x[i][j + 1];
-        x[i][j] = u0 * cs - u1 * sn;
-        x[i][j + 1] = u1 * cs + u0 * sn;
-      }
-    }
+    rotate8(x[i], c, pos, a);
 #pragma unroll
     for (int j = 0; j < 8; ++j) y[i][j] *= r;
     if (live && c < a.d) store_vec<__bf16, 8>(out + c, x[i]);
@@ -174,14 +190,7 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
 #pragma unroll
         for (int j = 0; j < 8; ++j) x[j] = rotated(qp, e + j, qpos[t], a);
       } else {
-#pragma unroll
-        for (int j = 0; j < 8; j += 2)
-          if (e + j < a.rot) {
-            const long ti = (long)qpos[t] * (a.rot / 2) + (e + j) / 2;
-            const float cs = a.cos_t[ti], sn = a.sin_t[ti], u0 = x[j], u1 = x[j + 1];
-            x[j] = u0 * cs - u1 * sn;
-            x[j + 1] = u1 * cs + u0 * sn;
-          }
+        rotate8(x, e, qpos[t], a);
       }
 #pragma unroll
       for (int j = 0; j < 8; ++j) qf[t][c][j] = (__bf16)(e < a.d ? x[j] : 0.f);
@@ -197,6 +206,7 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
 #pragma unroll
     for (int i = 0; i < 2 * VC; ++i) acc[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run[2] = {-INFINITY, -INFINITY}, l_run[2] = {0.f, 0.f};
+  const float scale2 = a.scale * 1.4426950408889634f;  // scores in powers of two
 
   const int first_pos = a.pos_host + r0 / qpk, last_pos = a.pos_host + (r_end - 1) / qpk;
   const int lo = first_pos - a.window + 1 > 0 ? first_pos - a.window + 1 : 0;
@@ -255,62 +265,70 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
     stage();
     __syncthreads();
     if (k0 + kTileKeys <= last_pos) fetch(k0 + kTileKeys);
-    // does any row of this wavefront see a key of this tile?
-    if (k0 > wave_hi_tok || k0 + kTileKeys - 1 <= wave_lo_tok - a.window) continue;
-    f32x4 s[2][4];
 #pragma unroll
-    for (int kt = 0; kt < 4; ++kt) {
+    for (int h = 0; h < 2; ++h) {
+      // 32 keys at a time: does any row of this wavefront see one of them, does every row see all?
+      const int kh = k0 + h * 32;
+      if (kh > wave_hi_tok || kh + 31 <= wave_lo_tok - a.window) continue;
+      const bool all = kh + 31 <= wave_lo_tok && kh > wave_hi_tok - a.window;
+      f32x4 s[2][2];
 #pragma unroll
-      for (int t = 0; t < 2; ++t) s[t][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int kt = 0; kt < 2; ++kt) {
 #pragma unroll
-      for (int c = 0; c < KC; ++c) {
-        const bf16x8 kf = *reinterpret_cast<const bf16x8*>(&lds_k[(kt * 16 + l16) * KS + c * 32 + quad * 8]);
+        for (int t = 0; t < 2; ++t) s[t][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int t = 0; t < 2; ++t) s[t][kt] = mfma_bf16(kf, qf[t][c], s[t][kt]);
+        for (int c = 0; c < KC; ++c) {
+          const bf16x8 kf = *reinterpret_cast<const bf16x8*>(&lds_k[(h * 32 + kt * 16 + l16) * KS + c * 32 + quad * 8]);
+#pragma unroll
+          for (int t = 0; t < 2; ++t) s[t][kt] = mfma_bf16(kf, qf[t][c], s[t][kt]);
+        }
       }
-    }
-    bf16x8 pf[2][2];
+      bf16x8 pf[2];
 #pragma unroll
-    for (int t = 0; t < 2; ++t) {
-      float mx = -INFINITY;
+      for (int t = 0; t < 2; ++t) {
+        float mx = -INFINITY;
+        const int d0 = qpos[t] - kh - quad * 4;
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
+        for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int dist = qpos[t] - (k0 + kt * 16 + quad * 4 + i);
-          const float sc = dist >= 0 && dist < a.window ? s[t][kt][i] * a.scale : -INFINITY;
-          s[t][kt][i] = sc;
-          mx = fmaxf(mx, sc);
+          for (int i = 0; i < 4; ++i) {
+            float sc = s[t][kt][i] * scale2;
+            if (!all) sc = (unsigned)(d0 - kt * 16 - i) < (unsigned)a.window ? sc : -INFINITY;
+            s[t][kt][i] = sc;
+            mx = fmaxf(mx, sc);
+          }
+        mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+        mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+        if (__any(mx > m_run[t])) {
+          const float m_new = fmaxf(m_run[t], mx);
+          // no key seen yet: every weight is 2^-inf = 0
+          const float alpha = __builtin_amdgcn_exp2f(m_run[t] - (m_new == -INFINITY ? 0.f : m_new));
+          m_run[t] = m_new;
+          l_run[t] *= alpha;
+#pragma unroll
+          for (int i = 0; i < 2 * VC; ++i) acc[t][i] *= alpha;
         }
-      mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-      mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-      const float m_new = fmaxf(m_run[t], mx);
-      const float m_use = m_new == -INFINITY ? 0.f : m_new;  // no key seen yet: every weight is exp(-inf) = 0
-      const float alpha = __expf(m_run[t] - m_use);
-      m_run[t] = m_new;
-      float sum = 0.f;
+        const float m_use = m_run[t] == -INFINITY ? 0.f : m_run[t];
+        float sum = 0.f;
 #pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
+        for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const float p = __expf(s[t][kt][i] - m_use);
-          sum += p;
-          pf[t][kt >> 1][(kt & 1) * 4 + i] = (__bf16)p;
-        }
-      l_run[t] = l_run[t] * alpha + sum;  // this lane's keys; the four lane groups are added at the end
+          for (int i = 0; i < 4; ++i) {
+            const float p = __builtin_amdgcn_exp2f(s[t][kt][i] - m_use);
+            sum += p;
+            pf[t][kt * 4 + i] = (__bf16)p;
+          }
+        l_run[t] += sum;  // this lane's keys; the four lane groups are added at the end
+      }
 #pragma unroll
-      for (int i = 0; i < 2 * VC; ++i) acc[t][i] *= alpha;
-    }
-#pragma unroll
-    for (int i = 0; i < 2 * VC; ++i)
-#pragma unroll
-      for (int h = 0; h < 2; ++h) {
+      for (int i = 0; i < 2 * VC; ++i) {
         const __bf16* vp = &lds_v[(i * 16 + l16) * VS + h * 32 + quad * 4];
         const bf16x4 v0 = *reinterpret_cast<const bf16x4*>(vp), v1 = *reinterpret_cast<const bf16x4*>(vp + 16);
         const bf16x8 vf = __builtin_shufflevector(v0, v1, 0, 1, 2, 3, 4, 5, 6, 7);
 #pragma unroll
-        for (int t = 0; t < 2; ++t) acc[t][i] = mfma_bf16(vf, pf[t][h], acc[t][i]);
+        for (int t = 0; t < 2; ++t) acc[t][i] = mfma_bf16(vf, pf[t], acc[t][i]);
       }
+    }
   }
 #pragma unroll
   for (int t = 0; t < 2; ++t) {
@@ -409,8 +427,7 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   float* qs = smem;                        // [QT][d]
   float* sc = qs + QT * a.d;               // [QT][kStepKeys]
   float* stat = sc + QT * kStepKeys;       // [3][QT]: running maximum, running sum, rescale of this round
-  float* part = stat + 3 * QT;             // [kStepThreads][N], reduction of the output (16-byte aligned: see the launch)
-  part += (4 - ((QT * a.d + QT * kStepKeys + 3 * QT) & 3)) & 3;
+  float* part = stat + 3 * QT;             // [QT][parts][vp2 * N], partial outputs
   const T* k = static_cast<const T*>(a.k) + b * a.k_sb + (long)g * a.d;
   const T* v = static_cast<const T*>(a.v) + b * a.v_sb + (long)g * a.dv;
   T* kv = static_cast<T*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
@@ -431,8 +448,13 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   int lpk = 1;
   while (lpk < pieces && lpk < 64) lpk <<= 1;
   const int keys_at_once = kStepThreads / lpk, my_key = tid / lpk, my_piece = tid % lpk;
-  const int v_pieces = (a.dv + N - 1) / N;                       // <= kStepThreads
-  const int v_groups = kStepThreads / v_pieces, my_vp = tid % v_pieces, my_vg = tid / v_pieces;
+  // lanes per value row, likewise; then the partial sums that are left for LDS
+  int vp2 = 1;
+  while (vp2 * N < a.dv) vp2 <<= 1;  // <= kStepThreads
+  const int v_groups = kStepThreads / vp2, my_vp = tid % vp2, my_vg = tid / vp2;
+  const int parts = vp2 < 64 ? kStepThreads / 64 : v_groups, my_part = vp2 < 64 ? wave : my_vg;
+  const bool v_in = my_vp * N < a.dv;
+  constexpr int KU = 4;  // rows whose loads are in flight together
 
   for (int h0 = 0; h0 < qpk; h0 += QT) {
     __syncthreads();  // the new row is visible; the round before is done with LDS
@@ -446,6 +468,12 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
       stat[tid] = -INFINITY;
       stat[QT + tid] = 0.f;
     }
+    __syncthreads();
+    float qr[QT][N];  // this lane's piece of every query
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+      for (int i = 0; i < N; ++i) qr[hh][i] = my_piece < pieces ? qs[hh * a.d + (my_piece < pieces ? my_piece : 0) * N + i] : 0.f;
     float acc[QT][N];
 #pragma unroll
     for (int hh = 0; hh < QT; ++hh)
@@ -453,41 +481,65 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
       for (int i = 0; i < N; ++i) acc[hh][i] = 0.f;
     for (int k0 = lo; k0 <= pos; k0 += kStepKeys) {
       const int n = pos - k0 + 1 < kStepKeys ? pos - k0 + 1 : kStepKeys;
-      __syncthreads();
-      for (int j0 = 0; j0 < n; j0 += keys_at_once) {
-        const int j = j0 + my_key;
-        float dot[QT];
+      const T* rows = kv + (long)k0 * a.kv_st;
+      if (k0 > lo) __syncthreads();
+      auto load_row = [&](const T* base, int j, int piece, float (&x)[N]) {
+        const T* r = base + (long)(j < n ? j : n - 1) * a.kv_st + piece * N;
+        if constexpr (VEC)
+          load_vec<T, N>(r, x);
+        else
+          x[0] = to_f32(*r);
+      };
+      for (int j0 = 0; j0 < n; j0 += KU * keys_at_once) {
+        float x[KU][N];
 #pragma unroll
-        for (int hh = 0; hh < QT; ++hh) dot[hh] = 0.f;
-        const T* kr = kv + (long)(k0 + (j < n ? j : 0)) * a.kv_st;
-        for (int p = my_piece; p < pieces; p += lpk) {
-          float x[N];
-          if constexpr (VEC)
-            load_vec<T, N>(kr + p * N, x);
-          else
-            x[0] = to_f32(kr[p]);
+        for (int u = 0; u < KU; ++u) load_row(rows, j0 + u * keys_at_once + my_key, my_piece < pieces ? my_piece : 0, x[u]);
 #pragma unroll
-          for (int hh = 0; hh < QT; ++hh)
+        for (int u = 0; u < KU; ++u) {
+          const int j = j0 + u * keys_at_once + my_key;
+          float dot[QT];
 #pragma unroll
-            for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(x[i], qs[hh * a.d + p * N + i], dot[hh]);
-        }
+          for (int hh = 0; hh < QT; ++hh) {
+            dot[hh] = 0.f;
 #pragma unroll
-        for (int hh = 0; hh < QT; ++hh) {
-          for (int m = 1; m < lpk; m <<= 1) dot[hh] += __shfl_xor(dot[hh], m, 64);
-          if (my_piece == 0 && j < n) sc[hh * kStepKeys + j] = dot[hh] * a.scale;
+            for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(x[u][i], qr[hh][i], dot[hh]);
+          }
+          for (int p = my_piece + lpk; p < pieces; p += lpk) {  // rows of more than 64 pieces
+            float y[N];
+            load_row(rows, j, p, y);
+#pragma unroll
+            for (int hh = 0; hh < QT; ++hh)
+#pragma unroll
+              for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(y[i], qs[hh * a.d + p * N + i], dot[hh]);
+          }
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh) {
+            for (int m = 1; m < lpk; m <<= 1) dot[hh] += __shfl_xor(dot[hh], m, 64);
+            if (my_piece == 0 && j < n) sc[hh * kStepKeys + j] = dot[hh] * a.scale;
+          }
         }
       }
+      // the first value rows are on their way during the softmax
+      float xv[KU][N];
+#pragma unroll
+      for (int u = 0; u < KU; ++u) load_row(rows + a.d, my_vg + u * v_groups, v_in ? my_vp : 0, xv[u]);
       __syncthreads();
       for (int hh = wave; hh < QT; hh += kStepThreads / 64) {
-        float mx = -INFINITY;
-        for (int j = lane; j < n; j += 64) mx = fmaxf(mx, sc[hh * kStepKeys + j]);
+        float s[kStepKeys / 64], mx = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < kStepKeys / 64; ++i) {
+          const int j = i * 64 + lane;
+          s[i] = j < n ? sc[hh * kStepKeys + j] : -INFINITY;
+          mx = fmaxf(mx, s[i]);
+        }
 #pragma unroll
         for (int m = 32; m >= 1; m >>= 1) mx = fmaxf(mx, __shfl_xor(mx, m, 64));
         const float m_old = stat[hh], m_new = fmaxf(m_old, mx);
         float sum = 0.f;
-        for (int j = lane; j < n; j += 64) {
-          const float p = expf(sc[hh * kStepKeys + j] - m_new);
-          sc[hh * kStepKeys + j] = p;
+#pragma unroll
+        for (int i = 0; i < kStepKeys / 64; ++i) {
+          const float p = expf(s[i] - m_new);
+          sc[hh * kStepKeys + i * 64 + lane] = p;
           sum += p;
         }
         sum = wave_sum(sum);
@@ -499,40 +551,48 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
         }
       }
       __syncthreads();
-      if (my_vg < v_groups) {
+      if (k0 > lo) {
 #pragma unroll
         for (int hh = 0; hh < QT; ++hh)
 #pragma unroll
           for (int i = 0; i < N; ++i) acc[hh][i] *= stat[2 * QT + hh];
-#pragma unroll 4
-        for (int j = my_vg; j < n; j += v_groups) {
-          const T* vr = kv + (long)(k0 + j) * a.kv_st + a.d;
-          float x[N];
-          if constexpr (VEC)
-            load_vec<T, N>(vr + my_vp * N, x);
-          else
-            x[0] = to_f32(vr[my_vp]);
+      }
+      for (int j0 = my_vg; j0 < n; j0 += KU * v_groups) {
+        if (j0 != my_vg) {
 #pragma unroll
-          for (int hh = 0; hh < QT; ++hh)
+          for (int u = 0; u < KU; ++u) load_row(rows + a.d, j0 + u * v_groups, v_in ? my_vp : 0, xv[u]);
+        }
 #pragma unroll
-            for (int i = 0; i < N; ++i) acc[hh][i] = __builtin_fmaf(sc[hh * kStepKeys + j], x[i], acc[hh][i]);
+        for (int u = 0; u < KU; ++u) {
+          const int j = j0 + u * v_groups;
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh) {
+            const float p = j < n ? sc[hh * kStepKeys + j] : 0.f;
+#pragma unroll
+            for (int i = 0; i < N; ++i) acc[hh][i] = __builtin_fmaf(p, xv[u][i], acc[hh][i]);
+          }
         }
       }
     }
 #pragma unroll
     for (int hh = 0; hh < QT; ++hh) {
-      __syncthreads();
+      for (int m = vp2; m < 64; m <<= 1) {
 #pragma unroll
-      for (int i = 0; i < N; ++i) part[tid * N + i] = acc[hh][i];
-      __syncthreads();
+        for (int i = 0; i < N; ++i) acc[hh][i] += __shfl_xor(acc[hh][i], m, 64);
+      }
+      if (vp2 >= 64 || lane < vp2) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) part[((hh * parts + my_part) * vp2 + my_vp) * N + i] = acc[hh][i];
+      }
+    }
+    __syncthreads();
+    for (int i = tid; i < QT * a.dv; i += kStepThreads) {
+      const int hh = i / a.dv, c = i % a.dv;
       if (h0 + hh < qpk) {
+        float s = 0.f;
+        for (int p = 0; p < parts; ++p) s += part[(hh * parts + p) * vp2 * N + c];
         T* o = static_cast<T*>(a.o) + b * a.o_sb + (long)(g * qpk + h0 + hh) * a.dv;
-        const float inv = a.out_scale / stat[QT + hh];
-        for (int c = tid; c < a.dv; c += kStepThreads) {
-          float s = 0.f;
-          for (int vg = 0; vg < v_groups; ++vg) s += part[(vg * v_pieces + c / N) * N + c % N];
-          o[c] = from_f32<T>(s * inv);
-        }
+        o[c] = from_f32<T>(s * (a.out_scale / stat[QT + hh]));
       }
     }
   }
@@ -541,14 +601,16 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
 template <typename T, bool VEC> void launch_window_step(const WindowArgs& a, hipStream_t s) {
   const int qpk = a.H / a.G;
   const dim3 grid((unsigned)(a.B * a.G)), block(kStepThreads);
-  auto bytes = [&](int qt) {
-    return (size_t)(qt * a.d + qt * kStepKeys + 3 * qt + 4 + kStepThreads * (VEC ? Pack<T>::kN : 1)) * sizeof(float);
-  };
+  constexpr int N = VEC ? Pack<T>::kN : 1;
+  int vp2 = 1;
+  while (vp2 * N < a.dv) vp2 <<= 1;
+  const int parts = vp2 < 64 ? kStepThreads / 64 : kStepThreads / vp2;
+  auto bytes = [&](int qt) { return (size_t)qt * (a.d + kStepKeys + 3 + parts * vp2 * N) * sizeof(float); };
   if (qpk == 1)
     hipLaunchKernelGGL((window_step_kernel<T, 1, VEC>), grid, block, bytes(1), s, a);
   else if (qpk == 2)
     hipLaunchKernelGGL((window_step_kernel<T, 2, VEC>), grid, block, bytes(2), s, a);
-  else if (qpk <= 4)
+  else if (qpk <= 4 || bytes(8) > 64 * 1024)
     hipLaunchKernelGGL((window_step_kernel<T, 4, VEC>), grid, block, bytes(4), s, a);
   else
     hipLaunchKernelGGL((window_step_kernel<T, 8, VEC>), grid, block, bytes(8), s, a);

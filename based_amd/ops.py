@@ -710,6 +710,7 @@ def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residu
 NORM_RMS, NORM_LAYER = 0, 1
 ACT_NONE, ACT_SILU = 0, 1
 STREAM_MAX_TAPS = 8  # BASED_STREAM_MAX_TAPS
+DELTA_BLOCK, DELTA_PREP_FLOATS = 16, 592  # tokens per block of based_gated_delta_scan, BASED_DELTA_PREP_FLOATS
 RGLRU_SEGMENT = 64   # tokens per segment of based_rglru_prefill
 
 
@@ -881,10 +882,11 @@ def gated_delta_scan(q, k, v, a_gate, b_gate, a_log, dt_bias, state, heads: int,
         raise ValueError(f"gates must be ({B}, {L}, {heads})")
     _check_delta(state, B, heads, d, dv)
     o = torch.empty(B, L, heads, dv, dtype=torch.float32, device=q.device)
+    work = torch.empty(B, heads, (L + DELTA_BLOCK - 1) // DELTA_BLOCK, DELTA_PREP_FLOATS, dtype=torch.float32, device=q.device)
     with _on_device(q.device):
         _lib.check(_lib.lib().based_gated_delta_scan(
             q.data_ptr(), k.data_ptr(), v.data_ptr(), a_gate.data_ptr(), b_gate.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),
-            state.data_ptr(), o.data_ptr(), B, L, heads, kv_heads, d, dv, state.shape[3], q.stride(0), q.stride(1),
+            state.data_ptr(), work.data_ptr(), o.data_ptr(), B, L, heads, kv_heads, d, dv, state.shape[3], q.stride(0), q.stride(1),
             a_gate.stride(0), a_gate.stride(1), int(fresh), _dtype_code(q), _stream_ptr(q)))
     return o
 
