@@ -220,6 +220,17 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
   int g = wg * WV + wave;
   const int g_step = n_wg * WV;
   const bool have = g < a.n_groups;
+  // positions of the streamed-input prologue: scalar loads, in front of the weight rows
+  constexpr int RW = (MT + WV - 1) / WV;  // activation rows per wavefront
+  int pos_of[RW];
+  if constexpr (PRO == kProStream) {
+    const int wave_u = __builtin_amdgcn_readfirstlane(wave);
+#pragma unroll
+    for (int i = 0; i < RW; ++i) {
+      const int m = wave_u + i * WV;
+      pos_of[i] = a.ic_taps == 0 ? 0 : a.pos != nullptr ? a.pos[a.m0 + (m < a.M ? m : 0)] : a.pos_host;
+    }
+  }
   u32x4 wcur[R][C];
   load_rows(have ? g : 0, wcur);  // in flight while the activations are prepared
 
@@ -293,7 +304,7 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       const __bf16* xrow = x_row(m, poison);
       const bool has_res = a.res_in != nullptr;
       const float mult = has_res ? a.mult : 1.0f;
-      const int pos = a.ic_taps > 0 ? (a.pos != nullptr ? a.pos[a.m0 + m] : a.pos_host) : 0;
+      const int pos = pos_of[(m - wave) / WV];
       float v[C][8], nw[C][8];
       float sum = 0.f;
 #pragma unroll

@@ -62,25 +62,29 @@ template <typename T> __device__ __forceinline__ float log_decay_of(float a, con
 
 __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0); }
 
-// 4 consecutive channels of a row of d, zeros past its end
-template <typename T> __device__ __forceinline__ f32x4 load4(const T* row, int e, int d, int vec) {
-  f32x4 x = {0.f, 0.f, 0.f, 0.f};
-  if (vec) {
-    typedef __attribute__((ext_vector_type(4))) T t4;
-    if (e < d) {
-      const t4 r = *reinterpret_cast<const t4*>(row + e);
+// 4 consecutive channels of a row of d as they lie in memory.  Fetched without a condition (channels
+// past the end come from the row's start) and cleared where they are used: a load in a branch or
+// in front of a select is waited for on the spot.  VEC: whole groups, aligned.
+template <typename T, bool VEC> struct Four {
+  typedef __attribute__((ext_vector_type(4))) T t4;
+  t4 r;
+  __device__ __forceinline__ void load(const T* row, int e, int d) {
+    if constexpr (VEC) {
+      r = *reinterpret_cast<const t4*>(row + (e < d ? e : 0));
+    } else {
 #pragma unroll
-      for (int i = 0; i < 4; ++i) x[i] = to_f32(r[i]);
+      for (int i = 0; i < 4; ++i) r[i] = row[e + i < d ? e + i : 0];
     }
-  } else {
-#pragma unroll
-    for (int i = 0; i < 4; ++i)
-      if (e + i < d) x[i] = to_f32(row[e + i]);
   }
-  return x;
-}
+  __device__ __forceinline__ f32x4 get(int e, int d) const {
+    f32x4 x;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) x[i] = e + i < d ? to_f32(r[i]) : 0.f;
+    return x;
+  }
+};
 
-template <typename T>
+template <typename T, bool VEC>
 __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArgs a) {
   __shared__ __attribute__((aligned(16))) float s_a[4][kBlk][kBlk + 4];
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, quad = lane >> 4;
@@ -102,14 +106,25 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArg
   lg = fmaxf(lg, -200.f);  // exp(-200) is zero in fp32
   f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
   float sq = 0.f, sk = 0.f;
-  for (int e = quad * 4; e < a.d + quad * 4; e += 16) {
-    const f32x4 x = load4(q, e, a.d, a.vec), y = load4(k, e, a.d, a.vec);
+  for (int e0 = 0; e0 < a.d; e0 += 64) {
+    Four<T, VEC> xr[4], yr[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      sq = __builtin_fmaf(x[i], x[i], sq);
-      sk = __builtin_fmaf(y[i], y[i], sk);
-      kk = mfma_f32(y[i], y[i], kk);
-      qk = mfma_f32(x[i], y[i], qk);
+    for (int j = 0; j < 4; ++j) {
+      xr[j].load(q, e0 + j * 16 + quad * 4, a.d);
+      yr[j].load(k, e0 + j * 16 + quad * 4, a.d);
+    }
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const f32x4 x = xr[j].get(e0 + j * 16 + quad * 4, a.d), y = yr[j].get(e0 + j * 16 + quad * 4, a.d);
+      if (e0 + j * 16 < a.d) {
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          sq = __builtin_fmaf(x[i], x[i], sq);
+          sk = __builtin_fmaf(y[i], y[i], sk);
+          kk = mfma_f32(y[i], y[i], kk);
+          qk = mfma_f32(x[i], y[i], qk);
+        }
+      }
     }
   }
   sq += __shfl_xor(sq, 16, 64), sk += __shfl_xor(sk, 16, 64);
@@ -164,7 +179,7 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArg
 
 // RB: 16-row blocks of the state; RS: wavefronts that share a 16-column tile, RB / RS row blocks each
 // (their partial products with the state are added up through LDS).  Four wavefronts per workgroup.
-template <typename T, int RB, int RS>
+template <typename T, int RB, int RS, bool VEC>
 __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a) {
   static_assert(RB % RS == 0 && 4 % RS == 0, "row blocks divide among the wavefronts of a tile");
   constexpr int D = RB * 16, CT = 4 / RS, RBW = RB / RS;
@@ -195,8 +210,9 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
       S[r][i] = in ? st[(long)row * a.dvp] : 0.f;
     }
 
-  // what a block needs from memory is asked for one block ahead
-  f32x4 rk[PP][2], rq[PP][2];
+  // what a block needs from memory is asked for ahead of its use: q and k (which are laid out in LDS one
+  // block early) two blocks, the rest one block
+  Four<T, VEC> rk[PP][2], rq[PP][2];
   float fk[PP], fq[PP];
   f32x4 tn, pn, gn, tailn, betan;
   T vn[4];
@@ -223,8 +239,8 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
       const long row = blk * kBlk + t < a.L ? blk * kBlk + t : a.L - 1;
 #pragma unroll
       for (int j = 0; j < 2; ++j) {
-        rk[p][j] = load4(k + row * a.x_sl, e + 4 * j, a.d, a.vec);
-        rq[p][j] = load4(q + row * a.x_sl, e + 4 * j, a.d, a.vec);
+        rk[p][j].load(k + row * a.x_sl, e + 4 * j, a.d);
+        rq[p][j].load(q + row * a.x_sl, e + 4 * j, a.d);
       }
       fk[p] = pr[kPrepFk + t];
       fq[p] = pr[kPrepFq + t];
@@ -237,19 +253,21 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
       if (PIECES % 256 == 0 || piece < PIECES) {
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
-          const f32x4 y = rk[p][j] * fk[p];
+          const f32x4 y = rk[p][j].get(e + 4 * j, a.d) * fk[p];
           *reinterpret_cast<f32x4*>(&s_k[buf][t * KS + e + 4 * j]) = y;
-          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j] * fq[p];
+          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j].get(e + 4 * j, a.d) * fq[p];
 #pragma unroll
           for (int i = 0; i < 4; ++i) s_kt[buf][(e + 4 * j + i) * TS + t] = y[i];
         }
       }
     }
   };
+  const int last_blk = a.blocks - 1;
 
   fetch_qk(0);
   fetch(0);
   stage(0);
+  fetch_qk(0 < last_blk ? 1 : last_blk);
   for (int blk = 0, buf = 0; blk < a.blocks; ++blk, buf ^= 1) {
     __syncthreads();  // this block is laid out; everyone is done with the other buffer
     const f32x4 tm = tn, pm = pn, gm = gn, tail = tailn, beta = betan;
@@ -257,9 +275,9 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
     float vv[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) vv[i] = to_f32(vn[i]);
-    const bool more = blk + 1 < a.blocks;
-    fetch_qk(more ? blk + 1 : blk);
-    fetch(more ? blk + 1 : blk);
+    stage(buf ^ 1);  // the next block (past the end: the last one again, unused)
+    fetch_qk(blk + 2 < last_blk ? blk + 2 : last_blk);
+    fetch(blk + 1 < last_blk ? blk + 1 : last_blk);
     f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
 #pragma unroll
     for (int r = 0; r < RBW; ++r) {
@@ -313,7 +331,6 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
         if (t < a.L) o[(long)t * a.H * a.dv] = oo[i];
       }
     }
-    if (more) stage(buf ^ 1);
   }
 #pragma unroll
   for (int r = 0; r < RBW; ++r)
@@ -324,7 +341,7 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
     }
 }
 
-// ---- o / rms(o) * w * silu(gate) * scale: 16 lanes per (token, head) ----
+// ---- o / rms(o) * w * silu(gate) * scale: LPR (8 or 16) lanes per (token, head) ----
 struct GatedNormArgs {
   const float* o;  // (B, L, H, dv)
   const void* w;
@@ -336,13 +353,13 @@ struct GatedNormArgs {
   float eps, scale;
 };
 
-template <typename T, bool VEC>
+template <typename T, bool VEC, int LPR>
 __global__ __launch_bounds__(256) void gated_rms_norm_kernel(const GatedNormArgs a) {
   constexpr int N = VEC ? Pack<T>::kN : 1;
-  const long row0 = (long)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const long row0 = (long)blockIdx.x * (256 / LPR) + threadIdx.x / LPR;
   const bool live = row0 < a.rows;
   const long row = live ? row0 : a.rows - 1;
-  const int lane = threadIdx.x & 15;
+  const int lane = threadIdx.x % LPR;
   const int h = (int)(row % a.H);
   const long bl = row / a.H;
   const long b = bl / a.L, l = bl % a.L;
@@ -351,7 +368,7 @@ __global__ __launch_bounds__(256) void gated_rms_norm_kernel(const GatedNormArgs
   T* y = static_cast<T*>(a.y) + b * a.y_sb + l * a.y_sl + (long)h * a.dv;
   const T* w = static_cast<const T*>(a.w);
   float ss = 0.f;
-  for (int p = lane; p * N < a.dv; p += 16) {
+  for (int p = lane; p * N < a.dv; p += LPR) {
     float x[N];
     if constexpr (VEC) {
       load_vec<float, N>(o + p * N, x);
@@ -361,8 +378,8 @@ __global__ __launch_bounds__(256) void gated_rms_norm_kernel(const GatedNormArgs
 #pragma unroll
     for (int j = 0; j < N; ++j) ss = __builtin_fmaf(x[j], x[j], ss);
   }
-  const float r = 1.0f / sqrtf(sum16(ss) / (float)a.dv + a.eps);
-  for (int p = lane; p * N < a.dv; p += 16) {
+  const float r = 1.0f / sqrtf((LPR == 16 ? sum16(ss) : sum8(ss)) / (float)a.dv + a.eps);
+  for (int p = lane; p * N < a.dv; p += LPR) {
     float x[N], g[N], wv[N], out[N];
     if constexpr (VEC) {
       load_vec<float, N>(o + p * N, x);
@@ -379,6 +396,23 @@ __global__ __launch_bounds__(256) void gated_rms_norm_kernel(const GatedNormArgs
       else
         y[p] = from_f32<T>(out[0]);
     }
+  }
+}
+
+template <typename T> void launch_gated_norm(const GatedNormArgs& a, bool vec, hipStream_t s) {
+  const bool narrow = a.dv <= 8 * (vec ? Pack<T>::kN : 1);
+  const int per = narrow ? 32 : 16;
+  const dim3 grid((unsigned)((a.rows + per - 1) / per)), block(256);
+  if (vec) {
+    if (narrow)
+      hipLaunchKernelGGL((gated_rms_norm_kernel<T, true, 8>), grid, block, 0, s, a);
+    else
+      hipLaunchKernelGGL((gated_rms_norm_kernel<T, true, 16>), grid, block, 0, s, a);
+  } else {
+    if (narrow)
+      hipLaunchKernelGGL((gated_rms_norm_kernel<T, false, 8>), grid, block, 0, s, a);
+    else
+      hipLaunchKernelGGL((gated_rms_norm_kernel<T, false, 16>), grid, block, 0, s, a);
   }
 }
 
@@ -441,11 +475,7 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaStepArg
   for (int i = tid; i < 2 * a.d + a.dv; i += NT) {
     const int ch = i < a.d ? hk * a.d + i : (i < 2 * a.d ? a.k_off + hk * a.d + i - a.d : a.v_off + h * a.dv + i - 2 * a.d);
     const T now = x[ch];
-    float acc = 0.f;
-    for (int j = 0; j < a.taps - 1; ++j) {
-      const int p = pos - (a.taps - 1) + j;
-      if (p >= 0) acc = __builtin_fmaf(to_f32(cw[(long)j * a.C + ch]), to_f32(ring[(long)(p % a.taps) * a.C + ch]), acc);
-    }
+    float acc = ring_dot<T>(ring + ch, cw + ch, a.C, a.taps, pos);
     acc = __builtin_fmaf(to_f32(cw[(long)(a.taps - 1) * a.C + ch]), to_f32(now), acc);
     const float val = round_to<T>(silu_exact(acc));
     (i < a.d ? sq[i] : i < 2 * a.d ? sk[i - a.d] : sv[i - 2 * a.d]) = val;
@@ -526,7 +556,11 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaStepArg
 
 template <typename T, int RB, int RS> void launch_delta_scan_split(const DeltaArgs& a, hipStream_t s) {
   const int cols = 16 * (4 / RS);
-  hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS>), dim3((unsigned)(a.B * a.H), (unsigned)((a.dv + cols - 1) / cols)), dim3(256), 0, s, a);
+  const dim3 grid((unsigned)(a.B * a.H), (unsigned)((a.dv + cols - 1) / cols));
+  if (a.vec)
+    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, true>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, false>), grid, dim3(256), 0, s, a);
 }
 
 // Tiles are shared by as many wavefronts as it takes to give every compute unit a workgroup.
@@ -549,7 +583,11 @@ template <typename T, int RB> void launch_delta_scan(const DeltaArgs& a, hipStre
 
 template <typename T> void launch_delta(const DeltaArgs& a, hipStream_t s) {
   const long items = (long)a.B * a.H * a.blocks;
-  hipLaunchKernelGGL(gated_delta_prepare_kernel<T>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
+  const dim3 grid((unsigned)((items + 3) / 4));
+  if (a.vec)
+    hipLaunchKernelGGL((gated_delta_prepare_kernel<T, true>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((gated_delta_prepare_kernel<T, false>), grid, dim3(256), 0, s, a);
   const int rb = (a.d + 15) / 16;
   if (rb <= 1)
     launch_delta_scan<T, 1>(a, s);
@@ -632,25 +670,17 @@ extern "C" BASED_API int based_gated_rms_norm(const float* o, const void* weight
   BASED_REQUIRE(B >= 0 && L >= 0 && H > 0 && DV > 0, BASED_ERR_ARG, "gated_rms_norm: bad sizes");
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "gated_rms_norm: bad dtype");
   const int64_t rows = B * L * H;
-  BASED_REQUIRE((rows + 15) / 16 < (1ll << 31), BASED_ERR_SHAPE, "gated_rms_norm: grid too large");
+  BASED_REQUIRE(rows < (1ll << 33), BASED_ERR_SHAPE, "gated_rms_norm: grid too large");
   if (rows == 0) return BASED_OK;
   const GatedNormArgs a{o, weight, gate, y, (long)rows, (int)L, (int)H, (int)DV, g_sb, g_sl, y_sb, y_sl, eps, scale};
   const int n = io_dtype == BASED_BF16 ? 8 : 4;
   const bool vec = DV % n == 0 && g_sb % n == 0 && g_sl % n == 0 && y_sb % n == 0 && y_sl % n == 0 && aligned_to(o, 16) &&
                    aligned_to(weight, 16) && aligned_to(gate, 16) && aligned_to(y, 16);
-  const dim3 grid((unsigned)((rows + 15) / 16)), block(256);
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (io_dtype == BASED_BF16) {
-    if (vec)
-      hipLaunchKernelGGL((gated_rms_norm_kernel<__bf16, true>), grid, block, 0, s, a);
-    else
-      hipLaunchKernelGGL((gated_rms_norm_kernel<__bf16, false>), grid, block, 0, s, a);
-  } else {
-    if (vec)
-      hipLaunchKernelGGL((gated_rms_norm_kernel<float, true>), grid, block, 0, s, a);
-    else
-      hipLaunchKernelGGL((gated_rms_norm_kernel<float, false>), grid, block, 0, s, a);
-  }
+  if (io_dtype == BASED_BF16)
+    launch_gated_norm<__bf16>(a, vec, s);
+  else
+    launch_gated_norm<float>(a, vec, s);
   return check_launch("gated_rms_norm");
 }
 

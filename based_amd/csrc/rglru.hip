@@ -57,20 +57,26 @@ template <> struct GateMma<float> {
 __device__ __forceinline__ void lru_gates(float zr, float zi, float sp, float u, float c, float& a, float& x) {
   const float r = sigmoid_f(zr), i = sigmoid_f(zi);
   const float log_a = -c * r * sp;
-  a = expf(log_a);
-  x = sqrtf(-expm1f(2.0f * log_a)) * i * u;
+  a = exp_f(log_a);
+  x = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a)) * i * u;
 }
 
 // grid: x = segment of the sequence, y = 64-channel tile within its block (ceil(n / 64) per block), z = sequence
 template <typename T>
 __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
   typedef GateMma<T> M;
-  constexpr int KT = 32;                               // contraction staged at a time
+  constexpr int KT = 128 / (int)sizeof(T);             // contraction staged at a time
   constexpr int PAD = 16 / (int)sizeof(T);
   constexpr int KS = KT + PAD;
   constexpr int SPAD = 4;
-  __shared__ __attribute__((aligned(16))) T s_u[64 * KS], s_r[64 * KS], s_i[64 * KS];
-  __shared__ float s_a[64][64 + SPAD], s_x[64][64 + SPAD];  // [token][channel]
+  // the operands, and after them the decays and inputs of the tile
+  constexpr int kOperands = 3 * 64 * KS * (int)sizeof(T), kTile = 2 * 64 * (64 + SPAD) * 4;
+  __shared__ __attribute__((aligned(16))) char s_mem[kOperands > kTile ? kOperands : kTile];
+  T* s_u = reinterpret_cast<T*>(s_mem);
+  T* s_r = s_u + 64 * KS;
+  T* s_i = s_r + 64 * KS;
+  float(*s_a)[64 + SPAD] = reinterpret_cast<float(*)[64 + SPAD]>(s_mem);  // [token][channel]
+  float(*s_x)[64 + SPAD] = s_a + 64;
   __shared__ float s_const[3][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
   const int tiles = (a.n + 63) / 64;
@@ -93,34 +99,43 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
                    ((uintptr_t)a.ri & 15) == 0;
   for (int k0 = 0; k0 < a.n; k0 += KT) {
     __syncthreads();
-    for (int p = tid; p < 64 * (KT / V); p += 256) {
-      const int row = p / (KT / V), e = (p % (KT / V)) * V;
-      const int tok = l0 + row < a.L ? l0 + row : a.L - 1;
-      const int ch = c0 + row < a.n ? c0 + row : a.n - 1;
-      typedef typename Pack<T>::type vec_t;
-      if (vec) {
-        const bool in = k0 + e < a.n;
-        const int k = in ? k0 + e : 0;
-        vec_t xu = *reinterpret_cast<const vec_t*>(u + tok * a.u_sl + k);
-        vec_t xr = *reinterpret_cast<const vec_t*>(ra + (long)ch * a.n + k);
-        vec_t xi = *reinterpret_cast<const vec_t*>(ri + (long)ch * a.n + k);
-        if (!in) {
+    typedef typename Pack<T>::type vec_t;
+    constexpr int PIECES = 64 * (KT / V) / 256;
+    if (vec) {
+      vec_t xu[PIECES], xr[PIECES], xi[PIECES];
 #pragma unroll
-          for (int j = 0; j < V; ++j) xu[j] = xr[j] = xi[j] = (T)0.0f;
-        }
-        *reinterpret_cast<vec_t*>(&s_u[row * KS + e]) = xu;
-        *reinterpret_cast<vec_t*>(&s_r[row * KS + e]) = xr;
-        *reinterpret_cast<vec_t*>(&s_i[row * KS + e]) = xi;
-      } else {
+      for (int i = 0; i < PIECES; ++i) {
+        const int p = i * 256 + tid, row = p / (KT / V), e = (p % (KT / V)) * V;
+        const int tok = l0 + row < a.L ? l0 + row : a.L - 1, ch = c0 + row < a.n ? c0 + row : a.n - 1;
+        const int k = k0 + e < a.n ? k0 + e : 0;
+        xu[i] = *reinterpret_cast<const vec_t*>(u + tok * a.u_sl + k);
+        xr[i] = *reinterpret_cast<const vec_t*>(ra + (long)ch * a.n + k);
+        xi[i] = *reinterpret_cast<const vec_t*>(ri + (long)ch * a.n + k);
+      }
+#pragma unroll
+      for (int i = 0; i < PIECES; ++i) {
+        const int p = i * 256 + tid, row = p / (KT / V), e = (p % (KT / V)) * V;
+        const bool in = k0 + e < a.n;
 #pragma unroll
         for (int j = 0; j < V; ++j) {
-          const bool in = k0 + e + j < a.n;
-          const int k = in ? k0 + e + j : 0;
-          const T xu = u[tok * a.u_sl + k], xr = ra[(long)ch * a.n + k], xi = ri[(long)ch * a.n + k];
-          s_u[row * KS + e + j] = in ? xu : (T)0.0f;
-          s_r[row * KS + e + j] = in ? xr : (T)0.0f;
-          s_i[row * KS + e + j] = in ? xi : (T)0.0f;
+          xu[i][j] = in ? xu[i][j] : (T)0.0f;
+          xr[i][j] = in ? xr[i][j] : (T)0.0f;
+          xi[i][j] = in ? xi[i][j] : (T)0.0f;
         }
+        *reinterpret_cast<vec_t*>(&s_u[row * KS + e]) = xu[i];
+        *reinterpret_cast<vec_t*>(&s_r[row * KS + e]) = xr[i];
+        *reinterpret_cast<vec_t*>(&s_i[row * KS + e]) = xi[i];
+      }
+    } else {
+      for (int p = tid; p < 64 * KT; p += 256) {
+        const int row = p / KT, e = p % KT;
+        const int tok = l0 + row < a.L ? l0 + row : a.L - 1, ch = c0 + row < a.n ? c0 + row : a.n - 1;
+        const bool in = k0 + e < a.n;
+        const int k = in ? k0 + e : 0;
+        const T xu = u[tok * a.u_sl + k], xr = ra[(long)ch * a.n + k], xi = ri[(long)ch * a.n + k];
+        s_u[row * KS + e] = in ? xu : (T)0.0f;
+        s_r[row * KS + e] = in ? xr : (T)0.0f;
+        s_i[row * KS + e] = in ? xi : (T)0.0f;
       }
     }
     __syncthreads();
@@ -135,6 +150,7 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
       }
     }
   }
+  __syncthreads();  // the operands are done with
   // lane: token wave*16 + l16, channels i*16 + quad*4 ..
   const int tl = wave * 16 + l16, tok = l0 + tl;
   const bool tok_in = tok < a.L;
@@ -184,42 +200,70 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
   }
 }
 
-// grid: x = 256-channel tile, y = segment, z = sequence
-template <typename T>
+// C consecutive channels as floats / from floats
+template <typename T, int C> __device__ __forceinline__ void load_ch(const T* p, float (&out)[C]) {
+  typedef __attribute__((ext_vector_type(C))) T vec_t;
+  const vec_t x = *reinterpret_cast<const vec_t*>(p);
+#pragma unroll
+  for (int c = 0; c < C; ++c) out[c] = to_f32(x[c]);
+}
+
+// grid: x = tile of 256 C channels, y = segment, z = sequence; C channels per thread
+template <typename T, int C>
 __global__ __launch_bounds__(256) void rglru_scan_kernel(const RglruArgs a) {
-  const int w = blockIdx.x * 256 + threadIdx.x;
+  const int w = (blockIdx.x * 256 + threadIdx.x) * C;
   if (w >= a.W) return;
   const int seg = blockIdx.y, b = blockIdx.z, l0 = seg * kSeg;
   const float* g = a.agg + (long)b * (a.segs + 1) * 2 * a.W + w;
-  float S = 0.f;
-#pragma unroll 8
-  for (int i = 0; i <= seg; ++i) S = __builtin_fmaf(g[(long)i * 2 * a.W], S, g[(long)i * 2 * a.W + a.W]);
+  float S[C];
+#pragma unroll
+  for (int c = 0; c < C; ++c) S[c] = 0.f;
+  constexpr int U = 8;
+  for (int i0 = 0; i0 <= seg; i0 += U) {
+    float P[U][C], X[U][C];
+#pragma unroll
+    for (int i = 0; i < U; ++i) {
+      const long at = (long)(i0 + i <= seg ? i0 + i : seg) * 2 * a.W;
+      load_ch<float, C>(g + at, P[i]);
+      load_ch<float, C>(g + at + a.W, X[i]);
+    }
+#pragma unroll
+    for (int i = 0; i < U; ++i)
+#pragma unroll
+      for (int c = 0; c < C; ++c) S[c] = i0 + i <= seg ? __builtin_fmaf(P[i][c], S[c], X[i][c]) : S[c];
+  }
   const int ntok = a.L - l0 < kSeg ? a.L - l0 : kSeg;
   const float* pa = a.ga + ((long)b * a.L + l0) * a.W + w;
   const float* px = a.gx + ((long)b * a.L + l0) * a.W + w;
   const T* py = static_cast<const T*>(a.y) + b * a.y_sb + l0 * a.y_sl + w;
   T* po = static_cast<T*>(a.out) + b * a.o_sb + l0 * a.o_sl + w;
-  constexpr int U = 8;
-  int t = 0;
-  for (; t + U <= ntok; t += U) {
-    float av[U], xv[U], yv[U];
+  for (int t0 = 0; t0 < ntok; t0 += U) {
+    float av[U][C], xv[U][C], yv[U][C];
 #pragma unroll
     for (int i = 0; i < U; ++i) {
-      av[i] = pa[(long)(t + i) * a.W];
-      xv[i] = px[(long)(t + i) * a.W];
-      yv[i] = to_f32(py[(t + i) * a.y_sl]);
+      const int t = t0 + i < ntok ? t0 + i : ntok - 1;
+      load_ch<float, C>(pa + (long)t * a.W, av[i]);
+      load_ch<float, C>(px + (long)t * a.W, xv[i]);
+      load_ch<T, C>(py + t * a.y_sl, yv[i]);
     }
 #pragma unroll
     for (int i = 0; i < U; ++i) {
-      S = __builtin_fmaf(av[i], S, xv[i]);
-      po[(t + i) * a.o_sl] = from_f32<T>(S * gelu_tanh_f(yv[i]));
+      if (t0 + i < ntok) {
+        typedef __attribute__((ext_vector_type(C))) T vec_t;
+        vec_t o;
+#pragma unroll
+        for (int c = 0; c < C; ++c) {
+          S[c] = __builtin_fmaf(av[i][c], S[c], xv[i][c]);
+          o[c] = from_f32<T>(S[c] * gelu_tanh_f(yv[i][c]));
+        }
+        *reinterpret_cast<vec_t*>(po + (t0 + i) * a.o_sl) = o;
+      }
     }
   }
-  for (; t < ntok; ++t) {
-    S = __builtin_fmaf(pa[(long)t * a.W], S, px[(long)t * a.W]);
-    po[t * a.o_sl] = from_f32<T>(S * gelu_tanh_f(to_f32(py[t * a.y_sl])));
+  if (seg == a.segs - 1) {
+#pragma unroll
+    for (int c = 0; c < C; ++c) a.state[(long)b * a.W + w + c] = S[c];
   }
-  if (seg == a.segs - 1) a.state[(long)b * a.W + w] = S;
 }
 
 // ---- one token per sequence ----
@@ -265,10 +309,7 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) 
       const T* cw = static_cast<const T*>(a.conv_w) + ch;
       T* ring = static_cast<T*>(a.ring) + b * a.ring_sb + ch;
       float acc = a.conv_b != nullptr ? to_f32(static_cast<const T*>(a.conv_b)[ch]) : 0.f;
-      for (int j = 0; j < a.taps - 1; ++j) {
-        const int p = pos - (a.taps - 1) + j;
-        if (p >= 0) acc = __builtin_fmaf(to_f32(cw[(long)j * a.W]), to_f32(ring[(long)(p % a.taps) * a.W]), acc);
-      }
+      acc += ring_dot<T>(ring, cw, a.W, a.taps, pos);
       acc = __builtin_fmaf(to_f32(cw[(long)(a.taps - 1) * a.W]), to_f32(now), acc);
       val = round_to<T>(acc);
       // a slot that no reader of this step looks at; one tile of the block writes it
@@ -330,6 +371,17 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) 
   }
 }
 
+template <typename T> void launch_rglru_prefill(const RglruArgs& a, int tiles, bool pairs, hipStream_t s) {
+  const int per = pairs ? 512 : 256;
+  const dim3 g1((unsigned)a.segs, (unsigned)tiles, (unsigned)a.B);
+  const dim3 g2((unsigned)((a.W + per - 1) / per), (unsigned)a.segs, (unsigned)a.B), block(256);
+  hipLaunchKernelGGL(rglru_gates_kernel<T>, g1, block, 0, s, a);
+  if (pairs)
+    hipLaunchKernelGGL((rglru_scan_kernel<T, 2>), g2, block, 0, s, a);
+  else
+    hipLaunchKernelGGL((rglru_scan_kernel<T, 1>), g2, block, 0, s, a);
+}
+
 }  // namespace based
 
 extern "C" BASED_API int based_rglru_prefill(const void* u, const void* y, const void* ra, const void* rb, const void* ri, const void* ib,
@@ -348,14 +400,12 @@ extern "C" BASED_API int based_rglru_prefill(const void* u, const void* y, const
   const RglruArgs a{u,      y,      ra,     rb,     ri,        ib,   lam,  work_a, work_x, work_agg, state, out, (int)B,
                     (int)L, (int)W, (int)n, (int)segs, u_sb, u_sl, y_sb,   y_sl,   o_sb,     o_sl,  c,   fresh};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const dim3 g1((unsigned)segs, (unsigned)tiles, (unsigned)B), g2((unsigned)((W + 255) / 256), (unsigned)segs, (unsigned)B), block(256);
-  if (io_dtype == BASED_BF16) {
-    hipLaunchKernelGGL(rglru_gates_kernel<__bf16>, g1, block, 0, s, a);
-    hipLaunchKernelGGL(rglru_scan_kernel<__bf16>, g2, block, 0, s, a);
-  } else {
-    hipLaunchKernelGGL(rglru_gates_kernel<float>, g1, block, 0, s, a);
-    hipLaunchKernelGGL(rglru_scan_kernel<float>, g2, block, 0, s, a);
-  }
+  const bool pairs = W % 2 == 0 && y_sb % 2 == 0 && y_sl % 2 == 0 && o_sb % 2 == 0 && o_sl % 2 == 0 && aligned_to(y, 8) &&
+                     aligned_to(out, 8) && aligned_to(work_a, 8) && aligned_to(work_x, 8) && aligned_to(work_agg, 8);
+  if (io_dtype == BASED_BF16)
+    launch_rglru_prefill<__bf16>(a, (int)tiles, pairs, s);
+  else
+    launch_rglru_prefill<float>(a, (int)tiles, pairs, s);
   return check_launch("rglru_prefill");
 }
 

@@ -1,7 +1,8 @@
 // Helpers shared by the kernels of the streaming layers (norms with a scaled residual, causal
 // convolutions on a ring of past inputs, grouped window attention, gated delta rule, gated linear
-// recurrent unit).  Transcendentals are the library's full-precision fp32 functions: everything
-// that enters a norm, a softmax or a recurrence is evaluated in 32 bits.
+// recurrent unit).  Everything that enters a norm, a softmax or a recurrence is evaluated in 32 bits;
+// exponentials, reciprocals and square roots are the hardware's (1 ulp) where a value per element and
+// token is needed.
 #pragma once
 
 #include "common.hpp"
@@ -18,12 +19,21 @@ template <> struct Pack<float> {
   typedef f32x4 type;
 };
 
-__device__ __forceinline__ float sigmoid_f(float z) { return 1.0f / (1.0f + expf(-z)); }
-__device__ __forceinline__ float silu_exact(float z) { return z / (1.0f + expf(-z)); }
+// exp of an argument whose rounding to a power of two may cost |z| ulps: callers have |z| small, or a result
+// that is far from the scale of what it is added to.
+__device__ __forceinline__ float exp_f(float z) { return __builtin_amdgcn_exp2f(z * 1.4426950408889634f); }
+__device__ __forceinline__ float sigmoid_f(float z) { return __builtin_amdgcn_rcpf(1.0f + exp_f(-z)); }
+__device__ __forceinline__ float silu_exact(float z) { return z * sigmoid_f(z); }
 __device__ __forceinline__ float softplus_f(float z) { return log1pf(expf(-fabsf(z))) + fmaxf(z, 0.0f); }
+// 0.5 z (1 + tanh(t)) = z sigmoid(2 t)
 __device__ __forceinline__ float gelu_tanh_f(float z) {
-  const float t = 0.7978845608028654f * (z + 0.044715f * z * z * z);
-  return 0.5f * z * (1.0f + tanhf(t));
+  return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z));
+}
+// 1 - exp(x) for x <= 0 without cancellation: the series below 1/4 (the next term is 5e-8 of the sum)
+__device__ __forceinline__ float one_minus_exp(float x) {
+  const float p = x * (1.f / 720.f) + 1.f / 120.f;
+  const float series = -x * (1.f + x * (0.5f + x * (1.f / 6.f + x * (1.f / 24.f + x * p))));
+  return x > -0.25f ? series : 1.0f - exp_f(x);
 }
 // x as the element type would keep it
 template <typename T> __device__ __forceinline__ float round_to(float x) { return to_f32(from_f32<T>(x)); }
@@ -71,6 +81,27 @@ __device__ __forceinline__ float sum16(float v) {
 }
 
 inline bool aligned_to(const void* p, uintptr_t n) { return (reinterpret_cast<uintptr_t>(p) & (n - 1)) == 0; }
+
+// Sum of w_j x_{t - taps + 1 + j} over the past inputs of one channel of a ring (taps slots, `stride` elements
+// apart; w likewise): three at a time, those before position 0 fetched from slot 0 and left out.
+template <typename T>
+__device__ __forceinline__ float ring_dot(const T* ring, const T* w, long stride, int taps, int pos) {
+  float acc = 0.f;
+  for (int j0 = 0; j0 < taps - 1; j0 += 3) {
+    T x[3], c[3];
+    bool ok[3];
+#pragma unroll
+    for (int j = 0; j < 3; ++j) {
+      const int p = pos - (taps - 1) + j0 + j;
+      ok[j] = j0 + j < taps - 1 && p >= 0;
+      x[j] = ring[(ok[j] ? p % taps : 0) * stride];
+      c[j] = w[(ok[j] ? j0 + j : 0) * stride];
+    }
+#pragma unroll
+    for (int j = 0; j < 3; ++j) acc = ok[j] ? __builtin_fmaf(to_f32(c[j]), to_f32(x[j]), acc) : acc;
+  }
+  return acc;
+}
 
 // Position of the token a single-token launch brings for batch row b: from the device when there is
 // an array of positions, otherwise the one the host passed.

@@ -62,29 +62,42 @@ __device__ __forceinline__ float rotated(const T* row, int c, int pos, const Win
   return x * a.cos_t[t] + sgn * to_f32(row[partner]) * a.sin_t[t];
 }
 
-// 8 channels from c on (a multiple of 8) of interleaved pairs, in registers.
-__device__ __forceinline__ void rotate8(float (&x)[8], int c, int pos, const WindowArgs& a) {
-  if (c >= a.rot) return;
-  const long t = (long)pos * (a.rot / 2) + c / 2;
-  float cs[4], sn[4];
-  if ((a.rot & 7) == 0) {
-    load_vec<float, 4>(a.cos_t + t, cs);
-    load_vec<float, 4>(a.sin_t + t, sn);
-  } else {
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const bool in = c + 2 * j < a.rot;
-      cs[j] = in ? a.cos_t[t + j] : 1.f;
-      sn[j] = in ? a.sin_t[t + j] : 0.f;
+// What turns 8 channels from c on (c and the rotary size multiples of 8): angles, and for half-split pairs
+// the partners.  Loaded without a condition (what is not rotated reads the table's start and its own
+// channels) and applied later, so that every load of a row is on its way before the first is waited for.
+template <bool HALF> struct Turn8 {
+  float cs[HALF ? 8 : 4], sn[HALF ? 8 : 4], partner[8];
+  __device__ __forceinline__ void load(const __bf16* row, int c, int pos, const WindowArgs& a) {
+    const bool in = c < a.rot;
+    const int half = a.rot / 2;
+    if constexpr (HALF) {
+      const int pair = in ? (c < half ? c : c - half) : 0;
+      const long t = in ? (long)pos * half + pair : 0;
+      load_vec<float, 8>((a.rot > 0 ? a.cos_t : reinterpret_cast<const float*>(a.kv)) + t, cs);
+      load_vec<float, 8>((a.rot > 0 ? a.sin_t : reinterpret_cast<const float*>(a.kv)) + t, sn);
+      load_vec<__bf16, 8>(row + (in ? (c < half ? c + half : c - half) : 0), partner);
+    } else {
+      const long t = in ? (long)pos * half + c / 2 : 0;
+      load_vec<float, 4>((a.rot > 0 ? a.cos_t : reinterpret_cast<const float*>(a.kv)) + t, cs);
+      load_vec<float, 4>((a.rot > 0 ? a.sin_t : reinterpret_cast<const float*>(a.kv)) + t, sn);
     }
   }
+  __device__ __forceinline__ void apply(float (&x)[8], int c, const WindowArgs& a) const {
+    if (c >= a.rot) return;
+    if constexpr (HALF) {
+      const float sgn = c < a.rot / 2 ? -1.f : 1.f;
 #pragma unroll
-  for (int j = 0; j < 4; ++j) {
-    const float u = x[2 * j], v = x[2 * j + 1];
-    x[2 * j] = u * cs[j] - v * sn[j];
-    x[2 * j + 1] = v * cs[j] + u * sn[j];
+      for (int j = 0; j < 8; ++j) x[j] = x[j] * cs[j] + sgn * partner[j] * sn[j];
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const float u = x[2 * j], v = x[2 * j + 1];
+        x[2 * j] = u * cs[j] - v * sn[j];
+        x[2 * j + 1] = v * cs[j] + u * sn[j];
+      }
+    }
   }
-}
+};
 
 // One wavefront per (token, key/value head).
 template <typename T>
@@ -106,14 +119,15 @@ __global__ __launch_bounds__(256) void window_kv_write_kernel(const WindowArgs a
   for (int c = lane; c < a.dv; c += 64) out[a.d + c] = from_f32<T>(to_f32(v[c]) * r);
 }
 
-// The same with 16-byte pieces: 16 lanes per (token, key/value head), interleaved pairs or none.
-// d, dv and every stride multiples of 8, pointers 16-byte aligned; d, dv <= 256.
+// The same with 16-byte pieces: LPI (8, 16 or 32) lanes per (token, key/value head), one piece of the key and
+// one of the value each.  d, dv and every stride multiples of 8, pointers 16-byte aligned.
+template <int LPI, bool HALF>
 __global__ __launch_bounds__(256) void window_kv_write_vec_kernel(const WindowArgs a) {
-  const long item0 = (long)blockIdx.x * 16 + (threadIdx.x >> 4);
+  const long item0 = (long)blockIdx.x * (256 / LPI) + threadIdx.x / LPI;
   const long n_items = (long)a.B * a.L * a.G;
   const bool live = item0 < n_items;
   const long item = live ? item0 : n_items - 1;
-  const int lane = threadIdx.x & 15;
+  const int c = (threadIdx.x % LPI) * 8;
   const int g = (int)(item % a.G);
   const long bl = item / a.G;
   const int l = (int)(bl % a.L), b = (int)(bl / a.L);
@@ -121,28 +135,24 @@ __global__ __launch_bounds__(256) void window_kv_write_vec_kernel(const WindowAr
   const __bf16* k = static_cast<const __bf16*>(a.k) + b * a.k_sb + l * a.k_sl + (long)g * a.d;
   const __bf16* v = static_cast<const __bf16*>(a.v) + b * a.v_sb + l * a.v_sl + (long)g * a.dv;
   __bf16* out = static_cast<__bf16*>(a.kv) + b * a.kv_sb + pos * a.kv_st + (long)g * (a.d + a.dv);
-  float x[2][8], y[2][8];
+  const int ck = c < a.d ? c : 0, cv = c < a.dv ? c : 0;
+  float x[8], y[8];
+  Turn8<HALF> turn;
+  load_vec<__bf16, 8>(k + ck, x);
+  load_vec<__bf16, 8>(v + cv, y);
+  turn.load(k, ck, pos, a);
   float ss = 0.f;
 #pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int c = (i * 16 + lane) * 8;
-    load_vec<__bf16, 8>(k + (c < a.d ? c : 0), x[i]);
-    load_vec<__bf16, 8>(v + (c < a.dv ? c : 0), y[i]);
-    if (c < a.dv) {
+  for (int j = 0; j < 8; ++j) ss = __builtin_fmaf(y[j], y[j], ss);
+  ss = c < a.dv ? ss : 0.f;
+  ss = LPI == 8 ? sum8(ss) : sum16(ss);
+  if (LPI == 32) ss += __shfl_xor(ss, 16, 64);
+  const float r = a.norm_v ? 1.0f / sqrtf(ss / (float)a.dv + a.eps) : 1.0f;
+  turn.apply(x, ck, a);
 #pragma unroll
-      for (int j = 0; j < 8; ++j) ss = __builtin_fmaf(y[i][j], y[i][j], ss);
-    }
-  }
-  const float r = a.norm_v ? 1.0f / sqrtf(sum16(ss) / (float)a.dv + a.eps) : 1.0f;
-#pragma unroll
-  for (int i = 0; i < 2; ++i) {
-    const int c = (i * 16 + lane) * 8;
-    rotate8(x[i], c, pos, a);
-#pragma unroll
-    for (int j = 0; j < 8; ++j) y[i][j] *= r;
-    if (live && c < a.d) store_vec<__bf16, 8>(out + c, x[i]);
-    if (live && c < a.dv) store_vec<__bf16, 8>(out + a.d + c, y[i]);
-  }
+  for (int j = 0; j < 8; ++j) y[j] *= r;
+  if (live && c < a.d) store_vec<__bf16, 8>(out + c, x);
+  if (live && c < a.dv) store_vec<__bf16, 8>(out + a.d + c, y);
 }
 
 // ---- prefill, bf16, MFMA ----
@@ -155,7 +165,7 @@ __device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0);
 }
 
-template <int KC, int VC>
+template <int KC, int VC, bool HALF>
 __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowArgs a) {
   constexpr int D = KC * 32, DV = VC * 32;
   constexpr int KS = D + 8, VS = kTileKeys + 8;  // LDS row strides: 16-lane reads of 16 bytes meet every bank once
@@ -170,9 +180,11 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
   const int row_w = r0 + wave * 32;  // first row of this wavefront
   const __bf16* kv = static_cast<const __bf16*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
 
-  // queries: lane holds channels quad*8 + 32 c .. of row l16 (+16): the MFMA's second operand
+  // queries: lane holds channels quad*8 + 32 c .. of row l16 (+16): the MFMA's second operand.  Turned and
+  // rounded after the first tile of keys has been asked for.
   bf16x8 qf[2][KC];
   int qpos[2], qtok[2], qhead[2];
+  const __bf16* qrow[2];
 #pragma unroll
   for (int t = 0; t < 2; ++t) {
     const int row = row_w + t * 16 + l16;
@@ -180,20 +192,11 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
     qtok[t] = rr / qpk;
     qhead[t] = g * qpk + rr % qpk;
     qpos[t] = a.pos_host + qtok[t];
-    const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + qtok[t] * a.q_sl + (long)qhead[t] * a.d;
+    qrow[t] = static_cast<const __bf16*>(a.q) + b * a.q_sb + qtok[t] * a.q_sl + (long)qhead[t] * a.d;
 #pragma unroll
     for (int c = 0; c < KC; ++c) {
       const int e = c * 32 + quad * 8;
-      float x[8];
-      load_vec<__bf16, 8>(qp + (e < a.d ? e : 0), x);
-      if (a.half_split && e < a.rot) {
-#pragma unroll
-        for (int j = 0; j < 8; ++j) x[j] = rotated(qp, e + j, qpos[t], a);
-      } else {
-        rotate8(x, e, qpos[t], a);
-      }
-#pragma unroll
-      for (int j = 0; j < 8; ++j) qf[t][c][j] = (__bf16)(e < a.d ? x[j] : 0.f);
+      qf[t][c] = *reinterpret_cast<const bf16x8*>(qrow[t] + (e < a.d ? e : 0));
     }
   }
   const int wave_lo_tok = a.pos_host + (row_w < n_rows ? row_w : n_rows - 1) / qpk;
@@ -218,13 +221,12 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
   u32x4 kbuf[KP];
   u32x4 vbuf[VP][4];
   const u32x4 zero4 = {0u, 0u, 0u, 0u};
+  // rows past the last key and channels past the sizes are fetched from valid places and cleared in `stage`
   auto fetch = [&](int k0) {
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
-      const bool ok = k0 + key <= last_pos && e < a.d;
-      const u32x4 x = *reinterpret_cast<const u32x4*>(kv + (long)(ok ? k0 + key : lo) * a.kv_st + (ok ? e : 0));
-      kbuf[i] = ok ? x : zero4;
+      const int p = i * 256 + tid, key = k0 + p / (D / 8), e = (p % (D / 8)) * 8;
+      kbuf[i] = *reinterpret_cast<const u32x4*>(kv + (long)(key <= last_pos ? key : last_pos) * a.kv_st + (e < a.d ? e : 0));
     }
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
@@ -232,22 +234,22 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
         const int key = k0 + k4 * 4 + r;
-        const bool ok = key <= last_pos && e < a.dv;
-        const u32x4 x = *reinterpret_cast<const u32x4*>(kv + (long)(ok ? key : lo) * a.kv_st + a.d + (ok ? e : 0));
-        vbuf[i][r] = ok ? x : zero4;
+        vbuf[i][r] = *reinterpret_cast<const u32x4*>(kv + (long)(key <= last_pos ? key : last_pos) * a.kv_st + a.d + (e < a.dv ? e : 0));
       }
     }
   };
-  auto stage = [&]() {
+  auto stage = [&](int k0) {
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
       const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
-      *reinterpret_cast<u32x4*>(&lds_k[key * KS + e]) = kbuf[i];
+      *reinterpret_cast<u32x4*>(&lds_k[key * KS + e]) = e < a.d ? kbuf[i] : zero4;
     }
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
       const int p = i * 256 + tid, k4 = p & 15, e = (p >> 4) * 8;
       if (e < DV) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) vbuf[i][r] = e < a.dv ? vbuf[i][r] : zero4;
 #pragma unroll
         for (int j = 0; j < 8; ++j) {
           bf16x4 col;
@@ -260,11 +262,43 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
   };
 
   fetch(lo);
+  if (a.rot > 0) {
+    constexpr int CB = KC < 4 ? KC : 4;
+#pragma unroll
+    for (int c0 = 0; c0 < KC; c0 += CB) {
+      Turn8<HALF> turn[2][CB];
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int c = 0; c < CB; ++c) turn[t][c].load(qrow[t], (c0 + c) * 32 + quad * 8, qpos[t], a);
+#pragma unroll
+      for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int c = 0; c < CB; ++c) {
+          float x[8];
+#pragma unroll
+          for (int j = 0; j < 8; ++j) x[j] = to_f32(qf[t][c0 + c][j]);
+          turn[t][c].apply(x, (c0 + c) * 32 + quad * 8, a);
+#pragma unroll
+          for (int j = 0; j < 8; ++j) qf[t][c0 + c][j] = (__bf16)x[j];
+        }
+    }
+  }
+  if (D > a.d) {
+#pragma unroll
+    for (int c = 0; c < KC; ++c)
+      if (c * 32 + quad * 8 >= a.d) {
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+          for (int j = 0; j < 8; ++j) qf[t][c][j] = (__bf16)0.f;
+      }
+  }
   for (int k0 = lo; k0 <= last_pos; k0 += kTileKeys) {
     __syncthreads();  // every wavefront is done with the tile before
-    stage();
+    stage(k0);
     __syncthreads();
-    if (k0 + kTileKeys <= last_pos) fetch(k0 + kTileKeys);
+    fetch(k0 + kTileKeys <= last_pos ? k0 + kTileKeys : last_pos);  // always, so that nothing is waited for at a branch
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
       // 32 keys at a time: does any row of this wavefront see one of them, does every row see all?
@@ -413,10 +447,19 @@ __global__ __launch_bounds__(64) void window_prefill_any_kernel(const WindowArgs
 constexpr int kStepThreads = 256;
 constexpr int kStepKeys = 256;  // keys per round of the running softmax
 
+template <typename T, int N> struct RawPiece {
+  typedef typename Pack<T>::type type;
+  static __device__ __forceinline__ float get(type x, int i) { return to_f32(x[i]); }
+};
+template <typename T> struct RawPiece<T, 1> {
+  typedef T type;
+  static __device__ __forceinline__ float get(type x, int) { return to_f32(x); }
+};
+
 // QT: query heads of the group served together (the group is walked QT heads at a time).
 // VEC: 16-byte pieces of the rows (sizes and strides multiples of the piece); otherwise element by element.
 template <typename T, int QT, bool VEC>
-__global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowArgs a) {
+__global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowArgs a, int part_floats) {
   constexpr int N = VEC ? Pack<T>::kN : 1;
   extern __shared__ float smem[];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
@@ -428,20 +471,11 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   float* sc = qs + QT * a.d;               // [QT][kStepKeys]
   float* stat = sc + QT * kStepKeys;       // [3][QT]: running maximum, running sum, rescale of this round
   float* part = stat + 3 * QT;             // [QT][parts][vp2 * N], partial outputs
+  float* knew = part + part_floats;        // [d] and [dv]: the row of the new token, as the cache holds it
+  float* vnew = knew + a.d;
   const T* k = static_cast<const T*>(a.k) + b * a.k_sb + (long)g * a.d;
   const T* v = static_cast<const T*>(a.v) + b * a.v_sb + (long)g * a.dv;
   T* kv = static_cast<T*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
-  {
-    T* out = kv + (long)pos * a.kv_st;
-    if (wave == 0) {
-      float ss = 0.f;
-      for (int c = lane; c < a.dv; c += 64) ss = __builtin_fmaf(to_f32(v[c]), to_f32(v[c]), ss);
-      const float r = a.norm_v ? 1.0f / sqrtf(wave_sum(ss) / (float)a.dv + a.eps) : 1.0f;
-      for (int c = lane; c < a.dv; c += 64) out[a.d + c] = from_f32<T>(to_f32(v[c]) * r);
-    } else {
-      for (int c = tid - 64; c < a.d; c += kStepThreads - 64) out[c] = from_f32<T>(rotated(k, c, pos, a));
-    }
-  }
   const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
   // lanes per key: the smallest power of two that covers the row in N-element pieces, 64 at most
   const int pieces = (a.d + N - 1) / N;
@@ -455,9 +489,41 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   const int parts = vp2 < 64 ? kStepThreads / 64 : v_groups, my_part = vp2 < 64 ? wave : my_vg;
   const bool v_in = my_vp * N < a.dv;
   constexpr int KU = 4;  // rows whose loads are in flight together
+  typedef typename RawPiece<T, N>::type raw_t;
+  auto load_row = [&](int j, int n, int first, int piece, int k0) -> raw_t {
+    return *reinterpret_cast<const raw_t*>(kv + (long)(k0 + (j < n ? j : n - 1)) * a.kv_st + first + piece * N);
+  };
+  // the first rows of the cache are asked for before anything else; the new token's row is not in it yet
+  // and is taken from LDS
+  const int n_first = pos - lo + 1 < kStepKeys ? pos - lo + 1 : kStepKeys;
+  const int kp = my_piece < pieces ? my_piece : 0, vp = v_in ? my_vp : 0;
+  raw_t xk[KU], xv[KU];
+#pragma unroll
+  for (int u = 0; u < KU; ++u) xk[u] = load_row(u * keys_at_once + my_key, n_first, 0, kp, lo);
+#pragma unroll
+  for (int u = 0; u < KU; ++u) xv[u] = load_row(u * v_groups + my_vg, n_first, a.d, vp, lo);
+  {
+    T* out = kv + (long)pos * a.kv_st;
+    if (wave == 0) {
+      float ss = 0.f;
+      for (int c = lane; c < a.dv; c += 64) ss = __builtin_fmaf(to_f32(v[c]), to_f32(v[c]), ss);
+      const float r = a.norm_v ? 1.0f / sqrtf(wave_sum(ss) / (float)a.dv + a.eps) : 1.0f;
+      for (int c = lane; c < a.dv; c += 64) {
+        const T x = from_f32<T>(to_f32(v[c]) * r);
+        out[a.d + c] = x;
+        vnew[c] = to_f32(x);
+      }
+    } else {
+      for (int c = tid - 64; c < a.d; c += kStepThreads - 64) {
+        const T x = from_f32<T>(rotated(k, c, pos, a));
+        out[c] = x;
+        knew[c] = to_f32(x);
+      }
+    }
+  }
 
   for (int h0 = 0; h0 < qpk; h0 += QT) {
-    __syncthreads();  // the new row is visible; the round before is done with LDS
+    if (h0 > 0) __syncthreads();  // the round before is done with LDS
     for (int i = tid; i < QT * a.d; i += kStepThreads) {
       const int hh = i / a.d, c = i % a.d;
       const int h = g * qpk + (h0 + hh < qpk ? h0 + hh : h0);
@@ -481,32 +547,37 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
       for (int i = 0; i < N; ++i) acc[hh][i] = 0.f;
     for (int k0 = lo; k0 <= pos; k0 += kStepKeys) {
       const int n = pos - k0 + 1 < kStepKeys ? pos - k0 + 1 : kStepKeys;
-      const T* rows = kv + (long)k0 * a.kv_st;
       if (k0 > lo) __syncthreads();
-      auto load_row = [&](const T* base, int j, int piece, float (&x)[N]) {
-        const T* r = base + (long)(j < n ? j : n - 1) * a.kv_st + piece * N;
-        if constexpr (VEC)
-          load_vec<T, N>(r, x);
-        else
-          x[0] = to_f32(*r);
-      };
-      for (int j0 = 0; j0 < n; j0 += KU * keys_at_once) {
-        float x[KU][N];
+      // the pieces of row j as floats; the last row of all is the new token's
+      auto floats = [&](raw_t x, const float* fresh, int piece, int j, float (&f)[N]) {
+        const bool is_new = k0 + j == pos;
 #pragma unroll
-        for (int u = 0; u < KU; ++u) load_row(rows, j0 + u * keys_at_once + my_key, my_piece < pieces ? my_piece : 0, x[u]);
+        for (int i = 0; i < N; ++i) {
+          const float nv = fresh[piece * N + i], ov = RawPiece<T, N>::get(x, i);
+          f[i] = is_new ? nv : ov;
+        }
+      };
+      const bool first = h0 == 0 && k0 == lo;
+      for (int j0 = 0; j0 < n; j0 += KU * keys_at_once) {
+        if (!first || j0 > 0) {
+#pragma unroll
+          for (int u = 0; u < KU; ++u) xk[u] = load_row(j0 + u * keys_at_once + my_key, n, 0, kp, k0);
+        }
 #pragma unroll
         for (int u = 0; u < KU; ++u) {
           const int j = j0 + u * keys_at_once + my_key;
+          float f[N];
+          floats(xk[u], knew, kp, j, f);
           float dot[QT];
 #pragma unroll
           for (int hh = 0; hh < QT; ++hh) {
             dot[hh] = 0.f;
 #pragma unroll
-            for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(x[u][i], qr[hh][i], dot[hh]);
+            for (int i = 0; i < N; ++i) dot[hh] = __builtin_fmaf(f[i], qr[hh][i], dot[hh]);
           }
           for (int p = my_piece + lpk; p < pieces; p += lpk) {  // rows of more than 64 pieces
             float y[N];
-            load_row(rows, j, p, y);
+            floats(load_row(j, n, 0, p, k0), knew, p, j, y);
 #pragma unroll
             for (int hh = 0; hh < QT; ++hh)
 #pragma unroll
@@ -514,15 +585,22 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
           }
 #pragma unroll
           for (int hh = 0; hh < QT; ++hh) {
-            for (int m = 1; m < lpk; m <<= 1) dot[hh] += __shfl_xor(dot[hh], m, 64);
+            if (lpk == 8) {
+              dot[hh] = sum8(dot[hh]);
+            } else if (lpk == 16) {
+              dot[hh] = sum16(dot[hh]);
+            } else {
+              for (int m = 1; m < lpk; m <<= 1) dot[hh] += __shfl_xor(dot[hh], m, 64);
+            }
             if (my_piece == 0 && j < n) sc[hh * kStepKeys + j] = dot[hh] * a.scale;
           }
         }
       }
-      // the first value rows are on their way during the softmax
-      float xv[KU][N];
+      if (!first) {
+        // the first value rows are on their way during the softmax
 #pragma unroll
-      for (int u = 0; u < KU; ++u) load_row(rows + a.d, my_vg + u * v_groups, v_in ? my_vp : 0, xv[u]);
+        for (int u = 0; u < KU; ++u) xv[u] = load_row(my_vg + u * v_groups, n, a.d, vp, k0);
+      }
       __syncthreads();
       for (int hh = wave; hh < QT; hh += kStepThreads / 64) {
         float s[kStepKeys / 64], mx = -INFINITY;
@@ -560,16 +638,18 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
       for (int j0 = my_vg; j0 < n; j0 += KU * v_groups) {
         if (j0 != my_vg) {
 #pragma unroll
-          for (int u = 0; u < KU; ++u) load_row(rows + a.d, j0 + u * v_groups, v_in ? my_vp : 0, xv[u]);
+          for (int u = 0; u < KU; ++u) xv[u] = load_row(j0 + u * v_groups, n, a.d, vp, k0);
         }
 #pragma unroll
         for (int u = 0; u < KU; ++u) {
           const int j = j0 + u * v_groups;
+          float f[N];
+          floats(xv[u], vnew, vp, j, f);
 #pragma unroll
           for (int hh = 0; hh < QT; ++hh) {
             const float p = j < n ? sc[hh * kStepKeys + j] : 0.f;
 #pragma unroll
-            for (int i = 0; i < N; ++i) acc[hh][i] = __builtin_fmaf(p, xv[u][i], acc[hh][i]);
+            for (int i = 0; i < N; ++i) acc[hh][i] = j < n ? __builtin_fmaf(p, f[i], acc[hh][i]) : acc[hh][i];
           }
         }
       }
@@ -605,27 +685,44 @@ template <typename T, bool VEC> void launch_window_step(const WindowArgs& a, hip
   int vp2 = 1;
   while (vp2 * N < a.dv) vp2 <<= 1;
   const int parts = vp2 < 64 ? kStepThreads / 64 : kStepThreads / vp2;
-  auto bytes = [&](int qt) { return (size_t)qt * (a.d + kStepKeys + 3 + parts * vp2 * N) * sizeof(float); };
+  auto part_floats = [&](int qt) { return qt * parts * vp2 * N; };
+  auto bytes = [&](int qt) { return (size_t)(qt * (a.d + kStepKeys + 3) + part_floats(qt) + a.d + a.dv) * sizeof(float); };
   if (qpk == 1)
-    hipLaunchKernelGGL((window_step_kernel<T, 1, VEC>), grid, block, bytes(1), s, a);
+    hipLaunchKernelGGL((window_step_kernel<T, 1, VEC>), grid, block, bytes(1), s, a, part_floats(1));
   else if (qpk == 2)
-    hipLaunchKernelGGL((window_step_kernel<T, 2, VEC>), grid, block, bytes(2), s, a);
+    hipLaunchKernelGGL((window_step_kernel<T, 2, VEC>), grid, block, bytes(2), s, a, part_floats(2));
   else if (qpk <= 4 || bytes(8) > 64 * 1024)
-    hipLaunchKernelGGL((window_step_kernel<T, 4, VEC>), grid, block, bytes(4), s, a);
+    hipLaunchKernelGGL((window_step_kernel<T, 4, VEC>), grid, block, bytes(4), s, a, part_floats(4));
   else
-    hipLaunchKernelGGL((window_step_kernel<T, 8, VEC>), grid, block, bytes(8), s, a);
+    hipLaunchKernelGGL((window_step_kernel<T, 8, VEC>), grid, block, bytes(8), s, a, part_floats(8));
+}
+
+template <int LPI> void launch_kv_write(const WindowArgs& a, hipStream_t s) {
+  const long items = (long)a.B * a.L * a.G;
+  const dim3 grid((unsigned)((items + 256 / LPI - 1) / (256 / LPI)));
+  if (a.half_split)
+    hipLaunchKernelGGL((window_kv_write_vec_kernel<LPI, true>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((window_kv_write_vec_kernel<LPI, false>), grid, dim3(256), 0, s, a);
+}
+
+template <int KC, int VC> void launch_window_mfma_pairs(const WindowArgs& a, dim3 grid, hipStream_t s) {
+  if (a.half_split)
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, VC, true>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, VC, false>), grid, dim3(256), 0, s, a);
 }
 
 template <int KC> void launch_window_mfma(const WindowArgs& a, dim3 grid, hipStream_t s) {
   const int vc = (a.dv + 31) / 32;
   if (vc <= 1)
-    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 1>), grid, dim3(256), 0, s, a);
+    launch_window_mfma_pairs<KC, 1>(a, grid, s);
   else if (vc <= 2)
-    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 2>), grid, dim3(256), 0, s, a);
+    launch_window_mfma_pairs<KC, 2>(a, grid, s);
   else if (vc <= 4)
-    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 4>), grid, dim3(256), 0, s, a);
+    launch_window_mfma_pairs<KC, 4>(a, grid, s);
   else
-    hipLaunchKernelGGL((window_prefill_mfma_kernel<KC, 8>), grid, dim3(256), 0, s, a);
+    launch_window_mfma_pairs<KC, 8>(a, grid, s);
 }
 
 static int window_check(const char* who, const WindowArgs& a, int64_t n_rope, int io_dtype, int64_t last) {
@@ -668,12 +765,14 @@ extern "C" BASED_API int based_window_attn_prefill(
   BASED_REQUIRE(B * G < 65536 && B < 65536 && H < 65536, BASED_ERR_SHAPE, "window_attn_prefill: grid too large");
   if (B == 0 || L == 0) return BASED_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const bool vec = io_dtype == BASED_BF16 && D <= 256 && DV <= 256 && window_vec(a, 8);
+  // pieces of 8 channels are turned whole: the rotary size is a multiple of 8 (16 in half-split pairs)
+  const bool vec = io_dtype == BASED_BF16 && D <= 256 && DV <= 256 && rotary_dim % (half_split ? 16 : 8) == 0 && window_vec(a, 8);
   const int64_t items = B * L * G;
-  BASED_REQUIRE((items + 3) / 4 < (1ll << 31), BASED_ERR_SHAPE, "window_attn_prefill: grid too large");
-  if (vec && !half_split)
-    hipLaunchKernelGGL(window_kv_write_vec_kernel, dim3((unsigned)((items + 15) / 16)), dim3(256), 0, s, a);
-  else if (io_dtype == BASED_BF16)
+  BASED_REQUIRE(items < (1ll << 32), BASED_ERR_SHAPE, "window_attn_prefill: grid too large");
+  if (vec) {
+    const int64_t widest = D > DV ? D : DV;
+    widest <= 64 ? launch_kv_write<8>(a, s) : widest <= 128 ? launch_kv_write<16>(a, s) : launch_kv_write<32>(a, s);
+  } else if (io_dtype == BASED_BF16)
     hipLaunchKernelGGL(window_kv_write_kernel<__bf16>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
   else
     hipLaunchKernelGGL(window_kv_write_kernel<float>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
