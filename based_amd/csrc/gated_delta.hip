@@ -246,21 +246,27 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
       fq[p] = pr[kPrepFq + t];
     }
   };
-  auto stage = [&](int buf) {
+  auto stage_rows = [&](int buf, int d) {
 #pragma unroll
     for (int p = 0; p < PP; ++p) {
       const int piece = p * 256 + tid, t = piece & 15, e = (piece >> 4) * 8;
       if (PIECES % 256 == 0 || piece < PIECES) {
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
-          const f32x4 y = rk[p][j].get(e + 4 * j, a.d) * fk[p];
+          const f32x4 y = rk[p][j].get(e + 4 * j, d) * fk[p];
           *reinterpret_cast<f32x4*>(&s_k[buf][t * KS + e + 4 * j]) = y;
-          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j].get(e + 4 * j, a.d) * fq[p];
+          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j].get(e + 4 * j, d) * fq[p];
 #pragma unroll
           for (int i = 0; i < 4; ++i) s_kt[buf][(e + 4 * j + i) * TS + t] = y[i];
         }
       }
     }
+  };
+  auto stage = [&](int buf) {
+    if (a.d == D)
+      stage_rows(buf, 1 << 30);  // nothing to clear
+    else
+      stage_rows(buf, a.d);
   };
   const int last_blk = a.blocks - 1;
 
@@ -278,7 +284,10 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
     stage(buf ^ 1);  // the next block (past the end: the last one again, unused)
     fetch_qk(blk + 2 < last_blk ? blk + 2 : last_blk);
     fetch(blk + 1 < last_blk ? blk + 1 : last_blk);
-    f32x4 ks = {0.f, 0.f, 0.f, 0.f}, qs = ks;
+    // two sums each for keys and queries: a product that waits for the one before it leaves the pipe idle
+    f32x4 kq[2][2];
+#pragma unroll
+    for (int j = 0; j < 2; ++j) kq[0][j] = kq[1][j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int r = 0; r < RBW; ++r) {
       const int e = (rs * RBW + r) * 16 + quad * 4;
@@ -286,10 +295,11 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
       const f32x4 qf = *reinterpret_cast<const f32x4*>(&s_q[buf][l16 * KS + e]);
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        ks = mfma_f32(kf[i], S[r][i], ks);
-        qs = mfma_f32(qf[i], S[r][i], qs);
+        kq[0][i & 1] = mfma_f32(kf[i], S[r][i], kq[0][i & 1]);
+        kq[1][i & 1] = mfma_f32(qf[i], S[r][i], kq[1][i & 1]);
       }
     }
+    f32x4 ks = kq[0][0] + kq[0][1], qs = kq[1][0] + kq[1][1];
     if constexpr (RS > 1) {
       f32x4* part = reinterpret_cast<f32x4*>(s_part) + ct * RS * 2 * 64;
       part[(rs * 2 + 0) * 64 + lane] = ks;
@@ -303,27 +313,31 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
         qs += part[(r * 2 + 1) * 64 + lane];
       }
     }
-    f32x4 u = {0.f, 0.f, 0.f, 0.f}, oo;
+    f32x4 kt[RBW];
+#pragma unroll
+    for (int r = 0; r < RBW; ++r) kt[r] = *reinterpret_cast<const f32x4*>(&s_kt[buf][((rs * RBW + r) * 16 + l16) * TS + quad * 4]);
+    const f32x4 none = {0.f, 0.f, 0.f, 0.f};
     float r4[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) r4[i] = beta[i] * (vv[i] - gm[i] * ks[i]);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) u = mfma_f32(tm[i], r4[i], u);
-#pragma unroll
-    for (int i = 0; i < 4; ++i) oo[i] = gm[i] * qs[i];
+    f32x4 u = mfma_f32(tm[0], r4[0], none), u1 = mfma_f32(tm[1], r4[1], none);
+    u = mfma_f32(tm[2], r4[2], u), u1 = mfma_f32(tm[3], r4[3], u1);
 #pragma unroll
     for (int r = 0; r < RBW; ++r) S[r] *= last;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) oo = mfma_f32(pm[i], u[i], oo);
+    u += u1;
     float ut[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) ut[i] = u[i] * tail[i];
 #pragma unroll
-    for (int r = 0; r < RBW; ++r) {
-      const f32x4 kt = *reinterpret_cast<const f32x4*>(&s_kt[buf][((rs * RBW + r) * 16 + l16) * TS + quad * 4]);
+    for (int i = 0; i < 4; ++i)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) S[r] = mfma_f32(kt[i], ut[i], S[r]);
-    }
+      for (int r = 0; r < RBW; ++r) S[r] = mfma_f32(kt[r][i], ut[i], S[r]);
+    f32x4 oo = gm * qs;
+    f32x4 o1 = mfma_f32(pm[1], u[1], none);
+    oo = mfma_f32(pm[0], u[0], oo);
+    o1 = mfma_f32(pm[3], u[3], o1);
+    oo = mfma_f32(pm[2], u[2], oo);
+    oo += o1;
     if (rs == 0 && col_in) {
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
@@ -563,17 +577,17 @@ template <typename T, int RB, int RS> void launch_delta_scan_split(const DeltaAr
     hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, false>), grid, dim3(256), 0, s, a);
 }
 
-// Tiles are shared by as many wavefronts as it takes to give every compute unit a workgroup.
+// Tiles are shared by as many wavefronts as it takes for two per SIMD: one alone shows every wait.
 template <typename T, int RB> void launch_delta_scan(const DeltaArgs& a, hipStream_t s) {
   const long tiles = (long)a.B * a.H * ((a.dv + 15) / 16);
   if constexpr (RB % 4 == 0) {
-    if (tiles < 512) {
+    if (tiles < 1024) {
       launch_delta_scan_split<T, RB, 4>(a, s);
       return;
     }
   }
   if constexpr (RB % 2 == 0) {
-    if (tiles < 1024) {
+    if (tiles < 2048) {
       launch_delta_scan_split<T, RB, 2>(a, s);
       return;
     }

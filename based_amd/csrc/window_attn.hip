@@ -166,7 +166,7 @@ __device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) {
 }
 
 template <int KC, int VC, bool HALF>
-__global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowArgs a) {
+__global__ __launch_bounds__(256, KC <= 2 && VC <= 2 ? 3 : 1) void window_prefill_mfma_kernel(const WindowArgs a) {
   constexpr int D = KC * 32, DV = VC * 32;
   constexpr int KS = D + 8, VS = kTileKeys + 8;  // LDS row strides: 16-lane reads of 16 bytes meet every bank once
   __shared__ __attribute__((aligned(16))) __bf16 lds_k[kTileKeys * KS];
@@ -209,7 +209,7 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
 #pragma unroll
     for (int i = 0; i < 2 * VC; ++i) acc[t][i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run[2] = {-INFINITY, -INFINITY}, l_run[2] = {0.f, 0.f};
-  const float scale2 = a.scale * 1.4426950408889634f;  // scores in powers of two
+  const float scale2 = fabsf(a.scale) * 1.4426950408889634f;  // scores in powers of two; the sign is the queries'
 
   const int first_pos = a.pos_host + r0 / qpk, last_pos = a.pos_host + (r_end - 1) / qpk;
   const int lo = first_pos - a.window + 1 > 0 ? first_pos - a.window + 1 : 0;
@@ -222,23 +222,26 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
   u32x4 vbuf[VP][4];
   const u32x4 zero4 = {0u, 0u, 0u, 0u};
   // rows past the last key and channels past the sizes are fetched from valid places and cleared in `stage`
+  const int st32 = (int)a.kv_st;
   auto fetch = [&](int k0) {
+    const __bf16* tile = kv + (long)k0 * a.kv_st;
+    const int last = last_pos - k0;
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
-      const int p = i * 256 + tid, key = k0 + p / (D / 8), e = (p % (D / 8)) * 8;
-      kbuf[i] = *reinterpret_cast<const u32x4*>(kv + (long)(key <= last_pos ? key : last_pos) * a.kv_st + (e < a.d ? e : 0));
+      const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
+      kbuf[i] = *reinterpret_cast<const u32x4*>(tile + ((key <= last ? key : last) * st32 + (e < a.d ? e : 0)));
     }
 #pragma unroll
     for (int i = 0; i < VP; ++i) {
       const int p = i * 256 + tid, k4 = p & 15, e = (p >> 4) * 8;
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int key = k0 + k4 * 4 + r;
-        vbuf[i][r] = *reinterpret_cast<const u32x4*>(kv + (long)(key <= last_pos ? key : last_pos) * a.kv_st + a.d + (e < a.dv ? e : 0));
+        const int key = k4 * 4 + r;
+        vbuf[i][r] = *reinterpret_cast<const u32x4*>(tile + ((key <= last ? key : last) * st32 + a.d + (e < a.dv ? e : 0)));
       }
     }
   };
-  auto stage = [&](int k0) {
+  auto stage = [&]() {
 #pragma unroll
     for (int i = 0; i < KP; ++i) {
       const int p = i * 256 + tid, key = p / (D / 8), e = (p % (D / 8)) * 8;
@@ -284,6 +287,14 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
         }
     }
   }
+  if (a.scale < 0.f) {
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+      for (int c = 0; c < KC; ++c)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) qf[t][c][j] = -qf[t][c][j];
+  }
   if (D > a.d) {
 #pragma unroll
     for (int c = 0; c < KC; ++c)
@@ -296,9 +307,9 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
   }
   for (int k0 = lo; k0 <= last_pos; k0 += kTileKeys) {
     __syncthreads();  // every wavefront is done with the tile before
-    stage(k0);
+    stage();
     __syncthreads();
-    fetch(k0 + kTileKeys <= last_pos ? k0 + kTileKeys : last_pos);  // always, so that nothing is waited for at a branch
+    if (k0 + kTileKeys <= last_pos) fetch(k0 + kTileKeys);
 #pragma unroll
     for (int h = 0; h < 2; ++h) {
       // 32 keys at a time: does any row of this wavefront see one of them, does every row see all?
@@ -326,7 +337,7 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
         for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            float sc = s[t][kt][i] * scale2;
+            float sc = s[t][kt][i];
             if (!all) sc = (unsigned)(d0 - kt * 16 - i) < (unsigned)a.window ? sc : -INFINITY;
             s[t][kt][i] = sc;
             mx = fmaxf(mx, sc);
@@ -336,19 +347,19 @@ __global__ __launch_bounds__(256) void window_prefill_mfma_kernel(const WindowAr
         if (__any(mx > m_run[t])) {
           const float m_new = fmaxf(m_run[t], mx);
           // no key seen yet: every weight is 2^-inf = 0
-          const float alpha = __builtin_amdgcn_exp2f(m_run[t] - (m_new == -INFINITY ? 0.f : m_new));
+          const float alpha = __builtin_amdgcn_exp2f((m_run[t] - (m_new == -INFINITY ? 0.f : m_new)) * scale2);
           m_run[t] = m_new;
           l_run[t] *= alpha;
 #pragma unroll
           for (int i = 0; i < 2 * VC; ++i) acc[t][i] *= alpha;
         }
-        const float m_use = m_run[t] == -INFINITY ? 0.f : m_run[t];
+        const float m2 = m_run[t] == -INFINITY ? 0.f : m_run[t] * scale2;
         float sum = 0.f;
 #pragma unroll
         for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
-            const float p = __builtin_amdgcn_exp2f(s[t][kt][i] - m_use);
+            const float p = __builtin_amdgcn_exp2f(__builtin_fmaf(s[t][kt][i], scale2, -m2));
             sum += p;
             pf[t][kt * 4 + i] = (__bf16)p;
           }
@@ -678,6 +689,245 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   }
 }
 
+// The same for bf16 rows of whole 16-byte pieces: queries, the new key and the new value are turned and
+// normalised in the registers of the lanes that use them, the new token starts the running softmax, and the
+// cached keys before it follow, so that everything the launch reads is asked for at its start and a window
+// of w needs w - 1 rows.  Products of queries and keys are dot-product instructions on bf16 pairs.
+template <int QT, bool HALF>
+__global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const WindowArgs a) {
+  constexpr int N = 8, KU = 4;
+  extern __shared__ float smem[];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const int b = blockIdx.x / a.G, g = blockIdx.x % a.G;
+  const int qpk = a.H / a.G;
+  const int pos = row_pos(a.pos, a.pos_host, b);
+  if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;  // a position the cache does not hold
+  float* sc = smem;                   // [QT][kStepKeys]
+  float* stat = sc + QT * kStepKeys;  // [3][QT]: running maximum, running sum, rescale of this round
+  float* part = stat + 3 * QT;        // [QT][parts][vp2 * 8], partial outputs
+  const __bf16* k = static_cast<const __bf16*>(a.k) + b * a.k_sb + (long)g * a.d;
+  const __bf16* v = static_cast<const __bf16*>(a.v) + b * a.v_sb + (long)g * a.dv;
+  __bf16* kv = static_cast<__bf16*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
+  const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
+  const int old = pos - lo;  // cached keys this token sees
+  int lpk = 1;
+  while (lpk * N < a.d) lpk <<= 1;
+  const int keys_at_once = kStepThreads / lpk, my_key = tid / lpk, my_piece = tid % lpk;
+  int vp2 = 1;
+  while (vp2 * N < a.dv) vp2 <<= 1;
+  const int v_groups = kStepThreads / vp2, my_vp = tid % vp2, my_vg = tid / vp2;
+  const int parts = kStepThreads / 64;
+  const bool k_in = my_piece * N < a.d, v_in = my_vp * N < a.dv;
+  const int ke = k_in ? my_piece * N : 0, ve = v_in ? my_vp * N : 0;
+  const int st32 = (int)a.kv_st;
+  auto row = [&](int k0, int j, int n) { return kv + (long)k0 * a.kv_st + (n > 0 ? (j < n ? j : n - 1) : 0) * st32; };
+
+  const int n_first = old < kStepKeys ? old : kStepKeys;
+  bf16x8 xk[KU], xv[KU], qraw[QT];
+#pragma unroll
+  for (int u = 0; u < KU; ++u) xk[u] = *reinterpret_cast<const bf16x8*>(row(lo, u * keys_at_once + my_key, n_first) + ke);
+#pragma unroll
+  for (int u = 0; u < KU; ++u) xv[u] = *reinterpret_cast<const bf16x8*>(row(lo, u * v_groups + my_vg, n_first) + a.d + ve);
+  const bf16x8 knew_raw = *reinterpret_cast<const bf16x8*>(k + ke), vnew_raw = *reinterpret_cast<const bf16x8*>(v + ve);
+  Turn8<HALF> turn;
+  turn.load(k, ke, pos, a);
+
+  // the new value: normalised by the lanes that share the row
+  float vn[N];
+  {
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      vn[i] = v_in ? to_f32(vnew_raw[i]) : 0.f;
+      ss = __builtin_fmaf(vn[i], vn[i], ss);
+    }
+    for (int m = 1; m < vp2; m <<= 1) ss += __shfl_xor(ss, m, 64);
+    const float r = a.norm_v ? 1.0f / sqrtf(ss / (float)a.dv + a.eps) : 1.0f;
+    bf16x8 o;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      o[i] = (__bf16)(vn[i] * r);
+      vn[i] = to_f32(o[i]);
+    }
+    if (my_vg == 0 && v_in) *reinterpret_cast<bf16x8*>(kv + (long)pos * a.kv_st + a.d + ve) = o;
+  }
+  typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
+  auto turned = [&](bf16x8 raw, const Turn8<HALF>& t) -> u32x4 {
+    float x[N];
+#pragma unroll
+    for (int i = 0; i < N; ++i) x[i] = to_f32(raw[i]);
+    t.apply(x, ke, a);
+    bf16x8 y;
+#pragma unroll
+    for (int i = 0; i < N; ++i) y[i] = (__bf16)(k_in ? x[i] : 0.f);
+    return __builtin_bit_cast(u32x4, y);
+  };
+  const u32x4 knew = turned(knew_raw, turn);
+  if (my_key == 0 && k_in) *reinterpret_cast<u32x4*>(kv + (long)pos * a.kv_st + ke) = knew;
+  auto dot8 = [](u32x4 x, u32x4 y) {
+    float s = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const uint32_t xi = x[i], yi = y[i];  // (a bit cast of a vector's element as such takes element 0)
+      s = __builtin_amdgcn_fdot2_f32_bf16(__builtin_bit_cast(bf16x2, xi), __builtin_bit_cast(bf16x2, yi), s, false);
+    }
+    return s;
+  };
+  auto over_pieces = [&](float x) {
+    if (lpk == 8) return sum8(x);
+    if (lpk == 16) return sum16(x);
+    for (int m = 1; m < lpk; m <<= 1) x += __shfl_xor(x, m, 64);
+    return x;
+  };
+
+  for (int h0 = 0; h0 < qpk; h0 += QT) {
+    if (h0 > 0) __syncthreads();  // the round before is done with LDS
+    u32x4 q[QT];
+    Turn8<HALF> tq = turn;
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)(g * qpk + (h0 + hh < qpk ? h0 + hh : h0)) * a.d;
+      qraw[hh] = *reinterpret_cast<const bf16x8*>(qp + ke);
+    }
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      if constexpr (HALF) {
+        const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)(g * qpk + (h0 + hh < qpk ? h0 + hh : h0)) * a.d;
+        load_vec<__bf16, 8>(qp + (ke < a.rot ? (ke < a.rot / 2 ? ke + a.rot / 2 : ke - a.rot / 2) : 0), tq.partner);
+      }
+      q[hh] = turned(qraw[hh], tq);
+    }
+    // the new token: maximum = its score, weight 1
+    float s_new[QT], acc[QT][N];
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      s_new[hh] = over_pieces(dot8(knew, q[hh])) * a.scale;
+#pragma unroll
+      for (int i = 0; i < N; ++i) acc[hh][i] = my_vg == 0 ? vn[i] : 0.f;
+      if (tid == 0) {
+        stat[hh] = s_new[hh];
+        stat[QT + hh] = 1.f;
+      }
+    }
+    for (int k0 = lo; k0 < pos; k0 += kStepKeys) {
+      const int n = pos - k0 < kStepKeys ? pos - k0 : kStepKeys;
+      const bool first = h0 == 0 && k0 == lo;
+      if (k0 > lo) __syncthreads();
+      for (int j0 = 0; j0 < n; j0 += KU * keys_at_once) {
+        if (!first || j0 > 0) {
+#pragma unroll
+          for (int u = 0; u < KU; ++u) xk[u] = *reinterpret_cast<const bf16x8*>(row(k0, j0 + u * keys_at_once + my_key, n) + ke);
+        }
+#pragma unroll
+        for (int u = 0; u < KU; ++u) {
+          const int j = j0 + u * keys_at_once + my_key;
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh) {
+            const float s = over_pieces(dot8(__builtin_bit_cast(u32x4, xk[u]), q[hh]));
+            if (my_piece == 0 && j < n) sc[hh * kStepKeys + j] = s * a.scale;
+          }
+        }
+      }
+      if (!first) {
+        // the first value rows are on their way during the softmax
+#pragma unroll
+        for (int u = 0; u < KU; ++u) xv[u] = *reinterpret_cast<const bf16x8*>(row(k0, u * v_groups + my_vg, n) + a.d + ve);
+      }
+      __syncthreads();
+      for (int hh = wave; hh < QT; hh += kStepThreads / 64) {
+        float s[kStepKeys / 64], mx = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < kStepKeys / 64; ++i) {
+          const int j = i * 64 + lane;
+          const float x = sc[hh * kStepKeys + j];
+          s[i] = j < n ? x : -INFINITY;
+          mx = fmaxf(mx, s[i]);
+        }
+#pragma unroll
+        for (int m = 32; m >= 1; m >>= 1) mx = fmaxf(mx, __shfl_xor(mx, m, 64));
+        const float m_old = stat[hh], m_new = fmaxf(m_old, mx);
+        float sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < kStepKeys / 64; ++i) {
+          const float p = exp_f(s[i] - m_new);
+          sc[hh * kStepKeys + i * 64 + lane] = p;
+          sum += p;
+        }
+        sum = wave_sum(sum);
+        const float alpha = exp_f(m_old - m_new);
+        if (lane == 0) {
+          stat[hh] = m_new;
+          stat[QT + hh] = stat[QT + hh] * alpha + sum;
+          stat[2 * QT + hh] = alpha;
+        }
+      }
+      __syncthreads();
+#pragma unroll
+      for (int hh = 0; hh < QT; ++hh) {
+        const float alpha = stat[2 * QT + hh];
+#pragma unroll
+        for (int i = 0; i < N; ++i) acc[hh][i] *= alpha;
+      }
+      for (int j0 = my_vg; j0 < n; j0 += KU * v_groups) {
+        if (j0 != my_vg) {
+#pragma unroll
+          for (int u = 0; u < KU; ++u) xv[u] = *reinterpret_cast<const bf16x8*>(row(k0, j0 + u * v_groups, n) + a.d + ve);
+        }
+#pragma unroll
+        for (int u = 0; u < KU; ++u) {
+          const int j = j0 + u * v_groups;
+#pragma unroll
+          for (int hh = 0; hh < QT; ++hh) {
+            const float p = j < n ? sc[hh * kStepKeys + (j < n ? j : 0)] : 0.f;
+#pragma unroll
+            for (int i = 0; i < N; ++i) acc[hh][i] = __builtin_fmaf(p, to_f32(xv[u][i]), acc[hh][i]);
+          }
+        }
+      }
+    }
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      for (int m = vp2; m < 64; m <<= 1) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) acc[hh][i] += __shfl_xor(acc[hh][i], m, 64);
+      }
+      if (lane < vp2) {
+#pragma unroll
+        for (int i = 0; i < N; ++i) part[((hh * parts + wave) * vp2 + my_vp) * N + i] = acc[hh][i];
+      }
+    }
+    __syncthreads();
+#pragma unroll
+    for (int hh = 0; hh < QT; ++hh) {
+      if (h0 + hh < qpk) {
+        const float inv = a.out_scale / stat[QT + hh];
+        for (int c = tid; c < a.dv; c += kStepThreads) {
+          float s = 0.f;
+#pragma unroll
+          for (int p = 0; p < kStepThreads / 64; ++p) s += part[(hh * parts + p) * vp2 * N + c];
+          static_cast<__bf16*>(a.o)[b * a.o_sb + (long)(g * qpk + h0 + hh) * a.dv + c] = (__bf16)(s * inv);
+        }
+      }
+    }
+  }
+}
+
+template <bool HALF> void launch_window_step_vec(const WindowArgs& a, hipStream_t s) {
+  const int qpk = a.H / a.G;
+  const dim3 grid((unsigned)(a.B * a.G)), block(kStepThreads);
+  int vp2 = 1;
+  while (vp2 * 8 < a.dv) vp2 <<= 1;
+  auto bytes = [&](int qt) { return (size_t)qt * (kStepKeys + 3 + kStepThreads / 64 * vp2 * 8) * sizeof(float); };
+  if (qpk == 1)
+    hipLaunchKernelGGL((window_step_vec_kernel<1, HALF>), grid, block, bytes(1), s, a);
+  else if (qpk == 2)
+    hipLaunchKernelGGL((window_step_vec_kernel<2, HALF>), grid, block, bytes(2), s, a);
+  else if (qpk <= 4 || bytes(8) > 64 * 1024)
+    hipLaunchKernelGGL((window_step_vec_kernel<4, HALF>), grid, block, bytes(4), s, a);
+  else
+    hipLaunchKernelGGL((window_step_vec_kernel<8, HALF>), grid, block, bytes(8), s, a);
+}
+
 template <typename T, bool VEC> void launch_window_step(const WindowArgs& a, hipStream_t s) {
   const int qpk = a.H / a.G;
   const dim3 grid((unsigned)(a.B * a.G)), block(kStepThreads);
@@ -817,7 +1067,9 @@ extern "C" BASED_API int based_window_attn_step(
                 (long)DV, kStepThreads);
   if (B == 0) return BASED_OK;
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (io_dtype == BASED_BF16)
+  if (io_dtype == BASED_BF16 && vec && rotary_dim % (half_split ? 16 : 8) == 0)
+    half_split ? launch_window_step_vec<true>(a, s) : launch_window_step_vec<false>(a, s);
+  else if (io_dtype == BASED_BF16)
     vec ? launch_window_step<__bf16, true>(a, s) : launch_window_step<__bf16, false>(a, s);
   else
     vec ? launch_window_step<float, true>(a, s) : launch_window_step<float, false>(a, s);
