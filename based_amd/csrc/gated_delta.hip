@@ -34,8 +34,8 @@ namespace based {
 constexpr float kUnitEps = 1e-6f;
 constexpr int kBlk = 16;            // tokens per block
 // what gated_delta_prepare leaves per (sequence, head, block): T and P row-major, then 16 each of G_t,
-// G_16 / G_t, beta_t, the factor of q_t and of k_t
-constexpr int kPrepT = 0, kPrepP = 256, kPrepG = 512, kPrepTail = 528, kPrepBeta = 544, kPrepFq = 560, kPrepFk = 576;
+// nk_t G_16 / G_t, beta_t, nq_t G_t and nk_t G_t, with nq_t and nk_t what turns q_t and k_t into unit vectors
+constexpr int kPrepT = 0, kPrepP = 256, kPrepG = 512, kPrepTail = 528, kPrepBeta = 544, kPrepGq = 560, kPrepGk = 576;
 constexpr int kPrepFloats = BASED_DELTA_PREP_FLOATS;
 
 struct DeltaArgs {
@@ -64,12 +64,15 @@ __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) { return __
 
 // 4 consecutive channels of a row of d as they lie in memory.  Fetched without a condition (channels
 // past the end come from the row's start) and cleared where they are used: a load in a branch or
-// in front of a select is waited for on the spot.  VEC: whole groups, aligned.
-template <typename T, bool VEC> struct Four {
+// in front of a select is waited for on the spot.  LAY: 0 element by element, 1 whole aligned groups, 2 whole
+// groups of rows that fill the tile (nothing to clear).
+template <typename T, int LAY> struct Four {
   typedef __attribute__((ext_vector_type(4))) T t4;
   t4 r;
   __device__ __forceinline__ void load(const T* row, int e, int d) {
-    if constexpr (VEC) {
+    if constexpr (LAY == 2) {
+      r = *reinterpret_cast<const t4*>(row + e);
+    } else if constexpr (LAY == 1) {
       r = *reinterpret_cast<const t4*>(row + (e < d ? e : 0));
     } else {
 #pragma unroll
@@ -79,7 +82,7 @@ template <typename T, bool VEC> struct Four {
   __device__ __forceinline__ f32x4 get(int e, int d) const {
     f32x4 x;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) x[i] = e + i < d ? to_f32(r[i]) : 0.f;
+    for (int i = 0; i < 4; ++i) x[i] = LAY == 2 || e + i < d ? to_f32(r[i]) : 0.f;
     return x;
   }
 };
@@ -107,7 +110,7 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArg
   f32x4 kk = {0.f, 0.f, 0.f, 0.f}, qk = kk;
   float sq = 0.f, sk = 0.f;
   for (int e0 = 0; e0 < a.d; e0 += 64) {
-    Four<T, VEC> xr[4], yr[4];
+    Four<T, VEC ? 1 : 0> xr[4], yr[4];
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
       xr[j].load(q, e0 + j * 16 + quad * 4, a.d);
@@ -150,11 +153,12 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArg
     if (live) out[kPrepP + t * kBlk + l16] = qk[i] * fq_t * fk * ratio;
   }
   if (live && quad == 0) {
-    out[kPrepG + l16] = expf((float)lc);
-    out[kPrepTail + l16] = expf(fminf((float)(lc_end - lc), 0.f));
+    const float G = expf((float)lc);
+    out[kPrepG + l16] = G;
+    out[kPrepTail + l16] = fk * expf(fminf((float)(lc_end - lc), 0.f));
     out[kPrepBeta + l16] = beta;
-    out[kPrepFq + l16] = fq;
-    out[kPrepFk + l16] = fk;
+    out[kPrepGq + l16] = fq * G;
+    out[kPrepGk + l16] = fk * G;
   }
   __syncthreads();
   // column l16 of T: x_t = [t = l16] - sum_{s<t} A_ts x_s
@@ -179,132 +183,117 @@ __global__ __launch_bounds__(256) void gated_delta_prepare_kernel(const DeltaArg
 
 // RB: 16-row blocks of the state; RS: wavefronts that share a 16-column tile, RB / RS row blocks each
 // (their partial products with the state are added up through LDS).  Four wavefronts per workgroup.
-template <typename T, int RB, int RS, bool VEC>
+// Queries and keys go from memory into the operands as they are: the factors that make unit vectors of
+// them are factors of rows of the products, and have been multiplied into the decays.
+template <typename T, int RB, int RS, int LAY>
 __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a) {
   static_assert(RB % RS == 0 && 4 % RS == 0, "row blocks divide among the wavefronts of a tile");
-  constexpr int D = RB * 16, CT = 4 / RS, RBW = RB / RS;
-  constexpr int KS = D + 4, TS = kBlk + 4;           // LDS row strides in floats: 16 lanes of 16 bytes meet every bank once
-  constexpr int PIECES = kBlk * (D / 8);             // 8 channels of a token, of q and of k
-  constexpr int PP = (PIECES + 255) / 256;           // per thread
-  __shared__ __attribute__((aligned(16))) float s_k[2][kBlk * KS], s_q[2][kBlk * KS], s_kt[2][D * TS];
-  __shared__ __attribute__((aligned(16))) float s_part[RS > 1 ? CT * RS * 2 * 256 : 4];
-  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
-  const int ct = wave / RS, rs = wave % RS;
-  const int b = blockIdx.x / a.H, h = blockIdx.x % a.H, hk = h / (a.H / a.G);
+  constexpr int CT = 4 / RS, RBW = RB / RS;
+  __shared__ __attribute__((aligned(16))) f32x4 s_part[2][RS > 1 ? CT * RS * 2 * 64 : 1];
+  const int tid = threadIdx.x, lane = tid & 63, l16 = lane & 15, quad = lane >> 4;
+  const int wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+  const int ct = wave / RS, rs = wave % RS, row0 = rs * RBW * 16;
+  // (the quotients are formed in vector registers: brought back so that every base address is a scalar)
+  const int b = __builtin_amdgcn_readfirstlane(blockIdx.x / a.H), h = blockIdx.x - b * a.H;
+  const int hk = __builtin_amdgcn_readfirstlane(h / (a.H / a.G));
   const int col = (blockIdx.y * CT + ct) * 16 + l16;
   const bool col_in = col < a.dv;
+  const int vcol = col_in ? col : 0;
   const T* q = static_cast<const T*>(a.q) + b * a.x_sb + (long)hk * a.d;
   const T* k = static_cast<const T*>(a.k) + b * a.x_sb + (long)hk * a.d;
-  const T* v = static_cast<const T*>(a.v) + b * a.x_sb + (long)h * a.dv + (col_in ? col : 0);
+  const T* v = static_cast<const T*>(a.v) + b * a.x_sb + (long)h * a.dv;
   const float* prep = a.prep + ((long)b * a.H + h) * a.blocks * kPrepFloats;
-  float* st = a.state + ((long)b * a.H + h) * a.d * a.dvp + (col_in ? col : 0);
-  float* o = a.o + ((long)b * a.L * a.H + h) * a.dv + (col_in ? col : 0);
+  float* st = a.state + ((long)b * a.H + h) * a.d * a.dvp + vcol;
+  float* o = a.o + ((long)b * a.L * a.H + h) * a.dv + vcol;
+  const int last_blk = (a.L - 1) / kBlk, x_sl = (int)a.x_sl, o_sl = a.H * a.dv;
 
   f32x4 S[RBW];
 #pragma unroll
   for (int r = 0; r < RBW; ++r)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int row = (rs * RBW + r) * 16 + quad * 4 + i;
+      const int row = row0 + r * 16 + quad * 4 + i;
       const bool in = !a.fresh && col_in && row < a.d;
       S[r][i] = in ? st[(long)row * a.dvp] : 0.f;
     }
 
-  // what a block needs from memory is asked for ahead of its use: q and k (which are laid out in LDS one
-  // block early) two blocks, the rest one block
-  Four<T, VEC> rk[PP][2], rq[PP][2];
-  float fk[PP], fq[PP];
-  f32x4 tn, pn, gn, tailn, betan;
-  T vn[4];
-  float lastn = 1.f;
-  auto fetch = [&](int blk) {
+  // What a block needs from memory, asked for two blocks ahead into two sets of registers that take turns.
+  struct Stage {
+    Four<T, LAY> k[RBW], q[RBW];
+    T kt[RBW][4], v[4];
+    f32x4 t, p, gk, gq, tail, beta;
+    float last;
+  };
+  auto fetch = [&](Stage& s, int blk) {
     const float* pr = prep + (long)blk * kPrepFloats;
-    tn = *reinterpret_cast<const f32x4*>(pr + kPrepT + l16 * kBlk + quad * 4);
-    pn = *reinterpret_cast<const f32x4*>(pr + kPrepP + l16 * kBlk + quad * 4);
-    gn = *reinterpret_cast<const f32x4*>(pr + kPrepG + quad * 4);
-    tailn = *reinterpret_cast<const f32x4*>(pr + kPrepTail + quad * 4);
-    betan = *reinterpret_cast<const f32x4*>(pr + kPrepBeta + quad * 4);
-    lastn = pr[kPrepG + kBlk - 1];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-      const int t = blk * kBlk + quad * 4 + i;
-      vn[i] = v[(long)(t < a.L ? t : a.L - 1) * a.x_sl];
-    }
-  };
-  auto fetch_qk = [&](int blk) {
-    const float* pr = prep + (long)blk * kPrepFloats;
-#pragma unroll
-    for (int p = 0; p < PP; ++p) {
-      const int piece = p * 256 + tid, t = piece & 15, e = (piece >> 4) * 8;
-      const long row = blk * kBlk + t < a.L ? blk * kBlk + t : a.L - 1;
-#pragma unroll
-      for (int j = 0; j < 2; ++j) {
-        rk[p][j].load(k + row * a.x_sl, e + 4 * j, a.d);
-        rq[p][j].load(q + row * a.x_sl, e + 4 * j, a.d);
-      }
-      fk[p] = pr[kPrepFk + t];
-      fq[p] = pr[kPrepFq + t];
-    }
-  };
-  auto stage_rows = [&](int buf, int d) {
-#pragma unroll
-    for (int p = 0; p < PP; ++p) {
-      const int piece = p * 256 + tid, t = piece & 15, e = (piece >> 4) * 8;
-      if (PIECES % 256 == 0 || piece < PIECES) {
-#pragma unroll
-        for (int j = 0; j < 2; ++j) {
-          const f32x4 y = rk[p][j].get(e + 4 * j, d) * fk[p];
-          *reinterpret_cast<f32x4*>(&s_k[buf][t * KS + e + 4 * j]) = y;
-          *reinterpret_cast<f32x4*>(&s_q[buf][t * KS + e + 4 * j]) = rq[p][j].get(e + 4 * j, d) * fq[p];
-#pragma unroll
-          for (int i = 0; i < 4; ++i) s_kt[buf][(e + 4 * j + i) * TS + t] = y[i];
-        }
-      }
-    }
-  };
-  auto stage = [&](int buf) {
-    if (a.d == D)
-      stage_rows(buf, 1 << 30);  // nothing to clear
-    else
-      stage_rows(buf, a.d);
-  };
-  const int last_blk = a.blocks - 1;
-
-  fetch_qk(0);
-  fetch(0);
-  stage(0);
-  fetch_qk(0 < last_blk ? 1 : last_blk);
-  for (int blk = 0, buf = 0; blk < a.blocks; ++blk, buf ^= 1) {
-    __syncthreads();  // this block is laid out; everyone is done with the other buffer
-    const f32x4 tm = tn, pm = pn, gm = gn, tail = tailn, beta = betan;
-    const float last = lastn;
-    float vv[4];
-#pragma unroll
-    for (int i = 0; i < 4; ++i) vv[i] = to_f32(vn[i]);
-    stage(buf ^ 1);  // the next block (past the end: the last one again, unused)
-    fetch_qk(blk + 2 < last_blk ? blk + 2 : last_blk);
-    fetch(blk + 1 < last_blk ? blk + 1 : last_blk);
-    // two sums each for keys and queries: a product that waits for the one before it leaves the pipe idle
-    f32x4 kq[2][2];
-#pragma unroll
-    for (int j = 0; j < 2; ++j) kq[0][j] = kq[1][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    // rows past the last token are fetched from it, and a block that lies behind it from the block before
+    const int at = (blk < last_blk ? blk : last_blk) * kBlk, left = a.L - 1 - at;
+    const T* kb = k + (long)at * a.x_sl;
+    const T* qb = q + (long)at * a.x_sl;
+    const T* vb = v + (long)at * a.x_sl;
+    const unsigned mine = (unsigned)((l16 < left ? l16 : left) * x_sl);
 #pragma unroll
     for (int r = 0; r < RBW; ++r) {
-      const int e = (rs * RBW + r) * 16 + quad * 4;
-      const f32x4 kf = *reinterpret_cast<const f32x4*>(&s_k[buf][l16 * KS + e]);
-      const f32x4 qf = *reinterpret_cast<const f32x4*>(&s_q[buf][l16 * KS + e]);
+      s.k[r].load(kb + mine, row0 + r * 16 + quad * 4, a.d);
+      s.q[r].load(qb + mine, row0 + r * 16 + quad * 4, a.d);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = quad * 4 + i;
+      const unsigned off = (unsigned)((t < left ? t : left) * x_sl);
+#pragma unroll
+      for (int r = 0; r < RBW; ++r) {
+        const int row = row0 + r * 16 + l16;
+        s.kt[r][i] = kb[off + (unsigned)(LAY == 2 || row < a.d ? row : 0)];
+      }
+      s.v[i] = vb[off + (unsigned)vcol];
+    }
+    s.t = *reinterpret_cast<const f32x4*>(pr + kPrepT + l16 * kBlk + quad * 4);
+    s.p = *reinterpret_cast<const f32x4*>(pr + kPrepP + l16 * kBlk + quad * 4);
+    s.gk = *reinterpret_cast<const f32x4*>(pr + kPrepGk + quad * 4);
+    s.gq = *reinterpret_cast<const f32x4*>(pr + kPrepGq + quad * 4);
+    s.tail = *reinterpret_cast<const f32x4*>(pr + kPrepTail + quad * 4);
+    s.beta = *reinterpret_cast<const f32x4*>(pr + kPrepBeta + quad * 4);
+    s.last = pr[kPrepG + kBlk - 1];
+  };
+
+  const f32x4 none = {0.f, 0.f, 0.f, 0.f};
+  auto block = [&](Stage& s, int blk, int buf) {
+    f32x4 kf[RBW], qf[RBW], kt[RBW];
+#pragma unroll
+    for (int r = 0; r < RBW; ++r) {
+      kf[r] = s.k[r].get(row0 + r * 16 + quad * 4, a.d);
+      qf[r] = s.q[r].get(row0 + r * 16 + quad * 4, a.d);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) kt[r][i] = LAY == 2 || row0 + r * 16 + l16 < a.d ? to_f32(s.kt[r][i]) : 0.f;
+    }
+    // copies of their own: values that are used later in the block would otherwise stay in the registers the
+    // next load wants, and the load's result be moved (and waited for) at the end of the loop
+    f32x4 tm = s.t, pm = s.p, gk = s.gk, gq = s.gq, tail = s.tail, beta = s.beta;
+    float last = s.last;
+    asm volatile("" : "+v"(tm), "+v"(pm), "+v"(gk), "+v"(gq), "+v"(tail), "+v"(beta), "+v"(last));
+    float vv[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) vv[i] = to_f32(s.v[i]);
+    fetch(s, blk + 2 < a.blocks ? blk + 2 : a.blocks - 1);
+    // two sums each for keys and queries: a product that waits for the one before it leaves the pipe idle
+    f32x4 kq[2][2] = {{none, none}, {none, none}};
+#pragma unroll
+    for (int r = 0; r < RBW; ++r)
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        kq[0][i & 1] = mfma_f32(kf[i], S[r][i], kq[0][i & 1]);
-        kq[1][i & 1] = mfma_f32(qf[i], S[r][i], kq[1][i & 1]);
+        kq[0][i & 1] = mfma_f32(kf[r][i], S[r][i], kq[0][i & 1]);
+        kq[1][i & 1] = mfma_f32(qf[r][i], S[r][i], kq[1][i & 1]);
       }
-    }
     f32x4 ks = kq[0][0] + kq[0][1], qs = kq[1][0] + kq[1][1];
     if constexpr (RS > 1) {
-      f32x4* part = reinterpret_cast<f32x4*>(s_part) + ct * RS * 2 * 64;
+      f32x4* part = &s_part[buf][ct * RS * 2 * 64];
       part[(rs * 2 + 0) * 64 + lane] = ks;
       part[(rs * 2 + 1) * 64 + lane] = qs;
-      __syncthreads();
+      // the waves exchange data through LDS only: what is on its way from memory is not waited for
+      __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+      __builtin_amdgcn_s_barrier();
+      __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
       ks = part[lane];
       qs = part[64 + lane];
 #pragma unroll
@@ -313,13 +302,9 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
         qs += part[(r * 2 + 1) * 64 + lane];
       }
     }
-    f32x4 kt[RBW];
-#pragma unroll
-    for (int r = 0; r < RBW; ++r) kt[r] = *reinterpret_cast<const f32x4*>(&s_kt[buf][((rs * RBW + r) * 16 + l16) * TS + quad * 4]);
-    const f32x4 none = {0.f, 0.f, 0.f, 0.f};
     float r4[4];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) r4[i] = beta[i] * (vv[i] - gm[i] * ks[i]);
+    for (int i = 0; i < 4; ++i) r4[i] = beta[i] * (vv[i] - gk[i] * ks[i]);
     f32x4 u = mfma_f32(tm[0], r4[0], none), u1 = mfma_f32(tm[1], r4[1], none);
     u = mfma_f32(tm[2], r4[2], u), u1 = mfma_f32(tm[3], r4[3], u1);
 #pragma unroll
@@ -332,25 +317,38 @@ __global__ __launch_bounds__(256) void gated_delta_scan_kernel(const DeltaArgs a
     for (int i = 0; i < 4; ++i)
 #pragma unroll
       for (int r = 0; r < RBW; ++r) S[r] = mfma_f32(kt[r][i], ut[i], S[r]);
-    f32x4 oo = gm * qs;
+    f32x4 oo = gq * qs;
     f32x4 o1 = mfma_f32(pm[1], u[1], none);
     oo = mfma_f32(pm[0], u[0], oo);
     o1 = mfma_f32(pm[3], u[3], o1);
     oo = mfma_f32(pm[2], u[2], oo);
     oo += o1;
     if (rs == 0 && col_in) {
+      float* ob = o + (long)blk * kBlk * o_sl;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int t = blk * kBlk + quad * 4 + i;
-        if (t < a.L) o[(long)t * a.H * a.dv] = oo[i];
-      }
+      for (int i = 0; i < 4; ++i)
+        if (blk * kBlk + quad * 4 + i < a.L) ob[(quad * 4 + i) * o_sl] = oo[i];
     }
+  };
+
+  Stage s0, s1;
+  // (kept apart: the wait for a set counts the loads behind it, and takes the least favourable order of
+  // those in front of the loop and in it)
+  fetch(s0, 0);
+  __builtin_amdgcn_sched_barrier(0);
+  fetch(s1, 1);
+  __builtin_amdgcn_sched_barrier(0);
+  // The number of blocks is even (an empty one changes nothing): a way out between the two would make
+  // copies of the registers that are being loaded, and wait for them.
+  for (int blk = 0; blk < a.blocks; blk += 2) {
+    block(s0, blk, 0);
+    block(s1, blk + 1, 1);
   }
 #pragma unroll
   for (int r = 0; r < RBW; ++r)
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
-      const int row = (rs * RBW + r) * 16 + quad * 4 + i;
+      const int row = row0 + r * 16 + quad * 4 + i;
       if (col_in && row < a.d) st[(long)row * a.dvp] = S[r][i];
     }
 }
@@ -568,31 +566,40 @@ __global__ __launch_bounds__(NT) void gated_delta_step_kernel(const DeltaStepArg
     y[c] = from_f32<T>(so[c] * r * to_f32(static_cast<const T*>(a.norm_w)[c]) * silu_exact(to_f32(gate[c])) * a.scale);
 }
 
-template <typename T, int RB, int RS> void launch_delta_scan_split(const DeltaArgs& a, hipStream_t s) {
+template <typename T, int RB, int RS, int LAY> void launch_delta_scan_split(const DeltaArgs& a, hipStream_t s) {
   const int cols = 16 * (4 / RS);
   const dim3 grid((unsigned)(a.B * a.H), (unsigned)((a.dv + cols - 1) / cols));
-  if (a.vec)
-    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, true>), grid, dim3(256), 0, s, a);
-  else
-    hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, false>), grid, dim3(256), 0, s, a);
+  hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, LAY>), grid, dim3(256), 0, s, a);
 }
 
-// Tiles are shared by as many wavefronts as it takes for two per SIMD: one alone shows every wait.
-template <typename T, int RB> void launch_delta_scan(const DeltaArgs& a, hipStream_t s) {
+// Tiles are shared by as many wavefronts as it takes to give every SIMD one (and tall ones always, for their
+// registers).
+template <typename T, int RB, int LAY> void launch_delta_scan_lay(const DeltaArgs& a, hipStream_t s) {
   const long tiles = (long)a.B * a.H * ((a.dv + 15) / 16);
   if constexpr (RB % 4 == 0) {
-    if (tiles < 1024) {
-      launch_delta_scan_split<T, RB, 4>(a, s);
+    if (tiles < 512 || LAY == 0) {
+      launch_delta_scan_split<T, RB, 4, LAY>(a, s);
       return;
     }
   }
-  if constexpr (RB % 2 == 0) {
-    if (tiles < 2048) {
-      launch_delta_scan_split<T, RB, 2>(a, s);
-      return;
+  if constexpr (LAY != 0 || RB % 4 != 0) {
+    if constexpr (RB % 2 == 0) {
+      if (tiles < 1024 || RB > 8) {
+        launch_delta_scan_split<T, RB, 2, LAY>(a, s);
+        return;
+      }
     }
+    if constexpr (RB <= 8) launch_delta_scan_split<T, RB, 1, LAY>(a, s);
   }
-  launch_delta_scan_split<T, RB, 1>(a, s);
+}
+
+template <typename T, int RB> void launch_delta_scan(const DeltaArgs& a, hipStream_t s) {
+  if (!a.vec)
+    launch_delta_scan_lay<T, RB, 0>(a, s);
+  else if (a.d < RB * 16)
+    launch_delta_scan_lay<T, RB, 1>(a, s);
+  else
+    launch_delta_scan_lay<T, RB, 2>(a, s);
 }
 
 template <typename T> void launch_delta(const DeltaArgs& a, hipStream_t s) {
@@ -661,8 +668,9 @@ extern "C" BASED_API int based_gated_delta_scan(const void* q, const void* k, co
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "gated_delta_scan: bad dtype");
   BASED_REQUIRE(B * H < (1ll << 31) && L < (1ll << 31) && DV < (1ll << 20), BASED_ERR_SHAPE, "gated_delta_scan: grid too large");
   if (B == 0 || L == 0) return BASED_OK;
-  const int64_t blocks = (L + kBlk - 1) / kBlk;
+  const int64_t blocks = 2 * ((L + 2 * kBlk - 1) / (2 * kBlk));
   BASED_REQUIRE(B * H * blocks < (1ll << 32), BASED_ERR_SHAPE, "gated_delta_scan: grid too large");
+  BASED_REQUIRE(x_sl < (1ll << 26) && H * DV < (1ll << 26), BASED_ERR_SHAPE, "gated_delta_scan: rows too long");
   BASED_REQUIRE(aligned_to(work, 16), BASED_ERR_ALIGN, "gated_delta_scan: the work space must be 16-byte aligned");
   // groups of four channels as one load
   const int vec = D % 4 == 0 && x_sb % 4 == 0 && x_sl % 4 == 0 && aligned_to(q, 16) && aligned_to(k, 16);

@@ -58,16 +58,7 @@ __device__ __forceinline__ void lru_gates(float zr, float zi, float sp, float u,
   const float r = sigmoid_f(zr), i = sigmoid_f(zi);
   const float log_a = -c * r * sp;
   a = exp_f(log_a);
-  x = __builtin_amdgcn_sqrtf(one_minus_exp(2.0f * log_a)) * i * u;
-}
-
-// (P, X) of this lane's tokens followed by those of the lane `CTRL` (a row_shl) brings: returns the product
-// of decays, updates x.  Lanes past the row's end bring nothing of use and are not used.
-template <int CTRL> __device__ __forceinline__ float then_later(float p, float& x) {
-  const float p2 = __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, p), CTRL, 0xf, 0xf, false));
-  const float x2 = __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, false));
-  x = __builtin_fmaf(p2, x, x2);
-  return p * p2;
+  x = __builtin_amdgcn_sqrtf(one_minus_square(a, log_a)) * i * u;
 }
 
 // grid: x = segment of the sequence, y = 64-channel tile within its block (ceil(n / 64) per block), z = sequence
@@ -77,8 +68,15 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
   constexpr int KT = 128 / (int)sizeof(T);             // contraction staged at a time
   constexpr int PAD = 16 / (int)sizeof(T);
   constexpr int KS = KT + PAD;
-  __shared__ __attribute__((aligned(16))) T s_u[64 * KS], s_r[64 * KS], s_i[64 * KS];
-  __shared__ float s_agg[2][4][64];  // (P, X) of each wavefront's 16 tokens
+  constexpr int SPAD = 4;
+  // the operands, and after them the decays and inputs of the tile
+  constexpr int kOperands = 3 * 64 * KS * (int)sizeof(T), kTile = 2 * 64 * (64 + SPAD) * 4;
+  __shared__ __attribute__((aligned(16))) char s_mem[kOperands > kTile ? kOperands : kTile];
+  T* s_u = reinterpret_cast<T*>(s_mem);
+  T* s_r = s_u + 64 * KS;
+  T* s_i = s_r + 64 * KS;
+  float(*s_a)[64 + SPAD] = reinterpret_cast<float(*)[64 + SPAD]>(s_mem);  // [token][channel]
+  float(*s_x)[64 + SPAD] = s_a + 64;
   __shared__ float s_const[3][64];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
   const int tiles = (a.n + 63) / 64;
@@ -152,68 +150,43 @@ __global__ __launch_bounds__(256) void rglru_gates_kernel(const RglruArgs a) {
       }
     }
   }
+  __syncthreads();  // the operands are done with
   // lane: token wave*16 + l16, channels i*16 + quad*4 ..
   const int tl = wave * 16 + l16, tok = l0 + tl;
   const bool tok_in = tok < a.L;
-  const int nch = a.n - c0 < 64 ? a.n - c0 : 64;
-  const T* ur = u + (long)(tok_in ? tok : a.L - 1) * a.u_sl + c0;
-  float uv[4][4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i)
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      const int ch = i * 16 + quad * 4 + j;
-      uv[i][j] = to_f32(ur[ch < nch ? ch : 0]);
-    }
-  const long base = ((long)b * a.L + (tok_in ? tok : 0)) * a.W + (long)blk * a.n + c0;
-  const bool rows16 = a.n % 4 == 0;  // four channels of a row lie together and aligned
 #pragma unroll
   for (int i = 0; i < 4; ++i) {
     const int ch = i * 16 + quad * 4;
-    f32x4 P, X;
+    f32x4 ov, xv;
 #pragma unroll
     for (int j = 0; j < 4; ++j) {
+      const int cc = c0 + ch + j < a.n ? c0 + ch + j : a.n - 1;
+      const float uv = to_f32(u[(tok_in ? tok : a.L - 1) * a.u_sl + cc]);
       float av, x;
-      lru_gates(zr[i][j] + s_const[0][ch + j], zi[i][j] + s_const[1][ch + j], s_const[2][ch + j], uv[i][j], a.c, av, x);
-      P[j] = av, X[j] = x;
+      lru_gates(zr[i][j] + s_const[0][ch + j], zi[i][j] + s_const[1][ch + j], s_const[2][ch + j], uv, a.c, av, x);
+      ov[j] = av, xv[j] = x;
     }
-    if (tok_in) {
-      if (rows16) {
-        if (ch < nch) {
-          *reinterpret_cast<f32x4*>(a.ga + base + ch) = P;
-          *reinterpret_cast<f32x4*>(a.gx + base + ch) = X;
-        }
-      } else {
-#pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (ch + j < nch) {
-            a.ga[base + ch + j] = P[j];
-            a.gx[base + ch + j] = X[j];
-          }
-      }
-    }
-    // what the 16 tokens do to a state that enters them, gathered in lane 0 of the row: token t first,
-    // then t + m
-#pragma unroll
-    for (int j = 0; j < 4; ++j) {
-      float p = tok_in ? P[j] : 1.f, x = tok_in ? X[j] : 0.f;
-      p = then_later<0x101>(p, x);  // row_shl:1
-      p = then_later<0x102>(p, x);
-      p = then_later<0x104>(p, x);
-      p = then_later<0x108>(p, x);
-      if (l16 == 0) {
-        s_agg[0][wave][ch + j] = p;
-        s_agg[1][wave][ch + j] = x;
-      }
-    }
+    *reinterpret_cast<f32x4*>(&s_a[tl][ch]) = ov;
+    *reinterpret_cast<f32x4*>(&s_x[tl][ch]) = xv;
   }
   __syncthreads();
+  // the tile in rows of 64 channels, and the segment's effect on a state that enters it
+  const int ntok = a.L - l0 < kSeg ? a.L - l0 : kSeg;
+  const int nch = a.n - c0 < 64 ? a.n - c0 : 64;
+  const long base = ((long)b * a.L + l0) * a.W + (long)blk * a.n + c0;
+  for (int p = tid; p < ntok * 64; p += 256) {
+    const int t = p >> 6, ch = p & 63;
+    if (ch < nch) {
+      a.ga[base + (long)t * a.W + ch] = s_a[t][ch];
+      a.gx[base + (long)t * a.W + ch] = s_x[t][ch];
+    }
+  }
   if (tid < nch) {
     float P = 1.f, X = 0.f;
-#pragma unroll
-    for (int k = 0; k < 4; ++k) {
-      X = __builtin_fmaf(s_agg[0][k][tid], X, s_agg[1][k][tid]);
-      P *= s_agg[0][k][tid];
+    for (int t = 0; t < ntok; ++t) {
+      const float av = s_a[t][tid];
+      P *= av;
+      X = __builtin_fmaf(av, X, s_x[t][tid]);
     }
     const int w = blk * a.n + c0 + tid;
     float* g = a.agg + ((long)b * (a.segs + 1) + seg + 1) * 2 * a.W + w;

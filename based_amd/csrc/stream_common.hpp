@@ -29,11 +29,12 @@ __device__ __forceinline__ float softplus_f(float z) { return log1pf(expf(-fabsf
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
-// 1 - exp(x) for x <= 0 without cancellation: the series below 1/4 (the next term is 5e-8 of the sum)
-__device__ __forceinline__ float one_minus_exp(float x) {
-  const float p = x * (1.f / 720.f) + 1.f / 120.f;
+// 1 - a^2 for a = exp(log_a) <= 1 without cancellation: the series of 1 - exp(x), x = 2 log_a, above -1/4 (the
+// next term is 5e-8 of the sum)
+__device__ __forceinline__ float one_minus_square(float a, float log_a) {
+  const float x = 2.0f * log_a, p = x * (1.f / 720.f) + 1.f / 120.f;
   const float series = -x * (1.f + x * (0.5f + x * (1.f / 6.f + x * (1.f / 24.f + x * p))));
-  return x > -0.25f ? series : 1.0f - exp_f(x);
+  return x > -0.25f ? series : __builtin_fmaf(-a, a, 1.0f);
 }
 // x as the element type would keep it
 template <typename T> __device__ __forceinline__ float round_to(float x) { return to_f32(from_f32<T>(x)); }

@@ -882,7 +882,7 @@ def gated_delta_scan(q, k, v, a_gate, b_gate, a_log, dt_bias, state, heads: int,
         raise ValueError(f"gates must be ({B}, {L}, {heads})")
     _check_delta(state, B, heads, d, dv)
     o = torch.empty(B, L, heads, dv, dtype=torch.float32, device=q.device)
-    work = torch.empty(B, heads, (L + DELTA_BLOCK - 1) // DELTA_BLOCK, DELTA_PREP_FLOATS, dtype=torch.float32, device=q.device)
+    work = torch.empty(B, heads, 2 * ((L + 2 * DELTA_BLOCK - 1) // (2 * DELTA_BLOCK)), DELTA_PREP_FLOATS, dtype=torch.float32, device=q.device)
     with _on_device(q.device):
         _lib.check(_lib.lib().based_gated_delta_scan(
             q.data_ptr(), k.data_ptr(), v.data_ptr(), a_gate.data_ptr(), b_gate.data_ptr(), a_log.data_ptr(), dt_bias.data_ptr(),

@@ -515,7 +515,7 @@ BASED_API int based_window_attn_step(const void* q, const void* k, const void* v
  * pair of strides for the three; a_gate, b_gate (B, L, H) projections; a_log, dt_bias (H).
  * g = exp(-exp(a_log) softplus(a + dt_bias)), beta = sigmoid(b); q and k made unit vectors, q times
  * D^(-1/2); S <- g S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q.
- * state (B, H, D, state_row) fp32, o (B, L, H, DV) fp32; work: B * H * ceil(L / 16) *
+ * state (B, H, D, state_row) fp32, o (B, L, H, DV) fp32; work: B * H * 2 ceil(L / 32) *
  * BASED_DELTA_PREP_FLOATS floats of scratch. */
 #define BASED_DELTA_PREP_FLOATS 592
 BASED_API int based_gated_delta_scan(const void* q, const void* k, const void* v, const void* a_gate, const void* b_gate,
