@@ -289,6 +289,16 @@ struct RglruStepArgs {
 
 constexpr int kLruRows = 8;  // sequences held at a time
 
+// a piece of a gate row: 16 bytes, or one element
+template <typename T, bool VEC> struct LruPiece {
+  typedef typename Pack<T>::type type;
+  static __device__ __forceinline__ float get(type x, int i) { return to_f32(x[i]); }
+};
+template <typename T> struct LruPiece<T, false> {
+  typedef T type;
+  static __device__ __forceinline__ float get(type x, int) { return to_f32(x); }
+};
+
 // A workgroup takes 32 output channels of one block (a wavefront 8 of them, 8 lanes per channel) and
 // up to kLruRows sequences; the convolved inputs of the whole block go through LDS.
 template <typename T, bool VEC>
@@ -300,40 +310,94 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) 
   const int blk = blockIdx.x / tiles, tile = blockIdx.x % tiles, m0 = blockIdx.y * kLruRows;
   const int rows = a.B - m0 < kLruRows ? a.B - m0 : kLruRows;
   const int ns = (a.n + 3) & ~3;  // rows of whole 16-byte pieces
-  for (int i = tid; i < kLruRows * a.n; i += 256) {
-    const int m = i / a.n, k = i % a.n, ch = blk * a.n + k;
-    float val = 0.f;
-    if (m < rows) {
-      const int b = m0 + m, pos = row_pos(a.pos, a.pos_host, b);
-      const T now = static_cast<const T*>(a.x)[b * a.x_sb + ch];
-      const T* cw = static_cast<const T*>(a.conv_w) + ch;
-      T* ring = static_cast<T*>(a.ring) + b * a.ring_sb + ch;
-      float acc = a.conv_b != nullptr ? to_f32(static_cast<const T*>(a.conv_b)[ch]) : 0.f;
-      acc += ring_dot<T>(ring, cw, a.W, a.taps, pos);
-      acc = __builtin_fmaf(to_f32(cw[(long)(a.taps - 1) * a.W]), to_f32(now), acc);
-      val = round_to<T>(acc);
-      // a slot that no reader of this step looks at; one tile of the block writes it
-      if (tile == 0 && pos >= 0) ring[(long)(pos % a.taps) * a.W] = now;
-    }
-    s_u[m * ns + k] = val;
-  }
-  __syncthreads();
   const int ch = tile * 32 + wave * 8 + (lane >> 3), part = lane & 7;
   const bool ok = ch < a.n;
   const int cc = ok ? ch : a.n - 1;
+  // What does not depend on a position is asked for first: the first pieces of the gate rows, and what the
+  // lane needs that finishes sequence m0 + part.
   const T* wr = static_cast<const T*>(a.ra) + ((long)blk * a.n + cc) * a.n;
   const T* wi = static_cast<const T*>(a.ri) + ((long)blk * a.n + cc) * a.n;
+  typedef typename LruPiece<T, VEC>::type piece_t;
+  piece_t pr[2], pi[2];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int k = (part + 8 * i) * N;
+    pr[i] = *reinterpret_cast<const piece_t*>(wr + (k < a.n ? k : 0));
+    pi[i] = *reinterpret_cast<const piece_t*>(wi + (k < a.n ? k : 0));
+  }
+  const int bp = m0 + (part < rows ? part : 0), wc = blk * a.n + cc;
+  const T rb = static_cast<const T*>(a.rb)[wc], ib = static_cast<const T*>(a.ib)[wc], lam = static_cast<const T*>(a.lam)[wc];
+  const T yv = static_cast<const T*>(a.y)[bp * a.y_sb + wc];
+  const float old = a.state[(long)bp * a.W + wc];
+  const int pos_p = row_pos(a.pos, a.pos_host, bp);
+
+  // the convolved inputs of the block: `share` threads per channel, each with every share-th sequence, four of
+  // them in flight together
+  const int share = a.n >= 256 ? 1 : 256 / a.n;
+  for (int k = tid % (256 / share); k < a.n; k += 256 / share) {
+    if (tid / (256 / share) >= share) break;
+    const int chn = blk * a.n + k;
+    const T* cw = static_cast<const T*>(a.conv_w) + chn;
+    const float bias = a.conv_b != nullptr ? to_f32(static_cast<const T*>(a.conv_b)[chn]) : 0.f;
+    for (int mb = tid / (256 / share); mb < rows; mb += 4 * share) {
+      int pos[4];
+      T now[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int m = mb + j * share < rows ? mb + j * share : rows - 1;
+        pos[j] = row_pos(a.pos, a.pos_host, m0 + m);
+        now[j] = static_cast<const T*>(a.x)[(m0 + m) * a.x_sb + chn];
+      }
+      float acc[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) acc[j] = bias;
+      for (int t0 = 0; t0 < a.taps - 1; t0 += 3) {
+        T xv[4][3], cv[3];
+#pragma unroll
+        for (int t = 0; t < 3; ++t) {
+          cv[t] = cw[(long)(t0 + t < a.taps - 1 ? t0 + t : 0) * a.W];
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int m = mb + j * share < rows ? mb + j * share : rows - 1;
+            const int p = pos[j] - (a.taps - 1) + t0 + t;
+            const bool in = t0 + t < a.taps - 1 && p >= 0;
+            xv[j][t] = static_cast<const T*>(a.ring)[(m0 + m) * a.ring_sb + (long)(in ? p % a.taps : 0) * a.W + chn];
+          }
+        }
+#pragma unroll
+        for (int t = 0; t < 3; ++t)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) {
+            const int p = pos[j] - (a.taps - 1) + t0 + t;
+            const bool in = t0 + t < a.taps - 1 && p >= 0;
+            acc[j] = in ? __builtin_fmaf(to_f32(cv[t]), to_f32(xv[j][t]), acc[j]) : acc[j];
+          }
+      }
+      const float c_last = to_f32(cw[(long)(a.taps - 1) * a.W]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        const int m = mb + j * share;
+        if (m < rows) {
+          s_u[m * ns + k] = round_to<T>(__builtin_fmaf(c_last, to_f32(now[j]), acc[j]));
+          // a slot that no reader of this step looks at; one tile of the block writes it
+          if (tile == 0 && pos[j] >= 0) static_cast<T*>(a.ring)[(m0 + m) * a.ring_sb + (long)(pos[j] % a.taps) * a.W + chn] = now[j];
+        }
+      }
+    }
+  }
+  for (int i = tid; i < (kLruRows - rows) * ns; i += 256) s_u[rows * ns + i] = 0.f;
+  __syncthreads();
   float zr[kLruRows], zi[kLruRows];
 #pragma unroll
   for (int m = 0; m < kLruRows; ++m) zr[m] = zi[m] = 0.f;
-#pragma unroll 2
-  for (int k = part * N; k < a.n; k += 8 * N) {
+  for (int k = part * N, it = 0; k < a.n; k += 8 * N, ++it) {
+    const piece_t rp = it == 0 ? pr[0] : it == 1 ? pr[1] : *reinterpret_cast<const piece_t*>(wr + k);
+    const piece_t ip = it == 0 ? pi[0] : it == 1 ? pi[1] : *reinterpret_cast<const piece_t*>(wi + k);
     float r[N], q[N];
-    if constexpr (VEC) {
-      load_vec<T, N>(wr + k, r);
-      load_vec<T, N>(wi + k, q);
-    } else {
-      r[0] = to_f32(wr[k]), q[0] = to_f32(wi[k]);
+#pragma unroll
+    for (int j = 0; j < N; ++j) {
+      r[j] = LruPiece<T, VEC>::get(rp, j);
+      q[j] = LruPiece<T, VEC>::get(ip, j);
     }
 #pragma unroll
     for (int m = 0; m < kLruRows; ++m) {
@@ -358,16 +422,11 @@ __global__ __launch_bounds__(256) void rglru_step_kernel(const RglruStepArgs a) 
   }
   // lane `part` finishes sequence m0 + part
   if (ok && part < rows) {
-    const int b = m0 + part, w = blk * a.n + ch;
-    const int pos = row_pos(a.pos, a.pos_host, b);
     float av, x;
-    lru_gates(my_r + to_f32(static_cast<const T*>(a.rb)[w]), my_i + to_f32(static_cast<const T*>(a.ib)[w]),
-              softplus_f(to_f32(static_cast<const T*>(a.lam)[w])), s_u[part * ns + ch], a.c, av, x);
-    float* sp = a.state + (long)b * a.W + w;
-    const float old = *sp;
-    const float S = pos > 0 ? __builtin_fmaf(av, old, x) : x;
-    *sp = S;
-    static_cast<T*>(a.out)[b * a.o_sb + w] = from_f32<T>(S * gelu_tanh_f(to_f32(static_cast<const T*>(a.y)[b * a.y_sb + w])));
+    lru_gates(my_r + to_f32(rb), my_i + to_f32(ib), softplus_f(to_f32(lam)), s_u[part * ns + ch], a.c, av, x);
+    const float S = pos_p > 0 ? __builtin_fmaf(av, old, x) : x;
+    a.state[(long)bp * a.W + wc] = S;
+    static_cast<T*>(a.out)[bp * a.o_sb + wc] = from_f32<T>(S * gelu_tanh_f(to_f32(yv)));
   }
 }
 

@@ -728,6 +728,9 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
   for (int u = 0; u < KU; ++u) xk[u] = *reinterpret_cast<const bf16x8*>(row(lo, u * keys_at_once + my_key, n_first) + ke);
 #pragma unroll
   for (int u = 0; u < KU; ++u) xv[u] = *reinterpret_cast<const bf16x8*>(row(lo, u * v_groups + my_vg, n_first) + a.d + ve);
+  auto q_row = [&](int hh) { return static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)(g * qpk + (hh < qpk ? hh : qpk - 1)) * a.d; };
+#pragma unroll
+  for (int hh = 0; hh < QT; ++hh) qraw[hh] = *reinterpret_cast<const bf16x8*>(q_row(hh) + ke);
   const bf16x8 knew_raw = *reinterpret_cast<const bf16x8*>(k + ke), vnew_raw = *reinterpret_cast<const bf16x8*>(v + ve);
   Turn8<HALF> turn;
   turn.load(k, ke, pos, a);
@@ -784,17 +787,14 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
     if (h0 > 0) __syncthreads();  // the round before is done with LDS
     u32x4 q[QT];
     Turn8<HALF> tq = turn;
+    if (h0 > 0) {
 #pragma unroll
-    for (int hh = 0; hh < QT; ++hh) {
-      const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)(g * qpk + (h0 + hh < qpk ? h0 + hh : h0)) * a.d;
-      qraw[hh] = *reinterpret_cast<const bf16x8*>(qp + ke);
+      for (int hh = 0; hh < QT; ++hh) qraw[hh] = *reinterpret_cast<const bf16x8*>(q_row(h0 + hh) + ke);
     }
 #pragma unroll
     for (int hh = 0; hh < QT; ++hh) {
-      if constexpr (HALF) {
-        const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)(g * qpk + (h0 + hh < qpk ? h0 + hh : h0)) * a.d;
-        load_vec<__bf16, 8>(qp + (ke < a.rot ? (ke < a.rot / 2 ? ke + a.rot / 2 : ke - a.rot / 2) : 0), tq.partner);
-      }
+      if constexpr (HALF)
+        load_vec<__bf16, 8>(q_row(h0 + hh) + (ke < a.rot ? (ke < a.rot / 2 ? ke + a.rot / 2 : ke - a.rot / 2) : 0), tq.partner);
       q[hh] = turned(qraw[hh], tq);
     }
     // the new token: maximum = its score, weight 1

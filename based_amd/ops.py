@@ -746,9 +746,11 @@ def _check_ring(ring, rows: int, taps: int, channels: int, like) -> None:
         raise ValueError(f"ring must be ({rows}, {taps}, {channels}) {like.dtype} with contiguous slots, got {tuple(ring.shape)} {ring.dtype}")
 
 
-def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: float = 1.0, want_residual: bool = True):
+def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: float = 1.0, want_residual: bool = True,
+             residual_out=None):
     """r = residual + mult * x in fp32 (r = x without a residual); y = norm(r) * weight in x's dtype.
-    x: (..., D); residual fp32 of the same shape or None.  Returns (y, r), r None if not wanted."""
+    x: (..., D); residual fp32 of the same shape or None.  Returns (y, r), r None if not wanted
+    (written into residual_out, fp32 with contiguous rows and not `residual`, when given)."""
     D = x.shape[-1]
     _require_cuda(x, weight)
     _check_same_dtype(x, weight)
@@ -767,10 +769,16 @@ def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: floa
             r2 = r2.contiguous()
     rows = x2.shape[0]
     y = torch.empty(rows, D, dtype=x.dtype, device=x.device)
-    out = torch.empty(rows, D, dtype=torch.float32, device=x.device) if want_residual else None
+    if residual_out is not None:
+        out = residual_out.view(rows, D)
+        if out.dtype != torch.float32 or out.stride(1) != 1 or out.device != x.device:
+            raise ValueError("residual_out must be float32 with contiguous rows on the device of x")
+    else:
+        out = torch.empty(rows, D, dtype=torch.float32, device=x.device) if want_residual else None
     with _on_device(x.device):
         _lib.check(_lib.lib().based_add_norm(x2.data_ptr(), _ptr(r2), weight.data_ptr(), y.data_ptr(), _ptr(out), rows, D,
-                                             x2.stride(0), 0 if r2 is None else r2.stride(0), D, D, float(eps), int(kind),
+                                             x2.stride(0), 0 if r2 is None else r2.stride(0), D, D if out is None else out.stride(0),
+                                             float(eps), int(kind),
                                              float(mult), _dtype_code(x), _stream_ptr(x)))
     return y.view(x.shape), None if out is None else out.view(x.shape)
 
@@ -985,6 +993,11 @@ def rglru_step(x, y, conv_weight, conv_bias, ring, ra, rb, ri, ib, lam, state, d
     return out
 
 
+# Rows up to which the streamed-input prologue is evaluated inside the projection.  Every workgroup of it
+# repeats the prologue for every row; beyond one register tile of rows that costs more than launches of its own.
+STREAM_PROLOGUE_MAX_ROWS = 8
+
+
 def _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult, norm_kind,
                           input_conv, out):
     """`decode_linear` behind PROLOGUE_STREAM."""
@@ -1014,6 +1027,12 @@ def _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, 
         _check_ring(ring, M, taps, K, x2)
         ring_stride = ring.stride(0)
         pos_ptr, pos_host = _pos_args(pos, M)
+    if M > STREAM_PROLOGUE_MAX_ROWS:
+        rows = x2 if row_index is None else x2.index_select(0, row_index)
+        h, _ = add_norm(rows, residual_in, norm_weight, eps, norm_kind, mult, residual_out is not None, residual_out)
+        if input_conv is not None:
+            h = stream_conv(h.unsqueeze(1), conv_w, None, ring, input_conv[2], add_input=True).squeeze(1)
+        return decode_linear(h, weight, bias, epilogue=epilogue, out=out)
     y = torch.empty(M, n_out, dtype=torch.bfloat16, device=x2.device) if out is None else out
     if tuple(y.shape) != (M, n_out) or y.dtype != torch.bfloat16 or y.stride(1) != 1:
         raise ValueError(f"out must be a ({M}, {n_out}) bfloat16 tensor with contiguous rows")
