@@ -572,17 +572,18 @@ template <typename T, int RB, int RS, int LAY> void launch_delta_scan_split(cons
   hipLaunchKernelGGL((gated_delta_scan_kernel<T, RB, RS, LAY>), grid, dim3(256), 0, s, a);
 }
 
-// Tiles are shared by as many wavefronts as it takes to give every SIMD one (and tall ones always, for their
-// registers).
+// Tiles are shared by as many wavefronts as it takes to give every SIMD one; tall ones always, for their
+// registers.
 template <typename T, int RB, int LAY> void launch_delta_scan_lay(const DeltaArgs& a, hipStream_t s) {
   const long tiles = (long)a.B * a.H * ((a.dv + 15) / 16);
-  if constexpr (RB % 4 == 0) {
-    if (tiles < 512 || LAY == 0) {
+  constexpr bool kFour = RB % 4 == 0, kOnlyFour = kFour && (LAY == 0 || (RB > 12 && sizeof(T) == 4));
+  if constexpr (kFour) {
+    if (tiles < 512 || kOnlyFour) {
       launch_delta_scan_split<T, RB, 4, LAY>(a, s);
       return;
     }
   }
-  if constexpr (LAY != 0 || RB % 4 != 0) {
+  if constexpr (!kOnlyFour) {
     if constexpr (RB % 2 == 0) {
       if (tiles < 1024 || RB > 8) {
         launch_delta_scan_split<T, RB, 2, LAY>(a, s);

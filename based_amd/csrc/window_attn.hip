@@ -693,7 +693,8 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
 // normalised in the registers of the lanes that use them, the new token starts the running softmax, and the
 // cached keys before it follow, so that everything the launch reads is asked for at its start and a window
 // of w needs w - 1 rows.  Products of queries and keys are dot-product instructions on bf16 pairs.
-template <int QT, bool HALF>
+// LPK, VP2: lanes per key row and per value row (powers of two), 0: whatever the sizes ask for.
+template <int QT, bool HALF, int LPK, int VP2>
 __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const WindowArgs a) {
   constexpr int N = 8, KU = 4;
   extern __shared__ float smem[];
@@ -710,11 +711,16 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
   __bf16* kv = static_cast<__bf16*>(a.kv) + b * a.kv_sb + (long)g * (a.d + a.dv);
   const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0;
   const int old = pos - lo;  // cached keys this token sees
-  int lpk = 1;
-  while (lpk * N < a.d) lpk <<= 1;
+  int lpk = LPK, vp2 = VP2;
+  if constexpr (LPK == 0) {
+    lpk = 1;
+    while (lpk * N < a.d) lpk <<= 1;
+  }
+  if constexpr (VP2 == 0) {
+    vp2 = 1;
+    while (vp2 * N < a.dv) vp2 <<= 1;
+  }
   const int keys_at_once = kStepThreads / lpk, my_key = tid / lpk, my_piece = tid % lpk;
-  int vp2 = 1;
-  while (vp2 * N < a.dv) vp2 <<= 1;
   const int v_groups = kStepThreads / vp2, my_vp = tid % vp2, my_vg = tid / vp2;
   const int parts = kStepThreads / 64;
   const bool k_in = my_piece * N < a.d, v_in = my_vp * N < a.dv;
@@ -744,7 +750,13 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
       vn[i] = v_in ? to_f32(vnew_raw[i]) : 0.f;
       ss = __builtin_fmaf(vn[i], vn[i], ss);
     }
-    for (int m = 1; m < vp2; m <<= 1) ss += __shfl_xor(ss, m, 64);
+    if constexpr (VP2 == 8) {
+      ss = sum8(ss);
+    } else if constexpr (VP2 == 16) {
+      ss = sum16(ss);
+    } else {
+      for (int m = 1; m < vp2; m <<= 1) ss += __shfl_xor(ss, m, 64);
+    }
     const float r = a.norm_v ? 1.0f / sqrtf(ss / (float)a.dv + a.eps) : 1.0f;
     bf16x8 o;
 #pragma unroll
@@ -777,9 +789,13 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
     return s;
   };
   auto over_pieces = [&](float x) {
-    if (lpk == 8) return sum8(x);
-    if (lpk == 16) return sum16(x);
-    for (int m = 1; m < lpk; m <<= 1) x += __shfl_xor(x, m, 64);
+    if constexpr (LPK == 8) {
+      x = sum8(x);
+    } else if constexpr (LPK == 16) {
+      x = sum16(x);
+    } else {
+      for (int m = 1; m < lpk; m <<= 1) x += __shfl_xor(x, m, 64);
+    }
     return x;
   };
 
@@ -887,9 +903,16 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
     }
 #pragma unroll
     for (int hh = 0; hh < QT; ++hh) {
-      for (int m = vp2; m < 64; m <<= 1) {
+      if constexpr (VP2 != 0) {
 #pragma unroll
-        for (int i = 0; i < N; ++i) acc[hh][i] += __shfl_xor(acc[hh][i], m, 64);
+        for (int m = VP2; m < 64; m <<= 1)
+#pragma unroll
+          for (int i = 0; i < N; ++i) acc[hh][i] += __shfl_xor(acc[hh][i], m, 64);
+      } else {
+        for (int m = vp2; m < 64; m <<= 1) {
+#pragma unroll
+          for (int i = 0; i < N; ++i) acc[hh][i] += __shfl_xor(acc[hh][i], m, 64);
+        }
       }
       if (lane < vp2) {
 #pragma unroll
@@ -912,20 +935,32 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
   }
 }
 
-template <bool HALF> void launch_window_step_vec(const WindowArgs& a, hipStream_t s) {
+template <bool HALF, int LPK, int VP2> void launch_window_step_lanes(const WindowArgs& a, int vp2, hipStream_t s) {
   const int qpk = a.H / a.G;
   const dim3 grid((unsigned)(a.B * a.G)), block(kStepThreads);
-  int vp2 = 1;
-  while (vp2 * 8 < a.dv) vp2 <<= 1;
   auto bytes = [&](int qt) { return (size_t)qt * (kStepKeys + 3 + kStepThreads / 64 * vp2 * 8) * sizeof(float); };
   if (qpk == 1)
-    hipLaunchKernelGGL((window_step_vec_kernel<1, HALF>), grid, block, bytes(1), s, a);
+    hipLaunchKernelGGL((window_step_vec_kernel<1, HALF, LPK, VP2>), grid, block, bytes(1), s, a);
   else if (qpk == 2)
-    hipLaunchKernelGGL((window_step_vec_kernel<2, HALF>), grid, block, bytes(2), s, a);
+    hipLaunchKernelGGL((window_step_vec_kernel<2, HALF, LPK, VP2>), grid, block, bytes(2), s, a);
   else if (qpk <= 4 || bytes(8) > 64 * 1024)
-    hipLaunchKernelGGL((window_step_vec_kernel<4, HALF>), grid, block, bytes(4), s, a);
+    hipLaunchKernelGGL((window_step_vec_kernel<4, HALF, LPK, VP2>), grid, block, bytes(4), s, a);
   else
-    hipLaunchKernelGGL((window_step_vec_kernel<8, HALF>), grid, block, bytes(8), s, a);
+    hipLaunchKernelGGL((window_step_vec_kernel<8, HALF, LPK, VP2>), grid, block, bytes(8), s, a);
+}
+
+template <bool HALF> void launch_window_step_vec(const WindowArgs& a, hipStream_t s) {
+  int lpk = 1, vp2 = 1;
+  while (lpk * 8 < a.d) lpk <<= 1;
+  while (vp2 * 8 < a.dv) vp2 <<= 1;
+  if (lpk == 8 && vp2 == 8)
+    launch_window_step_lanes<HALF, 8, 8>(a, vp2, s);
+  else if (lpk == 8 && vp2 == 16)
+    launch_window_step_lanes<HALF, 8, 16>(a, vp2, s);
+  else if (lpk == 16 && vp2 == 16)
+    launch_window_step_lanes<HALF, 16, 16>(a, vp2, s);
+  else
+    launch_window_step_lanes<HALF, 0, 0>(a, vp2, s);
 }
 
 template <typename T, bool VEC> void launch_window_step(const WindowArgs& a, hipStream_t s) {

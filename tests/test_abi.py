@@ -78,3 +78,48 @@ def test_argument_validation_without_gpu():
     rc = lib.based_linear_attn_prefill_split_static(p, p, p, p, None, None, 256, 16, 4096, 64, 0, 0, 16, 0, 0, 16,
                                                     0, 0, 64, 0, 0, 64, 1e-12, 0, 4, None)
     assert rc == 1 and b"scratch" in lib.based_hip_last_error()
+
+
+def test_parts_hold_what_they_are_for():
+    """The partial build for streamed models names existing sources, and these define every entry point
+    the streamed operations call."""
+    from based_amd import build
+
+    text = ""
+    for name in build.PARTS["streaming"]:
+        text += open(os.path.join(build.CSRC, f"{name}.hip")).read()
+    for entry in ("based_add_norm", "based_stream_conv", "based_window_attn_prefill", "based_window_attn_step",
+                  "based_gated_delta_scan", "based_gated_rms_norm", "based_gated_delta_step", "based_rglru_prefill",
+                  "based_rglru_step", "based_decode_linear_stream", "based_decode_linear", "based_swiglu", "based_greedy_step",
+                  "based_hip_last_error"):
+        assert re.search(rf"BASED_API [\w\*]+\s*\**{entry}\(|BASED_API const char\* {entry}\(", text), entry
+
+
+def test_header_matches_argument_lists():
+    """Every ctypes argument list has the number and kinds of arguments the header declares."""
+    text = re.sub(r"/\*.*?\*/", "", open(os.path.join(ROOT, "include", "based_hip.h")).read(), flags=re.S)
+    names = {"c_void_p": "p", "c_char_p": "p", "c_long": "l", "c_longlong": "l", "c_float": "f", "c_int": "i"}
+    for m in re.finditer(r"BASED_API\s+[\w\s\*]+?\b(based_\w+)\s*\(([^;]*?)\);", text, re.S):
+        args = [x for x in m.group(2).split(",") if x.strip() != "void"]
+        kinds = ["p" if "*" in x else "l" if "int64" in x else "f" if "float" in x else "i" for x in args]
+        assert kinds == [names.get(t.__name__, "p") for t in _lib.SIGNATURES[m.group(1)][1]], m.group(1)
+
+
+def test_streamed_argument_validation_without_gpu():
+    lib = _lib.lib()
+    buf = (ctypes.c_float * 64)()
+    p = ctypes.cast(buf, ctypes.c_void_p)
+    assert lib.based_add_norm(None, None, None, None, None, 1, 8, 8, 8, 8, 8, 1e-5, 1, 1.0, 0, None) == 4
+    # nine taps -> BASED_ERR_SHAPE; in place -> BASED_ERR_ARG
+    q = ctypes.c_void_p(p.value + 64)
+    assert lib.based_stream_conv(p, p, None, q, None, None, 0, 1, 1, 8, 9, 8, 8, 8, 8, 0, 0, 0, 0, None) == 1
+    assert lib.based_stream_conv(p, p, None, p, None, None, 0, 1, 1, 8, 4, 8, 8, 8, 8, 0, 0, 0, 0, None) == 4
+    # three query heads over two key/value heads; a portion that runs past the cache
+    tail = (0.1, 0, 0.0, 1.0, None, None, 0, 0, 0, 0, None)
+    assert lib.based_window_attn_prefill(p, p, p, p, p, 0, 1, 2, 3, 2, 8, 8, 4, *([8] * 10), 4, *tail) == 1
+    assert lib.based_window_attn_prefill(p, p, p, p, p, 3, 1, 2, 2, 2, 8, 8, 4, *([8] * 10), 4, *tail) == 1
+    # query/key size above 256
+    assert lib.based_gated_delta_scan(*([p] * 10), 1, 1, 1, 1, 264, 8, 8, 8, 8, 8, 8, 1, 0, None) == 1
+    # channels that do not divide into blocks
+    assert lib.based_rglru_prefill(*([p] * 12), 1, 1, 10, 3, *([8] * 6), 8.0, 1, 0, None) == 1
+    assert b"blocks" in lib.based_hip_last_error()
