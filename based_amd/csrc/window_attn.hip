@@ -480,7 +480,7 @@ __global__ __launch_bounds__(kStepThreads) void window_step_kernel(const WindowA
   if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;  // a position the cache does not hold
   float* qs = smem;                        // [QT][d]
   float* sc = qs + QT * a.d;               // [QT][kStepKeys]
-  float* stat = sc + QT * kStepKeys;       // [3][QT]: running maximum, running sum, rescale of this round
+  float* stat = sc + QT * kStepKeys;       // [3][QT]: running maximum, running sum, rescale of the current keys
   float* part = stat + 3 * QT;             // [QT][parts][vp2 * N], partial outputs
   float* knew = part + part_floats;        // [d] and [dv]: the row of the new token, as the cache holds it
   float* vnew = knew + a.d;
@@ -704,7 +704,7 @@ __global__ __launch_bounds__(kStepThreads) void window_step_vec_kernel(const Win
   const int pos = row_pos(a.pos, a.pos_host, b);
   if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;  // a position the cache does not hold
   float* sc = smem;                   // [QT][kStepKeys]
-  float* stat = sc + QT * kStepKeys;  // [3][QT]: running maximum, running sum, rescale of this round
+  float* stat = sc + QT * kStepKeys;  // [3][QT]: running maximum, running sum, rescale of the current keys
   float* part = stat + 3 * QT;        // [QT][parts][vp2 * 8], partial outputs
   const __bf16* k = static_cast<const __bf16*>(a.k) + b * a.k_sb + (long)g * a.d;
   const __bf16* v = static_cast<const __bf16*>(a.v) + b * a.v_sb + (long)g * a.dv;

@@ -145,7 +145,15 @@ def bench_kernels(torch, ops, B=8, L=4096, D=1024, decode_B=128):
                                         value_norm_eps=1e-5, out=o1)
     pair("window_attn_step B=%d H=16 G=4 window=129" % M,
          _entry(_graph_ms(torch, fn, 2), M * 2 * d * (2 * G * 129 + 2 * H + 2 * G)), "swa_step", swa1)
-    del kvs, c5, kv4
+    # the grouped form again with as many bytes per launch as the ungrouped one
+    M4 = 4 * M
+    q4, k4, pos4 = rnd(M4, H * d), rnd(M4, G * d), torch.full((M4,), 1000, dtype=torch.int32, device=dev)
+    o4 = torch.empty(M4, H * d, device=dev, dtype=bf)
+    kvb = [x.view(M4, 1024, 4, 2 * d) for x in kvs]
+    fn = lambda i: ops.window_attn_step(q4, k4, k4, kvb[i], H, G, 129, 0.125, pos4, rope=(*rope, True), value_norm_eps=1e-5, out=o4)
+    pair("window_attn_step B=%d H=16 G=4 window=129" % M4,
+         _entry(_graph_ms(torch, fn, 2), M4 * 2 * d * (2 * G * 129 + 2 * H + 2 * G)), "swa_step", swa1)
+    del kvs, c5, kv4, kvb
     kvst = [torch.zeros(M, 16, 1, 64, 273, device=dev) for _ in range(3)]
     kst = torch.ones(M, 16, 1, 1, 273, device=dev)
     q2, v2 = rnd(M, 16, 1, 16), rnd(M, 16, 1, 64)
