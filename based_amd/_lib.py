@@ -119,6 +119,26 @@ SIGNATURES = {
         [_P, _I64, _P, _I64, _P, _I64, _P, _P] + [_I64] * 4 + [_P, _I64, _P, _I64, C.c_float, C.c_int, _P, C.c_float,
                                                               _P, _P, _I64, C.c_int, _P, _I64, C.c_int, _P],
     ),
+    "based_add_norm_addends": (
+        C.c_int, [_P] * 5 + [_I64] * 6 + [C.c_float, C.c_int, C.c_float, _P, C.c_float, _P, _P, _P, _I64, _I64, C.c_int, _P]),
+    "based_token_mix": (C.c_int, [_P] * 5 + [_I64] * 8 + [C.c_int, _P]),
+    "based_channel_decay": (C.c_int, [_P] * 4 + [_I64] * 4 + [C.c_int, _P]),
+    "based_gelu_mul": (C.c_int, [_P] * 4 + [_I64] * 5 + [C.c_int, _P]),
+    "based_softcap": (C.c_int, [_P, _I64, C.c_float, C.c_int, _P]),
+    "based_decay_scan_work": (_I64, [_I64] * 6),
+    "based_decay_scan": (C.c_int, [_P] * 9 + [_I64] * 14 + [C.c_int, C.c_int, C.c_int, _P]),
+    "based_decay_step": (C.c_int, [_P] * 13 + [_I64] * 13 + [C.c_int, C.c_float, C.c_int, _P]),
+    "based_group_norm_gate": (C.c_int, [_P] * 4 + [_I64] * 10 + [C.c_float, C.c_float, C.c_int, C.c_int, _P]),
+    "based_window_attn_attend": (
+        C.c_int, [_P] * 3 + [_I64] * 15 + [C.c_float, C.c_float, _P, _P, _I64, _I64, C.c_int, C.c_int, _P]),
+    "based_latent_write": (C.c_int, [_P] * 3 + [_I64] * 10 + [C.c_float, _P, _P, _I64, C.c_int, C.c_int, _P]),
+    "based_latent_step": (
+        C.c_int, [_P] * 10 + [_I64] * 16 + [C.c_float, C.c_float, C.c_float, _P, _P, _I64, C.c_int, C.c_int, _P]),
+    "based_expert_route": (C.c_int, [_P] * 6 + [_I64] * 5 + [C.c_int, _P]),
+    "based_expert_tiles": (_I64, [_I64] * 3),
+    "based_expert_tile_rows": (_I64, [_I64] * 3),
+    "based_expert_grouped": (C.c_int, [_P] * 13 + [_I64] * 6 + [_P]),
+    "based_expert_rows": (C.c_int, [_P] * 7 + [_I64] * 5 + [C.c_int, _P]),
     "based_swa_step": (
         C.c_int,
         [_P, _P, _P, _P, _P, _P, _P, _I64] + [_I64] * 3 + [_I64] * 8 + [_I64] * 3

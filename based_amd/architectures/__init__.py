@@ -1,11 +1,12 @@
 """Model designs with a config.json format and tensor names of their own.  A design is a module with
-`stack_config(raw)` (config.json -> StackConfig keywords) and `convert_state(raw, tensors)` (its
-tensors -> the stack's state dict); config.json names it under "architecture"."""
+`stack_config(raw, shapes)` (config.json, and the shapes of the tensors by name for sizes that only they
+tell -> StackConfig keywords) and `convert_state(raw, tensors)` (its tensors -> the stack's state dict);
+config.json names it under "architecture"."""
 from __future__ import annotations
 
-from . import sozilix
+from . import peponex, sozilix
 
-DESIGNS = {"Sozilix": sozilix}
+DESIGNS = {"Peponex": peponex, "Sozilix": sozilix}
 
 
 def find(raw: dict):

@@ -47,7 +47,7 @@ def _mlp_spec(layer: dict):
     return {"hidden": mlp["ff"]}
 
 
-def stack_config(raw: dict) -> dict:
+def stack_config(raw: dict, shapes: dict = None) -> dict:
     """Keywords of StackConfig for a Sozilix config.json."""
     eps = raw["norm"]["eps"]
     return dict(

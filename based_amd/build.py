@@ -69,7 +69,8 @@ def _compile(src: str):
 
 # Sources a group of models needs, for a machine that serves nothing else: `build_part`.
 PARTS = {
-    "streaming": ("capi", "decode_linear", "gated_conv", "gated_delta", "greedy", "rglru", "stream_norm_conv", "window_attn"),
+    "streaming": ("capi", "decay_scan", "decode_linear", "experts", "gated_conv", "gated_delta", "greedy", "latent_attn", "rglru",
+                  "stream_norm_conv", "token_mix", "window_attn"),
 }
 
 

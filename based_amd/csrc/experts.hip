@@ -1,0 +1,520 @@
+// Mixture of experts with sigmoid routing for gfx950.  Of E small gated feed-forwards a token takes the `top`
+// with the largest scores s = sigmoid(W_router h); each reads s * h, and their outputs are added:
+//   y = sum_e down_e(silu(gate_e(s h)) * up_e(s h))
+// (s multiplies the sums of gate and up in fp32, which is the same thing.)
+//
+//   expert_route    scores in fp32, the choice, and for grouped products each choice's place among its
+//                   expert's rows
+//   expert_plan     rows of every expert rounded up to tiles; which expert a tile belongs to
+//   expert_scatter  the choices in that order
+//   expert_gemm     MFMA product of a tile of rows with its expert's matrices, gathered and scattered by that
+//                   order: gate and up with the activation behind them, then down
+//   expert_sum      the choices of a token added up (with one choice the product writes the token's row)
+//   expert_rows     few tokens, fp32, or rows that are no whole 16-byte pieces: dot products, one choice at a time
+#include "stream_common.hpp"
+
+namespace based {
+
+constexpr int kMaxExperts = 256;
+constexpr int kRouteTokens = 16;
+
+struct RouteArgs {
+  const void* h;  // (N, D)
+  const void* w;  // (E, D)
+  int32_t* ids;   // (N, top)
+  float* scores;  // (N, top)
+  int32_t* rank;  // (N, top) or null
+  int32_t* counts;  // (E), zero on entry, with rank
+  long n, h_sr;
+  int D, E, top;
+};
+
+__device__ __forceinline__ f32x4 expert_mfma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+// ET: tiles of 16 experts (bf16 MFMA, a quarter of the row per wavefront); 0: element by element.
+template <typename T, int ET>
+__global__ __launch_bounds__(256) void expert_route_kernel(const RouteArgs a) {
+  extern __shared__ float logits[];  // [4 (ET) or 1][kRouteTokens][E]
+  __shared__ int hist[kMaxExperts], base[kMaxExperts];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
+  const long n0 = (long)blockIdx.x * kRouteTokens;
+  const int n = a.n - n0 < kRouteTokens ? (int)(a.n - n0) : kRouteTokens;
+  for (int e = tid; e < a.E; e += 256) hist[e] = 0;
+  if constexpr (ET > 0) {
+    f32x4 acc[ET];
+#pragma unroll
+    for (int t = 0; t < ET; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const __bf16* h = static_cast<const __bf16*>(a.h) + (n0 + (l16 < n ? l16 : 0)) * a.h_sr;
+    const int pieces = (a.D + 31) / 32, per = (pieces + 3) / 4;
+    const int p1 = (wave + 1) * per < pieces ? (wave + 1) * per : pieces;
+    for (int p = wave * per; p < p1; ++p) {
+      const int c = p * 32 + quad * 8;
+      bf16x8 x = *reinterpret_cast<const bf16x8*>(h + (c < a.D ? c : 0));
+      if (c >= a.D) {
+#pragma unroll
+        for (int j = 0; j < 8; ++j) x[j] = (__bf16)0.f;
+      }
+#pragma unroll
+      for (int t = 0; t < ET; ++t) {
+        const int e = t * 16 + l16;
+        const bf16x8 w = *reinterpret_cast<const bf16x8*>(static_cast<const __bf16*>(a.w) + (long)(e < a.E ? e : 0) * a.D + (c < a.D ? c : 0));
+        acc[t] = expert_mfma(w, x, acc[t]);
+      }
+    }
+    // column = token l16, rows = experts 4 quad + i
+#pragma unroll
+    for (int t = 0; t < ET; ++t)
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int e = t * 16 + quad * 4 + i;
+        if (e < a.E) logits[(wave * kRouteTokens + l16) * a.E + e] = acc[t][i];
+      }
+    __syncthreads();
+    for (int i = tid; i < kRouteTokens * a.E; i += 256) {
+      const int s = kRouteTokens * a.E;
+      const float z = (logits[i] + logits[s + i]) + (logits[2 * s + i] + logits[3 * s + i]);
+      logits[i] = 1.0f / (1.0f + expf(-z));
+    }
+  } else {
+    for (int i = tid; i < kRouteTokens * a.E; i += 256) {
+      const int t = i / a.E, e = i % a.E;
+      const T* h = static_cast<const T*>(a.h) + (n0 + (t < n ? t : 0)) * a.h_sr;
+      const T* w = static_cast<const T*>(a.w) + (long)e * a.D;
+      float z = 0.f;
+      for (int c = 0; c < a.D; ++c) z = __builtin_fmaf(to_f32(w[c]), to_f32(h[c]), z);
+      logits[i] = 1.0f / (1.0f + expf(-z));
+    }
+  }
+  __syncthreads();
+  // 16 lanes per token
+  const int t = tid >> 4, sub = tid & 15;
+  float* s = logits + t * a.E;
+  for (int j = 0; j < a.top; ++j) {
+    float best = -2.f;
+    int at = 0;
+    for (int e = sub; e < a.E; e += 16)
+      if (s[e] > best) best = s[e], at = e;
+#pragma unroll
+    for (int m = 8; m >= 1; m >>= 1) {
+      const float ov = __shfl_xor(best, m, 16);
+      const int oa = __shfl_xor(at, m, 16);
+      if (ov > best || (ov == best && oa < at)) best = ov, at = oa;
+    }
+    if (at % 16 == sub) s[at] = -1.f;  // taken
+    if (sub == 0 && t < n) {
+      const long slot = (n0 + t) * a.top + j;
+      a.ids[slot] = at;
+      a.scores[slot] = best;
+      if (a.rank != nullptr) a.rank[slot] = atomicAdd(&hist[at], 1);
+    }
+  }
+  if (a.rank == nullptr) return;
+  __syncthreads();
+  for (int e = tid; e < a.E; e += 256) base[e] = hist[e] > 0 ? atomicAdd(&a.counts[e], hist[e]) : 0;
+  __syncthreads();
+  if (sub == 0 && t < n) {
+    for (int j = 0; j < a.top; ++j) {
+      const long slot = (n0 + t) * a.top + j;
+      a.rank[slot] += base[a.ids[slot]];
+    }
+  }
+}
+
+// One workgroup: tile_first[e] and, at the end, the number of tiles; tile_expert[tile].
+__global__ __launch_bounds__(256) void expert_plan_kernel(const int32_t* counts, int32_t* tile_first, int32_t* tile_expert, int E, int tile_rows) {
+  __shared__ int scan[256];
+  const int e = threadIdx.x;
+  const int tiles = e < E ? (counts[e] + tile_rows - 1) / tile_rows : 0;
+  scan[e] = tiles;
+  __syncthreads();
+  for (int m = 1; m < 256; m <<= 1) {
+    const int add = e >= m ? scan[e - m] : 0;
+    __syncthreads();
+    scan[e] += add;
+    __syncthreads();
+  }
+  const int first = scan[e] - tiles;
+  if (e < E) tile_first[e] = first;
+  if (e == 255) tile_first[E] = scan[255];
+  for (int t = 0; t < tiles; ++t) tile_expert[first + t] = e;
+}
+
+__global__ __launch_bounds__(256) void expert_scatter_kernel(const int32_t* ids, const int32_t* rank, const int32_t* tile_first, int32_t* order,
+                                                             long slots, int tile_rows) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i < slots) order[(long)tile_first[ids[i]] * tile_rows + rank[i]] = (int32_t)i;
+}
+
+// ---- grouped products ----
+struct ExpertGemmArgs {
+  const __bf16* x;       // PAIRED: (N, K) rows gathered by order / top; otherwise (tiles * rows, K) in order
+  const __bf16* w;       // PAIRED: (E, 2 F, K), up rows then gate rows; otherwise (E, F, K)
+  __bf16* y;             // PAIRED: (tiles * rows, F); otherwise (slots, F) scattered by order
+  const int32_t* order;
+  const int32_t* counts;
+  const int32_t* tile_first;
+  const int32_t* tile_expert;
+  const float* scores;   // (slots), PAIRED
+  long x_sr;
+  int E, F, K, top;
+};
+
+constexpr int kGemmK = 64;
+
+template <int BM, bool PAIRED>
+__global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a) {
+  constexpr int KS = kGemmK + 8;
+  constexpr int WM = BM >= 128 ? 2 : 1, WN = 4 / WM, MT = BM / 16 / WM, NT = 4 / WN;
+  constexpr int AP = BM / 32;  // 16-byte pieces of the rows per thread
+  __shared__ __attribute__((aligned(16))) __bf16 xs[BM * KS], ws[128 * KS];
+  __shared__ int slot_of[BM];
+  const int tile = blockIdx.y;
+  if (tile >= a.tile_first[a.E]) return;
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4, wm = wave % WM, wn = wave / WM;
+  const int e = a.tile_expert[tile], r0 = (tile - a.tile_first[e]) * BM;
+  const int rows = a.counts[e] - r0 < BM ? a.counts[e] - r0 : BM;
+  const int f0 = blockIdx.x * (PAIRED ? 64 : 128);
+  for (int i = tid; i < BM; i += 256) slot_of[i] = a.order[(long)tile * BM + (i < rows ? i : 0)];
+  __syncthreads();
+  typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
+  const int piece = (tid & 7) * 8;  // of the 64 channels of a round
+  const __bf16* xrow[AP];
+#pragma unroll
+  for (int i = 0; i < AP; ++i) {
+    const int r = i * 32 + (tid >> 3);
+    xrow[i] = a.x + (PAIRED ? (long)(slot_of[r] / a.top) * a.x_sr : ((long)tile * BM + (r < rows ? r : 0)) * a.x_sr);
+  }
+  const __bf16* wrow[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int r = i * 32 + (tid >> 3);
+    const int f = PAIRED ? f0 + (r & 63) : f0 + r;
+    wrow[i] = a.w + ((long)e * (PAIRED ? 2 * a.F : a.F) + (PAIRED && r >= 64 ? a.F : 0) + (f < a.F ? f : a.F - 1)) * a.K;
+  }
+  u32x4 xb[AP], wb[4];
+  const u32x4 zero = {0u, 0u, 0u, 0u};
+  auto fetch = [&](int k0) {
+    const int c = k0 + piece < a.K ? k0 + piece : 0;
+#pragma unroll
+    for (int i = 0; i < AP; ++i) xb[i] = *reinterpret_cast<const u32x4*>(xrow[i] + c);
+#pragma unroll
+    for (int i = 0; i < 4; ++i) wb[i] = *reinterpret_cast<const u32x4*>(wrow[i] + c);
+  };
+  f32x4 acc[2][NT][MT];
+#pragma unroll
+  for (int p = 0; p < 2; ++p)
+#pragma unroll
+    for (int i = 0; i < NT; ++i)
+#pragma unroll
+      for (int j = 0; j < MT; ++j) acc[p][i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  fetch(0);
+  for (int k0 = 0; k0 < a.K; k0 += kGemmK) {
+    const bool in = k0 + piece < a.K;
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < AP; ++i) *reinterpret_cast<u32x4*>(&xs[(i * 32 + (tid >> 3)) * KS + piece]) = in ? xb[i] : zero;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(&ws[(i * 32 + (tid >> 3)) * KS + piece]) = wb[i];
+    __syncthreads();
+    if (k0 + kGemmK < a.K) fetch(k0 + kGemmK);
+#pragma unroll
+    for (int kk = 0; kk < kGemmK; kk += 32) {
+      bf16x8 xf[MT];
+#pragma unroll
+      for (int j = 0; j < MT; ++j) xf[j] = *reinterpret_cast<const bf16x8*>(&xs[((wm * MT + j) * 16 + l16) * KS + kk + quad * 8]);
+#pragma unroll
+      for (int p = 0; p < 2; ++p)
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+          const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&ws[(p * 64 + (wn * NT + i) * 16 + l16) * KS + kk + quad * 8]);
+#pragma unroll
+          for (int j = 0; j < MT; ++j) acc[p][i][j] = expert_mfma(wf, xf[j], acc[p][i][j]);
+        }
+    }
+  }
+  // column = row l16 of the tile's rows, rows = features 4 quad + i
+#pragma unroll
+  for (int j = 0; j < MT; ++j) {
+    const int r = (wm * MT + j) * 16 + l16;
+    if (r >= rows) continue;
+    const int slot = slot_of[r];
+    if constexpr (PAIRED) {
+      const float s = a.scores[slot];
+      __bf16* y = a.y + ((long)tile * BM + r) * a.F;
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        const int f = f0 + (wn * NT + i) * 16 + quad * 4;
+        if (f < a.F) {
+          bf16x4 o;
+#pragma unroll
+          for (int m = 0; m < 4; ++m) o[m] = (__bf16)(silu_exact(acc[1][i][j][m] * s) * (acc[0][i][j][m] * s));
+          *reinterpret_cast<bf16x4*>(y + f) = o;
+        }
+      }
+    } else {
+      __bf16* y = a.y + (long)slot * a.F;
+#pragma unroll
+      for (int p = 0; p < 2; ++p)
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+          const int f = f0 + p * 64 + (wn * NT + i) * 16 + quad * 4;
+          if (f < a.F) {
+            bf16x4 o;
+#pragma unroll
+            for (int m = 0; m < 4; ++m) o[m] = (__bf16)acc[p][i][j][m];
+            *reinterpret_cast<bf16x4*>(y + f) = o;
+          }
+        }
+    }
+  }
+}
+
+// y[n] = sum of the rows of its choices
+__global__ __launch_bounds__(256) void expert_sum_kernel(const __bf16* x, __bf16* y, long n, int D, int top) {
+  const int pieces = D / 8;
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= n * pieces) return;
+  const long row = i / pieces;
+  const int c = (int)(i % pieces) * 8;
+  float s[8];
+#pragma unroll
+  for (int j = 0; j < 8; ++j) s[j] = 0.f;
+  for (int t = 0; t < top; ++t) {
+    float v[8];
+    load_vec<__bf16, 8>(x + (row * top + t) * D + c, v);
+#pragma unroll
+    for (int j = 0; j < 8; ++j) s[j] += v[j];
+  }
+  store_vec<__bf16, 8>(y + row * D + c, s);
+}
+
+// ---- one choice at a time ----
+struct ExpertRowsArgs {
+  const void* x;   // first product: (N, K); second: (N * top, K)
+  const void* w;   // (E, 2 F, K) / (E, F, K)
+  void* y;         // (N * top, F) / (N, F)
+  const int32_t* ids;
+  const float* scores;
+  long n, x_sr;
+  int F, K, top;
+};
+
+constexpr int kRowsFeatures = 16;  // features per workgroup
+
+template <int LPR> __device__ __forceinline__ float lanes_sum(float v) {
+  if constexpr (LPR == 8) return sum8(v);
+  v = sum16(v);
+  if constexpr (LPR >= 32) v += __shfl_xor(v, 16, 64);
+  if constexpr (LPR >= 64) v += __shfl_xor(v, 32, 64);
+  return v;
+}
+
+// LPR lanes share a dot product; a workgroup takes kRowsFeatures features of one choice (gate and up) or token (down).
+template <typename T, int N, int LPR, bool PAIRED>
+__global__ __launch_bounds__(256) void expert_rows_kernel(const ExpertRowsArgs a) {
+  const int lane = threadIdx.x % LPR, grp = threadIdx.x / LPR;
+  constexpr int GROUPS = 256 / LPR;
+  const long item = blockIdx.x;  // choice or token
+  const int f1 = (int)(blockIdx.y + 1) * kRowsFeatures < a.F ? (int)(blockIdx.y + 1) * kRowsFeatures : a.F;
+  constexpr int FU = GROUPS >= kRowsFeatures ? 1 : kRowsFeatures / GROUPS;  // features per group of lanes, in flight together
+  int f[FU];
+#pragma unroll
+  for (int u = 0; u < FU; ++u) f[u] = blockIdx.y * kRowsFeatures + u * GROUPS + grp;
+  auto load = [&](const T* p, float (&v)[N]) {
+    if constexpr (N == 1)
+      v[0] = to_f32(*p);
+    else
+      load_vec<T, N>(p, v);
+  };
+  if constexpr (PAIRED) {
+    const T* x = static_cast<const T*>(a.x) + item / a.top * a.x_sr;
+    const T* w = static_cast<const T*>(a.w) + (long)a.ids[item] * 2 * a.F * a.K;
+    float up[FU], gate[FU];
+#pragma unroll
+    for (int u = 0; u < FU; ++u) up[u] = gate[u] = 0.f;
+#pragma unroll 2
+    for (int c = lane * N; c < a.K; c += LPR * N) {
+      float xv[N];
+      load(x + c, xv);
+#pragma unroll
+      for (int u = 0; u < FU; ++u) {
+        const long row = f[u] < f1 ? f[u] : 0;
+        float uv[N], gv[N];
+        load(w + row * a.K + c, uv);
+        load(w + (a.F + row) * a.K + c, gv);
+#pragma unroll
+        for (int j = 0; j < N; ++j) {
+          up[u] = __builtin_fmaf(uv[j], xv[j], up[u]);
+          gate[u] = __builtin_fmaf(gv[j], xv[j], gate[u]);
+        }
+      }
+    }
+    const float s = a.scores[item];
+#pragma unroll
+    for (int u = 0; u < FU; ++u) {
+      const float uu = lanes_sum<LPR>(up[u]), gg = lanes_sum<LPR>(gate[u]);
+      if (lane == 0 && f[u] < f1) static_cast<T*>(a.y)[item * a.F + f[u]] = from_f32<T>(silu_exact(gg * s) * (uu * s));
+    }
+  } else {
+    float acc[FU];
+#pragma unroll
+    for (int u = 0; u < FU; ++u) acc[u] = 0.f;
+    for (int t = 0; t < a.top; ++t) {
+      const T* x = static_cast<const T*>(a.x) + (item * a.top + t) * a.x_sr;
+      const T* w = static_cast<const T*>(a.w) + (long)a.ids[item * a.top + t] * a.F * a.K;
+#pragma unroll 2
+      for (int c = lane * N; c < a.K; c += LPR * N) {
+        float xv[N];
+        load(x + c, xv);
+#pragma unroll
+        for (int u = 0; u < FU; ++u) {
+          float wv[N];
+          load(w + (long)(f[u] < f1 ? f[u] : 0) * a.K + c, wv);
+#pragma unroll
+          for (int j = 0; j < N; ++j) acc[u] = __builtin_fmaf(wv[j], xv[j], acc[u]);
+        }
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < FU; ++u) {
+      const float s = lanes_sum<LPR>(acc[u]);
+      if (lane == 0 && f[u] < f1) static_cast<T*>(a.y)[item * a.F + f[u]] = from_f32<T>(s);
+    }
+  }
+}
+
+template <typename T, int N, bool PAIRED> void launch_expert_rows(const ExpertRowsArgs& a, long items, hipStream_t s) {
+  const dim3 grid((unsigned)items, (unsigned)((a.F + kRowsFeatures - 1) / kRowsFeatures));
+  const int pieces = (a.K + N - 1) / N;
+  if (pieces <= 8)
+    hipLaunchKernelGGL((expert_rows_kernel<T, N, 8, PAIRED>), grid, dim3(256), 0, s, a);
+  else if (pieces <= 16)
+    hipLaunchKernelGGL((expert_rows_kernel<T, N, 16, PAIRED>), grid, dim3(256), 0, s, a);
+  else if (pieces <= 32)
+    hipLaunchKernelGGL((expert_rows_kernel<T, N, 32, PAIRED>), grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL((expert_rows_kernel<T, N, 64, PAIRED>), grid, dim3(256), 0, s, a);
+}
+
+template <typename T, bool PAIRED> void launch_expert_rows_vec(const ExpertRowsArgs& a, bool vec, long items, hipStream_t s) {
+  if (vec)
+    launch_expert_rows<T, Pack<T>::kN, PAIRED>(a, items, s);
+  else
+    launch_expert_rows<T, 1, PAIRED>(a, items, s);
+}
+
+static void launch_route_bf16(const RouteArgs& a, bool vec, dim3 grid, hipStream_t s) {
+  const size_t one = (size_t)kRouteTokens * a.E * sizeof(float);
+  const int et = (a.E + 15) / 16;
+  if (!vec)
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, 0>), grid, dim3(256), one, s, a);
+  else if (et <= 1)
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, 1>), grid, dim3(256), 4 * one, s, a);
+  else if (et <= 2)
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, 2>), grid, dim3(256), 4 * one, s, a);
+  else if (et <= 4)
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, 4>), grid, dim3(256), 4 * one, s, a);
+  else
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, 8>), grid, dim3(256), 4 * one, s, a);
+}
+
+}  // namespace based
+
+extern "C" BASED_API int based_expert_route(const void* h, const void* router, int32_t* ids, float* scores, int32_t* rank, int32_t* counts,
+                                            int64_t n, int64_t D, int64_t E, int64_t top, int64_t h_sr, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(h && router && ids && scores && (rank == nullptr || counts), BASED_ERR_ARG, "expert_route: null pointer argument");
+  BASED_REQUIRE(n >= 0 && D > 0 && E > 0 && top > 0 && top <= E, BASED_ERR_ARG, "expert_route: bad sizes");
+  BASED_REQUIRE(E <= kMaxExperts, BASED_ERR_SHAPE, "expert_route: %ld experts (at most %d)", (long)E, kMaxExperts);
+  BASED_REQUIRE(n * top < (1ll << 31) && D < (1ll << 28), BASED_ERR_SHAPE, "expert_route: too many choices");
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "expert_route: bad dtype");
+  if (n == 0) return BASED_OK;
+  const RouteArgs a{h, router, ids, scores, rank, counts, (long)n, (long)h_sr, (int)D, (int)E, (int)top};
+  const dim3 grid((unsigned)((n + kRouteTokens - 1) / kRouteTokens));
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16) {
+    launch_route_bf16(a, D % 8 == 0 && h_sr % 8 == 0 && E <= 128 && aligned_to(h, 16) && aligned_to(router, 16), grid, s);
+  } else {
+    hipLaunchKernelGGL((expert_route_kernel<float, 0>), grid, dim3(256), (size_t)kRouteTokens * E * sizeof(float), s, a);
+  }
+  return check_launch("expert_route");
+}
+
+/* Tiles of BASED_EXPERT_TILE_ROWS or BASED_EXPERT_TILE_ROWS_SMALL rows. */
+static int expert_tile_rows(int64_t slots, int64_t E) { return slots >= 64 * E ? BASED_EXPERT_TILE_ROWS : BASED_EXPERT_TILE_ROWS_SMALL; }
+
+extern "C" BASED_API int64_t based_expert_tiles(int64_t n, int64_t E, int64_t top) {
+  if (n <= 0 || E <= 0 || top <= 0) return 0;
+  const int64_t rows = expert_tile_rows(n * top, E);
+  return n * top / rows + (E < n * top ? E : n * top);
+}
+
+extern "C" BASED_API int64_t based_expert_tile_rows(int64_t n, int64_t E, int64_t top) { return expert_tile_rows(n * top, E); }
+
+extern "C" BASED_API int based_expert_grouped(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
+                                              const int32_t* rank, const int32_t* counts, int32_t* tile_first, int32_t* tile_expert,
+                                              int32_t* order, void* work_act, void* work_out, void* y, int64_t n, int64_t D, int64_t F,
+                                              int64_t E, int64_t top, int64_t h_sr, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(h && w1 && w2 && ids && scores && rank && counts && tile_first && tile_expert && order && work_act && y, BASED_ERR_ARG,
+                "expert_grouped: null pointer argument");
+  BASED_REQUIRE(n >= 0 && D > 0 && F > 0 && E > 0 && top > 0 && E <= kMaxExperts && n * top < (1ll << 31), BASED_ERR_ARG,
+                "expert_grouped: bad sizes");
+  BASED_REQUIRE(top == 1 || work_out != nullptr, BASED_ERR_ARG, "expert_grouped: several choices per token need work_out");
+  BASED_REQUIRE(D % 8 == 0 && F % 8 == 0 && h_sr % 8 == 0, BASED_ERR_SHAPE, "expert_grouped: sizes %ld and %ld must be multiples of 8",
+                (long)D, (long)F);
+  BASED_REQUIRE(aligned_to(h, 16) && aligned_to(w1, 16) && aligned_to(w2, 16) && aligned_to(work_act, 16) && aligned_to(work_out, 16) &&
+                    aligned_to(y, 16),
+                BASED_ERR_ALIGN, "expert_grouped: tensors must be 16-byte aligned");
+  if (n == 0) return BASED_OK;
+  const int64_t slots = n * top;
+  const int rows = expert_tile_rows(slots, E);
+  const int64_t tiles = based_expert_tiles(n, E, top);
+  BASED_REQUIRE(tiles < 65536, BASED_ERR_SHAPE, "expert_grouped: too many rows");
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(256), 0, s, counts, tile_first, tile_expert, (int)E, rows);
+  hipLaunchKernelGGL(expert_scatter_kernel, dim3((unsigned)((slots + 255) / 256)), dim3(256), 0, s, ids, rank, tile_first, order,
+                     (long)slots, rows);
+  ExpertGemmArgs a{static_cast<const __bf16*>(h), static_cast<const __bf16*>(w1), static_cast<__bf16*>(work_act), order, counts, tile_first,
+                   tile_expert, scores, (long)h_sr, (int)E, (int)F, (int)D, (int)top};
+  const dim3 grid1((unsigned)((F + 63) / 64), (unsigned)tiles), grid2((unsigned)((D + 127) / 128), (unsigned)tiles);
+  __bf16* out = static_cast<__bf16*>(top == 1 ? y : work_out);
+  ExpertGemmArgs a2{static_cast<const __bf16*>(work_act), static_cast<const __bf16*>(w2), out, order, counts, tile_first,
+                    tile_expert, scores, (long)F, (int)E, (int)D, (int)F, (int)top};
+  if (rows == BASED_EXPERT_TILE_ROWS) {
+    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS, true>), grid1, dim3(256), 0, s, a);
+    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS, false>), grid2, dim3(256), 0, s, a2);
+  } else {
+    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS_SMALL, true>), grid1, dim3(256), 0, s, a);
+    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS_SMALL, false>), grid2, dim3(256), 0, s, a2);
+  }
+  if (top > 1)
+    hipLaunchKernelGGL(expert_sum_kernel, dim3((unsigned)((n * (D / 8) + 255) / 256)), dim3(256), 0, s, out, static_cast<__bf16*>(y), (long)n,
+                       (int)D, (int)top);
+  return check_launch("expert_grouped");
+}
+
+extern "C" BASED_API int based_expert_rows(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
+                                           void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t top, int64_t h_sr,
+                                           int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(h && w1 && w2 && ids && scores && work_act && y, BASED_ERR_ARG, "expert_rows: null pointer argument");
+  BASED_REQUIRE(n >= 0 && D > 0 && F > 0 && top > 0 && n * top < (1ll << 31), BASED_ERR_ARG, "expert_rows: bad sizes");
+  BASED_REQUIRE(D < (1 << 20) && F < (1 << 20), BASED_ERR_SHAPE, "expert_rows: grid too large");
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "expert_rows: bad dtype");
+  if (n == 0) return BASED_OK;
+  const int p = io_dtype == BASED_BF16 ? 8 : 4;
+  const bool vec1 = D % p == 0 && h_sr % p == 0 && aligned_to(h, 16) && aligned_to(w1, 16);
+  const bool vec2 = F % p == 0 && aligned_to(work_act, 16) && aligned_to(w2, 16);
+  const ExpertRowsArgs a1{h, w1, work_act, ids, scores, (long)n, (long)h_sr, (int)F, (int)D, (int)top};
+  const ExpertRowsArgs a2{work_act, w2, y, ids, scores, (long)n, (long)F, (int)D, (int)F, (int)top};
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16) {
+    launch_expert_rows_vec<__bf16, true>(a1, vec1, n * top, s);
+    launch_expert_rows_vec<__bf16, false>(a2, vec2, n, s);
+  } else {
+    launch_expert_rows_vec<float, true>(a1, vec1, n * top, s);
+    launch_expert_rows_vec<float, false>(a2, vec2, n, s);
+  }
+  return check_launch("expert_rows");
+}

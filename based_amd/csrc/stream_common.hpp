@@ -104,6 +104,17 @@ __device__ __forceinline__ float ring_dot(const T* ring, const T* w, long stride
   return acc;
 }
 
+// What a residual sum may receive besides mult * x: x divided by its RMS (post_eps) and multiplied by post_w
+// first, a vector for every row, and rows of a table (by index, or one per row).
+struct StreamAddends {
+  const void* post_w;
+  const void* vec;
+  const void* rows;
+  const int64_t* rows_index;
+  long rows_sr, rows_n;
+  float post_eps;
+};
+
 // Position of the token a single-token launch brings for batch row b: from the device when there is
 // an array of positions, otherwise the one the host passed.
 __device__ __forceinline__ int row_pos(const int32_t* pos, int pos_host, int b) { return pos != nullptr ? pos[b] : pos_host; }

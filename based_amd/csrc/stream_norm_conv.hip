@@ -3,7 +3,9 @@
 //   add_norm:     r = residual + mult * x  (fp32; r = x without a residual),
 //                 y = norm(r) * w, norm the layer norm without a bias
 //                 (r - mean) / sqrt(var + eps) or the RMS norm r / sqrt(mean(r^2) + eps).
-//                 The norm sees the fp32 sum, not a rounded copy of it.
+//                 The norm sees the fp32 sum, not a rounded copy of it.  Optionally x is divided by its own
+//                 RMS and weighted before it is added, and r also receives a vector and a row of a table
+//                 (the embedding of the row's token, once more); without a norm y is the rounded sum.
 //   stream_conv:  y_t = [x_t +] act(bias + sum_j w[j] x_{t - taps + 1 + j}), a causal convolution
 //                 per channel over a sequence that arrives in portions of any length.  The inputs
 //                 of earlier portions come from a ring (B, taps, D): slot p % taps holds the input
@@ -17,7 +19,7 @@
 
 namespace based {
 
-enum { kNormRms = BASED_NORM_RMS, kNormLayer = BASED_NORM_LAYER };
+enum { kNormRms = BASED_NORM_RMS, kNormLayer = BASED_NORM_LAYER, kNormNone = BASED_NORM_NONE };
 
 struct AddNormArgs {
   const void* x;
@@ -30,10 +32,12 @@ struct AddNormArgs {
   long x_sr, ri_sr, y_sr, ro_sr;
   float eps, mult;
   int kind;
+  StreamAddends add;
 };
 
 // One wavefront per row, the row in registers: NV pieces of 8 elements per lane (D <= 512 NV, D % 8 == 0).
-template <typename T, int NV>
+// ADD: with what `StreamAddends` brings, or without a norm.
+template <typename T, int NV, bool ADD>
 __global__ __launch_bounds__(256) void add_norm_kernel(const AddNormArgs a) {
   const long row = (long)blockIdx.x * 4 + (threadIdx.x >> 6);
   if (row >= a.rows) return;
@@ -47,7 +51,46 @@ __global__ __launch_bounds__(256) void add_norm_kernel(const AddNormArgs a) {
     const int e = (c * 64 + lane) * 8;
     live[c] = e < a.D;
     load_vec<T, 8>(x + (live[c] ? e : 0), v[c]);
-    load_vec<T, 8>(w + (live[c] ? e : 0), wt[c]);
+    if (!ADD || w != nullptr) load_vec<T, 8>(w + (live[c] ? e : 0), wt[c]);
+  }
+  float extra[ADD ? NV : 1][8];
+  if constexpr (ADD) {
+    const StreamAddends& m = a.add;
+    long src = row;
+    bool poison = false;
+    if (m.rows != nullptr && m.rows_index != nullptr) {
+      src = m.rows_index[row];
+      poison = src < 0 || src >= m.rows_n;
+      src = poison ? 0 : src;
+    }
+    float pw[NV][8];
+    if (m.post_w != nullptr) {
+#pragma unroll
+      for (int c = 0; c < NV; ++c) load_vec<T, 8>(static_cast<const T*>(m.post_w) + (live[c] ? (c * 64 + lane) * 8 : 0), pw[c]);
+    }
+#pragma unroll
+    for (int c = 0; c < NV; ++c) {
+      const int e = live[c] ? (c * 64 + lane) * 8 : 0;
+      float a8[8], b8[8];
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a8[i] = b8[i] = 0.f;
+      if (m.vec != nullptr) load_vec<T, 8>(static_cast<const T*>(m.vec) + e, a8);
+      if (m.rows != nullptr) load_vec<T, 8>(static_cast<const T*>(m.rows) + src * m.rows_sr + e, b8);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) extra[c][i] = poison ? __builtin_nanf("") : a8[i] + b8[i];
+    }
+    if (m.post_w != nullptr) {
+      float ss = 0.f;
+#pragma unroll
+      for (int c = 0; c < NV; ++c)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) ss = live[c] ? __builtin_fmaf(v[c][i], v[c][i], ss) : ss;
+      const float r = 1.0f / sqrtf(wave_sum(ss) / (float)a.D + m.post_eps);
+#pragma unroll
+      for (int c = 0; c < NV; ++c)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) v[c][i] = v[c][i] * r * pw[c][i];
+    }
   }
   if (a.res_in != nullptr) {
     const float* r = a.res_in + row * a.ri_sr;
@@ -59,6 +102,12 @@ __global__ __launch_bounds__(256) void add_norm_kernel(const AddNormArgs a) {
       for (int i = 0; i < 8; ++i) v[c][i] = __builtin_fmaf(a.mult, v[c][i], rv[i]);
     }
   }
+  if constexpr (ADD) {
+#pragma unroll
+    for (int c = 0; c < NV; ++c)
+#pragma unroll
+      for (int i = 0; i < 8; ++i) v[c][i] += extra[c][i];
+  }
   float s = 0.f;
 #pragma unroll
   for (int c = 0; c < NV; ++c) {
@@ -66,6 +115,14 @@ __global__ __launch_bounds__(256) void add_norm_kernel(const AddNormArgs a) {
       if (a.res_out != nullptr) store_vec<float, 8>(a.res_out + row * a.ro_sr + (c * 64 + lane) * 8, v[c]);
 #pragma unroll
       for (int i = 0; i < 8; ++i) s += v[c][i];
+    }
+  }
+  if constexpr (ADD) {
+    if (a.kind == kNormNone) {
+#pragma unroll
+      for (int c = 0; c < NV; ++c)
+        if (live[c]) store_vec<T, 8>(static_cast<T*>(a.y) + row * a.y_sr + (c * 64 + lane) * 8, v[c]);
+      return;
     }
   }
   const float mean = a.kind == kNormLayer ? wave_sum(s) / (float)a.D : 0.f;
@@ -99,7 +156,6 @@ __global__ __launch_bounds__(256) void add_norm_any_kernel(const AddNormArgs a) 
   const T* x = static_cast<const T*>(a.x) + row * a.x_sr;
   const T* w = static_cast<const T*>(a.w);
   const float* r = a.res_in != nullptr ? a.res_in + row * a.ri_sr : nullptr;
-  auto sum_at = [&](int e) { return r != nullptr ? __builtin_fmaf(a.mult, to_f32(x[e]), r[e]) : to_f32(x[e]); };
   auto block_sum = [&](float v) {
     v = wave_sum(v);
     __syncthreads();
@@ -107,6 +163,37 @@ __global__ __launch_bounds__(256) void add_norm_any_kernel(const AddNormArgs a) 
     __syncthreads();
     return part[0] + part[1] + part[2] + part[3];
   };
+  const StreamAddends& m = a.add;
+  const T* pw = static_cast<const T*>(m.post_w);
+  const T* vec = static_cast<const T*>(m.vec);
+  const T* add_row = nullptr;
+  bool poison = false;
+  if (m.rows != nullptr) {
+    long src = m.rows_index != nullptr ? m.rows_index[row] : row;
+    poison = m.rows_index != nullptr && (src < 0 || src >= m.rows_n);
+    add_row = static_cast<const T*>(m.rows) + (poison ? 0 : src) * m.rows_sr;
+  }
+  float post = 1.f;
+  if (pw != nullptr) {
+    float ss = 0.f;
+    for (int e = threadIdx.x; e < a.D; e += 256) ss = __builtin_fmaf(to_f32(x[e]), to_f32(x[e]), ss);
+    post = 1.0f / sqrtf(block_sum(ss) / (float)a.D + m.post_eps);
+  }
+  auto sum_at = [&](int e) {
+    float v = to_f32(x[e]);
+    if (pw != nullptr) v = v * post * to_f32(pw[e]);
+    if (r != nullptr) v = __builtin_fmaf(a.mult, v, r[e]);
+    const float more = (vec != nullptr ? to_f32(vec[e]) : 0.f) + (add_row != nullptr ? to_f32(add_row[e]) : 0.f);
+    return poison ? __builtin_nanf("") : v + more;
+  };
+  if (a.kind == kNormNone) {
+    for (int e = threadIdx.x; e < a.D; e += 256) {
+      const float v = sum_at(e);
+      if (a.res_out != nullptr) a.res_out[row * a.ro_sr + e] = v;
+      static_cast<T*>(a.y)[row * a.y_sr + e] = from_f32<T>(v);
+    }
+    return;
+  }
   float mean = 0.f;
   if (a.kind == kNormLayer) {
     float s = 0.f;
@@ -126,7 +213,7 @@ __global__ __launch_bounds__(256) void add_norm_any_kernel(const AddNormArgs a) 
   }
 }
 
-template <typename T> void launch_add_norm(const AddNormArgs& a, bool vec, hipStream_t s) {
+template <typename T, bool ADD> void launch_add_norm_rows(const AddNormArgs& a, bool vec, hipStream_t s) {
   if (!vec || a.D > 4096) {
     hipLaunchKernelGGL(add_norm_any_kernel<T>, dim3((unsigned)a.rows), dim3(256), 0, s, a);
     return;
@@ -134,13 +221,20 @@ template <typename T> void launch_add_norm(const AddNormArgs& a, bool vec, hipSt
   const dim3 grid((unsigned)((a.rows + 3) / 4)), block(256);
   const int nv = (a.D + 511) / 512;
   if (nv <= 1)
-    hipLaunchKernelGGL((add_norm_kernel<T, 1>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((add_norm_kernel<T, 1, ADD>), grid, block, 0, s, a);
   else if (nv <= 2)
-    hipLaunchKernelGGL((add_norm_kernel<T, 2>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((add_norm_kernel<T, 2, ADD>), grid, block, 0, s, a);
   else if (nv <= 4)
-    hipLaunchKernelGGL((add_norm_kernel<T, 4>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((add_norm_kernel<T, 4, ADD>), grid, block, 0, s, a);
   else
-    hipLaunchKernelGGL((add_norm_kernel<T, 8>), grid, block, 0, s, a);
+    hipLaunchKernelGGL((add_norm_kernel<T, 8, ADD>), grid, block, 0, s, a);
+}
+
+template <typename T> void launch_add_norm(const AddNormArgs& a, bool vec, hipStream_t s) {
+  if (a.kind == kNormNone || a.add.post_w != nullptr || a.add.vec != nullptr || a.add.rows != nullptr)
+    launch_add_norm_rows<T, true>(a, vec, s);
+  else
+    launch_add_norm_rows<T, false>(a, vec, s);
 }
 
 struct StreamConvArgs {
@@ -262,27 +356,42 @@ template <typename T> void launch_stream_conv(const StreamConvArgs& a, int B, in
 
 }  // namespace based
 
-extern "C" BASED_API int based_add_norm(const void* x, const float* residual_in, const void* weight, void* y,
-                                        float* residual_out, int64_t rows, int64_t D, int64_t x_sr, int64_t ri_sr,
-                                        int64_t y_sr, int64_t ro_sr, float eps, int kind, float mult, int io_dtype,
-                                        void* stream) {
+extern "C" BASED_API int based_add_norm_addends(const void* x, const float* residual_in, const void* weight, void* y,
+                                                float* residual_out, int64_t rows, int64_t D, int64_t x_sr, int64_t ri_sr,
+                                                int64_t y_sr, int64_t ro_sr, float eps, int kind, float mult, const void* post_weight,
+                                                float post_eps, const void* add_vec, const void* add_rows, const int64_t* add_index,
+                                                int64_t add_sr, int64_t add_n, int io_dtype, void* stream) {
   using namespace based;
-  BASED_REQUIRE(x && weight && y, BASED_ERR_ARG, "add_norm: null pointer argument");
+  BASED_REQUIRE(x && y && (weight || kind == kNormNone), BASED_ERR_ARG, "add_norm: null pointer argument");
   BASED_REQUIRE(rows >= 0 && D > 0 && rows < (1ll << 31) && D < (1ll << 30), BASED_ERR_ARG, "add_norm: bad sizes");
-  BASED_REQUIRE(kind == kNormRms || kind == kNormLayer, BASED_ERR_ARG, "add_norm: unknown norm %d", kind);
+  BASED_REQUIRE(kind == kNormRms || kind == kNormLayer || kind == kNormNone, BASED_ERR_ARG, "add_norm: unknown norm %d", kind);
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "add_norm: bad dtype");
   BASED_REQUIRE(residual_in == nullptr || residual_out != residual_in, BASED_ERR_ARG,
                 "add_norm: residual_out must not be residual_in");
+  BASED_REQUIRE(add_rows == nullptr || add_n > 0, BASED_ERR_ARG, "add_norm: the added rows need their number");
+  BASED_REQUIRE(add_rows == nullptr || add_index != nullptr || add_n >= rows, BASED_ERR_ARG, "add_norm: too few rows to add");
   if (rows == 0) return BASED_OK;
-  const bool vec = D % 8 == 0 && x_sr % 8 == 0 && y_sr % 8 == 0 && ri_sr % 4 == 0 && ro_sr % 4 == 0 && aligned_to(x, 16) &&
-                   aligned_to(weight, 16) && aligned_to(y, 16) && aligned_to(residual_in, 16) && aligned_to(residual_out, 16);
-  const AddNormArgs a{x, residual_in, weight, y, residual_out, (long)rows, (int)D, x_sr, ri_sr, y_sr, ro_sr, eps, mult, kind};
+  const bool vec = D % 8 == 0 && x_sr % 8 == 0 && y_sr % 8 == 0 && ri_sr % 4 == 0 && ro_sr % 4 == 0 && add_sr % 8 == 0 &&
+                   aligned_to(x, 16) && aligned_to(weight, 16) && aligned_to(y, 16) && aligned_to(residual_in, 16) &&
+                   aligned_to(residual_out, 16) && aligned_to(post_weight, 16) && aligned_to(add_vec, 16) && aligned_to(add_rows, 16);
+  const AddNormArgs a{x,     residual_in, weight, y,   residual_out, (long)rows, (int)D, x_sr, ri_sr, y_sr, ro_sr, eps, mult, kind,
+                      {post_weight, add_vec, add_rows, add_index, add_sr, add_n, post_eps}};
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (io_dtype == BASED_BF16)
     launch_add_norm<__bf16>(a, vec, s);
   else
     launch_add_norm<float>(a, vec, s);
   return check_launch("add_norm");
+}
+
+extern "C" BASED_API int based_add_norm(const void* x, const float* residual_in, const void* weight, void* y,
+                                        float* residual_out, int64_t rows, int64_t D, int64_t x_sr, int64_t ri_sr,
+                                        int64_t y_sr, int64_t ro_sr, float eps, int kind, float mult, int io_dtype,
+                                        void* stream) {
+  using namespace based;
+  BASED_REQUIRE(kind == kNormRms || kind == kNormLayer, BASED_ERR_ARG, "add_norm: unknown norm %d", kind);
+  return based_add_norm_addends(x, residual_in, weight, y, residual_out, rows, D, x_sr, ri_sr, y_sr, ro_sr, eps, kind, mult, nullptr,
+                                0.f, nullptr, nullptr, nullptr, 0, 0, io_dtype, stream);
 }
 
 extern "C" BASED_API int based_stream_conv(const void* x, const void* weight, const void* bias, void* y, void* ring,

@@ -1,0 +1,310 @@
+// Token mixing in front of a time-mixing layer, the low-rank decay of its channels, and two element-wise
+// operations of a per-layer token input, for gfx950:
+//
+//   token_mix:      y_s,t = x_t + (x_{t-1} - x_t) * mu_s for several mixes s of the same input; the input
+//                   before a portion comes from a ring (B, 2, D), slot p % 2 holds position p.
+//   channel_decay:  log2 of exp(-exp(w2 tanh(h) + w0)) per channel, in fp32.
+//   gelu_mul:       gelu_tanh(g) * table[index], the gate of a per-token embedding.
+//   softcap:        cap * tanh(x / cap) in place.
+#include "stream_common.hpp"
+
+namespace based {
+
+struct TokenMixArgs {
+  const void* x;
+  const void* mu;  // (S, D)
+  void* y;         // (S, B, L, D)
+  void* ring;      // (B, 2, D) or null
+  const int32_t* pos;
+  int pos_host;
+  int B, L, D, S;
+  long x_sb, x_sl, ring_sb;
+};
+
+constexpr int kMixTile = 4;  // tokens per thread
+
+template <typename T, int N> __device__ __forceinline__ void load_some(const T* p, float (&out)[N]) {
+  if constexpr (N == 1)
+    out[0] = to_f32(*p);
+  else
+    load_vec<T, N>(p, out);
+}
+template <typename T, int N> __device__ __forceinline__ void store_some(T* p, const float (&in)[N]) {
+  if constexpr (N == 1)
+    *p = from_f32<T>(in[0]);
+  else
+    store_vec<T, N>(p, in);
+}
+
+// A thread owns N consecutive channels and walks kMixTile tokens.
+template <typename T, int N>
+__global__ __launch_bounds__(256) void token_mix_kernel(const TokenMixArgs a) {
+  const int c0 = (blockIdx.x * 256 + threadIdx.x) * N;
+  if (c0 >= a.D) return;
+  const int b = blockIdx.z, l0 = blockIdx.y * kMixTile;
+  const int start = row_pos(a.pos, a.pos_host, b);
+  if (start < 0) return;
+  const T* x = static_cast<const T*>(a.x) + b * a.x_sb + c0;
+  T* ring = a.ring != nullptr ? static_cast<T*>(a.ring) + b * a.ring_sb + c0 : nullptr;
+  const int ntok = a.L - l0 < kMixTile ? a.L - l0 : kMixTile;
+  float in[kMixTile][N], before[N];
+#pragma unroll
+  for (int t = 0; t < kMixTile; ++t) load_some<T, N>(x + (long)(l0 + (t < ntok ? t : ntok - 1)) * a.x_sl, in[t]);
+#pragma unroll
+  for (int c = 0; c < N; ++c) before[c] = 0.f;
+  if (l0 > 0)
+    load_some<T, N>(x + (long)(l0 - 1) * a.x_sl, before);
+  else if (ring != nullptr && start > 0)
+    load_some<T, N>(ring + (long)((start - 1) & 1) * a.D, before);
+  for (int s = 0; s < a.S; ++s) {
+    float mu[N];
+    load_some<T, N>(static_cast<const T*>(a.mu) + (long)s * a.D + c0, mu);
+    T* y = static_cast<T*>(a.y) + (((long)s * a.B + b) * a.L + l0) * a.D + c0;
+#pragma unroll
+    for (int t = 0; t < kMixTile; ++t)
+      if (t < ntok) {
+        float out[N];
+#pragma unroll
+        for (int c = 0; c < N; ++c) out[c] = __builtin_fmaf((t > 0 ? in[t > 0 ? t - 1 : 0][c] : before[c]) - in[t][c], mu[c], in[t][c]);
+        store_some<T, N>(y + (long)t * a.D, out);
+      }
+  }
+  // the portion's last input goes into the ring; the thread that has read the old one writes it
+  if (ring != nullptr && blockIdx.y == 0) {
+    float last[N];
+    load_some<T, N>(x + (long)(a.L - 1) * a.x_sl, last);
+    store_some<T, N>(ring + (long)((start + a.L - 1) & 1) * a.D, last);
+  }
+}
+
+// ---- log2 decay of every channel: -exp(w2 tanh(h) + w0) log2(e) ----
+struct ChannelDecayArgs {
+  const void* h;   // (rows, R)
+  const void* w2;  // (C, R)
+  const void* w0;  // (C)
+  float* y;        // (rows, C)
+  long rows, h_sr;
+  int C, R;
+};
+
+constexpr float kLog2e = 1.4426950408889634f;
+
+__device__ __forceinline__ float tanh_f(float z) {
+  // exp(2z) overflows to infinity and 1 - 0 is left; 2^-24 of the result below |z| = 0.05 comes from the series
+  const float e = expf(2.0f * z), q = z * z;
+  const float far = 1.0f - 2.0f / (e + 1.0f);
+  const float near = z * (1.0f - q * (1.0f / 3.0f - q * (2.0f / 15.0f)));
+  return fabsf(z) < 0.05f ? near : far;
+}
+
+constexpr int kDecayRows = 16;
+
+// Any element type and size: 16 rows of tanh(h) in LDS, a thread per channel.
+template <typename T>
+__global__ __launch_bounds__(256) void channel_decay_kernel(const ChannelDecayArgs a) {
+  extern __shared__ float th[];  // [kDecayRows][R]
+  const long r0 = (long)blockIdx.x * kDecayRows;
+  const int n = a.rows - r0 < kDecayRows ? (int)(a.rows - r0) : kDecayRows;
+  for (int i = threadIdx.x; i < n * a.R; i += 256)
+    th[i] = tanh_f(to_f32(static_cast<const T*>(a.h)[(r0 + i / a.R) * a.h_sr + i % a.R]));
+  __syncthreads();
+  const int c = blockIdx.y * 256 + threadIdx.x;
+  if (c >= a.C) return;
+  const T* w = static_cast<const T*>(a.w2) + (long)c * a.R;
+  const float w0 = to_f32(static_cast<const T*>(a.w0)[c]);
+  float acc[kDecayRows];
+#pragma unroll
+  for (int r = 0; r < kDecayRows; ++r) acc[r] = w0;
+  for (int j = 0; j < a.R; ++j) {
+    const float wj = to_f32(w[j]);
+#pragma unroll
+    for (int r = 0; r < kDecayRows; ++r) acc[r] = __builtin_fmaf(wj, th[(r < n ? r : 0) * a.R + j], acc[r]);
+  }
+#pragma unroll
+  for (int r = 0; r < kDecayRows; ++r)
+    if (r < n) a.y[(r0 + r) * a.C + c] = -expf(acc[r]) * kLog2e;
+}
+
+__device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+// bf16, R a multiple of 8 up to 256: 64 rows and 64 channels per workgroup.  tanh(h) enters as two bf16 numbers.
+template <int KC>
+__global__ __launch_bounds__(256) void channel_decay_mfma_kernel(const ChannelDecayArgs a) {
+  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, quad = lane >> 4;
+  const long row = (long)blockIdx.x * 64 + wave * 16 + l16;
+  const long rr = row < a.rows ? row : a.rows - 1;
+  const __bf16* h = static_cast<const __bf16*>(a.h) + rr * a.h_sr;
+  bf16x8 raw[KC], hi[KC], lo[KC];
+#pragma unroll
+  for (int k = 0; k < KC; ++k) {
+    const int e = k * 32 + quad * 8;
+    raw[k] = *reinterpret_cast<const bf16x8*>(h + (e < a.R ? e : 0));
+  }
+#pragma unroll
+  for (int k = 0; k < KC; ++k)
+#pragma unroll
+    for (int j = 0; j < 8; ++j) {
+      const float t = k * 32 + quad * 8 < a.R ? tanh_f(to_f32(raw[k][j])) : 0.f;
+      hi[k][j] = (__bf16)t;
+      lo[k][j] = (__bf16)(t - (float)hi[k][j]);
+    }
+#pragma unroll
+  for (int ct = 0; ct < 4; ++ct) {
+    const int c0 = blockIdx.y * 64 + ct * 16;
+    if (c0 >= a.C) break;
+    const int c = c0 + l16 < a.C ? c0 + l16 : a.C - 1;
+    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int k = 0; k < KC; ++k) {
+      const int e = k * 32 + quad * 8;
+      const bf16x8 w = *reinterpret_cast<const bf16x8*>(static_cast<const __bf16*>(a.w2) + (long)c * a.R + (e < a.R ? e : 0));
+      acc = mfma16(w, hi[k], acc);
+      acc = mfma16(w, lo[k], acc);
+    }
+    // lane: row l16 of the tile, channels quad * 4 + i
+    if (row < a.rows) {
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int ch = c0 + quad * 4 + i;
+        if (ch < a.C) a.y[row * a.C + ch] = -expf(acc[i] + to_f32(static_cast<const __bf16*>(a.w0)[ch])) * kLog2e;
+      }
+    }
+  }
+}
+
+// ---- gelu_tanh(g) * table[index] ----
+struct GeluMulArgs {
+  const void* g;
+  const void* table;
+  const int64_t* index;
+  void* y;
+  long rows, t_sr, t_n;
+  int n;
+  long g_sr;
+};
+
+template <typename T>
+__global__ __launch_bounds__(256) void gelu_mul_kernel(const GeluMulArgs a) {
+  const long i = (long)blockIdx.x * 256 + threadIdx.x;
+  if (i >= a.rows * a.n) return;
+  const long row = i / a.n;
+  const int c = (int)(i % a.n);
+  const long src = a.index[row];
+  const bool bad = src < 0 || src >= a.t_n;
+  const float e = to_f32(static_cast<const T*>(a.table)[(bad ? 0 : src) * a.t_sr + c]);
+  const float g = to_f32(static_cast<const T*>(a.g)[row * a.g_sr + c]);
+  static_cast<T*>(a.y)[i] = from_f32<T>(bad ? __builtin_nanf("") : gelu_tanh_f(g) * e);
+}
+
+template <typename T>
+__global__ __launch_bounds__(256) void softcap_kernel(T* x, long n, float cap) {
+  constexpr int N = Pack<T>::kN;
+  const long i0 = ((long)blockIdx.x * 256 + threadIdx.x) * N;
+  if (i0 + N <= n) {
+    float v[N];
+    load_vec<T, N>(x + i0, v);
+#pragma unroll
+    for (int j = 0; j < N; ++j) v[j] = cap * tanh_f(v[j] / cap);
+    store_vec<T, N>(x + i0, v);
+  } else {
+    for (long i = i0; i < n; ++i) x[i] = from_f32<T>(cap * tanh_f(to_f32(x[i]) / cap));
+  }
+}
+
+}  // namespace based
+
+extern "C" BASED_API int based_token_mix(const void* x, const void* mu, void* y, void* ring, const int32_t* pos, int64_t pos_host,
+                                         int64_t B, int64_t L, int64_t D, int64_t S, int64_t x_sb, int64_t x_sl, int64_t ring_sb,
+                                         int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x && mu && y, BASED_ERR_ARG, "token_mix: null pointer argument");
+  BASED_REQUIRE(B >= 0 && L >= 0 && D > 0 && S > 0 && pos_host >= 0 && pos_host + L < (1ll << 31), BASED_ERR_ARG, "token_mix: bad sizes");
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "token_mix: bad dtype");
+  BASED_REQUIRE(B < 65536 && (L + kMixTile - 1) / kMixTile < 65536 && D < (1ll << 28), BASED_ERR_SHAPE, "token_mix: grid too large");
+  if (B == 0 || L == 0) return BASED_OK;
+  const int n = io_dtype == BASED_BF16 ? 8 : 4;
+  const bool vec = D % n == 0 && x_sb % n == 0 && x_sl % n == 0 && ring_sb % n == 0 && aligned_to(x, 16) && aligned_to(mu, 16) &&
+                   aligned_to(y, 16) && aligned_to(ring, 16);
+  const TokenMixArgs a{x, mu, y, ring, pos, (int)pos_host, (int)B, (int)L, (int)D, (int)S, x_sb, x_sl, ring_sb};
+  const int per = vec ? n : 1;
+  const dim3 grid((unsigned)((D / per + 255) / 256), (unsigned)((L + kMixTile - 1) / kMixTile), (unsigned)B), block(256);
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16) {
+    if (vec)
+      hipLaunchKernelGGL((token_mix_kernel<__bf16, 8>), grid, block, 0, s, a);
+    else
+      hipLaunchKernelGGL((token_mix_kernel<__bf16, 1>), grid, block, 0, s, a);
+  } else {
+    if (vec)
+      hipLaunchKernelGGL((token_mix_kernel<float, 4>), grid, block, 0, s, a);
+    else
+      hipLaunchKernelGGL((token_mix_kernel<float, 1>), grid, block, 0, s, a);
+  }
+  return check_launch("token_mix");
+}
+
+extern "C" BASED_API int based_channel_decay(const void* h, const void* w2, const void* w0, float* y, int64_t rows, int64_t h_sr,
+                                             int64_t C, int64_t R, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(h && w2 && w0 && y, BASED_ERR_ARG, "channel_decay: null pointer argument");
+  BASED_REQUIRE(rows >= 0 && C > 0 && R > 0 && rows < (1ll << 31) && C < (1ll << 22), BASED_ERR_ARG, "channel_decay: bad sizes");
+  BASED_REQUIRE(R <= 1024, BASED_ERR_SHAPE, "channel_decay: rank %ld (at most 1024)", (long)R);
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "channel_decay: bad dtype");
+  if (rows == 0) return BASED_OK;
+  const ChannelDecayArgs a{h, w2, w0, y, (long)rows, (long)h_sr, (int)C, (int)R};
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16 && R % 8 == 0 && R <= 256 && h_sr % 8 == 0 && aligned_to(h, 16) && aligned_to(w2, 16)) {
+    const dim3 grid((unsigned)((rows + 63) / 64), (unsigned)((C + 63) / 64));
+    const int kc = (int)((R + 31) / 32);
+    if (kc <= 1)
+      hipLaunchKernelGGL((channel_decay_mfma_kernel<1>), grid, dim3(256), 0, s, a);
+    else if (kc <= 2)
+      hipLaunchKernelGGL((channel_decay_mfma_kernel<2>), grid, dim3(256), 0, s, a);
+    else if (kc <= 4)
+      hipLaunchKernelGGL((channel_decay_mfma_kernel<4>), grid, dim3(256), 0, s, a);
+    else
+      hipLaunchKernelGGL((channel_decay_mfma_kernel<8>), grid, dim3(256), 0, s, a);
+    return check_launch("channel_decay");
+  }
+  const dim3 grid((unsigned)((rows + kDecayRows - 1) / kDecayRows), (unsigned)((C + 255) / 256));
+  const size_t bytes = (size_t)kDecayRows * R * sizeof(float);
+  if (io_dtype == BASED_BF16)
+    hipLaunchKernelGGL(channel_decay_kernel<__bf16>, grid, dim3(256), bytes, s, a);
+  else
+    hipLaunchKernelGGL(channel_decay_kernel<float>, grid, dim3(256), bytes, s, a);
+  return check_launch("channel_decay");
+}
+
+extern "C" BASED_API int based_gelu_mul(const void* g, const void* table, const int64_t* index, void* y, int64_t rows, int64_t n,
+                                        int64_t g_sr, int64_t table_sr, int64_t table_n, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(g && table && index && y, BASED_ERR_ARG, "gelu_mul: null pointer argument");
+  BASED_REQUIRE(rows >= 0 && n > 0 && table_n > 0 && rows * n < (1ll << 38), BASED_ERR_ARG, "gelu_mul: bad sizes");
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "gelu_mul: bad dtype");
+  if (rows == 0) return BASED_OK;
+  const GeluMulArgs a{g, table, index, y, (long)rows, (long)table_sr, (long)table_n, (int)n, (long)g_sr};
+  const dim3 grid((unsigned)((rows * n + 255) / 256));
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  if (io_dtype == BASED_BF16)
+    hipLaunchKernelGGL(gelu_mul_kernel<__bf16>, grid, dim3(256), 0, s, a);
+  else
+    hipLaunchKernelGGL(gelu_mul_kernel<float>, grid, dim3(256), 0, s, a);
+  return check_launch("gelu_mul");
+}
+
+extern "C" BASED_API int based_softcap(void* x, int64_t n, float cap, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x, BASED_ERR_ARG, "softcap: null pointer argument");
+  BASED_REQUIRE(n >= 0 && n < (1ll << 38) && cap > 0.f, BASED_ERR_ARG, "softcap: bad sizes");
+  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "softcap: bad dtype");
+  BASED_REQUIRE(aligned_to(x, 16), BASED_ERR_ALIGN, "softcap: x must be 16-byte aligned");
+  if (n == 0) return BASED_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const int per = io_dtype == BASED_BF16 ? 8 : 4;
+  const dim3 grid((unsigned)((n + 256 * per - 1) / (256 * per)));
+  if (io_dtype == BASED_BF16)
+    hipLaunchKernelGGL(softcap_kernel<__bf16>, grid, dim3(256), 0, s, static_cast<__bf16*>(x), (long)n, cap);
+  else
+    hipLaunchKernelGGL(softcap_kernel<float>, grid, dim3(256), 0, s, static_cast<float*>(x), (long)n, cap);
+  return check_launch("softcap");
+}

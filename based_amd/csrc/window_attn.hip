@@ -1031,6 +1031,28 @@ static bool window_vec(const WindowArgs& a, int n) {
          aligned_to(a.q, 16) && aligned_to(a.k, 16) && aligned_to(a.v, 16) && aligned_to(a.kv, 16) && aligned_to(a.o, 16);
 }
 
+// The attention of a portion whose keys and values are in place.
+static void launch_window_attend(const WindowArgs& a, bool vec, int io_dtype, hipStream_t s) {
+  if (vec) {
+    const dim3 grid((unsigned)(((long)a.L * (a.H / a.G) + kTileRows - 1) / kTileRows), (unsigned)(a.B * a.G));
+    const int kc = (int)((a.d + 31) / 32);
+    if (kc <= 1)
+      launch_window_mfma<1>(a, grid, s);
+    else if (kc <= 2)
+      launch_window_mfma<2>(a, grid, s);
+    else if (kc <= 4)
+      launch_window_mfma<4>(a, grid, s);
+    else
+      launch_window_mfma<8>(a, grid, s);
+  } else {
+    const dim3 grid((unsigned)a.L, (unsigned)a.H, (unsigned)a.B);
+    if (io_dtype == BASED_BF16)
+      hipLaunchKernelGGL(window_prefill_any_kernel<__bf16>, grid, dim3(64), 0, s, a);
+    else
+      hipLaunchKernelGGL(window_prefill_any_kernel<float>, grid, dim3(64), 0, s, a);
+  }
+}
+
 }  // namespace based
 
 extern "C" BASED_API int based_window_attn_prefill(
@@ -1061,25 +1083,30 @@ extern "C" BASED_API int based_window_attn_prefill(
     hipLaunchKernelGGL(window_kv_write_kernel<__bf16>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
   else
     hipLaunchKernelGGL(window_kv_write_kernel<float>, dim3((unsigned)((items + 3) / 4)), dim3(256), 0, s, a);
-  if (vec) {
-    const dim3 grid((unsigned)((L * (H / G) + kTileRows - 1) / kTileRows), (unsigned)(B * G));
-    const int kc = (int)((D + 31) / 32);
-    if (kc <= 1)
-      launch_window_mfma<1>(a, grid, s);
-    else if (kc <= 2)
-      launch_window_mfma<2>(a, grid, s);
-    else if (kc <= 4)
-      launch_window_mfma<4>(a, grid, s);
-    else
-      launch_window_mfma<8>(a, grid, s);
-  } else {
-    const dim3 grid((unsigned)L, (unsigned)H, (unsigned)B);
-    if (io_dtype == BASED_BF16)
-      hipLaunchKernelGGL(window_prefill_any_kernel<__bf16>, grid, dim3(64), 0, s, a);
-    else
-      hipLaunchKernelGGL(window_prefill_any_kernel<float>, grid, dim3(64), 0, s, a);
-  }
+  launch_window_attend(a, vec, io_dtype, s);
   return check_launch("window_attn_prefill");
+}
+
+extern "C" BASED_API int based_window_attn_attend(const void* q, const void* kv, void* o, int64_t start, int64_t B, int64_t L, int64_t H,
+                                                  int64_t G, int64_t D, int64_t DV, int64_t S, int64_t q_sb, int64_t q_sl, int64_t o_sb,
+                                                  int64_t o_sl, int64_t kv_sb, int64_t kv_st, int64_t window, float scale,
+                                                  float out_scale, const float* rope_cos, const float* rope_sin, int64_t rope_len,
+                                                  int64_t rotary_dim, int half_split, int io_dtype, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(start >= 0 && start + L < (1ll << 31) && window < (1ll << 31) && L * H < (1ll << 31), BASED_ERR_SHAPE,
+                "window_attn_attend: sequence too long");
+  // k and v are not read: the rows are there already
+  const WindowArgs a{q,      q,      q,      const_cast<void*>(kv), o,       rope_cos, rope_sin, nullptr, (int)start, (int)rope_len,
+                     (int)B, (int)L, (int)H, (int)G,                (int)D,  (int)DV,  (int)S,   q_sb,    q_sl,       0,
+                     0,      0,      0,      o_sb,                  o_sl,    kv_sb,    kv_st,    (int)rotary_dim, half_split, (int)window,
+                     0,      scale,  0.f,    out_scale};
+  const int rc = window_check("window_attn_attend", a, rope_len, io_dtype, start + L - 1);
+  if (rc != BASED_OK) return rc;
+  BASED_REQUIRE(B * G < 65536 && B < 65536 && H < 65536, BASED_ERR_SHAPE, "window_attn_attend: grid too large");
+  if (B == 0 || L == 0) return BASED_OK;
+  const bool vec = io_dtype == BASED_BF16 && D <= 256 && DV <= 256 && rotary_dim % (half_split ? 16 : 8) == 0 && window_vec(a, 8);
+  launch_window_attend(a, vec, io_dtype, static_cast<hipStream_t>(stream));
+  return check_launch("window_attn_attend");
 }
 
 extern "C" BASED_API int based_window_attn_step(

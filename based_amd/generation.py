@@ -29,6 +29,11 @@ class InferenceParams:
     batch_size_offset: int = 0
     key_value_memory_dict: dict = field(default_factory=dict)
     lengths_per_sample: Optional[Tensor] = None
+    layer_pass: int = 0  # which pass of a layer that runs several times with the same weights is on
+
+    def layer_key(self, layer_idx):
+        """Where a layer's caches lie in key_value_memory_dict: every pass has its own."""
+        return layer_idx if self.layer_pass == 0 else (layer_idx, self.layer_pass)
 
     def reset(self, max_seqlen, max_batch_size):
         self.max_seqlen = max_seqlen

@@ -44,6 +44,7 @@ class ShortConvolution(nn.Module):
         be larger than the running batch; it is cleared whole)."""
         outer, inner = self.layer_idx if isinstance(self.layer_idx, tuple) else (self.layer_idx, None)
         d = inference_params.key_value_memory_dict
+        outer = inference_params.layer_key(outer)
         if inner is not None:
             d = d.setdefault(outer, {})
         key = outer if inner is None else inner
@@ -55,8 +56,8 @@ class ShortConvolution(nn.Module):
     def _get_state(self, inference_params):
         d = inference_params.key_value_memory_dict
         if isinstance(self.layer_idx, tuple):
-            return d[self.layer_idx[0]][self.layer_idx[1]]
-        return d[self.layer_idx]
+            return d[inference_params.layer_key(self.layer_idx[0])][self.layer_idx[1]]
+        return d[inference_params.layer_key(self.layer_idx)]
 
 
 class BaseConv(nn.Module):

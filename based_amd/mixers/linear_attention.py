@@ -128,9 +128,10 @@ class LinearAttention(nn.Module):
             y = self._cache_step(self._get_inference_cache(inference_params), q, k, v)
             return self.out_proj(y.transpose(1, 2).reshape(b, l, self.num_heads * self.head_dim))
         y, kv_state, k_state = self.parallel_forward(hidden_states, q, k, v)
-        if self.layer_idx in inference_params.key_value_memory_dict:
+        key = inference_params.layer_key(self.layer_idx)
+        if key in inference_params.key_value_memory_dict:
             # pre-allocated caches (graph-style decoding) are filled in place
-            cache = inference_params.key_value_memory_dict[self.layer_idx]
+            cache = inference_params.key_value_memory_dict[key]
             cache[0][:b].copy_(kv_state)
             cache[1][:b].copy_(k_state)
             if len(cache) > 2:
@@ -139,7 +140,7 @@ class LinearAttention(nn.Module):
             cache = (kv_state, k_state)
             if self.deferred_state_steps > 1:
                 cache += ops.deferred_step_buffers(b, self.num_heads, self.head_dim, kv_state.device)
-            inference_params.key_value_memory_dict[self.layer_idx] = cache
+            inference_params.key_value_memory_dict[key] = cache
         return y
 
     def _cache_step(self, cache, q, k, v):
@@ -258,4 +259,4 @@ class LinearAttention(nn.Module):
         return (kv_state, k_state)
 
     def _get_inference_cache(self, inference_params: InferenceParams):
-        return inference_params.key_value_memory_dict[self.layer_idx]
+        return inference_params.key_value_memory_dict[inference_params.layer_key(self.layer_idx)]

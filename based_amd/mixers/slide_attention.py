@@ -147,11 +147,11 @@ class SlidingAttention(nn.Module):
 
     def _cache(self, inference_params, like: torch.Tensor):
         assert self.layer_idx is not None, "Generation requires layer_idx in the constructor"
-        d = inference_params.key_value_memory_dict
-        if self.layer_idx not in d:
-            d[self.layer_idx] = torch.empty(inference_params.max_batch_size, inference_params.max_seqlen, 2,
+        d, key = inference_params.key_value_memory_dict, inference_params.layer_key(self.layer_idx)
+        if key not in d:
+            d[key] = torch.empty(inference_params.max_batch_size, inference_params.max_seqlen, 2,
                                             self.num_heads_kv, self.head_dim, dtype=torch.bfloat16, device=like.device)
-        return d[self.layer_idx]
+        return d[key]
 
     def supports_decode_step(self) -> bool:
         return ops.decode_linear_weight_ok(self.Wqkv.weight) and ops.decode_linear_weight_ok(self.out_proj.weight)

@@ -40,7 +40,7 @@ def portion_start(inference_params, batch: int, seqlen: int):
 
 def cached(inference_params, layer_idx, name: str, allocate, batch: int):
     """The rows of this batch of the tensor `name` of a layer, created for the largest batch when it is not there."""
-    store = inference_params.key_value_memory_dict.setdefault(layer_idx, {})
+    store = inference_params.key_value_memory_dict.setdefault(inference_params.layer_key(layer_idx), {})
     if name not in store:
         store[name] = allocate(inference_params.max_batch_size, inference_params.max_seqlen)
     b0 = inference_params.batch_size_offset

@@ -4,7 +4,7 @@ from __future__ import annotations
 
 import ctypes
 import math
-from typing import Optional, Tuple
+from typing import NamedTuple, Optional, Tuple
 
 import torch
 
@@ -707,8 +707,8 @@ def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residu
 # --------------------------------------------------------------------------------------------------
 # Streaming layers: portions of any length on caches, rings of past inputs and fp32 states
 # --------------------------------------------------------------------------------------------------
-NORM_RMS, NORM_LAYER = 0, 1
-ACT_NONE, ACT_SILU = 0, 1
+NORM_RMS, NORM_LAYER, NORM_NONE = 0, 1, 2
+ACT_NONE, ACT_SILU, ACT_SIGMOID = 0, 1, 2
 STREAM_MAX_TAPS = 8  # BASED_STREAM_MAX_TAPS
 DELTA_BLOCK, DELTA_PREP_FLOATS = 16, 592  # tokens per block of based_gated_delta_scan, BASED_DELTA_PREP_FLOATS
 RGLRU_SEGMENT = 64   # tokens per segment of based_rglru_prefill
@@ -746,16 +746,44 @@ def _check_ring(ring, rows: int, taps: int, channels: int, like) -> None:
         raise ValueError(f"ring must be ({rows}, {taps}, {channels}) {like.dtype} with contiguous slots, got {tuple(ring.shape)} {ring.dtype}")
 
 
+class Addends(NamedTuple):
+    """What a residual sum receives besides mult * x: x may first be divided by its own RMS and weighted (post_weight,
+    post_eps); a vector (D) for every row; a row of table (n, D) per row, index (rows) int64."""
+
+    post_weight: Optional[torch.Tensor] = None
+    post_eps: float = 0.0
+    vec: Optional[torch.Tensor] = None
+    table: Optional[torch.Tensor] = None
+    index: Optional[torch.Tensor] = None
+
+
+def _addend_args(addends: Addends, x, rows: int, D: int):
+    """(post_weight, post_eps, vec, table, index, table stride, table rows), checked."""
+    for t in (addends.post_weight, addends.vec):
+        if t is not None and (tuple(t.shape) != (D,) or not t.is_contiguous() or t.dtype != x.dtype or t.device != x.device):
+            raise ValueError(f"an added vector must be a contiguous ({D},) {x.dtype} on the device of x")
+    table, index = addends.table, addends.index
+    if table is not None:
+        if table.dim() != 2 or table.shape[1] != D or table.stride(1) != 1 or table.dtype != x.dtype or table.device != x.device:
+            raise ValueError(f"the table of added rows must be (n, {D}) {x.dtype} on the device of x")
+        if index is None or index.dtype != torch.int64 or index.numel() != rows or not index.is_contiguous() or index.device != x.device:
+            raise ValueError(f"the index of added rows must be {rows} contiguous int64 on the device of x")
+    return (_ptr(addends.post_weight), float(addends.post_eps), _ptr(addends.vec), _ptr(table), _ptr(index) if table is not None else None,
+            0 if table is None else table.stride(0), 0 if table is None else table.shape[0])
+
+
 def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: float = 1.0, want_residual: bool = True,
-             residual_out=None):
-    """r = residual + mult * x in fp32 (r = x without a residual); y = norm(r) * weight in x's dtype.
-    x: (..., D); residual fp32 of the same shape or None.  Returns (y, r), r None if not wanted
-    (written into residual_out, fp32 with contiguous rows and not `residual`, when given)."""
+             residual_out=None, addends: Optional[Addends] = None):
+    """r = residual + mult * x in fp32 (r = x without a residual), and what `addends` brings; y = norm(r) * weight in x's
+    dtype (NORM_NONE: r rounded, no weight).  x: (..., D); residual fp32 of the same shape or None.
+    Returns (y, r), r None if not wanted (written into residual_out, fp32 with contiguous rows and not `residual`, when given)."""
     D = x.shape[-1]
-    _require_cuda(x, weight)
-    _check_same_dtype(x, weight)
-    if tuple(weight.shape) != (D,) or not weight.is_contiguous():
-        raise ValueError(f"weight must be a contiguous ({D},), got {tuple(weight.shape)}")
+    _require_cuda(x)
+    if kind != NORM_NONE:
+        _require_cuda(x, weight)
+        _check_same_dtype(x, weight)
+        if tuple(weight.shape) != (D,) or not weight.is_contiguous():
+            raise ValueError(f"weight must be a contiguous ({D},), got {tuple(weight.shape)}")
     x2 = x.reshape(-1, D)
     if x2.stride(1) != 1:
         x2 = x2.contiguous()
@@ -775,11 +803,14 @@ def add_norm(x, residual, weight, eps: float, kind: int = NORM_LAYER, mult: floa
             raise ValueError("residual_out must be float32 with contiguous rows on the device of x")
     else:
         out = torch.empty(rows, D, dtype=torch.float32, device=x.device) if want_residual else None
+    args = (x2.data_ptr(), _ptr(r2), None if kind == NORM_NONE else weight.data_ptr(), y.data_ptr(), _ptr(out), rows, D, x2.stride(0),
+            0 if r2 is None else r2.stride(0), D, D if out is None else out.stride(0), float(eps), int(kind), float(mult))
     with _on_device(x.device):
-        _lib.check(_lib.lib().based_add_norm(x2.data_ptr(), _ptr(r2), weight.data_ptr(), y.data_ptr(), _ptr(out), rows, D,
-                                             x2.stride(0), 0 if r2 is None else r2.stride(0), D, D if out is None else out.stride(0),
-                                             float(eps), int(kind),
-                                             float(mult), _dtype_code(x), _stream_ptr(x)))
+        if addends is None and kind != NORM_NONE:
+            _lib.check(_lib.lib().based_add_norm(*args, _dtype_code(x), _stream_ptr(x)))
+        else:
+            _lib.check(_lib.lib().based_add_norm_addends(*args, *_addend_args(addends or Addends(), x, rows, D), _dtype_code(x),
+                                                         _stream_ptr(x)))
     return y.view(x.shape), None if out is None else out.view(x.shape)
 
 
@@ -991,6 +1022,283 @@ def rglru_step(x, y, conv_weight, conv_bias, ring, ra, rb, ri, ib, lam, state, d
             ri.data_ptr(), ib.data_ptr(), lam.data_ptr(), state.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B, W, blocks, taps,
             x.stride(0), y.stride(0), out.stride(0), ring.stride(0), float(decay_scale), _dtype_code(x), _stream_ptr(x)))
     return out
+
+
+def token_mix(x, mu, ring=None, pos=0) -> torch.Tensor:
+    """(S, B, L, D): x_t + (x_{t-1} - x_t) * mu_s of a portion x (B, L, D) that starts at `pos`; mu (S, D); ring (B, 2, D) or
+    None (nothing before the portion): read for the input before it, left with its last one."""
+    B, L, D = x.shape
+    _check_rows(x, mu)
+    _check_same_dtype(x, mu)
+    if mu.dim() != 2 or mu.shape[1] != D or not mu.is_contiguous():
+        raise ValueError(f"mu must be a contiguous (mixes, {D}), got {tuple(mu.shape)}")
+    if ring is not None:
+        _check_ring(ring, B, 2, D, x)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    y = torch.empty(mu.shape[0], B, L, D, dtype=x.dtype, device=x.device)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_token_mix(x.data_ptr(), mu.data_ptr(), y.data_ptr(), _ptr(ring), pos_ptr, pos_host, B, L, D, mu.shape[0],
+                                              x.stride(0), x.stride(1), 0 if ring is None else ring.stride(0), _dtype_code(x),
+                                              _stream_ptr(x)))
+    return y
+
+
+def channel_decay(hidden, w2, w0) -> torch.Tensor:
+    """log2 of exp(-exp(w2 tanh(hidden) + w0)): hidden (B, L, R) -> (B, L, C) fp32; w2 (C, R), w0 (C)."""
+    B, L, R = hidden.shape
+    _check_rows(hidden, w2)
+    _check_same_dtype(hidden, w2, w0)
+    C = w2.shape[0]
+    h2 = hidden.reshape(-1, R)
+    if tuple(w2.shape) != (C, R) or not w2.is_contiguous() or tuple(w0.shape) != (C,) or not w0.is_contiguous() or not w0.is_cuda:
+        raise ValueError(f"w2 {tuple(w2.shape)} and w0 {tuple(w0.shape)} must be contiguous (channels, {R}) and (channels,)")
+    y = torch.empty(B, L, C, dtype=torch.float32, device=hidden.device)
+    with _on_device(hidden.device):
+        _lib.check(_lib.lib().based_channel_decay(h2.data_ptr(), w2.data_ptr(), w0.data_ptr(), y.data_ptr(), B * L, h2.stride(0), C, R,
+                                                  _dtype_code(hidden), _stream_ptr(hidden)))
+    return y
+
+
+def gelu_mul(g, table, index) -> torch.Tensor:
+    """gelu_tanh(g) * table[index]: g (rows, n), table (entries, n) with rows at any stride, index (rows) int64."""
+    rows, n = g.shape
+    _check_rows(g, table)
+    _check_same_dtype(g, table)
+    if table.dim() != 2 or table.shape[1] != n or index.dtype != torch.int64 or index.numel() != rows or not index.is_contiguous() \
+            or not index.is_cuda:
+        raise ValueError(f"bad shapes g{tuple(g.shape)} table{tuple(table.shape)} index{tuple(index.shape)}")
+    y = torch.empty(rows, n, dtype=g.dtype, device=g.device)
+    with _on_device(g.device):
+        _lib.check(_lib.lib().based_gelu_mul(g.data_ptr(), table.data_ptr(), index.data_ptr(), y.data_ptr(), rows, n, g.stride(0),
+                                             table.stride(0), table.shape[0], _dtype_code(g), _stream_ptr(g)))
+    return y
+
+
+def softcap_(x, cap: float) -> torch.Tensor:
+    """x <- cap * tanh(x / cap), in place."""
+    _require_cuda(x)
+    if not x.is_contiguous():
+        raise ValueError("x must be contiguous")
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_softcap(x.data_ptr(), x.numel(), float(cap), _dtype_code(x), _stream_ptr(x)))
+    return x
+
+
+def _check_decay_state(state, rows: int, heads: int, d: int, dv: int) -> None:
+    if (state.dim() != 4 or tuple(state.shape[:3]) != (rows, heads, dv) or state.shape[3] < d or state.shape[3] % 4 != 0
+            or state.dtype != torch.float32 or not state.is_contiguous() or not state.is_cuda):
+        raise ValueError(f"state must be a contiguous float32 ({rows}, {heads}, {dv}, {d} rounded up to 4), got {tuple(state.shape)}")
+
+
+def head_decays(decay, device) -> torch.Tensor:
+    """(2, H) fp32 for the head form of decay_scan and decay_step: base-2 logarithms of the decays as fp32 holds them, and the decays.
+    A decay of zero is one whose powers are zero (0 * -inf would not be a number)."""
+    value = torch.tensor(list(decay), dtype=torch.float32)
+    log2 = torch.where(value > 0, value.double().log2(), torch.full_like(value, -1e4).double()).float()
+    return torch.stack([log2, value]).to(device)
+
+
+def _check_head_decay(head_decay, heads: int, device) -> None:
+    if head_decay.dtype != torch.float32 or tuple(head_decay.shape) != (2, heads) or head_decay.device != device \
+            or not head_decay.is_contiguous():
+        raise ValueError(f"head_decay must be a contiguous float32 (2, {heads}) on the device of q (head_decays)")
+
+
+def decay_scan(q, k, v, state, heads: int, *, channel_log2=None, bonus=None, head_decay=None, activation: int = ACT_NONE,
+               fresh: bool) -> torch.Tensor:
+    """Linear attention with decaying states over a portion: q, k (B, L, H * d), v (B, L, H * dv) -> o (B, L, H * dv); state (B, H, dv,
+    d rounded up to 4) fp32, updated in place, taken as zero when `fresh`.  channel_log2 (B, L, H * d) fp32 with bonus (H, d):
+    o_t = (S + diag(u) k v^T)^T q, S <- diag(w) S + k v^T; head_decay (2, H) of `head_decays`: S <- w S + k v^T, o = S^T q."""
+    _check_rows(q, k, v)
+    _check_same_dtype(q, k, v, bonus)
+    B, L = q.shape[:2]
+    d, dv = q.shape[-1] // heads, v.shape[-1] // heads
+    if q.shape != k.shape or tuple(q.shape) != (B, L, heads * d) or tuple(v.shape) != (B, L, heads * dv):
+        raise ValueError(f"bad shapes q{tuple(q.shape)} k{tuple(k.shape)} v{tuple(v.shape)}")
+    _check_decay_state(state, B, heads, d, dv)
+    if channel_log2 is not None:
+        if tuple(channel_log2.shape) != (B, L, heads * d) or channel_log2.dtype != torch.float32 or not channel_log2.is_contiguous() \
+                or bonus is None or tuple(bonus.shape) != (heads, d) or not bonus.is_contiguous():
+            raise ValueError(f"channel decays must be contiguous float32 ({B}, {L}, {heads * d}) with a bonus ({heads}, {d})")
+        _require_cuda(q, channel_log2, bonus)
+    else:
+        _check_head_decay(head_decay, heads, q.device)
+    lib = _lib.lib()
+    work = None
+    if q.dtype == torch.bfloat16:
+        n = lib.based_decay_scan_work(B, L, heads, d, dv, state.shape[3])
+        work = torch.empty(n, dtype=torch.float32, device=q.device) if n else None
+    o = torch.empty(B, L, heads * dv, dtype=q.dtype, device=q.device)
+    with _on_device(q.device):
+        _lib.check(lib.based_decay_scan(
+            q.data_ptr(), k.data_ptr(), v.data_ptr(), _ptr(channel_log2), _ptr(head_decay), _ptr(bonus), state.data_ptr(), _ptr(work),
+            o.data_ptr(), B, L, heads, d, dv, state.shape[3], q.stride(0), q.stride(1), k.stride(0), k.stride(1), v.stride(0), v.stride(1),
+            o.stride(0), o.stride(1), int(activation), int(fresh), _dtype_code(q), _stream_ptr(q)))
+    return o
+
+
+def decay_step(q, k, v, state, heads: int, pos, *, head_decay=None, bonus=None, hidden=None, w2=None, w0=None, gate=None, norm_weight=None,
+               eps: float = 0.0, activation: int = ACT_NONE, out) -> torch.Tensor:
+    """One token of it: q, k (B, H * d), v, out (B, H * dv).  With head_decay the head form; with `hidden` (B, R), w2 (H * d, R), w0 (H * d),
+    bonus (H, d) the channel form, its output divided by its RMS per head, times norm_weight (H * dv) and silu(gate) (B, H * dv)."""
+    _check_rows(q, k, v, out)
+    _check_same_dtype(q, k, v, out, bonus, hidden, w2, w0, gate, norm_weight)
+    B = q.shape[0]
+    d, dv = q.shape[-1] // heads, v.shape[-1] // heads
+    if q.shape != k.shape or tuple(q.shape) != (B, heads * d) or tuple(v.shape) != (B, heads * dv) or out.shape != v.shape:
+        raise ValueError(f"bad shapes q{tuple(q.shape)} k{tuple(k.shape)} v{tuple(v.shape)} out{tuple(out.shape)}")
+    _check_decay_state(state, B, heads, d, dv)
+    R = 0
+    if hidden is not None:
+        _check_rows(hidden, gate)
+        R = hidden.shape[-1]
+        if (tuple(hidden.shape) != (B, R) or tuple(w2.shape) != (heads * d, R) or w0.numel() != heads * d or bonus.numel() != heads * d
+                or tuple(gate.shape) != (B, heads * dv) or norm_weight.numel() != heads * dv):
+            raise ValueError("bad shapes of the decay's or the output's parameters")
+        for t in (w2, w0, bonus, norm_weight):
+            if not t.is_contiguous() or not t.is_cuda:
+                raise ValueError("parameters must be contiguous device tensors")
+    else:
+        _check_head_decay(head_decay, heads, q.device)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    with _on_device(q.device):
+        _lib.check(_lib.lib().based_decay_step(
+            q.data_ptr(), k.data_ptr(), v.data_ptr(), _ptr(head_decay), _ptr(bonus), _ptr(hidden), _ptr(w2), _ptr(w0), _ptr(gate),
+            _ptr(norm_weight), state.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B, heads, d, dv, state.shape[3], R, q.stride(0),
+            k.stride(0), v.stride(0), 0 if hidden is None else hidden.stride(0), 0 if gate is None else gate.stride(0), out.stride(0),
+            int(activation), float(eps), _dtype_code(q), _stream_ptr(q)))
+    return out
+
+
+def group_norm_gate(o, weight, gate, groups: int, eps: float, activation: int, scale: float = 1.0, *, out) -> torch.Tensor:
+    """out = o / sqrt(mean(o^2) + eps) * weight * act(gate) * scale over each of `groups` parts of a row; o, gate, out (B, L, groups * n),
+    weight (groups * n); ACT_SILU or ACT_SIGMOID."""
+    B, L, W = o.shape
+    _check_rows(o, gate, out)
+    _check_same_dtype(o, gate, out, weight)
+    if gate.shape != o.shape or out.shape != o.shape or weight.numel() != W or W % groups != 0 or not weight.is_contiguous():
+        raise ValueError(f"bad shapes o{tuple(o.shape)} gate{tuple(gate.shape)} out{tuple(out.shape)} weight{tuple(weight.shape)}")
+    with _on_device(o.device):
+        _lib.check(_lib.lib().based_group_norm_gate(o.data_ptr(), weight.data_ptr(), gate.data_ptr(), out.data_ptr(), B, L, groups, W // groups,
+                                                    o.stride(0), o.stride(1), gate.stride(0), gate.stride(1), out.stride(0), out.stride(1),
+                                                    float(eps), float(scale), int(activation), _dtype_code(o), _stream_ptr(o)))
+    return out
+
+
+def window_attn_attend(q, kv, heads: int, kv_heads: int, dim: int, window: int, scale: float, start: int = 0, rope=None,
+                       out_scale: float = 1.0, *, out):
+    """window_attn_prefill on rows that kv (B, S, G, d + dv) already holds: only q (B, L, H * d) is rotated."""
+    _check_rows(q, kv, out)
+    _check_same_dtype(q, kv, out)
+    B, L = q.shape[:2]
+    dv = out.shape[-1] // heads
+    if (tuple(q.shape) != (B, L, heads * dim) or tuple(out.shape) != (B, L, heads * dv) or kv.dim() != 4 or kv.shape[0] != B
+            or tuple(kv.shape[2:]) != (kv_heads, dim + dv) or kv.stride(2) != dim + dv):
+        raise ValueError(f"bad shapes q{tuple(q.shape)} kv{tuple(kv.shape)} out{tuple(out.shape)}")
+    cos_ptr, sin_ptr, n_pos, rot, half = _stream_rope(rope, q.device)
+    with _on_device(q.device):
+        _lib.check(_lib.lib().based_window_attn_attend(
+            q.data_ptr(), kv.data_ptr(), out.data_ptr(), int(start), B, L, heads, kv_heads, dim, dv, kv.shape[1], q.stride(0), q.stride(1),
+            out.stride(0), out.stride(1), kv.stride(0), kv.stride(1), int(window), float(scale), float(out_scale), cos_ptr, sin_ptr, n_pos,
+            rot, half, _dtype_code(q), _stream_ptr(q)))
+    return out
+
+
+def _latent_rows(x, norm_weight, cache, rope):
+    """Latent and rotated sizes of x (..., R + rot) and cache (B, S, R + rot), checked."""
+    _check_rows(x, cache)
+    _check_same_dtype(x, cache, norm_weight)
+    R, W = norm_weight.numel(), x.shape[-1]
+    cos_ptr, sin_ptr, n_pos, rot, half = _stream_rope(rope, x.device)
+    if R + rot != W or cache.dim() != 3 or cache.shape[0] != x.shape[0] or cache.shape[2] != W or not norm_weight.is_contiguous():
+        raise ValueError(f"bad shapes x{tuple(x.shape)} cache{tuple(cache.shape)} norm{tuple(norm_weight.shape)}, rotary size {rot}")
+    return R, rot, cos_ptr, sin_ptr, n_pos, half
+
+
+def latent_write(x, norm_weight, cache, start: int, eps: float, rope) -> None:
+    """Rows start .. start + L - 1 of a latent cache (B, S, R + rot) from x (B, L, R + rot): the first R channels divided by their RMS
+    and weighted, the others rotated."""
+    R, rot, cos_ptr, sin_ptr, n_pos, half = _latent_rows(x, norm_weight, cache, rope)
+    B, L = x.shape[:2]
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_latent_write(x.data_ptr(), norm_weight.data_ptr(), cache.data_ptr(), int(start), B, L, cache.shape[1], R, rot,
+                                                 x.stride(0), x.stride(1), cache.stride(0), cache.stride(1), float(eps), cos_ptr, sin_ptr,
+                                                 n_pos, half, _dtype_code(x), _stream_ptr(x)))
+
+
+LATENT_STEP_TARGET = 512  # workgroups that the keys of a step are dealt to, where there are enough
+
+
+def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: int, scale: float, pos, eps: float, rope,
+                out_scale: float = 1.0, *, out) -> torch.Tensor:
+    """One token per sequence on a latent cache: q (B, H * (rot + d)) with a head's rotated channels first, x (B, R + rot) the token's own
+    row before norm and rotation, weight (H * (rot + d + dv), >= R): of each head rot rows that are not read, uk, uv.
+    Written, times out_scale, into out (B, H * dv)."""
+    R, rot, cos_ptr, sin_ptr, n_pos, half = _latent_rows(x, norm_weight, cache, rope)
+    _check_rows(q, weight, out)
+    _check_same_dtype(x, q, weight, out)
+    B, S = x.shape[0], cache.shape[1]
+    dv = out.shape[-1] // heads
+    if tuple(q.shape) != (B, heads * (rot + dim)) or tuple(out.shape) != (B, heads * dv) or weight.shape[0] != heads * (rot + dim + dv) \
+            or weight.shape[1] < R:
+        raise ValueError(f"bad shapes q{tuple(q.shape)} weight{tuple(weight.shape)} out{tuple(out.shape)}")
+    groups = B * ((heads + 15) // 16)
+    splits = max(1, min(LATENT_STEP_TARGET // groups, (min(window, S) + 127) // 128))
+    f32 = dict(dtype=torch.float32, device=x.device)
+    work_q = torch.empty(B, heads, R + rot, **f32)
+    part, part_ml = torch.empty(B, splits, heads, R, **f32), torch.empty(B, splits, heads, 2, **f32)
+    pos_ptr, pos_host = _pos_args(pos, B)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_latent_step(
+            q.data_ptr(), x.data_ptr(), norm_weight.data_ptr(), weight.data_ptr(), cache.data_ptr(), work_q.data_ptr(), part.data_ptr(),
+            part_ml.data_ptr(), out.data_ptr(), pos_ptr, pos_host, B, heads, dim, dv, S, R, rot, splits, q.stride(0), x.stride(0),
+            weight.stride(0), cache.stride(0), cache.stride(1), out.stride(0), int(window), float(scale), float(eps), float(out_scale),
+            cos_ptr, sin_ptr, n_pos, half, _dtype_code(x), _stream_ptr(x)))
+    return out
+
+
+# Choices up to which experts are evaluated one choice at a time: beyond, rows of one expert share its matrices.
+EXPERT_ROWS_MAX = 128
+
+
+def experts(h, router, w1, w2, top: int) -> torch.Tensor:
+    """y = sum over the `top` experts of a token with the largest sigmoid(router h) of w2_e (silu(gate) * up), [up; gate] = score * w1_e h.
+    h (..., D), router (E, D), w1 (E, 2 F, D) up rows first, w2 (E, D, F)."""
+    D = h.shape[-1]
+    E, F = w2.shape[0], w2.shape[2]
+    h2 = h.reshape(-1, D)
+    _check_rows(h2, router, w1, w2)
+    _check_same_dtype(h2, router, w1, w2)
+    if tuple(router.shape) != (E, D) or tuple(w1.shape) != (E, 2 * F, D) or tuple(w2.shape) != (E, D, F):
+        raise ValueError(f"bad shapes router{tuple(router.shape)} w1{tuple(w1.shape)} w2{tuple(w2.shape)}")
+    if not (router.is_contiguous() and w1.is_contiguous() and w2.is_contiguous()):
+        raise ValueError("expert weights must be contiguous")
+    if not 1 <= top <= E:
+        raise ValueError(f"{top} of {E} experts")
+    n, dev = h2.shape[0], h2.device
+    lib = _lib.lib()
+    grouped = h2.dtype == torch.bfloat16 and n * top > EXPERT_ROWS_MAX and D % 8 == 0 and F % 8 == 0 and h2.stride(0) % 8 == 0
+    i32 = dict(dtype=torch.int32, device=dev)
+    ids, scores = torch.empty(n, top, **i32), torch.empty(n, top, dtype=torch.float32, device=dev)
+    rank, counts = (torch.empty(n, top, **i32), torch.zeros(E, **i32)) if grouped else (None, None)
+    y = torch.empty(n, D, dtype=h2.dtype, device=dev)
+    with _on_device(dev):
+        _lib.check(lib.based_expert_route(h2.data_ptr(), router.data_ptr(), ids.data_ptr(), scores.data_ptr(), _ptr(rank), _ptr(counts), n, D, E,
+                                          top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
+        if grouped:
+            tiles, rows = lib.based_expert_tiles(n, E, top), lib.based_expert_tile_rows(n, E, top)
+            plan = torch.empty(E + 1 + tiles + tiles * rows, **i32)
+            act = torch.empty(tiles * rows, F, dtype=h2.dtype, device=dev)
+            part = torch.empty(n * top, D, dtype=h2.dtype, device=dev) if top > 1 else None
+            _lib.check(lib.based_expert_grouped(
+                h2.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(), rank.data_ptr(), counts.data_ptr(), plan.data_ptr(),
+                plan[E + 1:].data_ptr(), plan[E + 1 + tiles:].data_ptr(), act.data_ptr(), _ptr(part), y.data_ptr(), n, D, F, E, top,
+                h2.stride(0), _stream_ptr(h2)))
+        else:
+            act = torch.empty(n * top, F, dtype=h2.dtype, device=dev)
+            _lib.check(lib.based_expert_rows(h2.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(), act.data_ptr(),
+                                             y.data_ptr(), n, D, F, top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
+    return y.view(h.shape)
 
 
 # Rows up to which the streamed-input prologue is evaluated inside the projection.  Every workgroup of it

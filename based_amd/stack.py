@@ -14,7 +14,7 @@ import math
 from collections import namedtuple
 from functools import partial
 from types import SimpleNamespace
-from typing import Optional
+from typing import NamedTuple, Optional
 
 import torch
 import torch.nn as nn
@@ -24,12 +24,15 @@ from . import ops
 
 from .generation import GenerationMixin
 from .mixers.convolution import BaseConv, ShortConvolution
+from .mixers.decay_attention import DecayAttention
 from .mixers.gated_delta import GatedDeltaRule
+from .mixers.latent_attention import LatentAttention
 from .mixers.linear_attention import LinearAttention, TaylorExp
 from .mixers.rglru import RGLRU
 from .mixers.side_by_side import SideBySide
 from .mixers.slide_attention import SlidingAttention
-from .mixers.streaming import StreamConv, portion_start
+from .mixers.streaming import StreamConv, portion_start, round_up
+from .mixers.time_mix import TimeMix
 from .mixers.window_attention import WindowAttention
 
 # `_target_` strings accepted in mixer config dicts: the reference's own paths and this package's.
@@ -44,9 +47,12 @@ _TARGETS = {
     "based_amd.mixers.slide_attention.SlidingAttention": SlidingAttention,
     "based_amd.mixers.convolution.BaseConv": BaseConv,
     "based_amd.mixers.convolution.ShortConvolution": ShortConvolution,
+    "based_amd.mixers.decay_attention.DecayAttention": DecayAttention,
     "based_amd.mixers.gated_delta.GatedDeltaRule": GatedDeltaRule,
+    "based_amd.mixers.latent_attention.LatentAttention": LatentAttention,
     "based_amd.mixers.rglru.RGLRU": RGLRU,
     "based_amd.mixers.side_by_side.SideBySide": SideBySide,
+    "based_amd.mixers.time_mix.TimeMix": TimeMix,
     "based_amd.mixers.window_attention.WindowAttention": WindowAttention,
 }
 
@@ -82,11 +88,16 @@ class StackConfig(SimpleNamespace):
             qkv_proj_bias=False, out_proj_bias=False, rotary_emb_fraction=0.0, rotary_emb_base=10000.0,
             rotary_emb_interleaved=False, scale_attn_weights=True, max_position_embeddings=0,
             mixer=None, alt_mixer=None, alt_mixer_layers=None, alt_mixer_2=None, alt_mixer_2_layers=None,
-            # Streamed designs.  layer_specs: one {"mixer": spec, "mlp": {"hidden": n} or None} per layer
-            # instead of the mixer / alt_mixer routing; stream_norm: "layer" or "rms" without a bias on the
-            # fp32 residual sum; residual_mult: factor of every sublayer's output; input_conv_taps: causal
-            # convolution added to what a mixer reads (0: none).
-            layer_specs=None, stream_norm=None, residual_mult=1.0, input_conv_taps=0,
+            # Streamed designs.  layer_specs: one {"mixer": spec, "mlp": spec} per layer instead of the mixer /
+            # alt_mixer routing, the feed-forward None, {"hidden": n} or {"hidden": n, "experts": e, "top": k};
+            # stream_norm: "layer" or "rms" without a bias on the fp32 residual sum; residual_mult: factor of
+            # every sublayer's output; input_conv_taps: causal convolution added to what a mixer reads (0: none).
+            # loop: {"start": i, "stop": j, "times": n}: layers i .. j - 1 run n times in a row with the same
+            # weights and caches of their own, a learned vector per pass (and, from the second on, the embedding)
+            # added before each; token_side_dim: size of the token input that every layer adds behind its
+            # feed-forward (0: none); logit_softcap: c tanh(logits / c).
+            layer_specs=None, stream_norm=None, residual_mult=1.0, input_conv_taps=0, loop=None, token_side_dim=0,
+            logit_softcap=None,
         )
         defaults.update(kw)
         super().__init__(**defaults)
@@ -251,13 +262,16 @@ def norm_fuses(norm) -> bool:
     return isinstance(norm, (RMSNorm, StreamNorm)) and norm.weight.dtype == torch.bfloat16
 
 
-def add_norm(norm, hidden_states, residual, residual_in_fp32: bool, want_residual: bool = True):
+def add_norm(norm, hidden_states, residual, residual_in_fp32: bool, want_residual: bool = True, addends=None):
     """residual + hidden, the norm of the sum, and the sum itself for the next block
     (block.py:134-139; gpt.py:676-694 for the closing norm).  RMSNorm on tensors the kernel takes
     is one launch; nn.LayerNorm (`rms_norm: False`, the reference's default) and everything the
-    kernel refuses run the reference's own torch statement."""
+    kernel refuses run the reference's own torch statement.  addends (`ops.Addends`): what else the sum of a
+    StreamNorm receives."""
     if isinstance(norm, StreamNorm):
-        return ops.add_norm(hidden_states, residual, norm.weight, norm.eps, norm.kind, norm.mult, want_residual)
+        return ops.add_norm(hidden_states, residual, norm.weight, norm.eps, norm.kind, norm.mult, want_residual, addends=addends)
+    if addends is not None:
+        raise NotImplementedError("only a StreamNorm takes addends")
     if isinstance(norm, RMSNorm) and _norm_kernel_takes(hidden_states, residual, norm.weight):
         if residual is None:
             return ops.add_rms_norm(hidden_states, None, norm.weight, norm.eps, residual_in_fp32, want_residual)
@@ -311,12 +325,60 @@ class GatedMlp(nn.Module):
         return self.fc2(y * _GATE_ACTIVATIONS[self.activation](gate))
 
 
+class ExpertMlp(nn.Module):
+    """Mixture of gated feed-forwards with sigmoid routing (`ops.experts`): of `experts` of them a token takes the `top` with the largest
+    scores, each of which multiplies its expert's input."""
+
+    def __init__(self, in_features, hidden_features, experts, top, device=None, dtype=None):
+        super().__init__()
+        fk = {"device": device, "dtype": dtype}
+        if not 1 <= top <= experts:
+            raise ValueError(f"{top} of {experts} experts")
+        # hidden sizes are rounded up to 16-byte pieces; the extra ones carry zero weights
+        hidden = round_up(hidden_features)
+        self.top = top
+        self.router = nn.Parameter(torch.empty(experts, in_features, **fk).normal_(std=in_features ** -0.5))
+        self.w1 = nn.Parameter(torch.empty(experts, 2 * hidden, in_features, **fk).normal_(std=0.02))
+        self.w2 = nn.Parameter(torch.empty(experts, in_features, hidden, **fk).normal_(std=0.02))
+
+    def forward(self, x):
+        return ops.experts(x, self.router, self.w1, self.w2, self.top)
+
+
+class TokenSide(nn.Module):
+    """A layer's own token input, added to the residual stream x behind the feed-forward:
+    norm(proj(gelu_tanh(gate x) * e)), e the layer's columns of a table by token.  The norm is taken where the next
+    layer's sum is formed (`out_addends`)."""
+
+    def __init__(self, d_model, dim, layer_idx, eps, device=None, dtype=None):
+        super().__init__()
+        fk = {"device": device, "dtype": dtype}
+        self.dim, self.first = dim, layer_idx * dim
+        self.gate = nn.Linear(d_model, dim, bias=False, **fk)
+        self.proj = nn.Linear(dim, d_model, bias=False, **fk)
+        self.norm = StreamNorm(d_model, eps=eps, kind="rms", **fk)
+
+    def table(self, side_table):
+        return side_table[:, self.first:self.first + self.dim]
+
+    def out_addends(self):
+        return ops.Addends(post_weight=self.norm.weight, post_eps=self.norm.eps)
+
+    def forward(self, hidden_states, residual, mult, ids, side_table):
+        """(what proj gives, the residual stream with hidden_states in it)."""
+        x, residual = ops.add_norm(hidden_states, residual, None, 0.0, ops.NORM_NONE, mult)
+        g = self.gate(x)
+        g = ops.gelu_mul(g.reshape(-1, self.dim), self.table(side_table), ids.reshape(-1)).view(g.shape)
+        return self.proj(g), residual
+
+
 class Block(nn.Module):
     """Prenorm block: add -> norm1 -> mixer -> add -> norm2 -> mlp, returning (hidden, residual)
     (block.py:134-163, dropout-free).  mlp_cls None: the mixer alone.  input_conv_cls: a causal
-    convolution between norm1 and the mixer whose output is added to its input."""
+    convolution between norm1 and the mixer whose output is added to its input.  side_cls: a token input
+    behind the feed-forward; what the next sum then does with `hidden` says `out_addends`."""
 
-    def __init__(self, dim, mixer_cls, mlp_cls, norm_cls, residual_in_fp32=True, layer_idx=None, input_conv_cls=None):
+    def __init__(self, dim, mixer_cls, mlp_cls, norm_cls, residual_in_fp32=True, layer_idx=None, input_conv_cls=None, side_cls=None):
         super().__init__()
         self.residual_in_fp32 = residual_in_fp32
         self.layer_idx = layer_idx
@@ -325,6 +387,11 @@ class Block(nn.Module):
         self.input_conv = None if input_conv_cls is None else input_conv_cls(dim, layer_idx=layer_idx)
         self.mlp = None if mlp_cls is None else mlp_cls(dim)
         self.norm2 = None if mlp_cls is None else norm_cls(dim)
+        self.side = None if side_cls is None else side_cls(dim, layer_idx=layer_idx)
+
+    def out_addends(self):
+        """How the sum behind this block takes its hidden states (None: as they are)."""
+        return None if self.side is None else self.side.out_addends()
 
     def allocate_inference_cache(self, batch_size, max_seqlen, dtype=None, **kwargs):
         cache = self.mixer.allocate_inference_cache(batch_size, max_seqlen, dtype=dtype, **kwargs)
@@ -332,13 +399,15 @@ class Block(nn.Module):
             cache[self.input_conv.name] = self.input_conv.allocate_ring(batch_size)
         return cache
 
-    def _add_norm(self, norm, hidden_states, residual):
+    def _add_norm(self, norm, hidden_states, residual, addends=None):
         """residual + hidden, the norm of the sum, and the sum kept for the next block
         (block.py:134-139)."""
-        return add_norm(norm, hidden_states, residual, self.residual_in_fp32)
+        return add_norm(norm, hidden_states, residual, self.residual_in_fp32, addends=addends)
 
     def supports_decode_step(self) -> bool:
         mlp = self.mlp
+        if self.side is not None or isinstance(mlp, ExpertMlp):
+            return False
         return (getattr(self.mixer, "supports_decode_step", lambda: False)()
                 and (mlp is None or (mlp.mlp_type == "base" and mlp.activation == "swiglu"
                                      and ops.decode_linear_weight_ok(mlp.fc1.weight)
@@ -377,8 +446,9 @@ class Block(nn.Module):
             hidden_states = ops.decode_linear(gate_in, fc2.weight, fc2.bias, prologue=ops.PROLOGUE_SWIGLU)
         return hidden_states, last, mid
 
-    def forward(self, hidden_states, residual=None, mixer_kwargs=None, position_ids=None, decay=None):
-        hidden_states, residual = self._add_norm(self.norm1, hidden_states, residual)
+    def forward(self, hidden_states, residual=None, mixer_kwargs=None, position_ids=None, decay=None, addends=None, ids=None,
+                side_table=None):
+        hidden_states, residual = self._add_norm(self.norm1, hidden_states, residual, addends)
         mixer_kwargs = mixer_kwargs or {}
         if self.input_conv is not None:
             hidden_states = self.input_conv(hidden_states, mixer_kwargs.get("inference_params"))
@@ -386,10 +456,12 @@ class Block(nn.Module):
             hidden_states = self.mixer(hidden_states, position_ids=position_ids, decay=decay, **mixer_kwargs)
         else:
             hidden_states = self.mixer(hidden_states, **mixer_kwargs)
-        if self.mlp is None:
-            return hidden_states, residual
-        hidden_states, residual = self._add_norm(self.norm2, hidden_states, residual)
-        return self.mlp(hidden_states), residual
+        if self.mlp is not None:
+            hidden_states, residual = self._add_norm(self.norm2, hidden_states, residual)
+            hidden_states = self.mlp(hidden_states)
+        if self.side is not None:
+            hidden_states, residual = self.side(hidden_states, residual, self.norm1.mult, ids, side_table)
+        return hidden_states, residual
 
 
 def _init_weights(module, n_layer, initializer_range=0.02):
@@ -402,6 +474,23 @@ def _init_weights(module, n_layer, initializer_range=0.02):
     for name, p in module.named_parameters():
         if name in ["out_proj.weight", "fc2.weight"]:
             nn.init.normal_(p, mean=0.0, std=initializer_range / math.sqrt(2 * n_layer))
+
+
+class LayerRun(NamedTuple):
+    """One run of a layer: which, in which pass of the loop, and whether the pass starts with it."""
+
+    layer: int
+    layer_pass: int
+    starts_pass: bool
+
+
+def layer_runs(n_layer: int, loop: Optional[dict]):
+    """The layers in the order they run; those of the loop once per pass."""
+    start, stop, times = (loop["start"], loop["stop"], loop["times"]) if loop else (0, 0, 1)
+    if not (0 <= start <= stop <= n_layer and times >= 1) or (loop and start == stop):
+        raise ValueError(f"loop {loop} over {n_layer} layers")
+    body = [LayerRun(i, t, i == start) for t in range(times) for i in range(start, stop)]
+    return [LayerRun(i, 0, False) for i in range(start)] + body + [LayerRun(i, 0, False) for i in range(stop, n_layer)]
 
 
 class GPTModel(nn.Module):
@@ -434,11 +523,21 @@ class GPTModel(nn.Module):
                 return mlp_cls
             spec = config.layer_specs[i]["mlp"]
             # hidden sizes are rounded up to the 16-byte pieces of the gate kernel; the extra ones carry zero weights
+            if spec is not None and "experts" in spec:
+                return partial(ExpertMlp, hidden_features=spec["hidden"], experts=spec["experts"], top=spec["top"], **fk)
             return None if spec is None else partial(mlp_cls, hidden_features=spec["hidden"], multiple_of=8)
 
+        self.runs = layer_runs(config.num_hidden_layers, config.loop)
+        side_cls = None
+        if config.token_side_dim > 0:
+            side_cls = partial(TokenSide, dim=config.token_side_dim, eps=config.layer_norm_epsilon, **fk)
+            self.embeddings.side_embeddings = nn.Embedding(vocab, config.num_hidden_layers * config.token_side_dim, **fk)
+        if (config.loop or side_cls) and config.stream_norm is None:
+            raise NotImplementedError("loop and token_side_dim need stream_norm")
+        self.loop_step = nn.Parameter(torch.zeros(config.loop["times"], config.hidden_size, **fk)) if config.loop else None
         self.layers = nn.ModuleList([
             Block(config.hidden_size, create_mixer_cls(config, layer_idx=i, **fk), layer_mlp(i), norm_cls,
-                  residual_in_fp32=config.residual_in_fp32, layer_idx=i, input_conv_cls=input_conv_cls)
+                  residual_in_fp32=config.residual_in_fp32, layer_idx=i, input_conv_cls=input_conv_cls, side_cls=side_cls)
             for i in range(config.num_hidden_layers)
         ])
         self.ln_f = norm_cls(config.hidden_size)
@@ -446,8 +545,20 @@ class GPTModel(nn.Module):
                            initializer_range=config.initializer_range))
 
     def allocate_inference_cache(self, batch_size, max_seqlen, dtype=None, **kwargs):
-        return {i: layer.allocate_inference_cache(batch_size, max_seqlen, dtype=dtype, **kwargs)
-                for i, layer in enumerate(self.layers)}
+        return {i if t == 0 else (i, t): self.layers[i].allocate_inference_cache(batch_size, max_seqlen, dtype=dtype, **kwargs)
+                for i, t, _ in self.runs}
+
+    def _side_table(self):
+        return self.embeddings.side_embeddings.weight if self.config.token_side_dim > 0 else None
+
+    def _run_addends(self, run: LayerRun, addends, ids):
+        """What the first sum of a run receives: `addends` from the block before, and what starts a pass of the loop."""
+        if self.loop_step is None or not run.starts_pass:
+            return addends
+        addends = (addends or ops.Addends())._replace(vec=self.loop_step[run.layer_pass])
+        if run.layer_pass > 0:
+            addends = addends._replace(table=self.embeddings.word_embeddings.weight, index=ids)
+        return addends
 
     # Single-token steps of a bf16 model run through `decode_layers`: every projection is an
     # `ops.decode_linear` launch with the element-wise work in front of it folded in.  Set to False
@@ -458,7 +569,7 @@ class GPTModel(nn.Module):
         if not (self.fused_decode and inference_params is not None and inference_params.seqlen_offset > 0
                 and input_ids.shape[1] == 1 and input_ids.shape[0] <= ops.DECODE_LINEAR_MAX_ROWS
                 and input_ids.is_cuda and not torch.is_grad_enabled()
-                and self.config.max_position_embeddings == 0):
+                and self.config.max_position_embeddings == 0 and self.loop_step is None):
             return False
         # the answer depends on dtypes and devices of the parameters only: worked out once per
         # (dtype, device) of the embedding table
@@ -501,10 +612,25 @@ class GPTModel(nn.Module):
         if inference_params is not None:
             mixer_kwargs["inference_params"] = inference_params
             mixer_kwargs["stream"] = stream
-        for layer in self.layers:
+        addends, more = None, {}
+        ids = None
+        if self.loop_step is not None or self.config.token_side_dim > 0:
+            ids = input_ids.reshape(-1).contiguous()
+            more = {"ids": ids, "side_table": self._side_table()}
+        for run in self.runs:
+            layer = self.layers[run.layer]
+            if inference_params is not None:
+                inference_params.layer_pass = run.layer_pass
+            addends = self._run_addends(run, addends, ids)
+            if addends is not None:
+                more["addends"] = addends
             hidden_states, residual = layer(hidden_states, residual=residual, position_ids=position_ids,
-                                            mixer_kwargs=mixer_kwargs)
-        return add_norm(self.ln_f, hidden_states, residual, self.residual_in_fp32, want_residual=False)[0]
+                                            mixer_kwargs=mixer_kwargs, **more)
+            more.pop("addends", None)
+            addends = layer.out_addends()
+        if inference_params is not None:
+            inference_params.layer_pass = 0
+        return add_norm(self.ln_f, hidden_states, residual, self.residual_in_fp32, want_residual=False, addends=addends)[0]
 
 
 class GPTLMHeadModel(nn.Module, GenerationMixin):
@@ -539,8 +665,6 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
         with open(os.path.join(directory, "config.json")) as f:
             raw = json.load(f)
         design = architectures.find(raw)
-        config = StackConfig(**design.stack_config(raw)) if design else StackConfig.from_reference_dict(raw)
-        model = cls(config, device=device, dtype=dtype)
         st_path = os.path.join(directory, "model.safetensors")
         if os.path.exists(st_path):
             from safetensors.torch import load_file
@@ -548,6 +672,11 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             state = load_file(st_path, device="cpu")
         else:
             state = torch.load(os.path.join(directory, "pytorch_model.bin"), map_location="cpu", weights_only=True)
+        if design:
+            config = StackConfig(**design.stack_config(raw, {name: tuple(t.shape) for name, t in state.items()}))
+        else:
+            config = StackConfig.from_reference_dict(raw)
+        model = cls(config, device=device, dtype=dtype)
         if design:
             model.load_state_dict(design.convert_state(raw, state), strict=strict)
             return model
@@ -590,11 +719,14 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             hidden_states, residual = self.transformer.decode_layers(input_ids, inference_params)
             ln_f = self.transformer.ln_f
             logits = ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias, **norm_prologue(ln_f, residual))
-            return CausalLMOutput(logits=logits.unsqueeze(1))
+            return CausalLMOutput(logits=self._capped(logits).unsqueeze(1))
         hidden_states = self.transformer(input_ids, position_ids=position_ids, inference_params=inference_params,
                                          stream=stream)
         if num_last_tokens > 0:
             hidden_states = hidden_states[:, -num_last_tokens:]
         if logits_at is not None:
             hidden_states = hidden_states[:, logits_at]
-        return CausalLMOutput(logits=self.lm_head(hidden_states))
+        return CausalLMOutput(logits=self._capped(self.lm_head(hidden_states)))
+
+    def _capped(self, logits):
+        return logits if self.config.logit_softcap is None else ops.softcap_(logits, self.config.logit_softcap)

@@ -472,8 +472,8 @@ BASED_API int based_greedy_step(const void* logits, int64_t B, int64_t V, int64_
  * or a recurrence is evaluated in fp32.
  */
 
-enum { BASED_NORM_RMS = 0, BASED_NORM_LAYER = 1 };
-enum { BASED_ACT_NONE = 0, BASED_ACT_SILU = 1 };
+enum { BASED_NORM_RMS = 0, BASED_NORM_LAYER = 1, BASED_NORM_NONE = 2 };
+enum { BASED_ACT_NONE = 0, BASED_ACT_SILU = 1, BASED_ACT_SIGMOID = 2 };
 #define BASED_STREAM_MAX_TAPS 8
 
 /* r = residual_in + mult * x in fp32 (r = x when residual_in is NULL), written to residual_out when
@@ -563,6 +563,106 @@ BASED_API int based_decode_linear_stream(const void* x, int64_t x_row_stride, co
                                          int norm_kind, const void* norm_weight, float eps, const void* conv_weight,
                                          void* conv_ring, int64_t conv_ring_row_stride, int taps, const int32_t* pos,
                                          int64_t pos_host, int epilogue, void* stream);
+
+/* based_add_norm where x may first be divided by its own RMS (post_eps) and multiplied by post_weight (D), and
+ * where the sum also receives a vector add_vec (D) and rows of add_rows (add_n, D): row add_index[r], or row r
+ * when add_index is NULL.  Each may be NULL.  kind BASED_NORM_NONE (weight NULL): y is the rounded sum. */
+BASED_API int based_add_norm_addends(const void* x, const float* residual_in, const void* weight, void* y,
+                                     float* residual_out, int64_t rows, int64_t D, int64_t x_sr, int64_t ri_sr,
+                                     int64_t y_sr, int64_t ro_sr, float eps, int kind, float mult,
+                                     const void* post_weight, float post_eps, const void* add_vec, const void* add_rows,
+                                     const int64_t* add_index, int64_t add_sr, int64_t add_n, int io_dtype, void* stream);
+
+/* y[s, b, t] = x_t + (x_{t-1} - x_t) * mu[s]: x (B, L, D), mu (S, D), y (S, B, L, D) contiguous; ring (B, 2, D) or NULL
+ * holds position p in slot p % 2, is read for the input before the portion and left with its last one. */
+BASED_API int based_token_mix(const void* x, const void* mu, void* y, void* ring, const int32_t* pos, int64_t pos_host,
+                              int64_t B, int64_t L, int64_t D, int64_t S, int64_t x_sb, int64_t x_sl, int64_t ring_sb,
+                              int io_dtype, void* stream);
+
+/* y (rows, C) fp32 = log2 of exp(-exp(w2 tanh(h) + w0)): h (rows, R), w2 (C, R), w0 (C). */
+BASED_API int based_channel_decay(const void* h, const void* w2, const void* w0, float* y, int64_t rows, int64_t h_sr,
+                                  int64_t C, int64_t R, int io_dtype, void* stream);
+
+/* y (rows, n) = gelu_tanh(g) * table[index], table rows of n elements table_sr apart. */
+BASED_API int based_gelu_mul(const void* g, const void* table, const int64_t* index, void* y, int64_t rows, int64_t n,
+                             int64_t g_sr, int64_t table_sr, int64_t table_n, int io_dtype, void* stream);
+
+/* x <- cap * tanh(x / cap), n contiguous elements. */
+BASED_API int based_softcap(void* x, int64_t n, float cap, int io_dtype, void* stream);
+
+/* Linear attention with decaying states over a portion; q, k (B, L, H * D), v, o (B, L, H * DV), silu on q, k
+ * and v first with BASED_ACT_SILU.  channel_log2 (B, L, H * D) contiguous, the log2 of a decay w per key channel, with
+ * bonus u (H, D): o_t = (S + diag(u) k v^T)^T q, S <- diag(w) S + k v^T.  Or head_decay (2, H), the log2 of constants w
+ * and w itself:
+ * S <- w S + k v^T, o = S^T q.  state (B, H, DV, state_row) fp32, by value channel; work: as many floats as
+ * based_decay_scan_work says (bf16 only). */
+BASED_API int64_t based_decay_scan_work(int64_t B, int64_t L, int64_t H, int64_t D, int64_t DV, int64_t state_row);
+BASED_API int based_decay_scan(const void* q, const void* k, const void* v, const float* channel_log2, const float* head_decay,
+                               const void* bonus, float* state, float* work, void* o, int64_t B, int64_t L, int64_t H,
+                               int64_t D, int64_t DV, int64_t state_row, int64_t q_sb, int64_t q_sl, int64_t k_sb,
+                               int64_t k_sl, int64_t v_sb, int64_t v_sl, int64_t o_sb, int64_t o_sl, int activation,
+                               int fresh, int io_dtype, void* stream);
+
+/* One token of it.  With `hidden` (B, R), w2, w0 as in based_channel_decay the channel form, its output divided by its
+ * RMS per head, times norm_w (H, DV) and silu(gate) (B, H * DV); otherwise the head form, its output as it is. */
+BASED_API int based_decay_step(const void* q, const void* k, const void* v, const float* head_decay, const void* bonus,
+                               const void* hidden, const void* w2, const void* w0, const void* gate, const void* norm_w,
+                               float* state, void* o, const int32_t* pos, int64_t pos_host, int64_t B, int64_t H, int64_t D,
+                               int64_t DV, int64_t state_row, int64_t R, int64_t q_sb, int64_t k_sb, int64_t v_sb,
+                               int64_t h_sb, int64_t g_sb, int64_t o_sb, int activation, float eps, int io_dtype,
+                               void* stream);
+
+/* y = o / sqrt(mean(o^2) + eps) * weight * act(gate) * scale over each of G groups of n elements of a row; weight
+ * (G, n); act BASED_ACT_SILU or BASED_ACT_SIGMOID. */
+BASED_API int based_group_norm_gate(const void* o, const void* weight, const void* gate, void* y, int64_t B, int64_t L,
+                                    int64_t G, int64_t n, int64_t o_sb, int64_t o_sl, int64_t g_sb, int64_t g_sl,
+                                    int64_t y_sb, int64_t y_sl, float eps, float scale, int activation, int io_dtype,
+                                    void* stream);
+
+/* based_window_attn_prefill on rows that the cache already holds (only q is rotated). */
+BASED_API int based_window_attn_attend(const void* q, const void* kv, void* o, int64_t start, int64_t B, int64_t L, int64_t H,
+                                       int64_t G, int64_t D, int64_t DV, int64_t S, int64_t q_sb, int64_t q_sl, int64_t o_sb,
+                                       int64_t o_sl, int64_t kv_sb, int64_t kv_st, int64_t window, float scale,
+                                       float out_scale, const float* rope_cos, const float* rope_sin, int64_t rope_len,
+                                       int64_t rotary_dim, int half_split, int io_dtype, void* stream);
+
+/* Rows of a latent cache (B, S, R + rot) from x (B, L, R + rot): the first R channels divided by their RMS and
+ * multiplied by norm_w, the others rotated (tables (rope_len, rot / 2)). */
+BASED_API int based_latent_write(const void* x, const void* norm_w, void* cache, int64_t start, int64_t B, int64_t L, int64_t S,
+                                 int64_t R, int64_t rot, int64_t x_sb, int64_t x_sl, int64_t c_sb, int64_t c_st, float eps,
+                                 const float* rope_cos, const float* rope_sin, int64_t rope_len, int half_split,
+                                 int io_dtype, void* stream);
+
+/* One token per sequence of attention over that cache, the token's own row written first.  q (B, H * (rot + D)), a head's
+ * rotated channels first; weight (H * (rot + D + DV), at least R columns): of each head rot rows that are not read, uk (D
+ * rows), uv (DV rows).  score = ((uk^T q) . c + q_rot . k_rot) * scale over the last `window` rows; o (B, H * DV) = uv times the
+ * weighted latents, times out_scale.  work_q: B H (R + rot) floats, work_part: B splits H R, work_ml: B splits H 2. */
+BASED_API int based_latent_step(const void* q, const void* x, const void* norm_w, const void* weight, void* cache, float* work_q,
+                                float* work_part, float* work_ml, void* o, const int32_t* pos, int64_t pos_host, int64_t B,
+                                int64_t H, int64_t D, int64_t DV, int64_t S, int64_t R, int64_t rot, int64_t splits,
+                                int64_t q_sb, int64_t x_sb, int64_t w_sr, int64_t c_sb, int64_t c_st, int64_t o_sb,
+                                int64_t window, float scale, float eps, float out_scale, const float* rope_cos,
+                                const float* rope_sin, int64_t rope_len, int half_split, int io_dtype, void* stream);
+
+/* Mixture of experts.  Route: scores = sigmoid(router h) in fp32, the `top` largest per token into ids, scores (n, top);
+ * with rank (n, top) also each choice's place among its expert's rows and counts (E, zero on entry).
+ * Grouped (bf16): y = sum over a token's choices of w2_e (silu(gate) * up), [up; gate] = score * w1_e h; w1 (E, 2 F, D), w2 (E, D, F);
+ * scratch: tile_first (E + 1), tile_expert (tiles), order (tiles * rows), work_act (tiles * rows, F), work_out (n * top, D) with
+ * top > 1, tiles and rows from based_expert_tiles / based_expert_tile_rows.  Rows: the same for few tokens and any element type;
+ * work_act (n * top, F). */
+#define BASED_EXPERT_TILE_ROWS 128
+#define BASED_EXPERT_TILE_ROWS_SMALL 32
+BASED_API int based_expert_route(const void* h, const void* router, int32_t* ids, float* scores, int32_t* rank, int32_t* counts,
+                                 int64_t n, int64_t D, int64_t E, int64_t top, int64_t h_sr, int io_dtype, void* stream);
+BASED_API int64_t based_expert_tiles(int64_t n, int64_t E, int64_t top);
+BASED_API int64_t based_expert_tile_rows(int64_t n, int64_t E, int64_t top);
+BASED_API int based_expert_grouped(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
+                                   const int32_t* rank, const int32_t* counts, int32_t* tile_first, int32_t* tile_expert,
+                                   int32_t* order, void* work_act, void* work_out, void* y, int64_t n, int64_t D, int64_t F,
+                                   int64_t E, int64_t top, int64_t h_sr, void* stream);
+BASED_API int based_expert_rows(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
+                                void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t top, int64_t h_sr, int io_dtype,
+                                void* stream);
 
 #ifdef __cplusplus
 }
