@@ -294,7 +294,7 @@ extern "C" BASED_API int based_gelu_mul(const void* g, const void* table, const 
 
 extern "C" BASED_API int based_softcap(void* x, int64_t n, float cap, int io_dtype, void* stream) {
   using namespace based;
-  BASED_REQUIRE(x, BASED_ERR_ARG, "softcap: null pointer argument");
+  BASED_REQUIRE(x || n == 0, BASED_ERR_ARG, "softcap: null pointer argument");
   BASED_REQUIRE(n >= 0 && n < (1ll << 38) && cap > 0.f, BASED_ERR_ARG, "softcap: bad sizes");
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "softcap: bad dtype");
   BASED_REQUIRE(aligned_to(x, 16), BASED_ERR_ALIGN, "softcap: x must be 16-byte aligned");
