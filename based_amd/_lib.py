@@ -22,6 +22,14 @@ PREFILL_SEGMENT_STATE_BYTES = 43008  # BASED_PREFILL_SEGMENT_STATE_BYTES of incl
 _I64 = C.c_int64
 _P = C.c_void_p
 
+class StreamExtras(C.Structure):
+    """based_stream_extras of include/based_hip.h."""
+
+    _fields_ = ([(n, _P) for n in ("post_weight", "add_vec", "add_rows", "add_index", "mix_mu", "mix_ring", "gate_table", "gate_index")]
+                + [(n, _I64) for n in ("add_sr", "add_n", "mix_rows", "mixes", "mix_ring_row_stride", "gate_sr", "gate_n")]
+                + [(n, C.c_float) for n in ("post_eps", "softcap")])
+
+
 # name -> (restype, argtypes); must list every symbol declared in include/based_hip.h
 SIGNATURES = {
     "based_hip_version": (C.c_int, []),
@@ -139,6 +147,12 @@ SIGNATURES = {
     "based_expert_tile_rows": (_I64, [_I64] * 3),
     "based_expert_grouped": (C.c_int, [_P] * 13 + [_I64] * 6 + [_P]),
     "based_expert_rows": (C.c_int, [_P] * 7 + [_I64] * 5 + [C.c_int, _P]),
+    "based_decode_linear_extras": (
+        C.c_int,
+        [_P, _I64, _P, _I64, _P, _I64, _P, _P] + [_I64] * 4 + [_P, _I64, _P, _I64, C.c_float, C.c_int, _P, C.c_float, _P, _I64, C.c_int,
+                                                              _P, _P],
+    ),
+    "based_decode_linear_mixes": (C.c_int, [_P, _P, _I64, _P] + [_I64] * 6 + [_P]),
     "based_swa_step": (
         C.c_int,
         [_P, _P, _P, _P, _P, _P, _P, _I64] + [_I64] * 3 + [_I64] * 8 + [_I64] * 3

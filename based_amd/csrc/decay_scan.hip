@@ -120,7 +120,8 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
   auto chan = [&](int c, int half) { return c * 32 + half * 16 + quad * 4; };
 
   float bonus[CHANNEL && !STATE_ONLY ? E : 1];
-  if constexpr (CHANNEL && !STATE_ONLY) {
+  auto load_bonus = [&]() {
+    if constexpr (CHANNEL && !STATE_ONLY) {
 #pragma unroll
     for (int c = 0; c < DT; ++c)
 #pragma unroll
@@ -130,7 +131,9 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
 #pragma unroll
         for (int j = 0; j < 4; ++j) bonus[c * 8 + f * 4 + j] = to_f32(x[j]);
       }
-  }
+    }
+  };
+  if constexpr (DT < 4) load_bonus();  // (tall heads load it where it is used, for their registers)
 
   // state: tile ct holds key channels 16 ct + 4 quad + i of value channel dv0 + l16
   f32x4 S[2 * DT];
@@ -177,12 +180,15 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
   };
   auto active = [&](float x) { return a.silu ? round_to<__bf16>(silu_exact(x)) : x; };
 
+  // the next 64 tokens are asked for while these are worked on, where the registers allow it
+  constexpr bool AHEAD = DT < 4 || !CHANNEL || STATE_ONLY;
   Stage cur;
-  if (first < last) fetch(cur, first);
+  if (AHEAD && first < last) fetch(cur, first);
   for (int chunk = first; chunk < last; ++chunk) {
     const int left = a.L - chunk * kScanTokens, n = left < kScanTokens ? left : kScanTokens;
     const int t = wave * 16 + l16;  // this lane's token
     const bool live = t < n;
+    if constexpr (!AHEAD) fetch(cur, chunk);
     float q[STATE_ONLY ? 1 : E], k[E], g_before[CHANNEL ? E : 1], g_after[CHANNEL ? E : 1], w[CHANNEL && !STATE_ONLY ? E : 1];
 #pragma unroll
     for (int c = 0; c < DT; ++c)
@@ -200,7 +206,7 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
 #pragma unroll
       for (int j = 0; j < 4; ++j)
         vv[f * 4 + j] = live && col_base + quad * 16 + f * 4 < a.dv ? from_f32<__bf16>(active(to_f32(cur.v[f][j]))) : (__bf16)0.f;
-    if (chunk + 1 < last) fetch(cur, chunk + 1);
+    if (AHEAD && chunk + 1 < last) fetch(cur, chunk + 1);
 
     __syncthreads();  // every wavefront is done with the 64 tokens before
 #pragma unroll
@@ -255,20 +261,14 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
 
     f32x4 P[STATE_ONLY ? 1 : 4];  // P^T tiles: column t of this wavefront's 16 tokens, rows s of 16 tokens j
     if constexpr (CHANNEL) {
-      float to_end[E];  // log decay over the 16-token groups behind this one
 #pragma unroll
       for (int i = 0; i < E; ++i) {
         const int ch = (i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3);
-        float sum = 0.f;
+        float to_end = 0.f;  // log decay over the 16-token groups behind this one
 #pragma unroll
-        for (int m = 1; m < 4; ++m) sum += m > wave ? lds.total[m][ch] : 0.f;
-        to_end[i] = sum;
-      }
-#pragma unroll
-      for (int i = 0; i < E; ++i) {
-        const int ch = (i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3);
+        for (int m = 1; m < 4; ++m) to_end += m > wave ? lds.total[m][ch] : 0.f;
         __bf16 x, y;
-        split(k[i] * __builtin_amdgcn_exp2f(g_after[i] + to_end[i]), x, y);
+        split(k[i] * __builtin_amdgcn_exp2f(g_after[i] + to_end), x, y);
         lds.kt_hi[ch * TS + t] = x;
         lds.kt_lo[ch * TS + t] = y;
       }
@@ -318,6 +318,7 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
         // the 16 tokens themselves: rows s = 4 quad + i
         f32x4 diag = {0.f, 0.f, 0.f, 0.f};
         {
+          if constexpr (DT >= 4) load_bonus();
           float sum = 0.f;
 #pragma unroll
           for (int i = 0; i < E; ++i) sum = __builtin_fmaf(q[i] * bonus[i], k[i], sum);
@@ -591,13 +592,6 @@ struct DecayStepArgs {
   float eps;
 };
 
-__device__ __forceinline__ float decay_tanh(float z) {
-  const float e = expf(2.0f * z), q = z * z;
-  const float far = 1.0f - 2.0f / (e + 1.0f);
-  const float near = z * (1.0f - q * (1.0f / 3.0f - q * (2.0f / 15.0f)));
-  return fabsf(z) < 0.05f ? near : far;
-}
-
 // NT threads; LPR lanes per value channel, four key channels each; RPT value channels per thread.
 template <typename T, int NT, int LPR, int RPT, bool CHANNEL>
 __global__ __launch_bounds__(NT) void decay_step_kernel(const DecayStepArgs a) {
@@ -639,7 +633,7 @@ __global__ __launch_bounds__(NT) void decay_step_kernel(const DecayStepArgs a) {
   for (int c = tid; c < RPT * kRows; c += NT)
     sv[c] = c < a.dv ? active(static_cast<const T*>(a.v)[b * a.v_sb + (long)h * a.dv + c]) : 0.f;
   if constexpr (CHANNEL) {
-    for (int j = tid; j < a.R; j += NT) th[j] = decay_tanh(to_f32(static_cast<const T*>(a.hid)[b * a.h_sb + j]));
+    for (int j = tid; j < a.R; j += NT) th[j] = tanh_f(to_f32(static_cast<const T*>(a.hid)[b * a.h_sb + j]));
     __syncthreads();
     // four lanes per key channel
     for (int c = tid >> 2; c < 4 * LPR; c += NT / 4) {

@@ -23,6 +23,9 @@
 //     RMS norm of that sum, and h + causal convolution of h on a ring of past norm outputs.  Every
 //     workgroup reads the ring; workgroup 0 writes the current row into the slot of its position,
 //     which no reader of the same step looks at.
+//   * the same with more around it (based_decode_linear_extras): x divided by its RMS first, a vector and a
+//     table row in the sum, no norm, or instead of the convolution several mixes of a row with the row of the
+//     token before, each read by its own weight rows (a workgroup's rows belong to one mix).
 // What FOLLOWS a projection whose output is consumed in (value, gate) pairs runs in its tail: a
 // wavefront then takes R/2 rows of the value half of the weight and the R/2 matching rows of the
 // gate half, so that after the sums one lane holds both numbers of an output element, and
@@ -34,7 +37,7 @@
 // All of them use the arithmetic (and the roundings to bf16) of the stand-alone kernels.
 #include <initializer_list>
 
-#include "common.hpp"
+#include "stream_common.hpp"
 
 namespace based {
 
@@ -72,6 +75,16 @@ struct DecodeLinearArgs {
   int ic_taps;
   const int32_t* pos;
   int pos_host;
+  // rows that read one of several mixes: mix_rows > 0 weight rows each (the last mix all that are left)
+  const __bf16* mix_mu;  // (mixes, K), with kProStreamAdd
+  __bf16* mix_ring;      // (rows, 2, K)
+  long mix_ring_sr, x_mix;  // x_mix: distance between the mixes of x, without a prologue
+  int mix_rows, mixes;
+  StreamAddends add;
+  const __bf16* gate_table;
+  const int64_t* gate_index;
+  long gate_sr, gate_n;
+  float softcap;
 };
 
 typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
@@ -144,7 +157,7 @@ __device__ __forceinline__ float wave_sum_dpp(float x) {
 __device__ __forceinline__ float silu_f(float a) { return a / (1.0f + __expf(-a)); }
 
 enum { kProNone = BASED_PROLOGUE_NONE, kProNorm = BASED_PROLOGUE_ADD_RMS_NORM, kProSwiglu = BASED_PROLOGUE_SWIGLU,
-       kProStream = 3 };
+       kProStream = 3, kProStreamAdd = 4 };
 enum { kEpiNone = BASED_EPILOGUE_NONE, kEpiSwiglu = BASED_EPILOGUE_SWIGLU, kEpiConv = BASED_EPILOGUE_GATED_CONV_STEP };
 
 __device__ __forceinline__ void lds_barrier() {
@@ -201,6 +214,11 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       for (int c = 0; c < C; ++c) dst[r][c] = *reinterpret_cast<const u32x4*>(src + e0[c]);
     }
   };
+  int mix = 0;  // which mix this workgroup's rows read
+  if ((PRO == kProNone || PRO == kProStreamAdd) && a.mix_rows > 0) {
+    mix = (int)blockIdx.x * WV * R / a.mix_rows;
+    mix = mix < a.mixes ? mix : a.mixes - 1;
+  }
   // row m of the activations (rows past M are never stored: any valid row will do); a row whose
   // index is out of range reads as NaN
   auto x_row = [&](int m, bool& poison) -> const __bf16* {
@@ -212,7 +230,7 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       poison = src < 0 || src >= a.x_index_rows;
       if (poison) src = 0;
     }
-    return a.x + src * a.x_sr;
+    return a.x + src * a.x_sr + (PRO == kProNone ? mix * a.x_mix : 0);
   };
   const __bf16* nans = reinterpret_cast<const __bf16*>(kNanPage);
 
@@ -223,12 +241,12 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
   // positions of the streamed-input prologue: scalar loads, in front of the weight rows
   constexpr int RW = (MT + WV - 1) / WV;  // activation rows per wavefront
   int pos_of[RW];
-  if constexpr (PRO == kProStream) {
+  if constexpr (PRO == kProStream || PRO == kProStreamAdd) {
     const int wave_u = __builtin_amdgcn_readfirstlane(wave);
 #pragma unroll
     for (int i = 0; i < RW; ++i) {
       const int m = wave_u + i * WV;
-      pos_of[i] = a.ic_taps == 0 ? 0 : a.pos != nullptr ? a.pos[a.m0 + (m < a.M ? m : 0)] : a.pos_host;
+      pos_of[i] = a.ic_taps == 0 && a.mix_rows == 0 ? 0 : a.pos != nullptr ? a.pos[a.m0 + (m < a.M ? m : 0)] : a.pos_host;
     }
   }
   u32x4 wcur[R][C];
@@ -296,7 +314,8 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
         xs[m][c][lane] = u32x4{pack_bf16(o[0], o[1]), pack_bf16(o[2], o[3]), pack_bf16(o[4], o[5]), pack_bf16(o[6], o[7])};
       }
     }
-  } else if constexpr (PRO == kProStream) {
+  } else if constexpr (PRO == kProStream || PRO == kProStreamAdd) {
+    constexpr bool ADD = PRO == kProStreamAdd;
 #pragma unroll
     for (int m = wave; m < MT; m += WV)
     if (m < a.M) {
@@ -305,20 +324,81 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       const bool has_res = a.res_in != nullptr;
       const float mult = has_res ? a.mult : 1.0f;
       const int pos = pos_of[(m - wave) / WV];
-      float v[C][8], nw[C][8];
+      float v[C][8], nw[C][8], more[ADD ? C : 1][8];
+      bf16x8 before[ADD ? C : 1], mu[ADD ? C : 1];
       float sum = 0.f;
 #pragma unroll
       for (int c = 0; c < C; ++c) {
         const bf16x8 h = *reinterpret_cast<const bf16x8*>(live[c] ? xrow + e0[c] : zeros);
-        const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.norm_w + e0[c] : zeros);
+        const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] && (!ADD || a.norm_w != nullptr) ? a.norm_w + e0[c] : zeros);
         const float* rp = has_res && live[c] ? a.res_in + (long)m * a.ri_sr + e0[c] : reinterpret_cast<const float*>(kZeroPage);
         const f32x4 r0 = reinterpret_cast<const f32x4*>(rp)[0], r1 = reinterpret_cast<const f32x4*>(rp)[1];
 #pragma unroll
         for (int i = 0; i < 8; ++i) {
           nw[c][i] = to_f32(w8[i]);
-          v[c][i] = __builtin_fmaf(mult, to_f32(h[i]), i < 4 ? r0[i & 3] : r1[i & 3]);
-          sum += v[c][i];
+          if constexpr (ADD) {
+            v[c][i] = to_f32(h[i]);
+            more[c][i] = i < 4 ? r0[i & 3] : r1[i & 3];
+          } else {
+            v[c][i] = __builtin_fmaf(mult, to_f32(h[i]), i < 4 ? r0[i & 3] : r1[i & 3]);
+            sum += v[c][i];
+          }
         }
+      }
+      if constexpr (ADD) {
+        // what else the sum receives, and the row of the token before, in flight together
+        const __bf16* vec = static_cast<const __bf16*>(a.add.vec);
+        const __bf16* post = static_cast<const __bf16*>(a.add.post_w);
+        const __bf16* row = static_cast<const __bf16*>(a.add.rows);
+        if (row != nullptr) {
+          const long src = a.add.rows_index[m];
+          const bool bad = src < 0 || src >= a.add.rows_n;
+          poison = poison || bad;
+          row += (bad ? 0 : src) * a.add.rows_sr;
+        }
+        const bool mixing = a.mix_rows > 0;
+        const __bf16* ring = mixing && pos > 0 ? a.mix_ring + (long)(a.m0 + m) * a.mix_ring_sr + (long)((pos - 1) & 1) * a.K : nullptr;
+        bf16x8 p8[C];
+        constexpr int CB = C >= 8 ? 2 : C;  // (wide rows: in batches, for their registers)
+#pragma unroll
+        for (int c0 = 0; c0 < C; c0 += CB) {
+          bf16x8 b8[CB], d8[CB];
+#pragma unroll
+          for (int cb = 0; cb < CB; ++cb) {
+            const int c = c0 + cb;
+            b8[cb] = *reinterpret_cast<const bf16x8*>(live[c] && vec != nullptr ? vec + e0[c] : zeros);
+            d8[cb] = *reinterpret_cast<const bf16x8*>(live[c] && row != nullptr ? row + e0[c] : zeros);
+            p8[c] = *reinterpret_cast<const bf16x8*>(live[c] && post != nullptr ? post + e0[c] : zeros);
+            if constexpr (C < 8) {
+              before[c] = *reinterpret_cast<const bf16x8*>(live[c] && ring != nullptr ? ring + e0[c] : zeros);
+              mu[c] = *reinterpret_cast<const bf16x8*>(live[c] && mixing ? a.mix_mu + (long)mix * a.K + e0[c] : zeros);
+            }
+          }
+#pragma unroll
+          for (int cb = 0; cb < CB; ++cb)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) more[c0 + cb][i] += to_f32(b8[cb][i]) + to_f32(d8[cb][i]);
+          if constexpr (C >= 8) __builtin_amdgcn_sched_barrier(0);
+        }
+        if (post != nullptr) {
+          float xs2 = 0.f;
+#pragma unroll
+          for (int c = 0; c < C; ++c)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) xs2 = __builtin_fmaf(v[c][i], v[c][i], xs2);
+          const float r = 1.0f / sqrtf(wave_sum_dpp(xs2) / (float)a.K + a.add.post_eps);
+#pragma unroll
+          for (int c = 0; c < C; ++c)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) v[c][i] *= r * to_f32(p8[c][i]);
+        }
+#pragma unroll
+        for (int c = 0; c < C; ++c)
+#pragma unroll
+          for (int i = 0; i < 8; ++i) {
+            v[c][i] = __builtin_fmaf(mult, v[c][i], more[c][i]);
+            sum += v[c][i];
+          }
       }
       // the ring rows of the past inputs, in flight during the reductions
       float past[C][8];
@@ -373,10 +453,30 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       for (int c = 0; c < C; ++c) {
         bf16x8 h;
         float o[8];
+        const bool plain = ADD && a.norm_kind == BASED_NORM_NONE;
+        if constexpr (ADD && C >= 8) {
+          const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] && a.norm_w != nullptr ? a.norm_w + e0[c] : zeros);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) h[i] = from_f32<__bf16>(v[c][i] * rstd * nw[c][i]);
+          for (int i = 0; i < 8; ++i) nw[c][i] = to_f32(w8[i]);
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i) h[i] = from_f32<__bf16>(plain ? (poison ? rstd : v[c][i]) : v[c][i] * rstd * nw[c][i]);
 #pragma unroll
         for (int i = 0; i < 8; ++i) o[i] = to_f32(h[i]);
+        if constexpr (ADD) {
+          if (a.mix_rows > 0) {
+            if constexpr (C >= 8) {
+              const __bf16* ring = a.mix_ring + (long)(a.m0 + m) * a.mix_ring_sr + (long)((pos - 1) & 1) * a.K;
+              before[c] = *reinterpret_cast<const bf16x8*>(live[c] && pos > 0 ? ring + e0[c] : zeros);
+              mu[c] = *reinterpret_cast<const bf16x8*>(live[c] ? a.mix_mu + (long)mix * a.K + e0[c] : zeros);
+            }
+#pragma unroll
+            for (int i = 0; i < 8; ++i) o[i] = __builtin_fmaf(to_f32(before[c][i]) - o[i], to_f32(mu[c][i]), o[i]);
+            // a slot that no reader of this step looks at
+            if (wg == 0 && live[c] && pos >= 0)
+              *reinterpret_cast<bf16x8*>(a.mix_ring + (long)(a.m0 + m) * a.mix_ring_sr + (long)(pos & 1) * a.K + e0[c]) = h;
+          }
+        }
         if (a.ic_taps > 0) {
           const bf16x8 w8 = *reinterpret_cast<const bf16x8*>(live[c] ? a.ic_w + (long)(a.ic_taps - 1) * a.K + e0[c] : zeros);
 #pragma unroll
@@ -467,7 +567,17 @@ __device__ __forceinline__ void decode_linear_tile(const DecodeLinearArgs& a, bo
       float mine = 0.f;
 #pragma unroll
       for (int j = 0; j < kOwners; ++j) mine = (j16 == j) ? tot[j] : mine;
-      if (owner) a.y[(long)own_m * a.y_sr + out_col] = from_f32<__bf16>(mine + bias_v);
+      mine += bias_v;
+      if constexpr (PRO == kProStreamAdd) {
+        if (a.gate_table != nullptr) {
+          const long src = a.gate_index[owner ? own_m : 0];
+          const bool bad = src < 0 || src >= a.gate_n;
+          const float e = to_f32(a.gate_table[(bad ? 0 : src) * a.gate_sr + col_c]);
+          mine = bad ? __builtin_nanf("") : gelu_tanh_f(to_f32(from_f32<__bf16>(mine))) * e;
+        }
+        if (a.softcap > 0.f) mine = a.softcap * tanh_f(mine / a.softcap);
+      }
+      if (owner) a.y[(long)own_m * a.y_sr + out_col] = from_f32<__bf16>(mine);
     } else {
       // value (r, m) and gate (r, m) are RH * MT sums apart: the same lane, kOwners slots on
       float val = 0.f, gate = 0.f;
@@ -546,6 +656,8 @@ __global__ __launch_bounds__(PRO == kProNone ? 64 : 256) void decode_linear_kern
     t.y = a.y + (long)m0 * a.y_sr;
     if (a.res_in != nullptr) t.res_in = a.res_in + (long)m0 * a.ri_sr;
     if (a.res_out != nullptr) t.res_out = a.res_out + (long)m0 * a.ro_sr;
+    if (a.add.rows_index != nullptr) t.add.rows_index = a.add.rows_index + m0;
+    if (a.gate_index != nullptr) t.gate_index = a.gate_index + m0;
     decode_linear_tile<C, MT, PRO, EPI>(t, m0 == 0);
   }
 }
@@ -555,7 +667,8 @@ constexpr int kDecodeLinearMaxWaves = 4096;  // row groups beyond this many are 
 template <int C, int MT, int EPI>
 void launch_decode_linear_pro(const DecodeLinearArgs& a, int prologue, hipStream_t s) {
   const int wv = prologue == kProNone ? 1 : 4;  // WV of the kernel
-  const int n_wg = (a.n_groups + wv - 1) / wv, cap = kDecodeLinearMaxWaves / wv;
+  // (a workgroup's activations belong to one mix: every row group has a wavefront of its own then)
+  const int n_wg = (a.n_groups + wv - 1) / wv, cap = a.mix_rows > 0 ? n_wg : kDecodeLinearMaxWaves / wv;
   const dim3 grid((unsigned)(n_wg < cap ? n_wg : cap)), block(64 * wv);
   if (prologue == kProNone) {
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProNone, EPI>), grid, block, 0, s, a);
@@ -563,6 +676,8 @@ void launch_decode_linear_pro(const DecodeLinearArgs& a, int prologue, hipStream
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProNorm, EPI>), grid, block, 0, s, a);
   } else if (prologue == kProStream) {
     if constexpr (EPI != kEpiConv) hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProStream, EPI>), grid, block, 0, s, a);
+  } else if (prologue == kProStreamAdd) {
+    if constexpr (EPI != kEpiConv) hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProStreamAdd, EPI>), grid, block, 0, s, a);
   } else if constexpr (EPI == kEpiNone) {
     hipLaunchKernelGGL((decode_linear_kernel<C, MT, kProSwiglu, EPI>), grid, block, 0, s, a);
   }
@@ -788,4 +903,115 @@ extern "C" BASED_API int based_decode_linear_stream(const void* x, int64_t x_row
   a.pos_host = (int)pos_host;
   launch_decode_linear_chunks(a, kProStream, epilogue, static_cast<hipStream_t>(stream));
   return check_launch("decode_linear_stream");
+}
+
+extern "C" BASED_API int based_decode_linear_extras(const void* x, int64_t x_row_stride, const int64_t* x_row_index, int64_t x_index_rows,
+                                                    const void* weight, int64_t w_row_stride, const void* bias, void* y,
+                                                    int64_t y_row_stride, int64_t M, int64_t N, int64_t K, const float* residual_in,
+                                                    int64_t ri_row_stride, float* residual_out, int64_t ro_row_stride, float mult,
+                                                    int norm_kind, const void* norm_weight, float eps, const int32_t* pos,
+                                                    int64_t pos_host, int epilogue, const based_stream_extras* extras, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x && weight && y && extras && (norm_weight || norm_kind == BASED_NORM_NONE), BASED_ERR_ARG,
+                "decode_linear_extras: null pointer argument");
+  const based_stream_extras& ex = *extras;
+  BASED_REQUIRE(M >= 0 && N > 0 && K > 0 && pos_host >= 0 && pos_host < (1ll << 31), BASED_ERR_ARG, "decode_linear_extras: bad sizes");
+  BASED_REQUIRE(M <= BASED_DECODE_LINEAR_MAX_ROWS, BASED_ERR_SHAPE, "decode_linear_extras: %ld activation rows, at most %d", (long)M,
+                BASED_DECODE_LINEAR_MAX_ROWS);
+  BASED_REQUIRE(K % 8 == 0 && K <= 4096, BASED_ERR_SHAPE,
+                "decode_linear_extras: contraction length %ld unsupported (multiple of 8, at most 4096)", (long)K);
+  BASED_REQUIRE(N < (1ll << 30), BASED_ERR_SHAPE, "decode_linear_extras: too many output features");
+  BASED_REQUIRE(norm_kind == BASED_NORM_RMS || norm_kind == BASED_NORM_LAYER || norm_kind == BASED_NORM_NONE, BASED_ERR_ARG,
+                "decode_linear_extras: unknown norm %d", norm_kind);
+  BASED_REQUIRE(epilogue == kEpiNone || epilogue == kEpiSwiglu, BASED_ERR_ARG, "decode_linear_extras: unknown epilogue %d", epilogue);
+  BASED_REQUIRE(epilogue == kEpiNone || (N % 2 == 0 && K <= 2048 && ex.mix_mu == nullptr && ex.gate_table == nullptr && ex.softcap == 0.f),
+                BASED_ERR_SHAPE, "decode_linear_extras: the paired epilogue takes an even number of rows of up to 2048 elements, and no other");
+  BASED_REQUIRE(ex.mix_mu == nullptr || (ex.mix_ring && ex.mixes > 0 && ex.mix_rows > 0 && ex.mix_rows % 32 == 0 && ex.mix_rows < (1ll << 30)),
+                BASED_ERR_SHAPE, "decode_linear_extras: mixes need a ring and a multiple of 32 rows each");
+  BASED_REQUIRE(ex.add_rows == nullptr || (ex.add_index && ex.add_n > 0), BASED_ERR_ARG, "decode_linear_extras: added rows need an index");
+  BASED_REQUIRE(ex.gate_table == nullptr || (ex.gate_index && ex.gate_n > 0), BASED_ERR_ARG, "decode_linear_extras: the gate needs an index");
+  BASED_REQUIRE(x_row_index == nullptr || x_index_rows > 0, BASED_ERR_ARG,
+                "decode_linear_extras: a row index needs the number of rows it may address");
+  BASED_REQUIRE(x_row_stride % 8 == 0 && w_row_stride % 8 == 0 && ri_row_stride % 4 == 0 && ro_row_stride % 4 == 0 && ex.add_sr % 8 == 0 &&
+                    ex.mix_ring_row_stride % 8 == 0,
+                BASED_ERR_ALIGN, "decode_linear_extras: rows must be whole 16-byte pieces");
+  BASED_REQUIRE(aligned16_all({x, weight, residual_in, residual_out, norm_weight, ex.post_weight, ex.add_vec, ex.add_rows, ex.mix_mu,
+                               ex.mix_ring}),
+                BASED_ERR_ALIGN, "decode_linear_extras: tensors must be 16-byte aligned");
+  if (M == 0) return BASED_OK;
+  {
+    const int64_t x_bytes = (((x_row_index ? x_index_rows : M) - 1) * x_row_stride + K) * 2;
+    const int64_t ri_bytes = ((M - 1) * ri_row_stride + K) * 4, ro_bytes = ((M - 1) * ro_row_stride + K) * 4;
+    const int64_t y_bytes = ((M - 1) * y_row_stride + (epilogue == kEpiNone ? N : N / 2)) * 2;
+    BASED_REQUIRE(!ranges_overlap(residual_out, ro_bytes, residual_in, ri_bytes) && !ranges_overlap(residual_out, ro_bytes, x, x_bytes) &&
+                      !ranges_overlap(y, y_bytes, x, x_bytes) && !ranges_overlap(y, y_bytes, residual_in, ri_bytes) &&
+                      !ranges_overlap(y, y_bytes, residual_out, ro_bytes),
+                  BASED_ERR_ARG, "decode_linear_extras: an output (y, residual_out) overlaps an input or the other output");
+  }
+  DecodeLinearArgs a = {};
+  a.x = static_cast<const __bf16*>(x);
+  a.x_sr = x_row_stride;
+  a.x_index = x_row_index;
+  a.x_index_rows = x_index_rows;
+  a.w = static_cast<const __bf16*>(weight);
+  a.w_sr = w_row_stride;
+  a.bias = static_cast<const __bf16*>(bias);
+  a.y = static_cast<__bf16*>(y);
+  a.y_sr = y_row_stride;
+  a.M = (int)M;
+  a.N = (int)N;
+  a.K = (int)K;
+  a.res_in = residual_in;
+  a.ri_sr = ri_row_stride;
+  a.res_out = residual_out;
+  a.ro_sr = ro_row_stride;
+  a.norm_w = static_cast<const __bf16*>(norm_weight);
+  a.eps = eps;
+  a.mult = mult;
+  a.norm_kind = norm_kind;
+  a.pos = pos;
+  a.pos_host = (int)pos_host;
+  a.mix_mu = static_cast<const __bf16*>(ex.mix_mu);
+  a.mix_ring = static_cast<__bf16*>(ex.mix_ring);
+  a.mix_ring_sr = ex.mix_ring_row_stride;
+  a.mix_rows = ex.mix_mu != nullptr ? (int)ex.mix_rows : 0;
+  a.mixes = (int)ex.mixes;
+  a.add = {ex.post_weight, ex.add_vec, ex.add_rows, ex.add_index, (long)ex.add_sr, (long)ex.add_n, ex.post_eps};
+  a.gate_table = static_cast<const __bf16*>(ex.gate_table);
+  a.gate_index = ex.gate_index;
+  a.gate_sr = ex.gate_sr;
+  a.gate_n = ex.gate_n;
+  a.softcap = ex.softcap;
+  launch_decode_linear_chunks(a, kProStreamAdd, epilogue, static_cast<hipStream_t>(stream));
+  return check_launch("decode_linear_extras");
+}
+
+extern "C" BASED_API int based_decode_linear_mixes(const void* x, const void* weight, int64_t w_row_stride, void* y, int64_t y_row_stride,
+                                                   int64_t M, int64_t N, int64_t K, int64_t mixes, int64_t mix_rows, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x && weight && y, BASED_ERR_ARG, "decode_linear_mixes: null pointer argument");
+  BASED_REQUIRE(M >= 0 && N > 0 && K > 0 && mixes > 0 && mix_rows > 0, BASED_ERR_ARG, "decode_linear_mixes: bad sizes");
+  BASED_REQUIRE(M <= BASED_DECODE_LINEAR_MAX_ROWS, BASED_ERR_SHAPE, "decode_linear_mixes: %ld activation rows, at most %d", (long)M,
+                BASED_DECODE_LINEAR_MAX_ROWS);
+  BASED_REQUIRE(K % 8 == 0 && K <= 4096 && N < (1ll << 30) && mix_rows % 32 == 0 && mix_rows < (1ll << 30), BASED_ERR_SHAPE,
+                "decode_linear_mixes: unsupported sizes");
+  BASED_REQUIRE(w_row_stride % 8 == 0 && aligned16_all({x, weight}), BASED_ERR_ALIGN, "decode_linear_mixes: rows must be whole 16-byte pieces");
+  if (M == 0) return BASED_OK;
+  BASED_REQUIRE(!ranges_overlap(y, ((M - 1) * y_row_stride + N) * 2, x, mixes * M * K * 2), BASED_ERR_ARG,
+                "decode_linear_mixes: the output overlaps the input");
+  DecodeLinearArgs a = {};
+  a.x = static_cast<const __bf16*>(x);
+  a.x_sr = K;
+  a.w = static_cast<const __bf16*>(weight);
+  a.w_sr = w_row_stride;
+  a.y = static_cast<__bf16*>(y);
+  a.y_sr = y_row_stride;
+  a.M = (int)M;
+  a.N = (int)N;
+  a.K = (int)K;
+  a.mixes = (int)mixes;
+  a.mix_rows = (int)mix_rows;
+  a.x_mix = M * K;
+  launch_decode_linear_chunks(a, kProNone, kEpiNone, static_cast<hipStream_t>(stream));
+  return check_launch("decode_linear_mixes");
 }

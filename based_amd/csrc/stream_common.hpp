@@ -29,6 +29,14 @@ __device__ __forceinline__ float softplus_f(float z) { return log1pf(expf(-fabsf
 __device__ __forceinline__ float gelu_tanh_f(float z) {
   return z * sigmoid_f(1.5957691216057308f * (z + 0.044715f * z * z * z));
 }
+// exp(2z) overflows to infinity and 1 - 0 is left; near zero, where that form cancels, the series (the next term is
+// 1e-9 of the sum)
+__device__ __forceinline__ float tanh_f(float z) {
+  const float e = expf(2.0f * z), q = z * z;
+  const float far = 1.0f - 2.0f / (e + 1.0f);
+  const float near = z * (1.0f - q * (1.0f / 3.0f - q * (2.0f / 15.0f)));
+  return fabsf(z) < 0.05f ? near : far;
+}
 // 1 - a^2 for a = exp(log_a) <= 1 without cancellation: the series of 1 - exp(x), x = 2 log_a, above -1/4 (the
 // next term is 5e-8 of the sum)
 __device__ __forceinline__ float one_minus_square(float a, float log_a) {

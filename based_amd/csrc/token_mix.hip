@@ -89,14 +89,6 @@ struct ChannelDecayArgs {
 
 constexpr float kLog2e = 1.4426950408889634f;
 
-__device__ __forceinline__ float tanh_f(float z) {
-  // exp(2z) overflows to infinity and 1 - 0 is left; 2^-24 of the result below |z| = 0.05 comes from the series
-  const float e = expf(2.0f * z), q = z * z;
-  const float far = 1.0f - 2.0f / (e + 1.0f);
-  const float near = z * (1.0f - q * (1.0f / 3.0f - q * (2.0f / 15.0f)));
-  return fabsf(z) < 0.05f ? near : far;
-}
-
 constexpr int kDecayRows = 16;
 
 // Any element type and size: 16 rows of tanh(h) in LDS, a thread per channel.

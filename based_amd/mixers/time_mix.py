@@ -63,6 +63,17 @@ class TimeMix(nn.Module):
                        norm_weight=self.norm_weight, eps=self.norm_eps, out=out[:, :self.width])
         return out
 
+    def supports_decode_step(self) -> bool:
+        return ops.decode_linear_weight_ok(self.in_proj.weight) and ops.decode_linear_weight_ok(self.out_proj.weight)
+
+    def decode_step(self, x, inference_params, **prologue):
+        """One token per sequence: norm and mixes inside the input projections (`ops.decode_linear`)."""
+        rows = x.shape[0] if prologue.get("row_index") is None else prologue["row_index"].numel()
+        pos, _ = portion_start(inference_params, rows, 1)
+        state, ring = self._cached(inference_params, rows)
+        proj = ops.decode_linear(x, self.in_proj.weight, mix=(self.mu, ring, pos, self.segment), **prologue)
+        return ops.decode_linear(self._step(*(proj[:, self._rows(i)] for i in range(len(self.MIXES))), state, pos), self.out_proj.weight)
+
     def forward(self, x, inference_params=None, **kwargs):
         """x (batch, seqlen, d_model) -> (batch, seqlen, d_model)."""
         B, L = x.shape[:2]

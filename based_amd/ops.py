@@ -594,7 +594,8 @@ def decode_linear_weight_ok(weight: torch.Tensor) -> bool:
 def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residual_in=None, residual_out=None,
                   norm_weight=None, eps: float = 1e-5, row_index=None, epilogue: int = EPILOGUE_NONE,
                   conv_state=None, conv_weight=None, conv_bias=None, out: Optional[torch.Tensor] = None,
-                  mult: float = 1.0, norm_kind: int = 0, input_conv=None) -> torch.Tensor:
+                  mult: float = 1.0, norm_kind: int = 0, input_conv=None, addends=None, mix=None, gate=None,
+                  softcap: float = 0.0) -> torch.Tensor:
     """y = epi(pro(x) @ weight.T (+ bias)) for the few rows of a single-token step, one launch.
 
     x: (M, K) bf16 rows (M <= 32; any leading shape is flattened), or for PROLOGUE_SWIGLU (M, 2K):
@@ -610,12 +611,21 @@ def decode_linear(x, weight, bias=None, *, prologue: int = PROLOGUE_NONE, residu
     PROLOGUE_STREAM: r = residual_in + mult * x in fp32 (written to residual_out), then the norm
     `norm_kind` of that sum times norm_weight, rounded to bf16, and with input_conv =
     (weight (taps, K), ring (M, taps, K), pos) that row plus its causal convolution; epilogues NONE and
-    SWIGLU."""
+    SWIGLU.  Instead of input_conv: `addends` (`Addends`) in the sum, NORM_NONE; mix = (mu (S, K), ring (M, 2, K), pos, rows):
+    weight rows i * rows .. read the i-th mix of the row with the one of the token before (`token_mix`), the last mix
+    all rows that are left; gate = (table (n, N), index (M)): gelu_tanh(y) * table[index]; softcap > 0: softcap * tanh(y / softcap)."""
     if prologue == PROLOGUE_STREAM:
         if conv_state is not None or conv_weight is not None or conv_bias is not None:
             raise ValueError("the streamed-input prologue has no convolution epilogue")
+        if addends is not None or mix is not None or gate is not None or softcap or norm_kind == NORM_NONE:
+            if input_conv is not None:
+                raise ValueError("an input convolution takes no addends, mixes, gate or cap")
+            return _decode_linear_extras(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult,
+                                         norm_kind, addends or Addends(), mix, gate, softcap, out)
         return _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult,
                                      norm_kind, input_conv, out)
+    if addends is not None or mix is not None or gate is not None or softcap:
+        raise ValueError("addends, mixes, gate and cap belong to PROLOGUE_STREAM")
     N, K = weight.shape
     x2 = x if x.dim() == 2 else x.reshape(-1, x.shape[-1])
     M = x2.shape[0] if row_index is None else row_index.numel()
@@ -1350,5 +1360,85 @@ def _decode_linear_stream(x, weight, bias, epilogue, residual_in, residual_out, 
             _ptr(bias), y.data_ptr(), y.stride(0), M, N, K, _ptr(residual_in), 0 if residual_in is None else residual_in.stride(0),
             _ptr(residual_out), 0 if residual_out is None else residual_out.stride(0), float(mult), int(norm_kind),
             norm_weight.data_ptr(), float(eps), _ptr(conv_w), _ptr(ring), ring_stride, taps, pos_ptr, pos_host, epilogue,
+            _stream_ptr(x2)))
+    return y
+
+
+def decode_linear_mixes(x, weight, mix_rows: int) -> torch.Tensor:
+    """(M, N): weight rows i * mix_rows .. times row m of x[i], x (mixes, M, K) bf16; the last mix all rows that are left."""
+    S, M, K = x.shape
+    N = weight.shape[0]
+    _require_cuda(x, weight)
+    if x.dtype != torch.bfloat16 or weight.dtype != torch.bfloat16 or weight.shape[1] != K or weight.stride(1) != 1 or not x.is_contiguous():
+        raise ValueError("x and weight must be bfloat16 rows of the contraction length, x contiguous")
+    y = torch.empty(M, N, dtype=torch.bfloat16, device=x.device)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_decode_linear_mixes(x.data_ptr(), weight.data_ptr(), weight.stride(0), y.data_ptr(), N, M, N, K, S,
+                                                        int(mix_rows), _stream_ptr(x)))
+    return y
+
+
+def _decode_linear_extras(x, weight, bias, epilogue, residual_in, residual_out, norm_weight, eps, row_index, mult, norm_kind, addends, mix,
+                          gate, softcap, out):
+    """`decode_linear` behind PROLOGUE_STREAM with what else may surround it."""
+    N, K = weight.shape
+    x2 = x if x.dim() == 2 else x.reshape(-1, x.shape[-1])
+    M = x2.shape[0] if row_index is None else row_index.numel()
+    n_out = N if epilogue == EPILOGUE_NONE else N // 2
+    _require_cuda(x2, weight)
+    if x2.dtype != torch.bfloat16 or weight.dtype != torch.bfloat16 or x2.shape[1] != K or weight.stride(1) != 1 or x2.stride(1) != 1:
+        raise ValueError("x and weight must be bfloat16 rows of the contraction length")
+    if norm_kind != NORM_NONE and (norm_weight is None or norm_weight.dtype != torch.bfloat16 or tuple(norm_weight.shape) != (K,)
+                                   or not norm_weight.is_contiguous() or not norm_weight.is_cuda):
+        raise ValueError(f"norm_weight must be a contiguous bfloat16 ({K},) on the device")
+    if bias is not None and (tuple(bias.shape) != (N,) or bias.dtype != torch.bfloat16 or not bias.is_contiguous()):
+        raise ValueError(f"bias must be a contiguous bfloat16 ({N},)")
+    for r in (residual_in, residual_out):
+        if r is not None and (r.dtype != torch.float32 or tuple(r.shape) != (M, K) or r.stride(1) != 1 or not r.is_cuda):
+            raise ValueError(f"residuals must be float32 ({M}, {K}) device tensors with contiguous rows")
+    if row_index is not None and (row_index.dtype != torch.int64 or row_index.dim() != 1 or not row_index.is_contiguous()
+                                  or not row_index.is_cuda):
+        raise ValueError("row_index must be a contiguous int64 device vector")
+    pos_ptr, pos_host = None, 0
+    if mix is not None:
+        mu, ring, pos, mix_rows = mix
+        _check_ring(ring, M, 2, K, x2)
+        if mu.dim() != 2 or mu.shape[1] != K or not mu.is_contiguous() or mu.dtype != torch.bfloat16 or not mu.is_cuda:
+            raise ValueError(f"mu must be a contiguous bfloat16 (mixes, {K})")
+        pos_ptr, pos_host = _pos_args(pos, M)
+    if gate is not None:
+        table, index = gate
+        if (epilogue != EPILOGUE_NONE or table.dim() != 2 or table.shape[1] != N or table.stride(1) != 1 or table.dtype != torch.bfloat16
+                or not table.is_cuda or index.dtype != torch.int64 or index.numel() != M or not index.is_contiguous() or not index.is_cuda):
+            raise ValueError(f"the gate must be a bfloat16 (entries, {N}) table with {M} contiguous int64 entries")
+    extra = _addend_args(addends, x2, M, K)
+    if M > STREAM_PROLOGUE_MAX_ROWS:
+        rows = x2 if row_index is None else x2.index_select(0, row_index)
+        h, _ = add_norm(rows, residual_in, norm_weight, eps, norm_kind, mult, residual_out is not None, residual_out, addends)
+        if mix is not None:
+            if bias is not None or out is not None or epilogue != EPILOGUE_NONE:
+                raise ValueError("mixes take no bias, epilogue or given output")
+            return decode_linear_mixes(token_mix(h.unsqueeze(1), mu, ring, pos).squeeze(2), weight, mix_rows)
+        y = decode_linear(h, weight, bias, epilogue=epilogue, out=out)
+        if gate is not None:
+            y = gelu_mul(y, table, index)
+        return softcap_(y, softcap) if softcap else y
+    y = torch.empty(M, n_out, dtype=torch.bfloat16, device=x2.device) if out is None else out
+    if tuple(y.shape) != (M, n_out) or y.dtype != torch.bfloat16 or y.stride(1) != 1:
+        raise ValueError(f"out must be a ({M}, {n_out}) bfloat16 tensor with contiguous rows")
+    post_weight, post_eps, vec, add_rows, add_index, add_sr, add_n = extra
+    ex = _lib.StreamExtras(post_weight=post_weight, post_eps=post_eps, add_vec=vec, add_rows=add_rows, add_index=add_index, add_sr=add_sr,
+                           add_n=add_n, softcap=float(softcap))
+    if mix is not None:
+        ex.mix_mu, ex.mix_ring, ex.mix_ring_row_stride = mu.data_ptr(), ring.data_ptr(), ring.stride(0)
+        ex.mixes, ex.mix_rows = mu.shape[0], int(mix_rows)
+    if gate is not None:
+        ex.gate_table, ex.gate_index, ex.gate_sr, ex.gate_n = table.data_ptr(), index.data_ptr(), table.stride(0), table.shape[0]
+    with _on_device(x2.device):
+        _lib.check(_lib.lib().based_decode_linear_extras(
+            x2.data_ptr(), x2.stride(0), _ptr(row_index), 0 if row_index is None else x2.shape[0], weight.data_ptr(), weight.stride(0),
+            _ptr(bias), y.data_ptr(), y.stride(0), M, N, K, _ptr(residual_in), 0 if residual_in is None else residual_in.stride(0),
+            _ptr(residual_out), 0 if residual_out is None else residual_out.stride(0), float(mult), int(norm_kind),
+            None if norm_kind == NORM_NONE else norm_weight.data_ptr(), float(eps), pos_ptr, pos_host, epilogue, ctypes.byref(ex),
             _stream_ptr(x2)))
     return y

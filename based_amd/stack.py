@@ -406,45 +406,61 @@ class Block(nn.Module):
 
     def supports_decode_step(self) -> bool:
         mlp = self.mlp
-        if self.side is not None or isinstance(mlp, ExpertMlp):
+        side = self.side
+        if side is not None and not (ops.decode_linear_weight_ok(side.gate.weight) and ops.decode_linear_weight_ok(side.proj.weight)):
             return False
         return (getattr(self.mixer, "supports_decode_step", lambda: False)()
-                and (mlp is None or (mlp.mlp_type == "base" and mlp.activation == "swiglu"
+                and (mlp is None or (isinstance(mlp, ExpertMlp) and norm_fuses(self.norm2)) or (
+                                     isinstance(mlp, GatedMlp) and mlp.mlp_type == "base" and mlp.activation == "swiglu"
                                      and ops.decode_linear_weight_ok(mlp.fc1.weight)
                                      and ops.decode_linear_weight_ok(mlp.fc2.weight) and norm_fuses(self.norm2)))
                 and norm_fuses(self.norm1) and self.residual_in_fp32)
 
-    def decode_step(self, hidden_states, residual, spare, inference_params, row_index=None):
-        """The block for one token per sequence in four to five launches: both norms run inside the
+    def decode_step(self, hidden_states, residual, spare, inference_params, row_index=None, addends=None, ids=None, side_table=None):
+        """The block for one token per sequence in four to seven launches: both norms run inside the
         projection that consumes them (`ops.decode_linear`), the SwiGLU gate in the tail of fc1.
         hidden_states (b, dim) bf16 (or the embedding table with `row_index`), residual fp32
         (b, dim) or None; `spare` is a second fp32 (b, dim) buffer: the two take turns as the
-        input and the output of the residual stream.  Returns (hidden, residual, spare)."""
+        input and the output of the residual stream.  addends: what else the first sum receives; ids and side_table:
+        tokens and table of the token input.  Returns (hidden, residual, spare)."""
         if residual is None:
-            residual_in, mid, last = None, spare[0], spare[1]
+            residual, (mid, last) = None, spare
         else:
-            residual_in, mid, last = residual, spare, residual
-        norm = norm_prologue(self.norm1, residual_in, mid)
+            mid, last = spare, residual
+        norm = norm_prologue(self.norm1, residual, mid)
         if row_index is not None:
             norm["row_index"] = row_index
+        if addends is not None:
+            norm["addends"] = addends
         if self.input_conv is not None:
             rows = mid.shape[0]
             pos, _ = portion_start(inference_params, rows, 1)
             norm["input_conv"] = (self.input_conv.weight, self.input_conv.ring(inference_params, rows), pos)
         hidden_states = self.mixer.decode_step(hidden_states, inference_params, **norm)
-        if self.mlp is None:
-            return hidden_states, mid, last
-        norm = norm_prologue(self.norm2, mid, last)
-        fc1, fc2 = self.mlp.fc1, self.mlp.fc2
-        if fc1.weight.shape[1] <= 2048:
-            # the gate in the tail of fc1
-            gated = ops.decode_linear(hidden_states, fc1.weight, fc1.bias, epilogue=ops.EPILOGUE_SWIGLU, **norm)
-            hidden_states = ops.decode_linear(gated, fc2.weight, fc2.bias)
-        else:
-            # wider models: the gate in front of fc2
-            gate_in = ops.decode_linear(hidden_states, fc1.weight, fc1.bias, **norm)
-            hidden_states = ops.decode_linear(gate_in, fc2.weight, fc2.bias, prologue=ops.PROLOGUE_SWIGLU)
-        return hidden_states, last, mid
+        if isinstance(self.mlp, ExpertMlp):
+            n = self.norm2
+            h, _ = ops.add_norm(hidden_states, mid, n.weight, n.eps, n.kind, n.mult, residual_out=last)
+            hidden_states = self.mlp(h)
+            mid, last = last, mid
+        elif self.mlp is not None:
+            norm = norm_prologue(self.norm2, mid, last)
+            fc1, fc2 = self.mlp.fc1, self.mlp.fc2
+            if fc1.weight.shape[1] <= 2048:
+                # the gate in the tail of fc1
+                gated = ops.decode_linear(hidden_states, fc1.weight, fc1.bias, epilogue=ops.EPILOGUE_SWIGLU, **norm)
+                hidden_states = ops.decode_linear(gated, fc2.weight, fc2.bias)
+            else:
+                # wider models: the gate in front of fc2
+                gate_in = ops.decode_linear(hidden_states, fc1.weight, fc1.bias, **norm)
+                hidden_states = ops.decode_linear(gate_in, fc2.weight, fc2.bias, prologue=ops.PROLOGUE_SWIGLU)
+            mid, last = last, mid
+        if self.side is not None:
+            side = self.side
+            g = ops.decode_linear(hidden_states, side.gate.weight, prologue=ops.PROLOGUE_STREAM, norm_kind=ops.NORM_NONE,
+                                  mult=self.norm1.mult, residual_in=mid, residual_out=last, gate=(side.table(side_table), ids))
+            hidden_states = ops.decode_linear(g, side.proj.weight)
+            mid, last = last, mid
+        return hidden_states, mid, last
 
     def forward(self, hidden_states, residual=None, mixer_kwargs=None, position_ids=None, decay=None, addends=None, ids=None,
                 side_table=None):
@@ -569,7 +585,7 @@ class GPTModel(nn.Module):
         if not (self.fused_decode and inference_params is not None and inference_params.seqlen_offset > 0
                 and input_ids.shape[1] == 1 and input_ids.shape[0] <= ops.DECODE_LINEAR_MAX_ROWS
                 and input_ids.is_cuda and not torch.is_grad_enabled()
-                and self.config.max_position_embeddings == 0 and self.loop_step is None):
+                and self.config.max_position_embeddings == 0):
             return False
         # the answer depends on dtypes and devices of the parameters only: worked out once per
         # (dtype, device) of the embedding table
@@ -593,15 +609,27 @@ class GPTModel(nn.Module):
             buffers = tuple(torch.empty(b, table.shape[1], dtype=torch.float32, device=table.device) for _ in range(2))
             self._decode_residuals[key] = buffers
         ids = input_ids.reshape(-1).contiguous()  # a column of a wider id tensor is a strided view
-        hidden_states, residual, spare = self.layers[0].decode_step(table, None, buffers, inference_params, row_index=ids)
-        for layer in self.layers[1:]:
-            hidden_states, residual, spare = layer.decode_step(hidden_states, residual, spare, inference_params)
+        hidden_states, residual, spare, addends = table, None, buffers, None
+        more = {"ids": ids, "side_table": self._side_table()} if self.config.token_side_dim > 0 else {}
+        for n, run in enumerate(self.runs):
+            layer = self.layers[run.layer]
+            inference_params.layer_pass = run.layer_pass
+            hidden_states, residual, spare = layer.decode_step(hidden_states, residual, spare, inference_params,
+                                                               row_index=ids if n == 0 else None,
+                                                               addends=self._run_addends(run, addends, ids), **more)
+            addends = layer.out_addends()
+        inference_params.layer_pass = 0
         return hidden_states, residual
+
+    def closing_addends(self):
+        """What the closing sum receives besides the last block's output."""
+        return self.layers[self.runs[-1].layer].out_addends()
 
     def forward(self, input_ids, position_ids=None, inference_params=None, stream=None):
         if self.decode_layers_ok(input_ids, inference_params):
             hidden_states, residual = self.decode_layers(input_ids, inference_params)
-            return add_norm(self.ln_f, hidden_states, residual, True, want_residual=False)[0].unsqueeze(1)
+            return add_norm(self.ln_f, hidden_states, residual, True, want_residual=False,
+                            addends=self.closing_addends())[0].unsqueeze(1)
         hidden_states = self.embeddings.word_embeddings(input_ids)
         if self.config.max_position_embeddings > 0:
             if position_ids is None:
@@ -718,7 +746,11 @@ class GPTLMHeadModel(nn.Module, GenerationMixin):
             # closing add + norm inside the LM head's projection
             hidden_states, residual = self.transformer.decode_layers(input_ids, inference_params)
             ln_f = self.transformer.ln_f
-            logits = ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias, **norm_prologue(ln_f, residual))
+            norm = norm_prologue(ln_f, residual)
+            if isinstance(ln_f, StreamNorm):
+                norm.update(addends=self.transformer.closing_addends(), softcap=self.config.logit_softcap or 0.0)
+                return CausalLMOutput(logits=ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias, **norm).unsqueeze(1))
+            logits = ops.decode_linear(hidden_states, self.lm_head.weight, self.lm_head.bias, **norm)
             return CausalLMOutput(logits=self._capped(logits).unsqueeze(1))
         hidden_states = self.transformer(input_ids, position_ids=position_ids, inference_params=inference_params,
                                          stream=stream)

@@ -664,6 +664,36 @@ BASED_API int based_expert_rows(const void* h, const void* w1, const void* w2, c
                                 void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t top, int64_t h_sr, int io_dtype,
                                 void* stream);
 
+/* based_decode_linear_stream with what else may surround a projection of single tokens; a pointer that is NULL leaves its part out.
+ *   post_weight, add_vec, add_rows: as in based_add_norm_addends (row m adds add_rows[add_index[m]]); norm_kind BASED_NORM_NONE
+ *     (norm_weight NULL) projects the sum itself.
+ *   mix_mu (mixes, K), mix_ring (M, 2, K): weight rows i * mix_rows .. (i + 1) * mix_rows - 1 read h + (h of the token before - h) * mu[i],
+ *     the last mix all rows that are left; the ring holds position p in slot p % 2.  mix_rows a multiple of 32.
+ *   gate_table (gate_n, N): the outputs become gelu_tanh(y) * gate_table[gate_index[m]].
+ *   softcap > 0: the outputs become softcap * tanh(y / softcap). */
+typedef struct {
+  const void* post_weight;
+  const void* add_vec;
+  const void* add_rows;
+  const int64_t* add_index;
+  const void* mix_mu;
+  void* mix_ring;
+  const void* gate_table;
+  const int64_t* gate_index;
+  int64_t add_sr, add_n, mix_rows, mixes, mix_ring_row_stride, gate_sr, gate_n;
+  float post_eps, softcap;
+} based_stream_extras;
+BASED_API int based_decode_linear_extras(const void* x, int64_t x_row_stride, const int64_t* x_row_index, int64_t x_index_rows,
+                                         const void* weight, int64_t w_row_stride, const void* bias, void* y,
+                                         int64_t y_row_stride, int64_t M, int64_t N, int64_t K, const float* residual_in,
+                                         int64_t ri_row_stride, float* residual_out, int64_t ro_row_stride, float mult,
+                                         int norm_kind, const void* norm_weight, float eps, const int32_t* pos,
+                                         int64_t pos_host, int epilogue, const based_stream_extras* extras, void* stream);
+
+/* y[m] = W x where weight rows i * mix_rows .. read row m of x (mixes, M, K), the last mix all rows that are left. */
+BASED_API int based_decode_linear_mixes(const void* x, const void* weight, int64_t w_row_stride, void* y, int64_t y_row_stride,
+                                        int64_t M, int64_t N, int64_t K, int64_t mixes, int64_t mix_rows, void* stream);
+
 #ifdef __cplusplus
 }
 #endif
