@@ -40,7 +40,7 @@ struct DecayScanArgs {
   const void* u;         // (H, d)
   float* state;          // (B, H, dv, dp)
   float* seg;            // (B, H, segs, dv, dp) work, null with one segment
-  float* seg_lw;         // (B, H, segs, dp) work
+  float* seg_lw;         // (B, H, segs, dp) work: channel decays over a segment
   void* o;               // (B, L, H * dv)
   int B, L, H, d, dv, dp;
   long q_sb, q_sl, k_sb, k_sl, v_sb, v_sl, o_sb, o_sl;
@@ -51,20 +51,36 @@ struct DecayScanArgs {
 template <int CTRL> __device__ __forceinline__ float row_moved(float x) {  // lanes without a source receive 0
   return __builtin_bit_cast(float, __builtin_amdgcn_update_dpp(0, __builtin_bit_cast(int, x), CTRL, 0xf, 0xf, true));
 }
-// sums over lanes 0 .. l of a 16-lane row
-__device__ __forceinline__ float row_prefix(float x) {
-  x += row_moved<0x111>(x);
-  x += row_moved<0x112>(x);
-  x += row_moved<0x114>(x);
-  return x + row_moved<0x118>(x);
+// Products along the 16 lanes of a row, of several independent numbers at once.  A DPP multiplication leaves a lane
+// without a source as it is, which is the multiplication by one that is wanted; the compiler has no builtin that
+// says so.  A register must not be read through DPP in the two issue slots after it was written: four numbers in turn
+// keep that distance by themselves, the first ones are kept from what stands before by the s_nop.
+//   prefix[i]: product over lanes 0 .. l of w[i];  suffix[i]: over lanes l .. 15
+//   before[i] *= prefix of the lane before (nothing for lane 0);  after[i] *= suffix of the lane behind (nothing for lane 15)
+#define BASED_ROW_STEP(ctrl) \
+  "v_mul_f32_dpp %0, %0, %0 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %1, %1, %1 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %2, %2, %2 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %3, %3, %3 " ctrl " row_mask:0xf bank_mask:0xf\n\t"
+#define BASED_ROW_LAST(ctrl) \
+  "v_mul_f32_dpp %4, %0, %4 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %5, %1, %5 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %6, %2, %6 " ctrl " row_mask:0xf bank_mask:0xf\n\t" \
+  "v_mul_f32_dpp %7, %3, %7 " ctrl " row_mask:0xf bank_mask:0xf"
+__device__ __forceinline__ void row_prefix4(float* prefix, float* before) {
+  asm volatile("s_nop 1\n\t" BASED_ROW_STEP("row_shr:1") BASED_ROW_STEP("row_shr:2") BASED_ROW_STEP("row_shr:4")
+               BASED_ROW_STEP("row_shr:8") BASED_ROW_LAST("row_shr:1")
+               : "+v"(prefix[0]), "+v"(prefix[1]), "+v"(prefix[2]), "+v"(prefix[3]), "+v"(before[0]), "+v"(before[1]), "+v"(before[2]),
+                 "+v"(before[3]));
 }
-// sums over lanes l .. 15
-__device__ __forceinline__ float row_suffix(float x) {
-  x += row_moved<0x101>(x);
-  x += row_moved<0x102>(x);
-  x += row_moved<0x104>(x);
-  return x + row_moved<0x108>(x);
+__device__ __forceinline__ void row_suffix4(float* suffix, float* after) {
+  asm volatile("s_nop 1\n\t" BASED_ROW_STEP("row_shl:1") BASED_ROW_STEP("row_shl:2") BASED_ROW_STEP("row_shl:4")
+               BASED_ROW_STEP("row_shl:8") BASED_ROW_LAST("row_shl:1")
+               : "+v"(suffix[0]), "+v"(suffix[1]), "+v"(suffix[2]), "+v"(suffix[3]), "+v"(after[0]), "+v"(after[1]), "+v"(after[2]),
+                 "+v"(after[3]));
 }
+#undef BASED_ROW_STEP
+#undef BASED_ROW_LAST
 // sum over the four lanes l16, l16 + 16, + 32, + 48, in all of them
 __device__ __forceinline__ float quad_rows_sum(float x) {
   x += __shfl_xor(x, 16, 64);
@@ -72,16 +88,36 @@ __device__ __forceinline__ float quad_rows_sum(float x) {
 }
 
 __device__ __forceinline__ f32x4 mfma_16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
-__device__ __forceinline__ void split(float x, __bf16& hi, __bf16& lo) {
-  hi = (__bf16)x;
-  lo = (__bf16)(x - (float)hi);
+// two numbers as packed pairs of bf16: rounded, and what the rounding left
+__device__ __forceinline__ void split2(float a, float b, uint32_t& hi, uint32_t& lo) {
+  hi = pack_bf16(a, b);
+  lo = pack_bf16(a - __builtin_bit_cast(float, hi << 16), b - __builtin_bit_cast(float, hi & 0xffff0000u));
+}
+typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
+// eight numbers in the order of an MFMA operand
+__device__ __forceinline__ void split8(const float* x, bf16x8& hi, bf16x8& lo) {
+  u32x4 h, l;
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    uint32_t a, b;
+    split2(x[2 * i], x[2 * i + 1], a, b);
+    h[i] = a, l[i] = b;
+  }
+  hi = __builtin_bit_cast(bf16x8, h);
+  lo = __builtin_bit_cast(bf16x8, l);
+}
+// the halves of a packed pair as they are
+__device__ __forceinline__ void store_pair(__bf16* p, __bf16* q, uint32_t x) {
+  *reinterpret_cast<uint16_t*>(p) = (uint16_t)x;
+  *reinterpret_cast<uint16_t*>(q) = (uint16_t)(x >> 16);
 }
 
-// DT: 32-channel pieces of the key size (d <= 32 DT, d % 4 == 0).  Channels of a piece are held by the lanes in the
+// HALVES wavefronts (1 or 2) share the key channels of 16 tokens, DT 32-channel pieces each (d <= 32 DT HALVES, d % 4 == 0), so
+// that what a lane holds of a token stays in registers; their parts of P are added through LDS.  Channels of a piece are held by the lanes in the
 // order of the accumulators: element e < 4 of a lane in 16-lane row `quad` is channel 4 quad + e, e >= 4
 // channel 16 + 4 quad + e - 4; every contraction over channels uses that order on both sides.
-template <int DT, bool CHANNEL> struct ScanLds {
-  static constexpr int CH = 32 * DT, RS = CH + 8, TS = kScanTokens + 8;
+template <int DT, int HALVES, bool CHANNEL> struct ScanLds {
+  static constexpr int CH = 32 * DT * HALVES, RS = CH + 8, TS = kScanTokens + 8;
   __bf16 q_hi[kScanTokens * RS];                 // q scaled to the start of the 64 tokens; head decays: q itself
   __bf16 q_lo[CHANNEL ? kScanTokens * RS : 8];
   union {
@@ -91,22 +127,24 @@ template <int DT, bool CHANNEL> struct ScanLds {
     } k;
     struct {
       __bf16 hi[kScanTokens * TS], lo[kScanTokens * TS];  // P, [t][s]
+      f32x4 part[HALVES > 1 ? 4 * 4 * 64 : 1];            // the second half's part of P, as its lanes hold it
     } p;
   };
   __bf16 kt_hi[CH * TS], kt_lo[CH * TS];         // k decayed to the end of the 64 tokens, [channel][token]
-  __bf16 vt[64 * TS];                            // v, [channel][token]
-  float total[4][CH];                            // log decay over each 16 tokens
+  __bf16 vt[64 * HALVES * TS];                            // v, [channel][token]
+  float total[4][CH], all[CH];                   // decay over each 16 tokens, and over the 64
 };
 
-template <int DT, bool CHANNEL, bool STATE_ONLY>
-__global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArgs a) {
-  typedef ScanLds<DT, CHANNEL> Lds;
-  constexpr int RS = Lds::RS, TS = Lds::TS, E = DT * 8;
+template <int DT, int HALVES, bool CHANNEL, bool STATE_ONLY>
+__global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const DecayScanArgs a) {
+  typedef ScanLds<DT, HALVES, CHANNEL> Lds;
+  constexpr int RS = Lds::RS, TS = Lds::TS, E = DT * 8, DA = DT * HALVES;
   extern __shared__ __attribute__((aligned(16))) char scan_lds[];
   Lds& lds = *reinterpret_cast<Lds*>(scan_lds);
   const int lane = threadIdx.x & 63, wave = __builtin_amdgcn_readfirstlane(threadIdx.x >> 6), l16 = lane & 15, quad = lane >> 4;
+  const int blk = wave & 3, half = wave >> 2, ch0 = half * 32 * DT;  // this wavefront's 16 tokens of 64, and its key channels
   const int b = blockIdx.x / a.H, h = blockIdx.x % a.H, sg = blockIdx.z;
-  const int col_base = blockIdx.y * 64, dv0 = col_base + wave * 16;
+  const int col_base = blockIdx.y * 64 * HALVES, dv0 = col_base + wave * 16;
   const bool has_cols = dv0 < a.dv, col_in = dv0 + l16 < a.dv;
   const __bf16* qp = static_cast<const __bf16*>(a.q) + b * a.q_sb + (long)h * a.d;
   const __bf16* kp = static_cast<const __bf16*>(a.k) + b * a.k_sb + (long)h * a.d;
@@ -117,41 +155,22 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
   float* st = a.state + (bh * a.dv + (col_in ? dv0 + l16 : 0)) * a.dp;
 
   // channel of element e of piece c
-  auto chan = [&](int c, int half) { return c * 32 + half * 16 + quad * 4; };
-
-  float bonus[CHANNEL && !STATE_ONLY ? E : 1];
-  auto load_bonus = [&]() {
-    if constexpr (CHANNEL && !STATE_ONLY) {
-#pragma unroll
-    for (int c = 0; c < DT; ++c)
-#pragma unroll
-      for (int f = 0; f < 2; ++f) {
-        const int ch = chan(c, f);
-        const bf16x4 x = *reinterpret_cast<const bf16x4*>(static_cast<const __bf16*>(a.u) + (long)h * a.d + (ch < a.d ? ch : 0));
-#pragma unroll
-        for (int j = 0; j < 4; ++j) bonus[c * 8 + f * 4 + j] = to_f32(x[j]);
-      }
-    }
-  };
-  if constexpr (DT < 4) load_bonus();  // (tall heads load it where it is used, for their registers)
+  auto chan = [&](int c, int f) { return ch0 + c * 32 + f * 16 + quad * 4; };
+  auto chan_of = [&](int i) { return ch0 + (i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3); };
 
   // state: tile ct holds key channels 16 ct + 4 quad + i of value channel dv0 + l16
-  f32x4 S[2 * DT];
+  f32x4 S[2 * DA];
   {
     const float* from = a.segs > 1 ? a.seg + ((bh * a.segs + sg) * a.dv + (col_in ? dv0 + l16 : 0)) * a.dp : st;
     const bool zero = STATE_ONLY || (a.segs == 1 && a.fresh);
 #pragma unroll
-    for (int ct = 0; ct < 2 * DT; ++ct) {
+    for (int ct = 0; ct < 2 * DA; ++ct) {
       const int ch = ct * 16 + quad * 4;
       S[ct] = f32x4{0.f, 0.f, 0.f, 0.f};
       if (!zero && col_in && ch < a.d) S[ct] = *reinterpret_cast<const f32x4*>(from + ch);
     }
   }
-  float seg_total[CHANNEL && STATE_ONLY ? E : 1];  // (state pass) log decay of the segment so far, channels as in S
-  if constexpr (CHANNEL && STATE_ONLY) {
-#pragma unroll
-    for (int i = 0; i < E; ++i) seg_total[i] = 0.f;
-  }
+  float seg_total = 1.f;  // (state pass, channel decays) decay of the segment so far, of the channel that is this thread's number
 
   struct Stage {
     bf16x4 q[STATE_ONLY ? 1 : 2 * DT], k[2 * DT], v[4];
@@ -159,145 +178,214 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
   };
   const int first = sg * a.seg_chunks, chunks = (a.L + kScanTokens - 1) / kScanTokens;
   const int last = first + a.seg_chunks < chunks ? first + a.seg_chunks : chunks;
-  // the rows of this wavefront's 16 tokens, unconditionally (places past the end are cleared at use)
+  // the rows of this wavefront's 16 tokens, unconditionally (places past the end are cleared at use): the place of the
+  // 64 tokens is the same for all lanes, and what lies behind it fits 32 bits
   auto fetch = [&](Stage& s, int chunk) {
-    int t = chunk * kScanTokens + wave * 16 + l16;
-    t = t < a.L ? t : a.L - 1;
+    const int left = a.L - chunk * kScanTokens, mine = blk * 16 + l16, t = mine < left ? mine : left - 1;
+    const long t0 = (long)chunk * kScanTokens;
+    const __bf16* q0 = qp + t0 * a.q_sl;
+    const __bf16* k0 = kp + t0 * a.k_sl;
+    const __bf16* v0 = vp + t0 * a.v_sl;
+    const float* w0 = CHANNEL ? lwp + t0 * a.H * a.d : nullptr;
+    const int tq = t * (int)a.q_sl, tk = t * (int)a.k_sl, tv = t * (int)a.v_sl, tw = t * a.H * a.d;
 #pragma unroll
-    for (int c = 0; c < DT; ++c)
-#pragma unroll
-      for (int f = 0; f < 2; ++f) {
-        const int ch = chan(c, f) < a.d ? chan(c, f) : 0;
-        if constexpr (!STATE_ONLY) s.q[c * 2 + f] = *reinterpret_cast<const bf16x4*>(qp + t * a.q_sl + ch);
-        s.k[c * 2 + f] = *reinterpret_cast<const bf16x4*>(kp + t * a.k_sl + ch);
-        if constexpr (CHANNEL) s.lw[c * 2 + f] = *reinterpret_cast<const f32x4*>(lwp + (long)t * a.H * a.d + ch);
-      }
+    for (int g = 0; g < 2 * DT; ++g) {
+      const int ch = chan(g >> 1, g & 1) < a.d ? chan(g >> 1, g & 1) : 0;
+      if constexpr (!STATE_ONLY) s.q[g] = *reinterpret_cast<const bf16x4*>(q0 + (tq + ch));
+      s.k[g] = *reinterpret_cast<const bf16x4*>(k0 + (tk + ch));
+      if constexpr (CHANNEL) s.lw[g] = *reinterpret_cast<const f32x4*>(w0 + (tw + ch));
+    }
 #pragma unroll
     for (int f = 0; f < 4; ++f) {
-      const int col = col_base + quad * 16 + f * 4;
-      s.v[f] = *reinterpret_cast<const bf16x4*>(vp + t * a.v_sl + (col < a.dv ? col : 0));
+      const int col = col_base + half * 64 + quad * 16 + f * 4;
+      s.v[f] = *reinterpret_cast<const bf16x4*>(v0 + (tv + (col < a.dv ? col : 0)));
     }
   };
-  auto active = [&](float x) { return a.silu ? round_to<__bf16>(silu_exact(x)) : x; };
 
-  // the next 64 tokens are asked for while these are worked on, where the registers allow it
-  constexpr bool AHEAD = DT < 4 || !CHANNEL || STATE_ONLY;
+  // the next 64 tokens are asked for as soon as these are in registers, or where those are scarce behind P
+  constexpr bool LATE = CHANNEL && !STATE_ONLY && HALVES > 1;
   Stage cur;
-  if (AHEAD && first < last) fetch(cur, first);
+  if (first < last) fetch(cur, first);
   for (int chunk = first; chunk < last; ++chunk) {
     const int left = a.L - chunk * kScanTokens, n = left < kScanTokens ? left : kScanTokens;
-    const int t = wave * 16 + l16;  // this lane's token
+    const int t = blk * 16 + l16;  // this lane's token
     const bool live = t < n;
-    if constexpr (!AHEAD) fetch(cur, chunk);
-    float q[STATE_ONLY ? 1 : E], k[E], g_before[CHANNEL ? E : 1], g_after[CHANNEL ? E : 1], w[CHANNEL && !STATE_ONLY ? E : 1];
+    float q[STATE_ONLY ? 1 : E], k[E], w[CHANNEL ? E : 1];
 #pragma unroll
-    for (int c = 0; c < DT; ++c)
-#pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        const int i = c * 8 + e;
-        const bool in = live && chan(c, e >> 2) < a.d;
-        if constexpr (!STATE_ONLY) q[i] = in ? active(to_f32(cur.q[c * 2 + (e >> 2)][e & 3])) : 0.f;
-        k[i] = in ? active(to_f32(cur.k[c * 2 + (e >> 2)][e & 3])) : 0.f;
-        if constexpr (CHANNEL) g_after[i] = in ? cur.lw[c * 2 + (e >> 2)][e & 3] : 0.f;
-      }
-    __bf16 vv[16];
-#pragma unroll
-    for (int f = 0; f < 4; ++f)
-#pragma unroll
-      for (int j = 0; j < 4; ++j)
-        vv[f * 4 + j] = live && col_base + quad * 16 + f * 4 < a.dv ? from_f32<__bf16>(active(to_f32(cur.v[f][j]))) : (__bf16)0.f;
-    if (AHEAD && chunk + 1 < last) fetch(cur, chunk + 1);
-
-    __syncthreads();  // every wavefront is done with the 64 tokens before
-#pragma unroll
-    for (int j = 0; j < 16; ++j) lds.vt[(quad * 16 + j) * TS + t] = vv[j];
-    if constexpr (CHANNEL) {
-      // log decays: of the tokens of these 16 before this one, and of those after it
+    for (int i = 0; i < E; ++i) {
+      if constexpr (!STATE_ONLY) q[i] = to_f32(cur.q[i >> 2][i & 3]);
+      k[i] = to_f32(cur.k[i >> 2][i & 3]);
+    }
+    if (a.silu) {  // (one branch for all of them)
 #pragma unroll
       for (int i = 0; i < E; ++i) {
-        const float lw = g_after[i];
-        const float incl = row_prefix(lw), suf = row_suffix(lw);
-        if constexpr (!STATE_ONLY) w[i] = row_moved<0x111>(lw);  // of the token before
-        g_before[i] = row_moved<0x111>(incl);
-        g_after[i] = row_moved<0x101>(suf);
-        if (l16 == 15) lds.total[wave][(i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3)] = incl;
+        if constexpr (!STATE_ONLY) q[i] = round_to<__bf16>(silu_exact(q[i]));
+        k[i] = round_to<__bf16>(silu_exact(k[i]));
+      }
+    }
+#pragma unroll
+    for (int g = 0; g < 2 * DT; ++g) {
+      const bool in = live && chan(g >> 1, g & 1) < a.d;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        if constexpr (!STATE_ONLY) q[g * 4 + j] = in ? q[g * 4 + j] : 0.f;
+        k[g * 4 + j] = in ? k[g * 4 + j] : 0.f;
+        if constexpr (CHANNEL) w[g * 4 + j] = in ? __builtin_amdgcn_exp2f(cur.lw[g][j]) : 1.f;
+      }
+    }
+
+    if constexpr (HALVES > 1) __builtin_amdgcn_sched_barrier(0);
+    f32x4 diag = {0.f, 0.f, 0.f, 0.f};  // the weights inside the 16 tokens: column t, rows s = 4 quad + i
+    if constexpr (CHANNEL && !STATE_ONLY) {
+      const int rel = l16 - quad * 4;  // row i is j tokens back where rel = j + i
+      float sum = 0.f;
+#pragma unroll
+      for (int g = 0; g < 2 * DT; ++g) {
+        const int ch = chan(g >> 1, g & 1) < a.d ? chan(g >> 1, g & 1) : 0;
+        const bf16x4 u = *reinterpret_cast<const bf16x4*>(static_cast<const __bf16*>(a.u) + (long)h * a.d + ch);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) sum = __builtin_fmaf(q[g * 4 + j] * to_f32(u[j]), k[g * 4 + j], sum);
+      }
+      sum = quad_rows_sum(sum);
+#pragma unroll
+      for (int i = 0; i < 4; ++i) diag[i] = rel == i ? sum : diag[i];
+      float x[E], before[E];
+#pragma unroll
+      for (int i = 0; i < E; ++i) {
+        x[i] = row_moved<0x111>(k[i]);
+        before[i] = row_moved<0x111>(w[i]);  // of the token before
+      }
+      constexpr int kUnroll = HALVES > 1 ? 3 : 15;  // (fewer steps in flight where registers are scarce)
+#pragma unroll kUnroll
+      for (int j = 1; j < 16; ++j) {
+        sum = 0.f;
+#pragma unroll
+        for (int i = 0; i < E; ++i) {
+          sum = __builtin_fmaf(q[i], x[i], sum);
+          x[i] = row_moved<0x111>(x[i]) * before[i];
+        }
+        sum = quad_rows_sum(sum);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) diag[i] = rel == j + i ? sum : diag[i];
+      }
+    }
+
+    __builtin_amdgcn_sched_barrier(0);
+    uint32_t vv[8];
+    {
+      float v[16];
+#pragma unroll
+      for (int j = 0; j < 16; ++j) v[j] = to_f32(cur.v[j >> 2][j & 3]);
+      if (a.silu) {
+#pragma unroll
+        for (int j = 0; j < 16; ++j) v[j] = silu_exact(v[j]);
+      }
+#pragma unroll
+      for (int f = 0; f < 4; ++f) {
+        const bool in = live && col_base + half * 64 + quad * 16 + f * 4 < a.dv;
+#pragma unroll
+        for (int j = 0; j < 2; ++j) vv[f * 2 + j] = in ? pack_bf16(v[f * 4 + 2 * j], v[f * 4 + 2 * j + 1]) : 0u;
+      }
+    }
+    if (!LATE && chunk + 1 < last) fetch(cur, chunk + 1);
+    __syncthreads();  // every wavefront is done with the 64 tokens before
+#pragma unroll
+    for (int j = 0; j < 8; ++j)
+      store_pair(&lds.vt[(half * 64 + quad * 16 + 2 * j) * TS + t], &lds.vt[(half * 64 + quad * 16 + 2 * j + 1) * TS + t], vv[j]);
+    if constexpr (CHANNEL) {
+      if constexpr (HALVES > 1) __builtin_amdgcn_sched_barrier(0);
+      // q decayed from the start of these 16 tokens, k to their end
+      if constexpr (!STATE_ONLY) {
+        float prefix[E];
+#pragma unroll
+        for (int i = 0; i < E; ++i) prefix[i] = w[i];
+#pragma unroll
+        for (int i = 0; i < E; i += 4) row_prefix4(prefix + i, q + i);
+      }
+#pragma unroll
+      for (int i = 0; i < E; i += 4) row_suffix4(w + i, k + i);
+      // (the product over all 16 is lane 0's suffix)
+      if (l16 == 0) {
+#pragma unroll
+        for (int i = 0; i < E; i += 4) *reinterpret_cast<f32x4*>(&lds.total[blk][chan_of(i)]) = f32x4{w[i], w[i + 1], w[i + 2], w[i + 3]};
       }
       if constexpr (!STATE_ONLY) {
 #pragma unroll
         for (int c = 0; c < DT; ++c) {
           bf16x8 hi, lo;
-#pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            __bf16 x, y;
-            split(k[c * 8 + e] * __builtin_amdgcn_exp2f(g_after[c * 8 + e]), x, y);
-            hi[e] = x, lo[e] = y;
-          }
-          *reinterpret_cast<bf16x8*>(&lds.k.hi[t * RS + c * 32 + quad * 8]) = hi;
-          *reinterpret_cast<bf16x8*>(&lds.k.lo[t * RS + c * 32 + quad * 8]) = lo;
+          split8(k + c * 8, hi, lo);
+          *reinterpret_cast<bf16x8*>(&lds.k.hi[t * RS + ch0 + c * 32 + quad * 8]) = hi;
+          *reinterpret_cast<bf16x8*>(&lds.k.lo[t * RS + ch0 + c * 32 + quad * 8]) = lo;
         }
       }
     } else {
       const float f = __builtin_amdgcn_exp2f(head_l2 * (float)(n - 1 - t > 0 ? n - 1 - t : 0));
 #pragma unroll
-      for (int c = 0; c < DT; ++c) {
-        bf16x8 q8, k8;
+      for (int i = 0; i < E; i += 2) {
+        uint32_t hi, lo;
+        split2(k[i] * f, k[i + 1] * f, hi, lo);
+        store_pair(&lds.kt_hi[chan_of(i) * TS + t], &lds.kt_hi[(chan_of(i) + 1) * TS + t], hi);
+        store_pair(&lds.kt_lo[chan_of(i) * TS + t], &lds.kt_lo[(chan_of(i) + 1) * TS + t], lo);
+      }
+      if constexpr (!STATE_ONLY) {
 #pragma unroll
-        for (int e = 0; e < 8; ++e) {
-          const int ch = c * 32 + (e >> 2) * 16 + quad * 4 + (e & 3);
-          __bf16 x, y;
-          split(k[c * 8 + e] * f, x, y);
-          lds.kt_hi[ch * TS + t] = x;
-          lds.kt_lo[ch * TS + t] = y;
-          k8[e] = (__bf16)k[c * 8 + e];
-          if constexpr (!STATE_ONLY) q8[e] = (__bf16)q[c * 8 + e];
-        }
-        if constexpr (!STATE_ONLY) {
-          *reinterpret_cast<bf16x8*>(&lds.k.hi[t * RS + c * 32 + quad * 8]) = k8;
-          *reinterpret_cast<bf16x8*>(&lds.q_hi[t * RS + c * 32 + quad * 8]) = q8;
+        for (int c = 0; c < DT; ++c) {
+          u32x4 q4, k4;
+#pragma unroll
+          for (int e = 0; e < 4; ++e) {
+            q4[e] = pack_bf16(q[c * 8 + 2 * e], q[c * 8 + 2 * e + 1]);
+            k4[e] = pack_bf16(k[c * 8 + 2 * e], k[c * 8 + 2 * e + 1]);
+          }
+          *reinterpret_cast<u32x4*>(&lds.k.hi[t * RS + ch0 + c * 32 + quad * 8]) = k4;
+          *reinterpret_cast<u32x4*>(&lds.q_hi[t * RS + ch0 + c * 32 + quad * 8]) = q4;
         }
       }
     }
     __syncthreads();
 
+    if constexpr (CHANNEL) {
+      const int ch = threadIdx.x;
+      if (ch < Lds::CH) {
+        const float all = (lds.total[0][ch] * lds.total[1][ch]) * (lds.total[2][ch] * lds.total[3][ch]);
+        lds.all[ch] = all;
+        if constexpr (STATE_ONLY) seg_total *= all;
+      }
+    }
     f32x4 P[STATE_ONLY ? 1 : 4];  // P^T tiles: column t of this wavefront's 16 tokens, rows s of 16 tokens j
     if constexpr (CHANNEL) {
 #pragma unroll
-      for (int i = 0; i < E; ++i) {
-        const int ch = (i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3);
-        float to_end = 0.f;  // log decay over the 16-token groups behind this one
+      for (int i = 0; i < E; i += 4) {
+        f32x4 x = {k[i], k[i + 1], k[i + 2], k[i + 3]};
 #pragma unroll
-        for (int m = 1; m < 4; ++m) to_end += m > wave ? lds.total[m][ch] : 0.f;
-        __bf16 x, y;
-        split(k[i] * __builtin_amdgcn_exp2f(g_after[i] + to_end), x, y);
-        lds.kt_hi[ch * TS + t] = x;
-        lds.kt_lo[ch * TS + t] = y;
+        for (int m = 1; m < 4; ++m)  // the 16-token groups behind this one
+          if (m > blk) x *= *reinterpret_cast<const f32x4*>(&lds.total[m][chan_of(i)]);
+#pragma unroll
+        for (int e = 0; e < 4; e += 2) {
+          const int ch = chan_of(i) + e;
+          uint32_t hi, lo;
+          split2(x[e], x[e + 1], hi, lo);
+          store_pair(&lds.kt_hi[ch * TS + t], &lds.kt_hi[(ch + 1) * TS + t], hi);
+          store_pair(&lds.kt_lo[ch * TS + t], &lds.kt_lo[(ch + 1) * TS + t], lo);
+        }
       }
       if constexpr (!STATE_ONLY) {
 #pragma unroll
         for (int j = 0; j < 4; ++j) P[j] = f32x4{0.f, 0.f, 0.f, 0.f};
         // q scaled to the start of its own 16 tokens, then by the groups in between, nearest first
-        float between[E];
-#pragma unroll
-        for (int i = 0; i < E; ++i) between[i] = 0.f;
 #pragma unroll
         for (int step = 1; step <= 4; ++step) {
-          const int j = wave - step;  // the last round scales to the start of the 64 tokens
+          __builtin_amdgcn_sched_barrier(0);
+          const int j = blk - step;  // the last round scales to the start of the 64 tokens
           if (j < -1) break;
           bf16x8 hi[DT], lo[DT];
 #pragma unroll
-          for (int c = 0; c < DT; ++c)
-#pragma unroll
-            for (int e = 0; e < 8; ++e) {
-              __bf16 x, y;
-              split(q[c * 8 + e] * __builtin_amdgcn_exp2f(g_before[c * 8 + e] + between[c * 8 + e]), x, y);
-              hi[c][e] = x, lo[c][e] = y;
-            }
+          for (int c = 0; c < DT; ++c) split8(q + c * 8, hi[c], lo[c]);
           if (j >= 0) {
             f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
             for (int c = 0; c < DT; ++c) {
-              const bf16x8 kh = *reinterpret_cast<const bf16x8*>(&lds.k.hi[(j * 16 + l16) * RS + c * 32 + quad * 8]);
-              const bf16x8 kl = *reinterpret_cast<const bf16x8*>(&lds.k.lo[(j * 16 + l16) * RS + c * 32 + quad * 8]);
+              const bf16x8 kh = *reinterpret_cast<const bf16x8*>(&lds.k.hi[(j * 16 + l16) * RS + ch0 + c * 32 + quad * 8]);
+              const bf16x8 kl = *reinterpret_cast<const bf16x8*>(&lds.k.lo[(j * 16 + l16) * RS + ch0 + c * 32 + quad * 8]);
               acc = mfma_16(kh, hi[c], acc);
               acc = mfma_16(kl, hi[c], acc);
               acc = mfma_16(kh, lo[c], acc);
@@ -305,57 +393,31 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
 #pragma unroll
             for (int m = 0; m < 3; ++m) P[m] = m == j ? acc : P[m];
 #pragma unroll
-            for (int i = 0; i < E; ++i)
-              between[i] += lds.total[j][(i >> 3) * 32 + ((i >> 2) & 1) * 16 + quad * 4 + (i & 3)];
+            for (int i = 0; i < E; i += 4) {
+              const f32x4 f = *reinterpret_cast<const f32x4*>(&lds.total[j][chan_of(i)]);
+#pragma unroll
+              for (int e = 0; e < 4; ++e) q[i + e] *= f[e];
+            }
           } else {
 #pragma unroll
             for (int c = 0; c < DT; ++c) {
-              *reinterpret_cast<bf16x8*>(&lds.q_hi[t * RS + c * 32 + quad * 8]) = hi[c];
-              *reinterpret_cast<bf16x8*>(&lds.q_lo[t * RS + c * 32 + quad * 8]) = lo[c];
+              *reinterpret_cast<bf16x8*>(&lds.q_hi[t * RS + ch0 + c * 32 + quad * 8]) = hi[c];
+              *reinterpret_cast<bf16x8*>(&lds.q_lo[t * RS + ch0 + c * 32 + quad * 8]) = lo[c];
             }
           }
         }
-        // the 16 tokens themselves: rows s = 4 quad + i
-        f32x4 diag = {0.f, 0.f, 0.f, 0.f};
-        {
-          if constexpr (DT >= 4) load_bonus();
-          float sum = 0.f;
 #pragma unroll
-          for (int i = 0; i < E; ++i) sum = __builtin_fmaf(q[i] * bonus[i], k[i], sum);
-          sum = quad_rows_sum(sum);
-#pragma unroll
-          for (int i = 0; i < 4; ++i) diag[i] = l16 == quad * 4 + i ? sum : diag[i];
-        }
-        float x[E];
-#pragma unroll
-        for (int i = 0; i < E; ++i) {
-          x[i] = row_moved<0x111>(k[i]);
-          w[i] = __builtin_amdgcn_exp2f(w[i]);
-        }
-#pragma unroll
-        for (int j = 1; j < 16; ++j) {
-          float sum = 0.f;
-#pragma unroll
-          for (int i = 0; i < E; ++i) {
-            sum = __builtin_fmaf(q[i], x[i], sum);
-            if (j < 15) x[i] = row_moved<0x111>(x[i]) * w[i];
-          }
-          sum = quad_rows_sum(sum);
-#pragma unroll
-          for (int i = 0; i < 4; ++i) diag[i] = l16 - quad * 4 - i == j ? sum : diag[i];
-        }
-#pragma unroll
-        for (int m = 0; m < 4; ++m) P[m] = m == wave ? diag : P[m];
+        for (int m = 0; m < 4; ++m) P[m] = m == blk ? diag : P[m];
       }
     } else if constexpr (!STATE_ONLY) {
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
         P[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (j > wave) continue;
+        if (j > blk) continue;
 #pragma unroll
         for (int c = 0; c < DT; ++c) {
-          const bf16x8 k8 = *reinterpret_cast<const bf16x8*>(&lds.k.hi[(j * 16 + l16) * RS + c * 32 + quad * 8]);
-          const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(&lds.q_hi[t * RS + c * 32 + quad * 8]);
+          const bf16x8 k8 = *reinterpret_cast<const bf16x8*>(&lds.k.hi[(j * 16 + l16) * RS + ch0 + c * 32 + quad * 8]);
+          const bf16x8 q8 = *reinterpret_cast<const bf16x8*>(&lds.q_hi[t * RS + ch0 + c * 32 + quad * 8]);
           P[j] = mfma_16(k8, q8, P[j]);
         }
 #pragma unroll
@@ -367,42 +429,53 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
     }
     __syncthreads();  // k is not read any more: P goes into its place
     if constexpr (!STATE_ONLY) {
+      if constexpr (HALVES > 1) {
+        if (half == 1) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) lds.p.part[(blk * 4 + j) * 64 + lane] = P[j];
+        }
+        __syncthreads();
+        if (half == 0) {
+#pragma unroll
+          for (int j = 0; j < 4; ++j) P[j] += lds.p.part[(blk * 4 + j) * 64 + lane];
+        }
+      }
 #pragma unroll
       for (int j = 0; j < 4; ++j) {
-        bf16x4 hi, lo;
+        typedef __attribute__((ext_vector_type(2))) uint32_t u32x2;
+        u32x2 hi, lo;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          __bf16 x, y;
-          split(P[j][i], x, y);
+        for (int i = 0; i < 2; ++i) {
+          uint32_t x, y;
+          split2(P[j][2 * i], P[j][2 * i + 1], x, y);
           hi[i] = x, lo[i] = y;
         }
-        if (j <= (wave | 1)) {
-          *reinterpret_cast<bf16x4*>(&lds.p.hi[t * TS + j * 16 + quad * 4]) = hi;
-          *reinterpret_cast<bf16x4*>(&lds.p.lo[t * TS + j * 16 + quad * 4]) = lo;
+        if (half == 0 && j <= (blk | 1)) {
+          *reinterpret_cast<u32x2*>(&lds.p.hi[t * TS + j * 16 + quad * 4]) = hi;
+          *reinterpret_cast<u32x2*>(&lds.p.lo[t * TS + j * 16 + quad * 4]) = lo;
         }
       }
       __syncthreads();
     }
+    if (LATE && chunk + 1 < last) fetch(cur, chunk + 1);
     if (has_cols) {
       bf16x8 v8[2];
 #pragma unroll
       for (int g = 0; g < 2; ++g) v8[g] = *reinterpret_cast<const bf16x8*>(&lds.vt[(wave * 16 + l16) * TS + g * 32 + quad * 8]);
       if constexpr (!STATE_ONLY) {
-        bf16x8 sh[DT], sl[DT];
+        bf16x8 sh[DA], sl[DA];
 #pragma unroll
-        for (int c = 0; c < DT; ++c)
-#pragma unroll
-          for (int e = 0; e < 8; ++e) {
-            __bf16 x, y;
-            split(S[c * 2 + (e >> 2)][e & 3], x, y);
-            sh[c][e] = x, sl[c][e] = y;
-          }
+        for (int c = 0; c < DA; ++c) {
+          const float x[8] = {S[2 * c][0], S[2 * c][1], S[2 * c][2], S[2 * c][3], S[2 * c + 1][0], S[2 * c + 1][1], S[2 * c + 1][2], S[2 * c + 1][3]};
+          split8(x, sh[c], sl[c]);
+        }
 #pragma unroll
         for (int tb = 0; tb < 4; ++tb) {
+          if (tb > 0 && DA > 1) __builtin_amdgcn_sched_barrier(0);  // (one group's operands in registers at a time)
           const int tok = tb * 16 + l16;
           f32x4 acc = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int c = 0; c < DT; ++c) {
+          for (int c = 0; c < DA; ++c) {
             const bf16x8 qh = *reinterpret_cast<const bf16x8*>(&lds.q_hi[tok * RS + c * 32 + quad * 8]);
             acc = mfma_16(sh[c], qh, acc);
             acc = mfma_16(sl[c], qh, acc);
@@ -431,15 +504,10 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
       }
       // the state behind the 64 tokens
 #pragma unroll
-      for (int ct = 0; ct < 2 * DT; ++ct) {
+      for (int ct = 0; ct < 2 * DA; ++ct) {
+        if (HALVES > 1 && ct % 2 == 0) __builtin_amdgcn_sched_barrier(0);
         if constexpr (CHANNEL) {
-#pragma unroll
-          for (int i = 0; i < 4; ++i) {
-            const int ch = ct * 16 + quad * 4 + i;
-            const float all = lds.total[0][ch] + lds.total[1][ch] + lds.total[2][ch] + lds.total[3][ch];
-            S[ct][i] *= __builtin_amdgcn_exp2f(all);
-            if constexpr (STATE_ONLY) seg_total[(ct >> 1) * 8 + (ct & 1) * 4 + i] += all;
-          }
+          S[ct] *= *reinterpret_cast<const f32x4*>(&lds.all[ct * 16 + quad * 4]);
         } else {
           S[ct] *= __builtin_amdgcn_exp2f(head_l2 * (float)n);
         }
@@ -453,25 +521,17 @@ __global__ __launch_bounds__(256) void decay_scan_mfma_kernel(const DecayScanArg
       }
     }
   }
+  if constexpr (CHANNEL && STATE_ONLY) {
+    if (blockIdx.y == 0 && threadIdx.x < a.d) a.seg_lw[(bh * a.segs + sg) * a.dp + threadIdx.x] = seg_total;
+  }
   if (!has_cols) return;
   float* to = st;
   if constexpr (STATE_ONLY) to = a.seg + ((bh * a.segs + sg) * a.dv + (col_in ? dv0 + l16 : 0)) * a.dp;
   if (STATE_ONLY || sg == a.segs - 1) {
 #pragma unroll
-    for (int ct = 0; ct < 2 * DT; ++ct) {
+    for (int ct = 0; ct < 2 * DA; ++ct) {
       const int ch = ct * 16 + quad * 4;
       if (col_in && ch < a.d) *reinterpret_cast<f32x4*>(to + ch) = S[ct];
-    }
-  }
-  if constexpr (CHANNEL && STATE_ONLY) {
-    if (dv0 == 0 && l16 == 0) {
-#pragma unroll
-      for (int ct = 0; ct < 2 * DT; ++ct)
-#pragma unroll
-        for (int i = 0; i < 4; ++i) {
-          const int ch = ct * 16 + quad * 4 + i;
-          if (ch < a.d) a.seg_lw[(bh * a.segs + sg) * a.dp + ch] = seg_total[(ct >> 1) * 8 + (ct & 1) * 4 + i];
-        }
     }
   }
 }
@@ -494,15 +554,16 @@ __global__ __launch_bounds__(256) void decay_join_kernel(const DecayScanArgs a) 
     if (s + 1 < a.segs) add = *reinterpret_cast<const f32x4*>(p);
     *reinterpret_cast<f32x4*>(p) = S;
     if (s + 1 == a.segs) return;
-    f32x4 l = {head_l2, head_l2, head_l2, head_l2};
+    f32x4 l;
     if (a.lw != nullptr) {
       l = *reinterpret_cast<const f32x4*>(a.seg_lw + (bh * a.segs + s) * a.dp + ch);
     } else {
       const int lo = s * a.seg_chunks * kScanTokens, hi = (s + 1) * a.seg_chunks * kScanTokens;
-      l *= (float)((hi < a.L ? hi : a.L) - lo);
+      const float f = __builtin_amdgcn_exp2f(head_l2 * (float)((hi < a.L ? hi : a.L) - lo));
+      l = f32x4{f, f, f, f};
     }
 #pragma unroll
-    for (int j = 0; j < 4; ++j) S[j] = __builtin_fmaf(S[j], __builtin_amdgcn_exp2f(l[j]), add[j]);
+    for (int j = 0; j < 4; ++j) S[j] = __builtin_fmaf(S[j], l[j], add[j]);
   }
 }
 
@@ -789,36 +850,35 @@ template <typename T, bool VEC> void launch_group_norm(const GroupNormArgs& a, h
     hipLaunchKernelGGL((group_norm_gate_kernel<T, VEC, 64>), grid, block, 0, s, a);
 }
 
-template <int DT, bool CHANNEL> int launch_decay_mfma(const DecayScanArgs& a, hipStream_t s) {
-  const size_t bytes = sizeof(ScanLds<DT, CHANNEL>);
+template <int DT, int HALVES, bool CHANNEL> int launch_decay_mfma(const DecayScanArgs& a, hipStream_t s) {
+  const size_t bytes = sizeof(ScanLds<DT, HALVES, CHANNEL>);
   if (bytes > 64 * 1024) {
     static const hipError_t once = [&] {
-      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(decay_scan_mfma_kernel<DT, CHANNEL, false>),
+      hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void*>(decay_scan_mfma_kernel<DT, HALVES, CHANNEL, false>),
                                          hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
       if (e != hipSuccess) return e;
-      return hipFuncSetAttribute(reinterpret_cast<const void*>(decay_scan_mfma_kernel<DT, CHANNEL, true>),
+      return hipFuncSetAttribute(reinterpret_cast<const void*>(decay_scan_mfma_kernel<DT, HALVES, CHANNEL, true>),
                                  hipFuncAttributeMaxDynamicSharedMemorySize, (int)bytes);
     }();
     BASED_REQUIRE(once == hipSuccess, BASED_ERR_LAUNCH, "decay_scan: %zu bytes of LDS refused: %s", bytes, hipGetErrorString(once));
   }
-  dim3 grid((unsigned)(a.B * a.H), (unsigned)((a.dv + 63) / 64), (unsigned)a.segs);
+  const int cols = 64 * HALVES;
+  dim3 grid((unsigned)(a.B * a.H), (unsigned)((a.dv + cols - 1) / cols), (unsigned)a.segs);
   if (a.segs > 1) {
     dim3 all_but_last = grid;
     all_but_last.z -= 1;
-    hipLaunchKernelGGL((decay_scan_mfma_kernel<DT, CHANNEL, true>), all_but_last, dim3(256), bytes, s, a);
+    hipLaunchKernelGGL((decay_scan_mfma_kernel<DT, HALVES, CHANNEL, true>), all_but_last, dim3(256 * HALVES), bytes, s, a);
     const long items = (long)a.B * a.H * a.dv * (a.dp / 4);
     hipLaunchKernelGGL(decay_join_kernel, dim3((unsigned)((items + 255) / 256)), dim3(256), 0, s, a);
   }
-  hipLaunchKernelGGL((decay_scan_mfma_kernel<DT, CHANNEL, false>), grid, dim3(256), bytes, s, a);
+  hipLaunchKernelGGL((decay_scan_mfma_kernel<DT, HALVES, CHANNEL, false>), grid, dim3(256 * HALVES), bytes, s, a);
   return BASED_OK;
 }
 
 template <bool CHANNEL> int launch_decay_scan_mfma(const DecayScanArgs& a, hipStream_t s) {
-  const int dt = (a.d + 31) / 32;
-  if (dt <= 1) return launch_decay_mfma<1, CHANNEL>(a, s);
-  if (dt <= 2) return launch_decay_mfma<2, CHANNEL>(a, s);
-  if (dt <= 3) return launch_decay_mfma<3, CHANNEL>(a, s);
-  return launch_decay_mfma<4, CHANNEL>(a, s);
+  if (a.d <= 32) return launch_decay_mfma<1, 1, CHANNEL>(a, s);
+  if (a.d <= 64) return launch_decay_mfma<2, 1, CHANNEL>(a, s);
+  return launch_decay_mfma<2, 2, CHANNEL>(a, s);
 }
 
 template <typename T, bool CHANNEL> void launch_decay_scan_any(const DecayScanArgs& a, hipStream_t s) {
@@ -864,10 +924,10 @@ template <typename T, bool CHANNEL> void launch_decay_step(const DecayStepArgs& 
     launch_decay_step_rows<T, 64, CHANNEL>(a, s);
 }
 
-// Segments of a scan: enough workgroups to give every compute unit two, none shorter than four pieces of 64 tokens.
-static int decay_segments(int64_t B, int64_t L, int64_t H, int64_t DV) {
-  const int64_t chunks = (L + kScanTokens - 1) / kScanTokens, wgs = B * H * ((DV + 63) / 64);
-  int64_t segs = (512 + wgs - 1) / wgs;
+// Segments of a scan: enough workgroups to give every SIMD two wavefronts, none shorter than four pieces of 64 tokens.
+static int decay_segments(int64_t B, int64_t L, int64_t H, int64_t D, int64_t DV) {
+  const int64_t cols = D <= 64 ? 64 : 128, chunks = (L + kScanTokens - 1) / kScanTokens, wgs = B * H * ((DV + cols - 1) / cols);
+  int64_t segs = ((D <= 64 ? 512 : 256) + wgs - 1) / wgs;
   if (segs > chunks / 4) segs = chunks / 4;
   if (segs > 64) segs = 64;
   return segs < 2 ? 1 : (int)segs;
@@ -877,7 +937,7 @@ static int decay_segments(int64_t B, int64_t L, int64_t H, int64_t DV) {
 
 extern "C" BASED_API int64_t based_decay_scan_work(int64_t B, int64_t L, int64_t H, int64_t D, int64_t DV, int64_t state_row) {
   if (B <= 0 || L <= 0 || H <= 0 || D <= 0 || DV <= 0) return 0;
-  const int64_t segs = based::decay_segments(B, L, H, DV);
+  const int64_t segs = based::decay_segments(B, L, H, D, DV);
   return segs <= 1 ? 0 : B * H * segs * (DV + 1) * state_row;
 }
 
@@ -897,6 +957,7 @@ extern "C" BASED_API int based_decay_scan(const void* q, const void* k, const vo
   BASED_REQUIRE(activation == BASED_ACT_NONE || activation == BASED_ACT_SILU, BASED_ERR_ARG, "decay_scan: unknown activation");
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "decay_scan: bad dtype");
   BASED_REQUIRE(B * H < (1ll << 31) && L < (1ll << 31) && DV < (1ll << 20), BASED_ERR_SHAPE, "decay_scan: grid too large");
+  BASED_REQUIRE(q_sl < (1ll << 24) && k_sl < (1ll << 24) && v_sl < (1ll << 24) && H * D < (1ll << 24), BASED_ERR_SHAPE, "decay_scan: rows too long");
   if (B == 0 || L == 0) return BASED_OK;
   DecayScanArgs a{q,    k,    v,    channel_log2, head_decay, bonus, state, nullptr, nullptr, o,    (int)B, (int)L, (int)H, (int)D, (int)DV,
                   (int)state_row, q_sb, q_sl, k_sb, k_sl, v_sb, v_sl, o_sb, o_sl, 1, (int)((L + kScanTokens - 1) / kScanTokens),
@@ -906,7 +967,7 @@ extern "C" BASED_API int based_decay_scan(const void* q, const void* k, const vo
                    k_sl % 4 == 0 && v_sb % 4 == 0 && v_sl % 4 == 0 && o_sb % 4 == 0 && o_sl % 4 == 0 && aligned_to(q, 8) &&
                    aligned_to(k, 8) && aligned_to(v, 8) && aligned_to(o, 8) && aligned_to(bonus, 8) && aligned_to(channel_log2, 16);
   if (vec) {
-    const int segs = decay_segments(B, L, H, DV);
+    const int segs = decay_segments(B, L, H, D, DV);
     if (segs > 1) {
       BASED_REQUIRE(work != nullptr, BASED_ERR_ARG, "decay_scan: no work space");
       a.seg_chunks = (a.seg_chunks + segs - 1) / segs;

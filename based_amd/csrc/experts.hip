@@ -4,9 +4,10 @@
 // (s multiplies the sums of gate and up in fp32, which is the same thing.)
 //
 //   expert_route    scores in fp32, the choice, and for grouped products each choice's place among its
-//                   expert's rows
-//   expert_plan     rows of every expert rounded up to tiles; which expert a tile belongs to
-//   expert_scatter  the choices in that order
+//                   expert's rows; a single workgroup (up to 32 tokens) also does what the next two do
+//   expert_plan     rows of every expert rounded up to tiles, which expert a tile belongs to, and the choices in
+//                   that order
+//   expert_scatter  the last part, where there are too many choices for one workgroup
 //   expert_gemm     MFMA product of a tile of rows with its expert's matrices, gathered and scattered by that
 //                   order: gate and up with the activation behind them, then down
 //   expert_sum      the choices of a token added up (with one choice the product writes the token's row)
@@ -16,7 +17,6 @@
 namespace based {
 
 constexpr int kMaxExperts = 256;
-constexpr int kRouteTokens = 16;
 
 struct RouteArgs {
   const void* h;  // (N, D)
@@ -24,59 +24,116 @@ struct RouteArgs {
   int32_t* ids;   // (N, top)
   float* scores;  // (N, top)
   int32_t* rank;  // (N, top) or null
-  int32_t* counts;  // (E), zero on entry, with rank
+  int32_t* counts;  // (E), with rank; zero on entry unless one workgroup does everything
+  // one workgroup for all tokens: the plan too
+  int32_t* tile_first;
+  int32_t* tile_expert;
+  int32_t* order;
+  int tile_rows;
   long n, h_sr;
   int D, E, top;
 };
 
 __device__ __forceinline__ f32x4 expert_mfma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
-// ET: tiles of 16 experts (bf16 MFMA, a quarter of the row per wavefront); 0: element by element.
-template <typename T, int ET>
-__global__ __launch_bounds__(256) void expert_route_kernel(const RouteArgs a) {
-  extern __shared__ float logits[];  // [4 (ET) or 1][kRouteTokens][E]
-  __shared__ int hist[kMaxExperts], base[kMaxExperts];
+// Tiles of every expert from its count, by threads 0 .. 255; scan: 256 ints of LDS.  Called by a whole workgroup.
+__device__ __forceinline__ void plan_tiles(const int* counts, int* scan, int* first_of, int32_t* tile_first, int32_t* tile_expert, int E, int tile_rows) {
+  const int e = threadIdx.x;
+  const int tiles = e < E ? (counts[e] + tile_rows - 1) / tile_rows : 0;
+  if (e < 256) scan[e] = tiles;
+  __syncthreads();
+  for (int m = 1; m < 256; m <<= 1) {
+    const int add = e < 256 && e >= m ? scan[e - m] : 0;
+    __syncthreads();
+    if (e < 256) scan[e] += add;
+    __syncthreads();
+  }
+  if (e < E) {
+    const int first = scan[e] - tiles;
+    first_of[e] = first;
+    tile_first[e] = first;
+    for (int t = 0; t < tiles; ++t) tile_expert[first + t] = e;
+  }
+  if (e == 255) tile_first[E] = scan[255];
+  __syncthreads();
+}
+
+// ET: tiles of 16 experts (bf16 MFMA); 0: element by element.  NW wavefronts.  SPLIT: they share 16 TT tokens, a part of the row each;
+// otherwise 16 tokens each.
+template <typename T, int ET, int NW, bool SPLIT, int TT>
+__global__ __launch_bounds__(64 * NW) void expert_route_kernel(const RouteArgs a) {
+  constexpr int NT = 64 * NW, TOK = ET == 0 ? 16 : SPLIT ? 16 * TT : 16 * NW;
+  extern __shared__ float logits[];  // [NW (SPLIT) or 1][TOK][E]
+  __shared__ int hist[kMaxExperts], base[kMaxExperts], scan[256];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
-  const long n0 = (long)blockIdx.x * kRouteTokens;
-  const int n = a.n - n0 < kRouteTokens ? (int)(a.n - n0) : kRouteTokens;
-  for (int e = tid; e < a.E; e += 256) hist[e] = 0;
+  const long n0 = (long)blockIdx.x * TOK;
+  const int n = a.n - n0 < TOK ? (int)(a.n - n0) : TOK;
+  for (int e = tid; e < a.E; e += NT) hist[e] = 0;
   if constexpr (ET > 0) {
-    f32x4 acc[ET];
+    f32x4 acc[ET][TT];
 #pragma unroll
-    for (int t = 0; t < ET; ++t) acc[t] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const __bf16* h = static_cast<const __bf16*>(a.h) + (n0 + (l16 < n ? l16 : 0)) * a.h_sr;
-    const int pieces = (a.D + 31) / 32, per = (pieces + 3) / 4;
-    const int p1 = (wave + 1) * per < pieces ? (wave + 1) * per : pieces;
-    for (int p = wave * per; p < p1; ++p) {
-      const int c = p * 32 + quad * 8;
-      bf16x8 x = *reinterpret_cast<const bf16x8*>(h + (c < a.D ? c : 0));
-      if (c >= a.D) {
+    for (int t = 0; t < ET; ++t)
 #pragma unroll
-        for (int j = 0; j < 8; ++j) x[j] = (__bf16)0.f;
+      for (int x = 0; x < TT; ++x) acc[t][x] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const __bf16* h[TT];
+#pragma unroll
+    for (int x = 0; x < TT; ++x) {
+      const int tok = (SPLIT ? 0 : wave * 16) + x * 16 + l16;
+      h[x] = static_cast<const __bf16*>(a.h) + (n0 + (tok < n ? tok : 0)) * a.h_sr;
+    }
+    const __bf16* w[ET];
+#pragma unroll
+    for (int t = 0; t < ET; ++t) {
+      const int e = t * 16 + l16;
+      w[t] = static_cast<const __bf16*>(a.w) + (long)(e < a.E ? e : 0) * a.D;
+    }
+    const int pieces = (a.D + 31) / 32, per = SPLIT ? (pieces + NW - 1) / NW : pieces;
+    const int p0 = SPLIT ? wave * per : 0, p1 = p0 + per < pieces ? p0 + per : pieces;
+    constexpr int PU = ET <= 4 ? 4 : 2;  // pieces whose loads are in flight together
+    for (int p = p0; p < p1; p += PU) {
+      bf16x8 x8[PU][TT], w8[PU][ET];
+#pragma unroll
+      for (int u = 0; u < PU; ++u) {
+        const int c = (p + u) * 32 + quad * 8;
+        const bool in = p + u < p1 && c < a.D;
+#pragma unroll
+        for (int x = 0; x < TT; ++x) x8[u][x] = *reinterpret_cast<const bf16x8*>(h[x] + (in ? c : 0));
+#pragma unroll
+        for (int t = 0; t < ET; ++t) w8[u][t] = *reinterpret_cast<const bf16x8*>(w[t] + (in ? c : 0));
       }
 #pragma unroll
-      for (int t = 0; t < ET; ++t) {
-        const int e = t * 16 + l16;
-        const bf16x8 w = *reinterpret_cast<const bf16x8*>(static_cast<const __bf16*>(a.w) + (long)(e < a.E ? e : 0) * a.D + (c < a.D ? c : 0));
-        acc[t] = expert_mfma(w, x, acc[t]);
+      for (int u = 0; u < PU; ++u) {
+        const bool in = p + u < p1 && (p + u) * 32 + quad * 8 < a.D;
+#pragma unroll
+        for (int x = 0; x < TT; ++x) {
+#pragma unroll
+          for (int j = 0; j < 8; ++j) x8[u][x][j] = in ? x8[u][x][j] : (__bf16)0.f;
+#pragma unroll
+          for (int t = 0; t < ET; ++t) acc[t][x] = expert_mfma(w8[u][t], x8[u][x], acc[t][x]);
+        }
       }
     }
     // column = token l16, rows = experts 4 quad + i
 #pragma unroll
     for (int t = 0; t < ET; ++t)
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int e = t * 16 + quad * 4 + i;
-        if (e < a.E) logits[(wave * kRouteTokens + l16) * a.E + e] = acc[t][i];
-      }
+      for (int x = 0; x < TT; ++x)
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int e = t * 16 + quad * 4 + i;
+          if (e < a.E) logits[((SPLIT ? wave * TOK : wave * 16) + x * 16 + l16) * a.E + e] = acc[t][x][i];
+        }
     __syncthreads();
-    for (int i = tid; i < kRouteTokens * a.E; i += 256) {
-      const int s = kRouteTokens * a.E;
-      const float z = (logits[i] + logits[s + i]) + (logits[2 * s + i] + logits[3 * s + i]);
+    for (int i = tid; i < TOK * a.E; i += NT) {
+      float z = logits[i];
+      if constexpr (SPLIT) {
+#pragma unroll
+        for (int v = 1; v < NW; ++v) z += logits[v * TOK * a.E + i];
+      }
       logits[i] = 1.0f / (1.0f + expf(-z));
     }
   } else {
-    for (int i = tid; i < kRouteTokens * a.E; i += 256) {
+    for (int i = tid; i < TOK * a.E; i += NT) {
       const int t = i / a.E, e = i % a.E;
       const T* h = static_cast<const T*>(a.h) + (n0 + (t < n ? t : 0)) * a.h_sr;
       const T* w = static_cast<const T*>(a.w) + (long)e * a.D;
@@ -87,56 +144,58 @@ __global__ __launch_bounds__(256) void expert_route_kernel(const RouteArgs a) {
   }
   __syncthreads();
   // 16 lanes per token
-  const int t = tid >> 4, sub = tid & 15;
-  float* s = logits + t * a.E;
-  for (int j = 0; j < a.top; ++j) {
-    float best = -2.f;
-    int at = 0;
-    for (int e = sub; e < a.E; e += 16)
-      if (s[e] > best) best = s[e], at = e;
+  const int sub = tid & 15;
+  for (int t = tid >> 4; t < TOK; t += NT / 16) {
+    float* s = logits + t * a.E;
+    for (int j = 0; j < a.top; ++j) {
+      float best = -2.f;
+      int at = 0;
+      for (int e = sub; e < a.E; e += 16)
+        if (s[e] > best) best = s[e], at = e;
 #pragma unroll
-    for (int m = 8; m >= 1; m >>= 1) {
-      const float ov = __shfl_xor(best, m, 16);
-      const int oa = __shfl_xor(at, m, 16);
-      if (ov > best || (ov == best && oa < at)) best = ov, at = oa;
-    }
-    if (at % 16 == sub) s[at] = -1.f;  // taken
-    if (sub == 0 && t < n) {
-      const long slot = (n0 + t) * a.top + j;
-      a.ids[slot] = at;
-      a.scores[slot] = best;
-      if (a.rank != nullptr) a.rank[slot] = atomicAdd(&hist[at], 1);
+      for (int m = 8; m >= 1; m >>= 1) {
+        const float ov = __shfl_xor(best, m, 16);
+        const int oa = __shfl_xor(at, m, 16);
+        if (ov > best || (ov == best && oa < at)) best = ov, at = oa;
+      }
+      if (at % 16 == sub) s[at] = -1.f;  // taken
+      if (sub == 0 && t < n) {
+        const long slot = (n0 + t) * a.top + j;
+        a.ids[slot] = at;
+        a.scores[slot] = best;
+        if (a.rank != nullptr) a.rank[slot] = atomicAdd(&hist[at], 1);
+      }
     }
   }
   if (a.rank == nullptr) return;
   __syncthreads();
-  for (int e = tid; e < a.E; e += 256) base[e] = hist[e] > 0 ? atomicAdd(&a.counts[e], hist[e]) : 0;
-  __syncthreads();
-  if (sub == 0 && t < n) {
+  if (a.order != nullptr) {
+    plan_tiles(hist, scan, base, a.tile_first, a.tile_expert, a.E, a.tile_rows);
+    for (int e = tid; e < a.E; e += NT) a.counts[e] = hist[e];
+  } else {
+    for (int e = tid; e < a.E; e += NT) base[e] = hist[e] > 0 ? atomicAdd(&a.counts[e], hist[e]) : 0;
+    __syncthreads();
+  }
+  for (int t = tid >> 4; t < n; t += NT / 16) {
+    if (sub != 0) continue;
     for (int j = 0; j < a.top; ++j) {
-      const long slot = (n0 + t) * a.top + j;
-      a.rank[slot] += base[a.ids[slot]];
+      const long slot = (n0 + t) * a.top + j;  // (this thread has written it)
+      if (a.order != nullptr)
+        a.order[(long)base[a.ids[slot]] * a.tile_rows + a.rank[slot]] = (int32_t)slot;
+      else
+        a.rank[slot] += base[a.ids[slot]];
     }
   }
 }
 
-// One workgroup: tile_first[e] and, at the end, the number of tiles; tile_expert[tile].
-__global__ __launch_bounds__(256) void expert_plan_kernel(const int32_t* counts, int32_t* tile_first, int32_t* tile_expert, int E, int tile_rows) {
-  __shared__ int scan[256];
-  const int e = threadIdx.x;
-  const int tiles = e < E ? (counts[e] + tile_rows - 1) / tile_rows : 0;
-  scan[e] = tiles;
-  __syncthreads();
-  for (int m = 1; m < 256; m <<= 1) {
-    const int add = e >= m ? scan[e - m] : 0;
-    __syncthreads();
-    scan[e] += add;
-    __syncthreads();
-  }
-  const int first = scan[e] - tiles;
-  if (e < E) tile_first[e] = first;
-  if (e == 255) tile_first[E] = scan[255];
-  for (int t = 0; t < tiles; ++t) tile_expert[first + t] = e;
+constexpr long kPlanSlots = 8192;  // choices that the planning workgroup puts in order by itself
+
+__global__ __launch_bounds__(256) void expert_plan_kernel(const int32_t* counts, const int32_t* ids, const int32_t* rank, int32_t* tile_first,
+                                                          int32_t* tile_expert, int32_t* order, long slots, int E, int tile_rows) {
+  __shared__ int scan[256], first_of[kMaxExperts];
+  plan_tiles(counts, scan, first_of, tile_first, tile_expert, E, tile_rows);
+  if (slots <= kPlanSlots)
+    for (long i = threadIdx.x; i < slots; i += 256) order[(long)first_of[ids[i]] * tile_rows + rank[i]] = (int32_t)i;
 }
 
 __global__ __launch_bounds__(256) void expert_scatter_kernel(const int32_t* ids, const int32_t* rank, const int32_t* tile_first, int32_t* order,
@@ -156,24 +215,31 @@ struct ExpertGemmArgs {
   const int32_t* tile_expert;
   const float* scores;   // (slots), PAIRED
   long x_sr;
-  int E, F, K, top;
+  int E, F, K, top, col_tiles, tiles;
 };
 
 constexpr int kGemmK = 64;
 
-template <int BM, bool PAIRED>
-__global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a) {
+// Workgroups are dealt to the eight dies in turn: those of one die take neighbouring tiles, which share rows and matrices.
+__device__ __forceinline__ int tile_of_block(int i, int n) {
+  const int die = i & 7, k = i >> 3, per = n / 8, more = n % 8;
+  return die * per + (die < more ? die : more) + k;
+}
+
+// BM rows and BN rows of the weights (PAIRED: half of them up, half gate) per workgroup; AHEAD rounds of 64 channels on their
+// way from memory.
+template <int BM, int BN, int AHEAD, bool PAIRED>
+__global__ __launch_bounds__(256, 2) void expert_gemm_kernel(const ExpertGemmArgs a) {
   constexpr int KS = kGemmK + 8;
-  constexpr int WM = BM >= 128 ? 2 : 1, WN = 4 / WM, MT = BM / 16 / WM, NT = 4 / WN;
-  constexpr int AP = BM / 32;  // 16-byte pieces of the rows per thread
-  __shared__ __attribute__((aligned(16))) __bf16 xs[BM * KS], ws[128 * KS];
+  constexpr int WM = BM >= 128 ? 2 : 1, WN = 4 / WM, MT = BM / 16 / WM, NT = BN / 32 / WN, HALF = BN / 2;
+  constexpr int AP = BM / 32, BP = BN / 32;  // 16-byte pieces per thread
+  __shared__ __attribute__((aligned(16))) __bf16 xs[BM * KS], ws[BN * KS];
   __shared__ int slot_of[BM];
-  const int tile = blockIdx.y;
+  const int id = tile_of_block(blockIdx.x, gridDim.x), tile = id / a.col_tiles, f0 = id % a.col_tiles * (PAIRED ? HALF : BN);
   if (tile >= a.tile_first[a.E]) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4, wm = wave % WM, wn = wave / WM;
   const int e = a.tile_expert[tile], r0 = (tile - a.tile_first[e]) * BM;
   const int rows = a.counts[e] - r0 < BM ? a.counts[e] - r0 : BM;
-  const int f0 = blockIdx.x * (PAIRED ? 64 : 128);
   for (int i = tid; i < BM; i += 256) slot_of[i] = a.order[(long)tile * BM + (i < rows ? i : 0)];
   __syncthreads();
   typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
@@ -184,21 +250,22 @@ __global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a
     const int r = i * 32 + (tid >> 3);
     xrow[i] = a.x + (PAIRED ? (long)(slot_of[r] / a.top) * a.x_sr : ((long)tile * BM + (r < rows ? r : 0)) * a.x_sr);
   }
-  const __bf16* wrow[4];
+  const __bf16* wbase = a.w + (long)e * (PAIRED ? 2 * a.F : a.F) * a.K;
+  int wrow[BP];
 #pragma unroll
-  for (int i = 0; i < 4; ++i) {
+  for (int i = 0; i < BP; ++i) {
     const int r = i * 32 + (tid >> 3);
-    const int f = PAIRED ? f0 + (r & 63) : f0 + r;
-    wrow[i] = a.w + ((long)e * (PAIRED ? 2 * a.F : a.F) + (PAIRED && r >= 64 ? a.F : 0) + (f < a.F ? f : a.F - 1)) * a.K;
+    const int f = PAIRED ? f0 + (r % HALF) : f0 + r;
+    wrow[i] = ((PAIRED && r >= HALF ? a.F : 0) + (f < a.F ? f : a.F - 1)) * a.K;
   }
-  u32x4 xb[AP], wb[4];
+  u32x4 xb[AHEAD][AP], wb[AHEAD][BP];
   const u32x4 zero = {0u, 0u, 0u, 0u};
-  auto fetch = [&](int k0) {
+  auto fetch = [&](int k0, u32x4 (&x)[AP], u32x4 (&w)[BP]) {
     const int c = k0 + piece < a.K ? k0 + piece : 0;
 #pragma unroll
-    for (int i = 0; i < AP; ++i) xb[i] = *reinterpret_cast<const u32x4*>(xrow[i] + c);
+    for (int i = 0; i < AP; ++i) x[i] = *reinterpret_cast<const u32x4*>(xrow[i] + c);
 #pragma unroll
-    for (int i = 0; i < 4; ++i) wb[i] = *reinterpret_cast<const u32x4*>(wrow[i] + c);
+    for (int i = 0; i < BP; ++i) w[i] = *reinterpret_cast<const u32x4*>(wbase + (wrow[i] + c));
   };
   f32x4 acc[2][NT][MT];
 #pragma unroll
@@ -207,29 +274,35 @@ __global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a
     for (int i = 0; i < NT; ++i)
 #pragma unroll
       for (int j = 0; j < MT; ++j) acc[p][i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  fetch(0);
-  for (int k0 = 0; k0 < a.K; k0 += kGemmK) {
-    const bool in = k0 + piece < a.K;
-    __syncthreads();
 #pragma unroll
-    for (int i = 0; i < AP; ++i) *reinterpret_cast<u32x4*>(&xs[(i * 32 + (tid >> 3)) * KS + piece]) = in ? xb[i] : zero;
+  for (int s = 0; s < AHEAD; ++s) fetch(s * kGemmK, xb[s], wb[s]);
+  // (rounds past the end multiply by zeros: every stage of the loop is the same)
+  for (int k00 = 0; k00 < a.K; k00 += AHEAD * kGemmK) {
 #pragma unroll
-    for (int i = 0; i < 4; ++i) *reinterpret_cast<u32x4*>(&ws[(i * 32 + (tid >> 3)) * KS + piece]) = wb[i];
-    __syncthreads();
-    if (k0 + kGemmK < a.K) fetch(k0 + kGemmK);
+    for (int s = 0; s < AHEAD; ++s) {
+      const int k0 = k00 + s * kGemmK;
+      const bool in = k0 + piece < a.K;
+      __syncthreads();
 #pragma unroll
-    for (int kk = 0; kk < kGemmK; kk += 32) {
-      bf16x8 xf[MT];
+      for (int i = 0; i < AP; ++i) *reinterpret_cast<u32x4*>(&xs[(i * 32 + (tid >> 3)) * KS + piece]) = in ? xb[s][i] : zero;
 #pragma unroll
-      for (int j = 0; j < MT; ++j) xf[j] = *reinterpret_cast<const bf16x8*>(&xs[((wm * MT + j) * 16 + l16) * KS + kk + quad * 8]);
+      for (int i = 0; i < BP; ++i) *reinterpret_cast<u32x4*>(&ws[(i * 32 + (tid >> 3)) * KS + piece]) = wb[s][i];
+      __syncthreads();
+      fetch(k0 + AHEAD * kGemmK, xb[s], wb[s]);
 #pragma unroll
-      for (int p = 0; p < 2; ++p)
+      for (int kk = 0; kk < kGemmK; kk += 32) {
+        bf16x8 xf[MT];
 #pragma unroll
-        for (int i = 0; i < NT; ++i) {
-          const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&ws[(p * 64 + (wn * NT + i) * 16 + l16) * KS + kk + quad * 8]);
+        for (int j = 0; j < MT; ++j) xf[j] = *reinterpret_cast<const bf16x8*>(&xs[((wm * MT + j) * 16 + l16) * KS + kk + quad * 8]);
 #pragma unroll
-          for (int j = 0; j < MT; ++j) acc[p][i][j] = expert_mfma(wf, xf[j], acc[p][i][j]);
-        }
+        for (int p = 0; p < 2; ++p)
+#pragma unroll
+          for (int i = 0; i < NT; ++i) {
+            const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&ws[(p * HALF + (wn * NT + i) * 16 + l16) * KS + kk + quad * 8]);
+#pragma unroll
+            for (int j = 0; j < MT; ++j) acc[p][i][j] = expert_mfma(wf, xf[j], acc[p][i][j]);
+          }
+      }
     }
   }
   // column = row l16 of the tile's rows, rows = features 4 quad + i
@@ -257,7 +330,7 @@ __global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a
       for (int p = 0; p < 2; ++p)
 #pragma unroll
         for (int i = 0; i < NT; ++i) {
-          const int f = f0 + p * 64 + (wn * NT + i) * 16 + quad * 4;
+          const int f = f0 + p * HALF + (wn * NT + i) * 16 + quad * 4;
           if (f < a.F) {
             bf16x4 o;
 #pragma unroll
@@ -267,6 +340,21 @@ __global__ __launch_bounds__(256) void expert_gemm_kernel(const ExpertGemmArgs a
         }
     }
   }
+}
+
+template <int BM, int BN, int AHEAD, bool PAIRED> void launch_expert_gemm(ExpertGemmArgs a, hipStream_t s) {
+  const int cols = PAIRED ? BN / 2 : BN;
+  a.col_tiles = (a.F + cols - 1) / cols;
+  hipLaunchKernelGGL((expert_gemm_kernel<BM, BN, AHEAD, PAIRED>), dim3((unsigned)(a.col_tiles * a.tiles)), dim3(256), 0, s, a);
+}
+
+template <bool PAIRED> void launch_expert_product(const ExpertGemmArgs& a, int rows, hipStream_t s) {
+  if (rows == BASED_EXPERT_TILE_ROWS_SMALL)
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS_SMALL, 128, 4, PAIRED>(a, s);
+  else if (a.F >= 256)
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 256, 1, PAIRED>(a, s);
+  else
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 128, 2, PAIRED>(a, s);
 }
 
 // y[n] = sum of the rows of its choices
@@ -403,42 +491,54 @@ template <typename T, bool PAIRED> void launch_expert_rows_vec(const ExpertRowsA
     launch_expert_rows<T, 1, PAIRED>(a, items, s);
 }
 
-static void launch_route_bf16(const RouteArgs& a, bool vec, dim3 grid, hipStream_t s) {
-  const size_t one = (size_t)kRouteTokens * a.E * sizeof(float);
-  const int et = (a.E + 15) / 16;
-  if (!vec)
-    hipLaunchKernelGGL((expert_route_kernel<__bf16, 0>), grid, dim3(256), one, s, a);
-  else if (et <= 1)
-    hipLaunchKernelGGL((expert_route_kernel<__bf16, 1>), grid, dim3(256), 4 * one, s, a);
-  else if (et <= 2)
-    hipLaunchKernelGGL((expert_route_kernel<__bf16, 2>), grid, dim3(256), 4 * one, s, a);
-  else if (et <= 4)
-    hipLaunchKernelGGL((expert_route_kernel<__bf16, 4>), grid, dim3(256), 4 * one, s, a);
+constexpr int kRouteOneWg = 32;  // tokens that one workgroup routes, of up to 32 experts (16 of more): it makes the plan too
+
+template <int ET> void launch_route_tiles(const RouteArgs& a, hipStream_t s) {
+  const size_t one = (size_t)16 * a.E * sizeof(float);
+  constexpr int NW = ET <= 4 ? 8 : 4;
+  if constexpr (ET <= 2) {
+    if (a.n > 16 && a.n <= kRouteOneWg) {
+      hipLaunchKernelGGL((expert_route_kernel<__bf16, ET, NW, true, 2>), dim3(1), dim3(64 * NW), 2 * NW * one, s, a);
+      return;
+    }
+  }
+  if (a.n >= 4096)
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, ET, 4, false, 1>), dim3((unsigned)((a.n + 63) / 64)), dim3(256), 4 * one, s, a);
   else
-    hipLaunchKernelGGL((expert_route_kernel<__bf16, 8>), grid, dim3(256), 4 * one, s, a);
+    hipLaunchKernelGGL((expert_route_kernel<__bf16, ET, NW, true, 1>), dim3((unsigned)((a.n + 15) / 16)), dim3(64 * NW), NW * one, s, a);
+}
+
+static bool route_is_single(const RouteArgs& a, bool vec) { return a.n <= (vec && a.E <= 32 ? kRouteOneWg : 16); }
+
+template <typename T> void launch_route(RouteArgs a, bool vec, hipStream_t s) {
+  const dim3 grid((unsigned)((a.n + 15) / 16));
+  if (!route_is_single(a, vec)) a.order = nullptr;
+  if constexpr (sizeof(T) == 2) {
+    const int et = (a.E + 15) / 16;
+    if (vec && et <= 1)
+      return launch_route_tiles<1>(a, s);
+    if (vec && et <= 2)
+      return launch_route_tiles<2>(a, s);
+    if (vec && et <= 4)
+      return launch_route_tiles<4>(a, s);
+    if (vec && et <= 8)
+      return launch_route_tiles<8>(a, s);
+  }
+  hipLaunchKernelGGL((expert_route_kernel<T, 0, 4, false, 1>), grid, dim3(256), (size_t)16 * a.E * sizeof(float), s, a);
+}
+
+static bool route_vec(const RouteArgs& a) {
+  return a.D % 8 == 0 && a.h_sr % 8 == 0 && a.E <= 128 && aligned_to(a.h, 16) && aligned_to(a.w, 16);
+}
+
+static int route_check(const char* who, const RouteArgs& a) {
+  BASED_REQUIRE(a.n >= 0 && a.D > 0 && a.E > 0 && a.top > 0 && a.top <= a.E, BASED_ERR_ARG, "%s: bad sizes", who);
+  BASED_REQUIRE(a.E <= kMaxExperts, BASED_ERR_SHAPE, "%s: %d experts (at most %d)", who, a.E, kMaxExperts);
+  BASED_REQUIRE(a.n * a.top < (1ll << 31), BASED_ERR_SHAPE, "%s: too many choices", who);
+  return BASED_OK;
 }
 
 }  // namespace based
-
-extern "C" BASED_API int based_expert_route(const void* h, const void* router, int32_t* ids, float* scores, int32_t* rank, int32_t* counts,
-                                            int64_t n, int64_t D, int64_t E, int64_t top, int64_t h_sr, int io_dtype, void* stream) {
-  using namespace based;
-  BASED_REQUIRE(h && router && ids && scores && (rank == nullptr || counts), BASED_ERR_ARG, "expert_route: null pointer argument");
-  BASED_REQUIRE(n >= 0 && D > 0 && E > 0 && top > 0 && top <= E, BASED_ERR_ARG, "expert_route: bad sizes");
-  BASED_REQUIRE(E <= kMaxExperts, BASED_ERR_SHAPE, "expert_route: %ld experts (at most %d)", (long)E, kMaxExperts);
-  BASED_REQUIRE(n * top < (1ll << 31) && D < (1ll << 28), BASED_ERR_SHAPE, "expert_route: too many choices");
-  BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "expert_route: bad dtype");
-  if (n == 0) return BASED_OK;
-  const RouteArgs a{h, router, ids, scores, rank, counts, (long)n, (long)h_sr, (int)D, (int)E, (int)top};
-  const dim3 grid((unsigned)((n + kRouteTokens - 1) / kRouteTokens));
-  hipStream_t s = static_cast<hipStream_t>(stream);
-  if (io_dtype == BASED_BF16) {
-    launch_route_bf16(a, D % 8 == 0 && h_sr % 8 == 0 && E <= 128 && aligned_to(h, 16) && aligned_to(router, 16), grid, s);
-  } else {
-    hipLaunchKernelGGL((expert_route_kernel<float, 0>), grid, dim3(256), (size_t)kRouteTokens * E * sizeof(float), s, a);
-  }
-  return check_launch("expert_route");
-}
 
 /* Tiles of BASED_EXPERT_TILE_ROWS or BASED_EXPERT_TILE_ROWS_SMALL rows. */
 static int expert_tile_rows(int64_t slots, int64_t E) { return slots >= 64 * E ? BASED_EXPERT_TILE_ROWS : BASED_EXPERT_TILE_ROWS_SMALL; }
@@ -451,57 +551,62 @@ extern "C" BASED_API int64_t based_expert_tiles(int64_t n, int64_t E, int64_t to
 
 extern "C" BASED_API int64_t based_expert_tile_rows(int64_t n, int64_t E, int64_t top) { return expert_tile_rows(n * top, E); }
 
-extern "C" BASED_API int based_expert_grouped(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
-                                              const int32_t* rank, const int32_t* counts, int32_t* tile_first, int32_t* tile_expert,
-                                              int32_t* order, void* work_act, void* work_out, void* y, int64_t n, int64_t D, int64_t F,
-                                              int64_t E, int64_t top, int64_t h_sr, void* stream) {
+extern "C" BASED_API int based_expert_grouped(const void* h, const void* router, const void* w1, const void* w2, int32_t* ids, float* scores,
+                                              int32_t* rank, int32_t* counts, int32_t* tile_first, int32_t* tile_expert, int32_t* order,
+                                              void* work_act, void* work_out, void* y, int64_t n, int64_t D, int64_t F, int64_t E, int64_t top,
+                                              int64_t h_sr, void* stream) {
   using namespace based;
-  BASED_REQUIRE(h && w1 && w2 && ids && scores && rank && counts && tile_first && tile_expert && order && work_act && y, BASED_ERR_ARG,
-                "expert_grouped: null pointer argument");
-  BASED_REQUIRE(n >= 0 && D > 0 && F > 0 && E > 0 && top > 0 && E <= kMaxExperts && n * top < (1ll << 31), BASED_ERR_ARG,
-                "expert_grouped: bad sizes");
+  BASED_REQUIRE(h && router && w1 && w2 && ids && scores && rank && counts && tile_first && tile_expert && order && work_act && y,
+                BASED_ERR_ARG, "expert_grouped: null pointer argument");
+  BASED_REQUIRE(F > 0 && D < (1ll << 28), BASED_ERR_ARG, "expert_grouped: bad sizes");
   BASED_REQUIRE(top == 1 || work_out != nullptr, BASED_ERR_ARG, "expert_grouped: several choices per token need work_out");
-  BASED_REQUIRE(D % 8 == 0 && F % 8 == 0 && h_sr % 8 == 0, BASED_ERR_SHAPE, "expert_grouped: sizes %ld and %ld must be multiples of 8",
-                (long)D, (long)F);
+  BASED_REQUIRE(D % 8 == 0 && F % 8 == 0 && h_sr % 8 == 0 && 2 * F * D < (1ll << 31), BASED_ERR_SHAPE,
+                "expert_grouped: sizes %ld and %ld must be multiples of 8", (long)D, (long)F);
   BASED_REQUIRE(aligned_to(h, 16) && aligned_to(w1, 16) && aligned_to(w2, 16) && aligned_to(work_act, 16) && aligned_to(work_out, 16) &&
                     aligned_to(y, 16),
                 BASED_ERR_ALIGN, "expert_grouped: tensors must be 16-byte aligned");
+  RouteArgs r{h, router, ids, scores, rank, counts, tile_first, tile_expert, order, 0, (long)n, (long)h_sr, (int)D, (int)E, (int)top};
+  const int rc = route_check("expert_grouped", r);
+  if (rc != BASED_OK) return rc;
   if (n == 0) return BASED_OK;
   const int64_t slots = n * top;
   const int rows = expert_tile_rows(slots, E);
   const int64_t tiles = based_expert_tiles(n, E, top);
-  BASED_REQUIRE(tiles < 65536, BASED_ERR_SHAPE, "expert_grouped: too many rows");
+  BASED_REQUIRE(tiles * ((F > D ? F : D) / 64 + 1) < (1ll << 31), BASED_ERR_SHAPE, "expert_grouped: too many rows");
   hipStream_t s = static_cast<hipStream_t>(stream);
-  hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(256), 0, s, counts, tile_first, tile_expert, (int)E, rows);
-  hipLaunchKernelGGL(expert_scatter_kernel, dim3((unsigned)((slots + 255) / 256)), dim3(256), 0, s, ids, rank, tile_first, order,
-                     (long)slots, rows);
-  ExpertGemmArgs a{static_cast<const __bf16*>(h), static_cast<const __bf16*>(w1), static_cast<__bf16*>(work_act), order, counts, tile_first,
-                   tile_expert, scores, (long)h_sr, (int)E, (int)F, (int)D, (int)top};
-  const dim3 grid1((unsigned)((F + 63) / 64), (unsigned)tiles), grid2((unsigned)((D + 127) / 128), (unsigned)tiles);
-  __bf16* out = static_cast<__bf16*>(top == 1 ? y : work_out);
-  ExpertGemmArgs a2{static_cast<const __bf16*>(work_act), static_cast<const __bf16*>(w2), out, order, counts, tile_first,
-                    tile_expert, scores, (long)F, (int)E, (int)D, (int)F, (int)top};
-  if (rows == BASED_EXPERT_TILE_ROWS) {
-    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS, true>), grid1, dim3(256), 0, s, a);
-    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS, false>), grid2, dim3(256), 0, s, a2);
-  } else {
-    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS_SMALL, true>), grid1, dim3(256), 0, s, a);
-    hipLaunchKernelGGL((expert_gemm_kernel<BASED_EXPERT_TILE_ROWS_SMALL, false>), grid2, dim3(256), 0, s, a2);
+  r.tile_rows = rows;
+  const bool vec = route_vec(r);
+  launch_route<__bf16>(r, vec, s);
+  if (!route_is_single(r, vec)) {
+    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(256), 0, s, counts, ids, rank, tile_first, tile_expert, order, (long)slots, (int)E,
+                       rows);
+    if (slots > kPlanSlots)
+      hipLaunchKernelGGL(expert_scatter_kernel, dim3((unsigned)((slots + 255) / 256)), dim3(256), 0, s, ids, rank, tile_first, order,
+                         (long)slots, rows);
   }
+  const ExpertGemmArgs a{static_cast<const __bf16*>(h), static_cast<const __bf16*>(w1), static_cast<__bf16*>(work_act), order, counts, tile_first,
+                         tile_expert, scores, (long)h_sr, (int)E, (int)F, (int)D, (int)top, 0, (int)tiles};
+  __bf16* out = static_cast<__bf16*>(top == 1 ? y : work_out);
+  const ExpertGemmArgs a2{static_cast<const __bf16*>(work_act), static_cast<const __bf16*>(w2), out, order, counts, tile_first,
+                          tile_expert, scores, (long)F, (int)E, (int)D, (int)F, (int)top, 0, (int)tiles};
+  launch_expert_product<true>(a, rows, s);
+  launch_expert_product<false>(a2, rows, s);
   if (top > 1)
     hipLaunchKernelGGL(expert_sum_kernel, dim3((unsigned)((n * (D / 8) + 255) / 256)), dim3(256), 0, s, out, static_cast<__bf16*>(y), (long)n,
                        (int)D, (int)top);
   return check_launch("expert_grouped");
 }
 
-extern "C" BASED_API int based_expert_rows(const void* h, const void* w1, const void* w2, const int32_t* ids, const float* scores,
-                                           void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t top, int64_t h_sr,
+extern "C" BASED_API int based_expert_rows(const void* h, const void* router, const void* w1, const void* w2, int32_t* ids, float* scores,
+                                           void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t E, int64_t top, int64_t h_sr,
                                            int io_dtype, void* stream) {
   using namespace based;
-  BASED_REQUIRE(h && w1 && w2 && ids && scores && work_act && y, BASED_ERR_ARG, "expert_rows: null pointer argument");
-  BASED_REQUIRE(n >= 0 && D > 0 && F > 0 && top > 0 && n * top < (1ll << 31), BASED_ERR_ARG, "expert_rows: bad sizes");
-  BASED_REQUIRE(D < (1 << 20) && F < (1 << 20), BASED_ERR_SHAPE, "expert_rows: grid too large");
+  BASED_REQUIRE(h && router && w1 && w2 && ids && scores && work_act && y, BASED_ERR_ARG, "expert_rows: null pointer argument");
+  BASED_REQUIRE(F > 0 && D < (1 << 20) && F < (1 << 20), BASED_ERR_SHAPE, "expert_rows: grid too large");
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "expert_rows: bad dtype");
+  const RouteArgs r{h, router, ids, scores, nullptr, nullptr, nullptr, nullptr, nullptr, 0, (long)n, (long)h_sr, (int)D, (int)E, (int)top};
+  const int rc = route_check("expert_rows", r);
+  if (rc != BASED_OK) return rc;
   if (n == 0) return BASED_OK;
   const int p = io_dtype == BASED_BF16 ? 8 : 4;
   const bool vec1 = D % p == 0 && h_sr % p == 0 && aligned_to(h, 16) && aligned_to(w1, 16);
@@ -510,9 +615,11 @@ extern "C" BASED_API int based_expert_rows(const void* h, const void* w1, const 
   const ExpertRowsArgs a2{work_act, w2, y, ids, scores, (long)n, (long)F, (int)D, (int)F, (int)top};
   hipStream_t s = static_cast<hipStream_t>(stream);
   if (io_dtype == BASED_BF16) {
+    launch_route<__bf16>(r, route_vec(r), s);
     launch_expert_rows_vec<__bf16, true>(a1, vec1, n * top, s);
     launch_expert_rows_vec<__bf16, false>(a2, vec2, n, s);
   } else {
+    launch_route<float>(r, false, s);
     launch_expert_rows_vec<float, true>(a1, vec1, n * top, s);
     launch_expert_rows_vec<float, false>(a2, vec2, n, s);
   }

@@ -115,8 +115,8 @@ __global__ __launch_bounds__(256) void latent_write_vec_kernel(const LatentArgs 
 constexpr int kQueryCols = 128;  // latent channels per workgroup of latent_query
 constexpr int kQueryRows = 4;    // sequences at a time
 
-// N: elements per load (8 or 1).  Workgroups 0 .. H * ceil(R / kQueryCols) - 1 form q~, the rest (one per sequence) write
-// the cache row and rotate the queries.
+// N: elements per load (8 or 1); kQueryRows sequences per workgroup.  In x, workgroups 0 .. H * ceil(R / kQueryCols) - 1 form q~, the
+// rest (one per sequence) write the cache row and rotate the queries.
 template <typename T, int N>
 __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
   constexpr int LANES = kQueryCols / N, GROUPS = 256 / LANES > 0 ? 256 / LANES : 1;
@@ -124,7 +124,8 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
   __shared__ float part[GROUPS][kQueryRows][kQueryCols];
   const int tid = threadIdx.x, W = a.R + a.rot, col_blocks = (a.R + kQueryCols - 1) / kQueryCols;
   if ((int)blockIdx.x >= a.H * col_blocks) {
-    const int b = blockIdx.x - a.H * col_blocks;
+    const int b = blockIdx.y * kQueryRows + blockIdx.x - a.H * col_blocks;
+    if (b >= a.B) return;
     const int pos = row_pos(a.pos, a.pos_host, b);
     if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;
     if (tid < 64) {
@@ -139,9 +140,10 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
     return;
   }
   const int h = blockIdx.x / col_blocks, r0 = (blockIdx.x % col_blocks) * kQueryCols;
+  const int b0 = blockIdx.y * kQueryRows;
   const int piece = tid % LANES, grp = tid / LANES, col = r0 + piece * N;
   const T* w = static_cast<const T*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot) * a.w_sr;
-  for (int b0 = 0; b0 < a.B; b0 += kQueryRows) {
+  {
     const int rows = a.B - b0 < kQueryRows ? a.B - b0 : kQueryRows;
     float acc[kQueryRows][N];
 #pragma unroll
@@ -393,6 +395,7 @@ __global__ __launch_bounds__(256, 1) void latent_step_mfma_kernel(const LatentAr
 
 constexpr int kValueRows = 4;   // sequences at a time
 constexpr int kValueCols = 32;  // value channels per workgroup
+constexpr int kMaxSplits = 64;
 
 template <typename T, int N>
 __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) {
@@ -400,49 +403,84 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int h = blockIdx.x, b0 = blockIdx.y * kValueRows, j0 = blockIdx.z * kValueCols;
   const int rows = a.B - b0 < kValueRows ? a.B - b0 : kValueRows;
-  for (int m = 0; m < rows; ++m) {
+  // what each split counts for: exp(m_s - max) / sum
+  __shared__ float share[kValueRows][kMaxSplits];
+  for (int m = wave; m < rows; m += 4) {
     const int pos = row_pos(a.pos, a.pos_host, b0 + m);
     const bool ok = pos >= 0 && pos < a.S;
-    const long at0 = (long)(b0 + m) * a.splits * a.H + h;
-    float mx = -INFINITY;
-    for (int s = 0; ok && s < a.splits; ++s) mx = fmaxf(mx, a.part_ml[2 * (at0 + (long)s * a.H)]);
-    float l = 0.f;
-    for (int s = 0; ok && s < a.splits; ++s) {
-      const float ms = a.part_ml[2 * (at0 + (long)s * a.H)];
-      l += ms == -INFINITY ? 0.f : expf(ms - mx) * a.part_ml[2 * (at0 + (long)s * a.H) + 1];
+    const float* ml = a.part_ml + 2 * ((long)(b0 + m) * a.splits * a.H + h);
+    float ms[kMaxSplits / 64], ls[kMaxSplits / 64], mx = -INFINITY, l = 0.f;
+#pragma unroll
+    for (int i = 0; i < kMaxSplits / 64; ++i) {
+      const int s = i * 64 + lane;
+      const bool in = ok && s < a.splits;
+      ms[i] = in ? ml[2 * (long)s * a.H] : -INFINITY;
+      ls[i] = in ? ml[2 * (long)s * a.H + 1] : 0.f;
+      mx = fmaxf(mx, ms[i]);
     }
-    for (int c = tid; c < a.R; c += 256) {
-      float v = 0.f;
-      for (int s = 0; ok && s < a.splits; ++s) {
-        const float ms = a.part_ml[2 * (at0 + (long)s * a.H)];
-        if (ms != -INFINITY) v = __builtin_fmaf(expf(ms - mx), a.part[(at0 + (long)s * a.H) * a.R + c], v);
-      }
-      lat[m][c] = ok ? v / l : 0.f;
+#pragma unroll
+    for (int x = 32; x >= 1; x >>= 1) mx = fmaxf(mx, __shfl_xor(mx, x, 64));
+#pragma unroll
+    for (int i = 0; i < kMaxSplits / 64; ++i) {
+      ms[i] = ms[i] == -INFINITY ? 0.f : expf(ms[i] - mx);
+      l = __builtin_fmaf(ms[i], ls[i], l);
     }
+    l = wave_sum(l);
+#pragma unroll
+    for (int i = 0; i < kMaxSplits / 64; ++i) share[m][i * 64 + lane] = l > 0.f ? ms[i] / l : 0.f;
+  }
+  __syncthreads();
+  // (a split without keys has left nothing in its part: it is not read)
+  for (int i = tid; i < rows * a.R; i += 256) {
+    const int m = i / a.R, c = i % a.R;
+    const float* p = a.part + ((long)(b0 + m) * a.splits * a.H + h) * a.R + c;
+    float v = 0.f;
+#pragma unroll 4
+    for (int s = 0; s < a.splits; ++s) {
+      const float f = share[m][s], x = p[f != 0.f ? (long)s * a.H * a.R : 0];
+      v = f != 0.f ? __builtin_fmaf(f, x, v) : v;
+    }
+    lat[m][c] = v;
   }
   __syncthreads();
   const T* w = static_cast<const T*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot + a.d) * a.w_sr;
   const int j1 = j0 + kValueCols < a.dv ? j0 + kValueCols : a.dv;
-  for (int j = j0 + wave; j < j1; j += 4) {
-    float acc[kValueRows];
+  constexpr int JU = 4;  // value channels whose rows are in flight together
+  for (int j = j0 + wave * JU; j < j1; j += 4 * JU) {
+    float acc[JU][kValueRows];
 #pragma unroll
-    for (int m = 0; m < kValueRows; ++m) acc[m] = 0.f;
+    for (int u = 0; u < JU; ++u)
+#pragma unroll
+      for (int m = 0; m < kValueRows; ++m) acc[u][m] = 0.f;
+#pragma unroll 2
     for (int c = lane * N; c < a.R; c += 64 * N) {
-      float wv[N];
-      if constexpr (N == 1)
-        wv[0] = to_f32(w[(long)j * a.w_sr + c]);
-      else
-        load_vec<T, N>(w + (long)j * a.w_sr + c, wv);
+      float wv[JU][N];
+#pragma unroll
+      for (int u = 0; u < JU; ++u) {
+        const T* p = w + (long)(j + u < j1 ? j + u : j) * a.w_sr + c;
+        if constexpr (N == 1)
+          wv[u][0] = to_f32(*p);
+        else
+          load_vec<T, N>(p, wv[u]);
+      }
 #pragma unroll
       for (int m = 0; m < kValueRows; ++m)
 #pragma unroll
-        for (int i = 0; i < N; ++i) acc[m] = __builtin_fmaf(wv[i], lat[m < rows ? m : 0][c + i], acc[m]);
+        for (int i = 0; i < N; ++i) {
+          const float x = lat[m < rows ? m : 0][c + i];
+#pragma unroll
+          for (int u = 0; u < JU; ++u) acc[u][m] = __builtin_fmaf(wv[u][i], x, acc[u][m]);
+        }
     }
 #pragma unroll
-    for (int m = 0; m < kValueRows; ++m) {
-      const float s = wave_sum(acc[m]);
-      if (m < rows && lane == 0) static_cast<T*>(a.o)[(long)(b0 + m) * a.o_sb + (long)h * a.dv + j] = from_f32<T>(s * a.out_scale);
-    }
+    for (int u = 0; u < JU; ++u)
+#pragma unroll
+      for (int m = 0; m < kValueRows; ++m) {
+        float s = sum16(acc[u][m]);
+        s += __shfl_xor(s, 16, 64);
+        s += __shfl_xor(s, 32, 64);
+        if (m < rows && lane == 0 && j + u < j1) static_cast<T*>(a.o)[(long)(b0 + m) * a.o_sb + (long)h * a.dv + j + u] = from_f32<T>(s * a.out_scale);
+      }
   }
 }
 
@@ -463,7 +501,7 @@ template <int KC, int RT> void launch_latent_mfma(const LatentArgs& a, hipStream
 }
 
 template <typename T> void launch_latent_query(const LatentArgs& a, bool vec, hipStream_t s) {
-  const dim3 grid((unsigned)(a.H * ((a.R + kQueryCols - 1) / kQueryCols) + a.B));
+  const dim3 grid((unsigned)(a.H * ((a.R + kQueryCols - 1) / kQueryCols) + kQueryRows), (unsigned)((a.B + kQueryRows - 1) / kQueryRows));
   if (vec)
     hipLaunchKernelGGL((latent_query_kernel<T, Pack<T>::kN>), grid, dim3(256), 0, s, a);
   else
@@ -537,6 +575,7 @@ extern "C" BASED_API int based_latent_step(const void* q, const void* x, const v
   BASED_REQUIRE(H > 0 && D > 0 && DV > 0 && window > 0 && window < (1ll << 31) && splits > 0 && splits < 65536 && pos_host >= 0 &&
                     pos_host < (1ll << 31),
                 BASED_ERR_ARG, "latent_step: bad sizes");
+  BASED_REQUIRE(splits <= kMaxSplits, BASED_ERR_SHAPE, "latent_step: %ld splits (at most %d)", (long)splits, kMaxSplits);
   BASED_REQUIRE(B < 65536 * kValueRows && B * H * splits < (1ll << 31) && H < 65536, BASED_ERR_SHAPE, "latent_step: grid too large");
   LatentArgs a{};
   a.x = x, a.norm_w = norm_w, a.cache = cache, a.cos_t = rope_cos, a.sin_t = rope_sin, a.pos = pos, a.pos_host = (int)pos_host;

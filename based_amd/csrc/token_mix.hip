@@ -119,7 +119,8 @@ __global__ __launch_bounds__(256) void channel_decay_kernel(const ChannelDecayAr
 
 __device__ __forceinline__ f32x4 mfma16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
-// bf16, R a multiple of 8 up to 256: 64 rows and 64 channels per workgroup.  tanh(h) enters as two bf16 numbers.
+// bf16, R a multiple of 8 up to 256, C of 4: a wavefront keeps tanh(h) of 16 rows, as two bf16 numbers each, and walks the
+// channels of its part 16 at a time.
 template <int KC>
 __global__ __launch_bounds__(256) void channel_decay_mfma_kernel(const ChannelDecayArgs a) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6, l16 = lane & 15, quad = lane >> 4;
@@ -132,6 +133,20 @@ __global__ __launch_bounds__(256) void channel_decay_mfma_kernel(const ChannelDe
     const int e = k * 32 + quad * 8;
     raw[k] = *reinterpret_cast<const bf16x8*>(h + (e < a.R ? e : 0));
   }
+  const int per = ((a.C + (int)gridDim.y - 1) / (int)gridDim.y + 15) / 16 * 16;
+  const int c_lo = blockIdx.y * per, c_hi = c_lo + per < a.C ? c_lo + per : a.C;
+  bf16x8 w[KC];
+  bf16x4 w0;
+  auto fetch = [&](int c0) {
+    const int c = c0 + l16 < a.C ? c0 + l16 : a.C - 1, cq = c0 + quad * 4 < a.C ? c0 + quad * 4 : 0;
+#pragma unroll
+    for (int k = 0; k < KC; ++k) {
+      const int e = k * 32 + quad * 8;
+      w[k] = *reinterpret_cast<const bf16x8*>(static_cast<const __bf16*>(a.w2) + (c * a.R + (e < a.R ? e : 0)));
+    }
+    w0 = *reinterpret_cast<const bf16x4*>(static_cast<const __bf16*>(a.w0) + cq);
+  };
+  if (c_lo < c_hi) fetch(c_lo);
 #pragma unroll
   for (int k = 0; k < KC; ++k)
 #pragma unroll
@@ -140,27 +155,21 @@ __global__ __launch_bounds__(256) void channel_decay_mfma_kernel(const ChannelDe
       hi[k][j] = (__bf16)t;
       lo[k][j] = (__bf16)(t - (float)hi[k][j]);
     }
+  for (int c0 = c_lo; c0 < c_hi; c0 += 16) {
+    f32x4 acc;
 #pragma unroll
-  for (int ct = 0; ct < 4; ++ct) {
-    const int c0 = blockIdx.y * 64 + ct * 16;
-    if (c0 >= a.C) break;
-    const int c = c0 + l16 < a.C ? c0 + l16 : a.C - 1;
-    f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+    for (int i = 0; i < 4; ++i) acc[i] = to_f32(w0[i]);
 #pragma unroll
     for (int k = 0; k < KC; ++k) {
-      const int e = k * 32 + quad * 8;
-      const bf16x8 w = *reinterpret_cast<const bf16x8*>(static_cast<const __bf16*>(a.w2) + (long)c * a.R + (e < a.R ? e : 0));
-      acc = mfma16(w, hi[k], acc);
-      acc = mfma16(w, lo[k], acc);
+      acc = mfma16(w[k], hi[k], acc);
+      acc = mfma16(w[k], lo[k], acc);
     }
-    // lane: row l16 of the tile, channels quad * 4 + i
-    if (row < a.rows) {
+    if (c0 + 16 < c_hi) fetch(c0 + 16);
+    // lane: row l16, channels 4 quad + i
+    f32x4 out;
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        const int ch = c0 + quad * 4 + i;
-        if (ch < a.C) a.y[row * a.C + ch] = -expf(acc[i] + to_f32(static_cast<const __bf16*>(a.w0)[ch])) * kLog2e;
-      }
-    }
+    for (int i = 0; i < 4; ++i) out[i] = -exp_f(acc[i]) * kLog2e;
+    if (row < a.rows && c0 + quad * 4 < c_hi) *reinterpret_cast<f32x4*>(a.y + row * a.C + c0 + quad * 4) = out;
   }
 }
 
@@ -245,8 +254,11 @@ extern "C" BASED_API int based_channel_decay(const void* h, const void* w2, cons
   if (rows == 0) return BASED_OK;
   const ChannelDecayArgs a{h, w2, w0, y, (long)rows, (long)h_sr, (int)C, (int)R};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  if (io_dtype == BASED_BF16 && R % 8 == 0 && R <= 256 && h_sr % 8 == 0 && aligned_to(h, 16) && aligned_to(w2, 16)) {
-    const dim3 grid((unsigned)((rows + 63) / 64), (unsigned)((C + 63) / 64));
+  if (io_dtype == BASED_BF16 && R % 8 == 0 && R <= 256 && C % 4 == 0 && C * R < (1ll << 31) && h_sr % 8 == 0 &&
+      aligned_to(h, 16) && aligned_to(w2, 16) && aligned_to(w0, 8) && aligned_to(y, 16)) {
+    // parts of the channels: enough workgroups for short portions, few times tanh for long ones
+    const int64_t blocks = (rows + 63) / 64, parts = blocks >= 1024 ? 2 : (2048 + blocks - 1) / blocks;
+    const dim3 grid((unsigned)blocks, (unsigned)(parts < (C + 63) / 64 ? parts : (C + 63) / 64));
     const int kc = (int)((R + 31) / 32);
     if (kc <= 1)
       hipLaunchKernelGGL((channel_decay_mfma_kernel<1>), grid, dim3(256), 0, s, a);

@@ -166,7 +166,7 @@ __device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) {
 }
 
 template <int KC, int VC, bool HALF>
-__global__ __launch_bounds__(256, KC <= 2 && VC <= 2 ? 3 : 1) void window_prefill_mfma_kernel(const WindowArgs a) {
+__global__ __launch_bounds__(256, KC <= 3 && VC <= 2 ? 3 : 1) void window_prefill_mfma_kernel(const WindowArgs a) {
   constexpr int D = KC * 32, DV = VC * 32;
   constexpr int KS = D + 8, VS = kTileKeys + 8;  // LDS row strides: 16-lane reads of 16 bytes meet every bank once
   __shared__ __attribute__((aligned(16))) __bf16 lds_k[kTileKeys * KS];
@@ -266,7 +266,7 @@ __global__ __launch_bounds__(256, KC <= 2 && VC <= 2 ? 3 : 1) void window_prefil
 
   fetch(lo);
   if (a.rot > 0) {
-    constexpr int CB = KC < 4 ? KC : 4;
+    constexpr int CB = KC == 3 ? 1 : KC < 4 ? KC : 4;
 #pragma unroll
     for (int c0 = 0; c0 < KC; c0 += CB) {
       Turn8<HALF> turn[2][CB];
@@ -1040,6 +1040,8 @@ static void launch_window_attend(const WindowArgs& a, bool vec, int io_dtype, hi
       launch_window_mfma<1>(a, grid, s);
     else if (kc <= 2)
       launch_window_mfma<2>(a, grid, s);
+    else if (kc <= 3)
+      launch_window_mfma<3>(a, grid, s);
     else if (kc <= 4)
       launch_window_mfma<4>(a, grid, s);
     else

@@ -1237,6 +1237,7 @@ def latent_write(x, norm_weight, cache, start: int, eps: float, rope) -> None:
 
 
 LATENT_STEP_TARGET = 512  # workgroups that the keys of a step are dealt to, where there are enough
+LATENT_STEP_MAX_SPLITS = 64
 
 
 def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: int, scale: float, pos, eps: float, rope,
@@ -1253,7 +1254,7 @@ def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: 
             or weight.shape[1] < R:
         raise ValueError(f"bad shapes q{tuple(q.shape)} weight{tuple(weight.shape)} out{tuple(out.shape)}")
     groups = B * ((heads + 15) // 16)
-    splits = max(1, min(LATENT_STEP_TARGET // groups, (min(window, S) + 127) // 128))
+    splits = max(1, min(LATENT_STEP_TARGET // groups, (min(window, S) + 127) // 128, LATENT_STEP_MAX_SPLITS))
     f32 = dict(dtype=torch.float32, device=x.device)
     work_q = torch.empty(B, heads, R + rot, **f32)
     part, part_ml = torch.empty(B, splits, heads, R, **f32), torch.empty(B, splits, heads, 2, **f32)
@@ -1268,7 +1269,7 @@ def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: 
 
 
 # Choices up to which experts are evaluated one choice at a time: beyond, rows of one expert share its matrices.
-EXPERT_ROWS_MAX = 128
+EXPERT_ROWS_MAX = 16
 
 
 def experts(h, router, w1, w2, top: int) -> torch.Tensor:
@@ -1290,24 +1291,23 @@ def experts(h, router, w1, w2, top: int) -> torch.Tensor:
     grouped = h2.dtype == torch.bfloat16 and n * top > EXPERT_ROWS_MAX and D % 8 == 0 and F % 8 == 0 and h2.stride(0) % 8 == 0
     i32 = dict(dtype=torch.int32, device=dev)
     ids, scores = torch.empty(n, top, **i32), torch.empty(n, top, dtype=torch.float32, device=dev)
-    rank, counts = (torch.empty(n, top, **i32), torch.zeros(E, **i32)) if grouped else (None, None)
     y = torch.empty(n, D, dtype=h2.dtype, device=dev)
     with _on_device(dev):
-        _lib.check(lib.based_expert_route(h2.data_ptr(), router.data_ptr(), ids.data_ptr(), scores.data_ptr(), _ptr(rank), _ptr(counts), n, D, E,
-                                          top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
         if grouped:
             tiles, rows = lib.based_expert_tiles(n, E, top), lib.based_expert_tile_rows(n, E, top)
+            rank = torch.empty(n, top, **i32)
+            counts = (torch.empty if n <= 16 else torch.zeros)(E, **i32)  # (so few tokens are counted by one workgroup)
             plan = torch.empty(E + 1 + tiles + tiles * rows, **i32)
             act = torch.empty(tiles * rows, F, dtype=h2.dtype, device=dev)
             part = torch.empty(n * top, D, dtype=h2.dtype, device=dev) if top > 1 else None
             _lib.check(lib.based_expert_grouped(
-                h2.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(), rank.data_ptr(), counts.data_ptr(), plan.data_ptr(),
-                plan[E + 1:].data_ptr(), plan[E + 1 + tiles:].data_ptr(), act.data_ptr(), _ptr(part), y.data_ptr(), n, D, F, E, top,
-                h2.stride(0), _stream_ptr(h2)))
+                h2.data_ptr(), router.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(), rank.data_ptr(),
+                counts.data_ptr(), plan.data_ptr(), plan[E + 1:].data_ptr(), plan[E + 1 + tiles:].data_ptr(), act.data_ptr(), _ptr(part),
+                y.data_ptr(), n, D, F, E, top, h2.stride(0), _stream_ptr(h2)))
         else:
             act = torch.empty(n * top, F, dtype=h2.dtype, device=dev)
-            _lib.check(lib.based_expert_rows(h2.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(), act.data_ptr(),
-                                             y.data_ptr(), n, D, F, top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
+            _lib.check(lib.based_expert_rows(h2.data_ptr(), router.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(),
+                                             act.data_ptr(), y.data_ptr(), n, D, F, E, top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
     return y.view(h.shape)
 
 

@@ -376,7 +376,8 @@ def expert_case(n, D, F, E, top, dtype, seed=0):
 
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("n,D,F,E,top", [(1, 64, 16, 4, 1), (9, 192, 40, 5, 2), (3, 84, 22, 3, 3), (200, 128, 64, 8, 1), (333, 192, 72, 6, 2),
-                                         (700, 64, 200, 3, 2), (150, 256, 136, 130, 3), (260, 84, 30, 4, 2), (5, 64, 8, 1, 1), (1100, 136, 64, 4, 4)])
+                                         (700, 64, 200, 3, 2), (150, 256, 136, 130, 3), (260, 84, 30, 4, 2), (5, 64, 8, 1, 1), (1100, 136, 64, 4, 4), (16, 128, 64, 8, 2), (24, 128, 40, 20, 2),
+                                         (32, 1024, 64, 40, 4), (31, 64, 64, 3, 1), (5000, 64, 72, 6, 2), (4100, 128, 264, 100, 2)])
 def test_experts(dev, n, D, F, E, top, dtype):
     from based_amd import ops
 
