@@ -145,7 +145,7 @@ SIGNATURES = {
     "based_expert_tiles": (_I64, [_I64] * 3),
     "based_expert_tile_rows": (_I64, [_I64] * 3),
     "based_expert_grouped": (C.c_int, [_P] * 14 + [_I64] * 6 + [_P]),
-    "based_expert_rows": (C.c_int, [_P] * 8 + [_I64] * 6 + [C.c_int, _P]),
+    "based_expert_rows": (C.c_int, [_P] * 5 + [C.c_float, C.c_int, C.c_float] + [_P] * 7 + [_I64] * 6 + [C.c_int, _P]),
     "based_decode_linear_extras": (
         C.c_int,
         [_P, _I64, _P, _I64, _P, _I64, _P, _P] + [_I64] * 4 + [_P, _I64, _P, _I64, C.c_float, C.c_int, _P, C.c_float, _P, _I64, C.c_int,

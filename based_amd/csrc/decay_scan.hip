@@ -255,7 +255,7 @@ __global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const 
         x[i] = row_moved<0x111>(k[i]);
         before[i] = row_moved<0x111>(w[i]);  // of the token before
       }
-      constexpr int kUnroll = HALVES > 1 ? 3 : 15;  // (fewer steps in flight where registers are scarce)
+      constexpr int kUnroll = 3;  // (few steps in flight: registers are scarce)
 #pragma unroll kUnroll
       for (int j = 1; j < 16; ++j) {
         sum = 0.f;

@@ -11,6 +11,7 @@
 //   expert_gemm     MFMA product of a tile of rows with its expert's matrices, gathered and scattered by that
 //                   order: gate and up with the activation behind them, then down
 //   expert_sum      the choices of a token added up (with one choice the product writes the token's row)
+//   expert_route_row  the same for few tokens, with the norm in front of the layer
 //   expert_rows     few tokens, fp32, or rows that are no whole 16-byte pieces: dot products, one choice at a time
 #include "stream_common.hpp"
 
@@ -188,6 +189,120 @@ __global__ __launch_bounds__(64 * NW) void expert_route_kernel(const RouteArgs a
   }
 }
 
+// Few tokens: one workgroup each, router rows as whole lines.  With norm_w (bf16) the token's row is formed first: r = res_in + mult * x
+// (fp32, into res_out), h = norm(r) * norm_w (into h_out).
+struct RouteRowArgs {
+  RouteArgs r;
+  const float* res_in;
+  float* res_out;
+  const __bf16* norm_w;
+  __bf16* h_out;
+  float mult, eps;
+  int kind;
+};
+
+constexpr int kRouteRowMax = 4096;  // channels
+
+__global__ __launch_bounds__(512) void expert_route_row_kernel(const RouteRowArgs a) {
+  __shared__ __attribute__((aligned(16))) __bf16 row[kRouteRowMax];
+  __shared__ float s[kMaxExperts], part[16];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, D = a.r.D, E = a.r.E;
+  const long n = blockIdx.x;
+  const __bf16* x = static_cast<const __bf16*>(a.r.h) + n * a.r.h_sr;
+  const int e8 = tid * 8;
+  const bool in = e8 < D;
+  float v[8];
+  load_vec<__bf16, 8>(x + (in ? e8 : 0), v);
+  if (a.norm_w != nullptr) {
+    float w8[8], r8[8];
+    load_vec<__bf16, 8>(a.norm_w + (in ? e8 : 0), w8);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) r8[i] = 0.f;
+    if (a.res_in != nullptr) load_vec<float, 8>(a.res_in + n * D + (in ? e8 : 0), r8);
+    const float mult = a.res_in != nullptr ? a.mult : 1.0f;
+    float sum = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      v[i] = in ? __builtin_fmaf(mult, v[i], r8[i]) : 0.f;
+      sum += v[i];
+    }
+    auto all = [&](float q, int at) {
+      q = sum16(q);
+      q += __shfl_xor(q, 16, 64);
+      q += __shfl_xor(q, 32, 64);
+      if (lane == 0) part[at + wave] = q;
+      __syncthreads();
+      float t = 0.f;
+#pragma unroll
+      for (int i = 0; i < 8; ++i) t += part[at + i];
+      return t;
+    };
+    if (a.res_out != nullptr && in) store_vec<float, 8>(a.res_out + n * D + e8, v);
+    const float mean = a.kind == BASED_NORM_LAYER ? all(sum, 0) / (float)D : 0.f;
+    float ss = 0.f;
+#pragma unroll
+    for (int i = 0; i < 8; ++i) {
+      v[i] = in ? v[i] - mean : 0.f;
+      ss = __builtin_fmaf(v[i], v[i], ss);
+    }
+    const float rstd = 1.0f / sqrtf(all(ss, 8) / (float)D + a.eps);
+#pragma unroll
+    for (int i = 0; i < 8; ++i) v[i] *= rstd * w8[i];
+    if (in) store_vec<__bf16, 8>(a.h_out + n * D + e8, v);
+  }
+  if (in) store_vec<__bf16, 8>(row + e8, v);
+  __syncthreads();
+  constexpr int EU = 4;  // experts whose rows are in flight together
+  for (int e0 = wave * EU; e0 < E; e0 += 8 * EU) {
+    float acc[EU];
+#pragma unroll
+    for (int u = 0; u < EU; ++u) acc[u] = 0.f;
+#pragma unroll 2
+    for (int c = lane * 8; c < D; c += 512) {
+      float h8[8];
+      load_vec<__bf16, 8>(row + c, h8);
+#pragma unroll
+      for (int u = 0; u < EU; ++u) {
+        float w8[8];
+        load_vec<__bf16, 8>(static_cast<const __bf16*>(a.r.w) + (long)(e0 + u < E ? e0 + u : 0) * D + c, w8);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[u] = __builtin_fmaf(w8[i], h8[i], acc[u]);
+      }
+    }
+#pragma unroll
+    for (int u = 0; u < EU; ++u) {
+      float z = sum16(acc[u]);
+      z += __shfl_xor(z, 16, 64);
+      z += __shfl_xor(z, 32, 64);
+      if (lane == 0 && e0 + u < E) s[e0 + u] = 1.0f / (1.0f + expf(-z));
+    }
+  }
+  __syncthreads();
+  if (wave != 0) return;
+  float mine[kMaxExperts / 64];
+#pragma unroll
+  for (int i = 0; i < kMaxExperts / 64; ++i) mine[i] = i * 64 + lane < E ? s[i * 64 + lane] : -2.f;
+  for (int j = 0; j < a.r.top; ++j) {
+    float best = -3.f;
+    int at = 0;
+#pragma unroll
+    for (int i = 0; i < kMaxExperts / 64; ++i)
+      if (mine[i] > best) best = mine[i], at = i * 64 + lane;
+#pragma unroll
+    for (int m = 32; m >= 1; m >>= 1) {
+      const float ov = __shfl_xor(best, m, 64);
+      const int oa = __shfl_xor(at, m, 64);
+      if (ov > best || (ov == best && oa < at)) best = ov, at = oa;
+    }
+#pragma unroll
+    for (int i = 0; i < kMaxExperts / 64; ++i) mine[i] = i * 64 + lane == at ? -2.f : mine[i];
+    if (lane == 0) {
+      a.r.ids[n * a.r.top + j] = at;
+      a.r.scores[n * a.r.top + j] = best;
+    }
+  }
+}
+
 constexpr long kPlanSlots = 8192;  // choices that the planning workgroup puts in order by itself
 
 __global__ __launch_bounds__(256) void expert_plan_kernel(const int32_t* counts, const int32_t* ids, const int32_t* rank, int32_t* tile_first,
@@ -351,7 +466,7 @@ template <int BM, int BN, int AHEAD, bool PAIRED> void launch_expert_gemm(Expert
 template <bool PAIRED> void launch_expert_product(const ExpertGemmArgs& a, int rows, hipStream_t s) {
   if (rows == BASED_EXPERT_TILE_ROWS_SMALL)
     launch_expert_gemm<BASED_EXPERT_TILE_ROWS_SMALL, 128, 4, PAIRED>(a, s);
-  else if (a.F >= 256)
+  else if (a.F >= 256 && (long)a.tiles * a.F >= (PAIRED ? 512 * 128 : 512 * 256))
     launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 256, 1, PAIRED>(a, s);
   else
     launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 128, 2, PAIRED>(a, s);
@@ -541,7 +656,7 @@ static int route_check(const char* who, const RouteArgs& a) {
 }  // namespace based
 
 /* Tiles of BASED_EXPERT_TILE_ROWS or BASED_EXPERT_TILE_ROWS_SMALL rows. */
-static int expert_tile_rows(int64_t slots, int64_t E) { return slots >= 64 * E ? BASED_EXPERT_TILE_ROWS : BASED_EXPERT_TILE_ROWS_SMALL; }
+static int expert_tile_rows(int64_t slots, int64_t E) { return slots >= 256 * E ? BASED_EXPERT_TILE_ROWS : BASED_EXPERT_TILE_ROWS_SMALL; }
 
 extern "C" BASED_API int64_t based_expert_tiles(int64_t n, int64_t E, int64_t top) {
   if (n <= 0 || E <= 0 || top <= 0) return 0;
@@ -597,29 +712,46 @@ extern "C" BASED_API int based_expert_grouped(const void* h, const void* router,
   return check_launch("expert_grouped");
 }
 
-extern "C" BASED_API int based_expert_rows(const void* h, const void* router, const void* w1, const void* w2, int32_t* ids, float* scores,
-                                           void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t E, int64_t top, int64_t h_sr,
-                                           int io_dtype, void* stream) {
+extern "C" BASED_API int based_expert_rows(const void* x, const float* residual_in, float* residual_out, const void* norm_weight, void* work_h,
+                                           float mult, int norm_kind, float eps, const void* router, const void* w1, const void* w2,
+                                           int32_t* ids, float* scores, void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t E,
+                                           int64_t top, int64_t x_sr, int io_dtype, void* stream) {
   using namespace based;
-  BASED_REQUIRE(h && router && w1 && w2 && ids && scores && work_act && y, BASED_ERR_ARG, "expert_rows: null pointer argument");
+  BASED_REQUIRE(x && router && w1 && w2 && ids && scores && work_act && y, BASED_ERR_ARG, "expert_rows: null pointer argument");
   BASED_REQUIRE(F > 0 && D < (1 << 20) && F < (1 << 20), BASED_ERR_SHAPE, "expert_rows: grid too large");
   BASED_REQUIRE(io_dtype == BASED_BF16 || io_dtype == BASED_F32, BASED_ERR_DTYPE, "expert_rows: bad dtype");
-  const RouteArgs r{h, router, ids, scores, nullptr, nullptr, nullptr, nullptr, nullptr, 0, (long)n, (long)h_sr, (int)D, (int)E, (int)top};
+  RouteArgs r{x, router, ids, scores, nullptr, nullptr, nullptr, nullptr, nullptr, 0, (long)n, (long)x_sr, (int)D, (int)E, (int)top};
   const int rc = route_check("expert_rows", r);
   if (rc != BASED_OK) return rc;
+  const bool by_row = io_dtype == BASED_BF16 && D % 8 == 0 && D <= kRouteRowMax && x_sr % 8 == 0 && aligned_to(x, 16) && aligned_to(router, 16);
+  if (norm_weight != nullptr) {
+    BASED_REQUIRE(by_row, BASED_ERR_SHAPE, "expert_rows: the norm takes bf16 rows of a multiple of 8 up to %d channels", kRouteRowMax);
+    BASED_REQUIRE(work_h && (norm_kind == BASED_NORM_RMS || norm_kind == BASED_NORM_LAYER) && residual_out != residual_in, BASED_ERR_ARG,
+                  "expert_rows: bad norm arguments");
+    BASED_REQUIRE(aligned_to(norm_weight, 16) && aligned_to(residual_in, 16) && aligned_to(residual_out, 16) && aligned_to(work_h, 16),
+                  BASED_ERR_ALIGN, "expert_rows: tensors must be 16-byte aligned");
+  }
   if (n == 0) return BASED_OK;
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const void* h = norm_weight != nullptr ? work_h : x;
+  const int64_t h_sr = norm_weight != nullptr ? D : x_sr;
+  if (norm_weight != nullptr || (by_row && n <= 16)) {
+    const RouteRowArgs a{r, residual_in, residual_out, static_cast<const __bf16*>(norm_weight), static_cast<__bf16*>(work_h), mult, eps, norm_kind};
+    hipLaunchKernelGGL(expert_route_row_kernel, dim3((unsigned)n), dim3(512), 0, s, a);
+  } else if (io_dtype == BASED_BF16) {
+    launch_route<__bf16>(r, route_vec(r), s);
+  } else {
+    launch_route<float>(r, false, s);
+  }
   const int p = io_dtype == BASED_BF16 ? 8 : 4;
   const bool vec1 = D % p == 0 && h_sr % p == 0 && aligned_to(h, 16) && aligned_to(w1, 16);
   const bool vec2 = F % p == 0 && aligned_to(work_act, 16) && aligned_to(w2, 16);
   const ExpertRowsArgs a1{h, w1, work_act, ids, scores, (long)n, (long)h_sr, (int)F, (int)D, (int)top};
   const ExpertRowsArgs a2{work_act, w2, y, ids, scores, (long)n, (long)F, (int)D, (int)F, (int)top};
-  hipStream_t s = static_cast<hipStream_t>(stream);
   if (io_dtype == BASED_BF16) {
-    launch_route<__bf16>(r, route_vec(r), s);
     launch_expert_rows_vec<__bf16, true>(a1, vec1, n * top, s);
     launch_expert_rows_vec<__bf16, false>(a2, vec2, n, s);
   } else {
-    launch_route<float>(r, false, s);
     launch_expert_rows_vec<float, true>(a1, vec1, n * top, s);
     launch_expert_rows_vec<float, false>(a2, vec2, n, s);
   }

@@ -394,7 +394,7 @@ __global__ __launch_bounds__(256, 1) void latent_step_mfma_kernel(const LatentAr
 }
 
 constexpr int kValueRows = 4;   // sequences at a time
-constexpr int kValueCols = 32;  // value channels per workgroup
+constexpr int kValueCols = 16;  // value channels per workgroup
 constexpr int kMaxSplits = 64;
 
 template <typename T, int N>
@@ -403,6 +403,22 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int h = blockIdx.x, b0 = blockIdx.y * kValueRows, j0 = blockIdx.z * kValueCols;
   const int rows = a.B - b0 < kValueRows ? a.B - b0 : kValueRows;
+  // this wavefront's rows of uv are asked for first
+  constexpr int JU = kValueCols / 4;
+  const T* w = static_cast<const T*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot + a.d) * a.w_sr;
+  const int j1 = j0 + kValueCols < a.dv ? j0 + kValueCols : a.dv, j = j0 + wave * JU;
+  float wv[JU][N];
+  auto load_rows = [&](int c) {
+#pragma unroll
+    for (int u = 0; u < JU; ++u) {
+      const T* p = w + (long)(j + u < j1 ? j + u : j0) * a.w_sr + (c < a.R ? c : 0);
+      if constexpr (N == 1)
+        wv[u][0] = to_f32(*p);
+      else
+        load_vec<T, N>(p, wv[u]);
+    }
+  };
+  load_rows(lane * N);
   // what each split counts for: exp(m_s - max) / sum
   __shared__ float share[kValueRows][kMaxSplits];
   for (int m = wave; m < rows; m += 4) {
@@ -431,38 +447,49 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   }
   __syncthreads();
   // (a split without keys has left nothing in its part: it is not read)
-  for (int i = tid; i < rows * a.R; i += 256) {
-    const int m = i / a.R, c = i % a.R;
-    const float* p = a.part + ((long)(b0 + m) * a.splits * a.H + h) * a.R + c;
-    float v = 0.f;
-#pragma unroll 4
-    for (int s = 0; s < a.splits; ++s) {
-      const float f = share[m][s], x = p[f != 0.f ? (long)s * a.H * a.R : 0];
-      v = f != 0.f ? __builtin_fmaf(f, x, v) : v;
+  const float* p0 = a.part + ((long)b0 * a.splits * a.H + h) * a.R;
+  const long p_row = (long)a.splits * a.H * a.R, p_split = (long)a.H * a.R;
+  constexpr int SU = 8;  // splits whose parts are in flight together
+  if (a.R % 4 == 0 && (reinterpret_cast<uintptr_t>(a.part) & 15) == 0) {
+    const int pieces = a.R / 4;
+    for (int i = tid; i < rows * pieces; i += 256) {
+      const int m = i / pieces, c = i % pieces * 4;
+      f32x4 v = {0.f, 0.f, 0.f, 0.f};
+      for (int s0 = 0; s0 < a.splits; s0 += SU) {
+        f32x4 x[SU];
+        float f[SU];
+#pragma unroll
+        for (int s = 0; s < SU; ++s) {
+          f[s] = s0 + s < a.splits ? share[m][s0 + s] : 0.f;
+          x[s] = *reinterpret_cast<const f32x4*>(p0 + m * p_row + (f[s] != 0.f ? (s0 + s) * p_split : 0) + c);
+        }
+#pragma unroll
+        for (int s = 0; s < SU; ++s)
+#pragma unroll
+          for (int j = 0; j < 4; ++j) v[j] = f[s] != 0.f ? __builtin_fmaf(f[s], x[s][j], v[j]) : v[j];
+      }
+      *reinterpret_cast<f32x4*>(&lat[m][c]) = v;
     }
-    lat[m][c] = v;
+  } else {
+    for (int i = tid; i < rows * a.R; i += 256) {
+      const int m = i / a.R, c = i % a.R;
+      float v = 0.f;
+      for (int s = 0; s < a.splits; ++s) {
+        const float f = share[m][s];
+        if (f != 0.f) v = __builtin_fmaf(f, p0[m * p_row + s * p_split + c], v);
+      }
+      lat[m][c] = v;
+    }
   }
   __syncthreads();
-  const T* w = static_cast<const T*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot + a.d) * a.w_sr;
-  const int j1 = j0 + kValueCols < a.dv ? j0 + kValueCols : a.dv;
-  constexpr int JU = 4;  // value channels whose rows are in flight together
-  for (int j = j0 + wave * JU; j < j1; j += 4 * JU) {
+  {
     float acc[JU][kValueRows];
 #pragma unroll
     for (int u = 0; u < JU; ++u)
 #pragma unroll
       for (int m = 0; m < kValueRows; ++m) acc[u][m] = 0.f;
-#pragma unroll 2
     for (int c = lane * N; c < a.R; c += 64 * N) {
-      float wv[JU][N];
-#pragma unroll
-      for (int u = 0; u < JU; ++u) {
-        const T* p = w + (long)(j + u < j1 ? j + u : j) * a.w_sr + c;
-        if constexpr (N == 1)
-          wv[u][0] = to_f32(*p);
-        else
-          load_vec<T, N>(p, wv[u]);
-      }
+      if (c >= 64 * N) load_rows(c);
 #pragma unroll
       for (int m = 0; m < kValueRows; ++m)
 #pragma unroll

@@ -1270,11 +1270,13 @@ def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: 
 
 # Choices up to which experts are evaluated one choice at a time: beyond, rows of one expert share its matrices.
 EXPERT_ROWS_MAX = 16
+EXPERT_NORM_MAX_DIM = 4096
 
 
-def experts(h, router, w1, w2, top: int) -> torch.Tensor:
+def experts(h, router, w1, w2, top: int, norm=None) -> torch.Tensor:
     """y = sum over the `top` experts of a token with the largest sigmoid(router h) of w2_e (silu(gate) * up), [up; gate] = score * w1_e h.
-    h (..., D), router (E, D), w1 (E, 2 F, D) up rows first, w2 (E, D, F)."""
+    h (..., D), router (E, D), w1 (E, 2 F, D) up rows first, w2 (E, D, F).  norm = (residual fp32 or None, residual_out fp32 or None, weight,
+    eps, kind, mult): h is the input of `add_norm` with these and the layer reads its norm."""
     D = h.shape[-1]
     E, F = w2.shape[0], w2.shape[2]
     h2 = h.reshape(-1, D)
@@ -1290,6 +1292,20 @@ def experts(h, router, w1, w2, top: int) -> torch.Tensor:
     lib = _lib.lib()
     grouped = h2.dtype == torch.bfloat16 and n * top > EXPERT_ROWS_MAX and D % 8 == 0 and F % 8 == 0 and h2.stride(0) % 8 == 0
     i32 = dict(dtype=torch.int32, device=dev)
+    norm_args = (None, None, None, None, 1.0, NORM_RMS, 0.0)
+    if norm is not None:
+        residual, residual_out, weight, eps, kind, mult = norm
+        if grouped or h2.dtype != torch.bfloat16 or D % 8 != 0 or D > EXPERT_NORM_MAX_DIM or n * top > EXPERT_ROWS_MAX:
+            h2, _ = add_norm(h2, residual, weight, eps, kind, mult, residual_out is not None, residual_out)
+        else:
+            for r in (residual, residual_out):
+                if r is not None and (r.dtype != torch.float32 or tuple(r.shape) != (n, D) or not r.is_contiguous() or not r.is_cuda):
+                    raise ValueError(f"residuals must be contiguous float32 ({n}, {D}) device tensors")
+            _check_same_dtype(h2, weight)
+            if tuple(weight.shape) != (D,) or not weight.is_contiguous() or not weight.is_cuda:
+                raise ValueError(f"the norm's weight must be a contiguous ({D},) on the device")
+            normed = torch.empty_like(h2)
+            norm_args = (_ptr(residual), _ptr(residual_out), weight.data_ptr(), normed.data_ptr(), float(mult), int(kind), float(eps))
     ids, scores = torch.empty(n, top, **i32), torch.empty(n, top, dtype=torch.float32, device=dev)
     y = torch.empty(n, D, dtype=h2.dtype, device=dev)
     with _on_device(dev):
@@ -1306,8 +1322,9 @@ def experts(h, router, w1, w2, top: int) -> torch.Tensor:
                 y.data_ptr(), n, D, F, E, top, h2.stride(0), _stream_ptr(h2)))
         else:
             act = torch.empty(n * top, F, dtype=h2.dtype, device=dev)
-            _lib.check(lib.based_expert_rows(h2.data_ptr(), router.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(), scores.data_ptr(),
-                                             act.data_ptr(), y.data_ptr(), n, D, F, E, top, h2.stride(0), _dtype_code(h2), _stream_ptr(h2)))
+            _lib.check(lib.based_expert_rows(h2.data_ptr(), *norm_args, router.data_ptr(), w1.data_ptr(), w2.data_ptr(), ids.data_ptr(),
+                                             scores.data_ptr(), act.data_ptr(), y.data_ptr(), n, D, F, E, top, h2.stride(0), _dtype_code(h2),
+                                             _stream_ptr(h2)))
     return y.view(h.shape)
 
 

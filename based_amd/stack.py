@@ -341,8 +341,8 @@ class ExpertMlp(nn.Module):
         self.w1 = nn.Parameter(torch.empty(experts, 2 * hidden, in_features, **fk).normal_(std=0.02))
         self.w2 = nn.Parameter(torch.empty(experts, in_features, hidden, **fk).normal_(std=0.02))
 
-    def forward(self, x):
-        return ops.experts(x, self.router, self.w1, self.w2, self.top)
+    def forward(self, x, norm=None):
+        return ops.experts(x, self.router, self.w1, self.w2, self.top, norm)
 
 
 class TokenSide(nn.Module):
@@ -410,7 +410,7 @@ class Block(nn.Module):
         if side is not None and not (ops.decode_linear_weight_ok(side.gate.weight) and ops.decode_linear_weight_ok(side.proj.weight)):
             return False
         return (getattr(self.mixer, "supports_decode_step", lambda: False)()
-                and (mlp is None or (isinstance(mlp, ExpertMlp) and norm_fuses(self.norm2)) or (
+                and (mlp is None or (isinstance(mlp, ExpertMlp) and isinstance(self.norm2, StreamNorm) and norm_fuses(self.norm2)) or (
                                      isinstance(mlp, GatedMlp) and mlp.mlp_type == "base" and mlp.activation == "swiglu"
                                      and ops.decode_linear_weight_ok(mlp.fc1.weight)
                                      and ops.decode_linear_weight_ok(mlp.fc2.weight) and norm_fuses(self.norm2)))
@@ -439,8 +439,7 @@ class Block(nn.Module):
         hidden_states = self.mixer.decode_step(hidden_states, inference_params, **norm)
         if isinstance(self.mlp, ExpertMlp):
             n = self.norm2
-            h, _ = ops.add_norm(hidden_states, mid, n.weight, n.eps, n.kind, n.mult, residual_out=last)
-            hidden_states = self.mlp(h)
+            hidden_states = self.mlp(hidden_states, norm=(mid, last, n.weight, n.eps, n.kind, n.mult))
             mid, last = last, mid
         elif self.mlp is not None:
             norm = norm_prologue(self.norm2, mid, last)

@@ -648,7 +648,8 @@ BASED_API int based_latent_step(const void* q, const void* x, const void* norm_w
  * y = sum over them of w2_e (silu(gate) * up), [up; gate] = score * w1_e h; router (E, D), w1 (E, 2 F, D), w2 (E, D, F).
  * Grouped (bf16): rows of one expert share its matrices; scratch: rank (n, top), counts (E, zero on entry), tile_first (E + 1),
  * tile_expert (tiles), order (tiles * rows), work_act (tiles * rows, F), work_out (n * top, D) with top > 1, tiles and rows from
- * based_expert_tiles / based_expert_tile_rows.  Rows: one choice at a time, for few tokens and any element type; work_act (n * top, F). */
+ * based_expert_tiles / based_expert_tile_rows.  Rows: one choice at a time, for few tokens and any element type; work_act (n * top, F).
+ * With norm_weight (D; bf16, D up to 4096) h is the norm of residual_in + mult * x as in based_add_norm, in work_h (n, D). */
 #define BASED_EXPERT_TILE_ROWS 128
 #define BASED_EXPERT_TILE_ROWS_SMALL 32
 BASED_API int64_t based_expert_tiles(int64_t n, int64_t E, int64_t top);
@@ -657,9 +658,10 @@ BASED_API int based_expert_grouped(const void* h, const void* router, const void
                                    int32_t* rank, int32_t* counts, int32_t* tile_first, int32_t* tile_expert, int32_t* order,
                                    void* work_act, void* work_out, void* y, int64_t n, int64_t D, int64_t F, int64_t E, int64_t top,
                                    int64_t h_sr, void* stream);
-BASED_API int based_expert_rows(const void* h, const void* router, const void* w1, const void* w2, int32_t* ids, float* scores,
-                                void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t E, int64_t top, int64_t h_sr,
-                                int io_dtype, void* stream);
+BASED_API int based_expert_rows(const void* x, const float* residual_in, float* residual_out, const void* norm_weight, void* work_h,
+                                float mult, int norm_kind, float eps, const void* router, const void* w1, const void* w2,
+                                int32_t* ids, float* scores, void* work_act, void* y, int64_t n, int64_t D, int64_t F, int64_t E,
+                                int64_t top, int64_t x_sr, int io_dtype, void* stream);
 
 /* based_decode_linear_stream with what else may surround a projection of single tokens; a pointer that is NULL leaves its part out.
  *   post_weight, add_vec, add_rows: as in based_add_norm_addends (row m adds add_rows[add_index[m]]); norm_kind BASED_NORM_NONE

@@ -407,6 +407,26 @@ def test_expert_products_do_not_depend_on_the_batch(dev):
     assert float((whole.double() - alone.double()).norm() / alone.double().norm()) < 4e-3
 
 
+@pytest.mark.parametrize("n,D,top", [(1, 64, 1), (4, 1024, 2), (3, 4096, 3), (9, 192, 2)])
+def test_experts_behind_their_norm(dev, n, D, top):
+    from based_amd import ops
+
+    x, router, w1, w2, w = expert_case(n, D, 40, 5, top, BF16)
+    router = router * 3  # (clear choices)
+    w["m.router"] = router.double()
+    res, nw = rnd(n, D, seed=7), rnd(D, seed=8, dtype=BF16, scale=0.2, mean=1.0)
+    d = lambda t: t.to(dev)
+    for kind in (ops.NORM_RMS, ops.NORM_LAYER):
+        for r in (res, None):
+            out = torch.empty(n, D, device=dev)
+            y = ops.experts(d(x), d(router), d(w1), d(w2), top, norm=(None if r is None else d(r), out, d(nw), 1e-5, kind, 0.5))
+            total = x.double() if r is None else r.double() + 0.5 * x.double()
+            close(out, total, 1e-6)
+            h = (total if kind == ops.NORM_RMS else total - total.mean(-1, keepdim=True))
+            h = (O.rms(h, 1e-5) * nw.double()).bfloat16().double()
+            close(y, O.expert_mlp(h, w, "m", {"router": {"top": top}}), 3 * TOL[BF16])
+
+
 # ---- projections of single tokens ----
 @pytest.mark.parametrize("M", [1, 3, 8, 9, 32])
 @pytest.mark.parametrize("K,rows,rank", [(64, 32, 8), (192, 64, 24), (1024, 96, 40), (2048, 32, 16), (4096, 64, 64)])
