@@ -1,7 +1,7 @@
 #!/usr/bin/env python3
 """Benchmark of the Based sequence-mixer hot path on one MI355X.
 
-    python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-cpu] [--only decode|prefill|swa|conv|stack|projections|copy|machine|sozilix]
+    python bench.py [--gpus 1] [--steps K] [--warmup W] [--no-cpu] [--only decode|prefill|swa|conv|stack|projections|copy|machine|sozilix|peponex]
 
 Headline workload (`value`): the recurrent decode step of Taylor linear attention at
 B=128, H=16, dv=64 — fp32 kv_state (128,16,1,64,273) + k_state, initialised from a seeded
@@ -793,10 +793,12 @@ def main():
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--no-graph", action="store_true",
                     help="decode legs: launches issued one by one, HIP events (for counter runs under a profiler)")
-    ap.add_argument("--only", choices=["decode", "prefill", "swa", "conv", "stack", "projections", "copy", "machine", "sozilix"], default=None,
+    ap.add_argument("--only", choices=["decode", "prefill", "swa", "conv", "stack", "projections", "copy", "machine", "sozilix", "peponex"],
+                    default=None,
                     help="one workload only; 'copy' is a plain 256 MiB device copy (the copy probe of bench_probes.hip) used to "
                          "calibrate the FETCH_SIZE / WRITE_SIZE counters of a rocprofv3 --pmc run; 'machine' the memory "
-                         "probes alone; 'sozilix' the streamed layers and a model of them beside the Based ones (bench_sozilix.py)")
+                         "probes alone; 'sozilix' and 'peponex' the layers of these designs and a model of them beside the Based "
+                         "ones (bench_sozilix.py, bench_peponex.py)")
     ap.add_argument("--prefill-batches", default="1,8,32,96",
                     help="comma-separated batch sizes of the L=4096 prefill lines")
     args = ap.parse_args()
@@ -827,14 +829,14 @@ def main():
         print(json.dumps({"machine": bench_machine(torch)}))
         return
 
-    if args.only == "sozilix":
-        import bench_sozilix
+    if args.only in ("sozilix", "peponex"):
+        import importlib
 
-        r = bench_sozilix.bench(torch)
-        m = r["models"]["sozilix"]
-        print(json.dumps({"metric": "decode tok/s, 27-layer Sozilix model, B=4, 1 GPU", "value": m["decode_B4_tok_s"], "unit": "tokens/s",
-                          "n_gpus": 1, "ms_per_step": m["decode_B4_ms_per_token"], "higher_is_better": True, "vs_baseline": None,
-                          "dtype": "bf16", "data": "synthetic", **r}))
+        r = importlib.import_module(f"bench_{args.only}").bench(torch)
+        m = r["models"][args.only]
+        print(json.dumps({"metric": f"decode tok/s, 27-layer {args.only.capitalize()} model, B=4, 1 GPU", "value": m["decode_B4_tok_s"],
+                          "unit": "tokens/s", "n_gpus": 1, "ms_per_step": m["decode_B4_ms_per_token"], "higher_is_better": True,
+                          "vs_baseline": None, "dtype": "bf16", "data": "synthetic", **r}))
         return
 
     out = {

@@ -206,14 +206,20 @@ def sozilix_config(D=1024, layers=27, vocab=50280, ff=2048):
             "layers": [par if i % 3 == 2 else rec for i in range(layers)]}
 
 
-def bench_models(torch, B=4, prefill_len=2048, new_tokens=128):
-    """Prefill and greedy decoding (recorded graph) of both models, and decoding at batch 32."""
+def model_configs():
+    """Name -> function that makes the StackConfig of the two models."""
     from based_amd import architectures
-    from based_amd.stack import GPTLMHeadModel, StackConfig, based_360m_config
+    from based_amd.stack import StackConfig, based_360m_config
+
+    raw = sozilix_config()
+    return {"sozilix": lambda: StackConfig(**architectures.find(raw).stack_config(raw)), "based_360m": based_360m_config}
+
+
+def bench_models(torch, makes, B=4, prefill_len=2048, new_tokens=128):
+    """Prefill and greedy decoding (recorded graph) of every model, and decoding at batch 32."""
+    from based_amd.stack import GPTLMHeadModel
 
     dev = torch.device("cuda:0")
-    raw = sozilix_config()
-    makes = {"sozilix": lambda: StackConfig(**architectures.find(raw).stack_config(raw)), "based_360m": based_360m_config}
     out = {"B": B, "prefill_len": prefill_len, "new_tokens": new_tokens}
     for name, make in makes.items():
         torch.manual_seed(0)
@@ -254,4 +260,4 @@ def bench(torch):
     with torch.inference_mode():
         kernels = bench_kernels(torch, ops)
     torch.cuda.empty_cache()
-    return {"kernels": kernels, "models": bench_models(torch)}
+    return {"kernels": kernels, "models": bench_models(torch, model_configs())}
