@@ -132,6 +132,7 @@ SIGNATURES = {
     "based_token_mix": (C.c_int, [_P] * 5 + [_I64] * 8 + [C.c_int, _P]),
     "based_channel_decay": (C.c_int, [_P] * 4 + [_I64] * 4 + [C.c_int, _P]),
     "based_gelu_mul": (C.c_int, [_P] * 4 + [_I64] * 5 + [C.c_int, _P]),
+    "based_token_side_step": (C.c_int, [_P] * 8 + [_I64] * 6 + [C.c_float, _P]),
     "based_softcap": (C.c_int, [_P, _I64, C.c_float, C.c_int, _P]),
     "based_decay_scan_work": (_I64, [_I64] * 6),
     "based_decay_scan": (C.c_int, [_P] * 9 + [_I64] * 14 + [C.c_int, C.c_int, C.c_int, _P]),

@@ -288,7 +288,7 @@ __global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const 
       }
     }
     if (!LATE && chunk + 1 < last) fetch(cur, chunk + 1);
-    __syncthreads();  // every wavefront is done with the 64 tokens before
+    lds_barrier();  // every wavefront is done with the 64 tokens before
 #pragma unroll
     for (int j = 0; j < 8; ++j)
       store_pair(&lds.vt[(half * 64 + quad * 16 + 2 * j) * TS + t], &lds.vt[(half * 64 + quad * 16 + 2 * j + 1) * TS + t], vv[j]);
@@ -341,7 +341,7 @@ __global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const 
         }
       }
     }
-    __syncthreads();
+    lds_barrier();
 
     if constexpr (CHANNEL) {
       const int ch = threadIdx.x;
@@ -427,14 +427,14 @@ __global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const 
         }
       }
     }
-    __syncthreads();  // k is not read any more: P goes into its place
+    lds_barrier();  // k is not read any more: P goes into its place
     if constexpr (!STATE_ONLY) {
       if constexpr (HALVES > 1) {
         if (half == 1) {
 #pragma unroll
           for (int j = 0; j < 4; ++j) lds.p.part[(blk * 4 + j) * 64 + lane] = P[j];
         }
-        __syncthreads();
+        lds_barrier();
         if (half == 0) {
 #pragma unroll
           for (int j = 0; j < 4; ++j) P[j] += lds.p.part[(blk * 4 + j) * 64 + lane];
@@ -455,7 +455,7 @@ __global__ __launch_bounds__(256 * HALVES, 2) void decay_scan_mfma_kernel(const 
           *reinterpret_cast<u32x2*>(&lds.p.lo[t * TS + j * 16 + quad * 4]) = lo;
         }
       }
-      __syncthreads();
+      lds_barrier();
     }
     if (LATE && chunk + 1 < last) fetch(cur, chunk + 1);
     if (has_cols) {

@@ -160,14 +160,6 @@ enum { kProNone = BASED_PROLOGUE_NONE, kProNorm = BASED_PROLOGUE_ADD_RMS_NORM, k
        kProStream = 3, kProStreamAdd = 4 };
 enum { kEpiNone = BASED_EPILOGUE_NONE, kEpiSwiglu = BASED_EPILOGUE_SWIGLU, kEpiConv = BASED_EPILOGUE_GATED_CONV_STEP };
 
-__device__ __forceinline__ void lds_barrier() {
-  // the waves only exchange data through LDS here; a fence over global memory as well would wait
-  // for the weight rows that are still on their way
-  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
-  __builtin_amdgcn_s_barrier();
-  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
-}
-
 // C: 512-element chunks of the contraction length a lane holds (K <= 512 C); MT: activation rows
 // held (M <= MT); a row group is R = 8 / C weight rows, one per wavefront at a time.  A prologue
 // is evaluated ONCE per workgroup (norm: wavefront w owns rows w, w + 4; gate: the (row, chunk)

@@ -334,6 +334,7 @@ struct ExpertGemmArgs {
 };
 
 constexpr int kGemmK = 64;
+constexpr int kBand = 8;
 
 // Workgroups are dealt to the eight dies in turn: those of one die take neighbouring tiles, which share rows and matrices.
 __device__ __forceinline__ int tile_of_block(int i, int n) {
@@ -343,20 +344,26 @@ __device__ __forceinline__ int tile_of_block(int i, int n) {
 
 // BM rows and BN rows of the weights (PAIRED: half of them up, half gate) per workgroup; AHEAD rounds of 64 channels on their
 // way from memory.
-template <int BM, int BN, int AHEAD, bool PAIRED>
+template <int BM, int BN, int AHEAD, int BUF, bool PAIRED>
 __global__ __launch_bounds__(256, 2) void expert_gemm_kernel(const ExpertGemmArgs a) {
-  constexpr int KS = kGemmK + 8;
+  // rows of 128 bytes lie side by side, the eight 16-byte pieces of a row turned by half its number: neither the rows that
+  // eight lanes write nor the sixteen that a tile reads meet a bank twice
+  constexpr int KS = kGemmK;
+  auto place = [](int r, int p) { return r * KS + ((p ^ (r >> 1)) & 7) * 8; };
   constexpr int WM = BM >= 128 ? 2 : 1, WN = 4 / WM, MT = BM / 16 / WM, NT = BN / 32 / WN, HALF = BN / 2;
   constexpr int AP = BM / 32, BP = BN / 32;  // 16-byte pieces per thread
-  __shared__ __attribute__((aligned(16))) __bf16 xs[BM * KS], ws[BN * KS];
+  __shared__ __attribute__((aligned(16))) __bf16 xs[BUF][BM * KS], ws[BUF][BN * KS];
   __shared__ int slot_of[BM];
-  const int id = tile_of_block(blockIdx.x, gridDim.x), tile = id / a.col_tiles, f0 = id % a.col_tiles * (PAIRED ? HALF : BN);
+  // bands of kBand row tiles, walked down the rows first: what is in flight on a die shares its rows and its matrices
+  const int id = tile_of_block(blockIdx.x, gridDim.x), band = id / (kBand * a.col_tiles), in_band = id % (kBand * a.col_tiles);
+  const int deep = a.tiles - band * kBand < kBand ? a.tiles - band * kBand : kBand;
+  const int tile = band * kBand + in_band % deep, f0 = in_band / deep * (PAIRED ? HALF : BN);
   if (tile >= a.tile_first[a.E]) return;
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4, wm = wave % WM, wn = wave / WM;
   const int e = a.tile_expert[tile], r0 = (tile - a.tile_first[e]) * BM;
   const int rows = a.counts[e] - r0 < BM ? a.counts[e] - r0 : BM;
   for (int i = tid; i < BM; i += 256) slot_of[i] = a.order[(long)tile * BM + (i < rows ? i : 0)];
-  __syncthreads();
+  lds_barrier();
   typedef __attribute__((ext_vector_type(4))) uint32_t u32x4;
   const int piece = (tid & 7) * 8;  // of the 64 channels of a round
   const __bf16* xrow[AP];
@@ -389,34 +396,58 @@ __global__ __launch_bounds__(256, 2) void expert_gemm_kernel(const ExpertGemmArg
     for (int i = 0; i < NT; ++i)
 #pragma unroll
       for (int j = 0; j < MT; ++j) acc[p][i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  auto stage = [&](int k0, int buf, const u32x4 (&x)[AP], const u32x4 (&w)[BP]) {
+    const bool in = k0 + piece < a.K;
+#pragma unroll
+    for (int i = 0; i < AP; ++i) *reinterpret_cast<u32x4*>(&xs[buf][place(i * 32 + (tid >> 3), tid & 7)]) = in ? x[i] : zero;
+#pragma unroll
+    for (int i = 0; i < BP; ++i) *reinterpret_cast<u32x4*>(&ws[buf][place(i * 32 + (tid >> 3), tid & 7)]) = w[i];
+  };
+  auto multiply = [&](int buf) {
+#pragma unroll
+    for (int kk = 0; kk < kGemmK; kk += 32) {
+      bf16x8 xf[MT];
+#pragma unroll
+      for (int j = 0; j < MT; ++j) xf[j] = *reinterpret_cast<const bf16x8*>(&xs[buf][place((wm * MT + j) * 16 + l16, kk / 8 + quad)]);
+#pragma unroll
+      for (int p = 0; p < 2; ++p)
+#pragma unroll
+        for (int i = 0; i < NT; ++i) {
+          const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&ws[buf][place(p * HALF + (wn * NT + i) * 16 + l16, kk / 8 + quad)]);
+#pragma unroll
+          for (int j = 0; j < MT; ++j) acc[p][i][j] = expert_mfma(wf, xf[j], acc[p][i][j]);
+        }
+    }
+  };
 #pragma unroll
   for (int s = 0; s < AHEAD; ++s) fetch(s * kGemmK, xb[s], wb[s]);
-  // (rounds past the end multiply by zeros: every stage of the loop is the same)
-  for (int k00 = 0; k00 < a.K; k00 += AHEAD * kGemmK) {
+  // (rounds past the end multiply by zeros: every stage of the loops is the same)
+  if constexpr (BUF == 1) {
+    for (int k00 = 0; k00 < a.K; k00 += AHEAD * kGemmK) {
 #pragma unroll
-    for (int s = 0; s < AHEAD; ++s) {
-      const int k0 = k00 + s * kGemmK;
-      const bool in = k0 + piece < a.K;
-      __syncthreads();
+      for (int s = 0; s < AHEAD; ++s) {
+        const int k0 = k00 + s * kGemmK;
+        lds_barrier();
+        stage(k0, 0, xb[s], wb[s]);
+        lds_barrier();
+        fetch(k0 + AHEAD * kGemmK, xb[s], wb[s]);
+        multiply(0);
+      }
+    }
+  } else {
+    // one barrier per round: the next round goes into the other half of LDS while this one is multiplied
+    constexpr int U = AHEAD % 2 == 0 ? AHEAD : 2 * AHEAD;
+    stage(0, 0, xb[0], wb[0]);
+    fetch(AHEAD * kGemmK, xb[0], wb[0]);
+    lds_barrier();
+    for (int k00 = 0; k00 < a.K; k00 += U * kGemmK) {
 #pragma unroll
-      for (int i = 0; i < AP; ++i) *reinterpret_cast<u32x4*>(&xs[(i * 32 + (tid >> 3)) * KS + piece]) = in ? xb[s][i] : zero;
-#pragma unroll
-      for (int i = 0; i < BP; ++i) *reinterpret_cast<u32x4*>(&ws[(i * 32 + (tid >> 3)) * KS + piece]) = wb[s][i];
-      __syncthreads();
-      fetch(k0 + AHEAD * kGemmK, xb[s], wb[s]);
-#pragma unroll
-      for (int kk = 0; kk < kGemmK; kk += 32) {
-        bf16x8 xf[MT];
-#pragma unroll
-        for (int j = 0; j < MT; ++j) xf[j] = *reinterpret_cast<const bf16x8*>(&xs[((wm * MT + j) * 16 + l16) * KS + kk + quad * 8]);
-#pragma unroll
-        for (int p = 0; p < 2; ++p)
-#pragma unroll
-          for (int i = 0; i < NT; ++i) {
-            const bf16x8 wf = *reinterpret_cast<const bf16x8*>(&ws[(p * HALF + (wn * NT + i) * 16 + l16) * KS + kk + quad * 8]);
-#pragma unroll
-            for (int j = 0; j < MT; ++j) acc[p][i][j] = expert_mfma(wf, xf[j], acc[p][i][j]);
-          }
+      for (int s = 0; s < U; ++s) {
+        const int k1 = k00 + (s + 1) * kGemmK;
+        multiply(s & 1);
+        stage(k1, (s + 1) & 1, xb[(s + 1) % AHEAD], wb[(s + 1) % AHEAD]);
+        fetch(k1 + AHEAD * kGemmK, xb[(s + 1) % AHEAD], wb[(s + 1) % AHEAD]);
+        lds_barrier();
       }
     }
   }
@@ -457,19 +488,19 @@ __global__ __launch_bounds__(256, 2) void expert_gemm_kernel(const ExpertGemmArg
   }
 }
 
-template <int BM, int BN, int AHEAD, bool PAIRED> void launch_expert_gemm(ExpertGemmArgs a, hipStream_t s) {
+template <int BM, int BN, int AHEAD, int BUF, bool PAIRED> void launch_expert_gemm(ExpertGemmArgs a, hipStream_t s) {
   const int cols = PAIRED ? BN / 2 : BN;
   a.col_tiles = (a.F + cols - 1) / cols;
-  hipLaunchKernelGGL((expert_gemm_kernel<BM, BN, AHEAD, PAIRED>), dim3((unsigned)(a.col_tiles * a.tiles)), dim3(256), 0, s, a);
+  hipLaunchKernelGGL((expert_gemm_kernel<BM, BN, AHEAD, BUF, PAIRED>), dim3((unsigned)(a.col_tiles * a.tiles)), dim3(256), 0, s, a);
 }
 
 template <bool PAIRED> void launch_expert_product(const ExpertGemmArgs& a, int rows, hipStream_t s) {
   if (rows == BASED_EXPERT_TILE_ROWS_SMALL)
-    launch_expert_gemm<BASED_EXPERT_TILE_ROWS_SMALL, 128, 4, PAIRED>(a, s);
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS_SMALL, 128, 4, 1, PAIRED>(a, s);
   else if (a.F >= 256 && (long)a.tiles * a.F >= (PAIRED ? 512 * 128 : 512 * 256))
-    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 256, 1, PAIRED>(a, s);
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 256, 1, 1, PAIRED>(a, s);
   else
-    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 128, 2, PAIRED>(a, s);
+    launch_expert_gemm<BASED_EXPERT_TILE_ROWS, 128, 2, 1, PAIRED>(a, s);
 }
 
 // y[n] = sum of the rows of its choices

@@ -325,7 +325,7 @@ __global__ __launch_bounds__(256, 1) void latent_step_mfma_kernel(const LatentAr
   for (int i = 0; i < RT; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m_run = -INFINITY, l_run = 0.f;
   for (int k0 = 0; k0 < n; k0 += 64) {
-    __syncthreads();
+    lds_barrier();
 #pragma unroll
     for (int i = 0; i < VU; ++i) {
       const int p = i * 256 + tid, k4 = p & 15, e = (p >> 4) * 8;
@@ -353,7 +353,7 @@ __global__ __launch_bounds__(256, 1) void latent_step_mfma_kernel(const LatentAr
     mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
     mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
     if (quad == 0) wmax[wave][l16] = mx;
-    __syncthreads();
+    lds_barrier();
     const float m_new = fmaxf(m_run, fmaxf(fmaxf(wmax[0][l16], wmax[1][l16]), fmaxf(wmax[2][l16], wmax[3][l16])));
     const float alpha = __builtin_amdgcn_exp2f(m_run - m_new);
     m_run = m_new;
@@ -369,7 +369,7 @@ __global__ __launch_bounds__(256, 1) void latent_step_mfma_kernel(const LatentAr
     sum += __shfl_xor(sum, 16, 64);
     sum += __shfl_xor(sum, 32, 64);
     if (quad == 0) wsum[wave][l16] = sum;
-    __syncthreads();
+    lds_barrier();
     l_run = l_run * alpha + wsum[0][l16] + wsum[1][l16] + wsum[2][l16] + wsum[3][l16];
     const bf16x8 pf0 = *reinterpret_cast<const bf16x8*>(&ps[l16 * KS + quad * 8]);
     const bf16x8 pf1 = *reinterpret_cast<const bf16x8*>(&ps[l16 * KS + 32 + quad * 8]);
@@ -445,7 +445,7 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
 #pragma unroll
     for (int i = 0; i < kMaxSplits / 64; ++i) share[m][i * 64 + lane] = l > 0.f ? ms[i] / l : 0.f;
   }
-  __syncthreads();
+  lds_barrier();
   // (a split without keys has left nothing in its part: it is not read)
   const float* p0 = a.part + ((long)b0 * a.splits * a.H + h) * a.R;
   const long p_row = (long)a.splits * a.H * a.R, p_split = (long)a.H * a.R;
@@ -481,7 +481,7 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
       lat[m][c] = v;
     }
   }
-  __syncthreads();
+  lds_barrier();
   {
     float acc[JU][kValueRows];
 #pragma unroll

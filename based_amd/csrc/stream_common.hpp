@@ -123,6 +123,14 @@ struct StreamAddends {
   float post_eps;
 };
 
+// A barrier between wavefronts that only exchange data through LDS: a fence over global memory as well would wait
+// for loads that are meant to stay on their way.
+__device__ __forceinline__ void lds_barrier() {
+  __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+  __builtin_amdgcn_s_barrier();
+  __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+}
+
 // Position of the token a single-token launch brings for batch row b: from the device when there is
 // an array of positions, otherwise the one the host passed.
 __device__ __forceinline__ int row_pos(const int32_t* pos, int pos_host, int b) { return pos != nullptr ? pos[b] : pos_host; }

@@ -6,6 +6,8 @@
 //   channel_decay:  log2 of exp(-exp(w2 tanh(h) + w0)) per channel, in fp32.
 //   gelu_mul:       gelu_tanh(g) * table[index], the gate of a per-token embedding.
 //   softcap:        cap * tanh(x / cap) in place.
+//   token_side_step: a per-layer token input for single tokens, r = residual + mult * x and
+//                   proj(gelu_tanh(gate r) * table[index]) in one launch, a workgroup per token.
 #include "stream_common.hpp"
 
 namespace based {
@@ -212,6 +214,107 @@ __global__ __launch_bounds__(256) void softcap_kernel(T* x, long n, float cap) {
   }
 }
 
+// ---- a token input for single tokens ----
+struct SideStepArgs {
+  const __bf16* x;       // (M, D)
+  const float* res_in;   // (M, D)
+  float* res_out;        // (M, D)
+  const __bf16* gate_w;  // (n, D)
+  const __bf16* proj_w;  // (D, n)
+  const __bf16* table;
+  const int64_t* index;
+  __bf16* y;             // (M, D)
+  long x_sr, t_sr, t_n;
+  int D, n;
+  float mult;
+};
+
+constexpr int kSideThreads = 1024, kSideWaves = kSideThreads / 64;
+constexpr int kSideMaxDim = 4096, kSideMaxInner = 512;
+
+// C: 512-channel pieces of a row a lane holds of each gate row (D <= 512 C).
+template <int C>
+__global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const SideStepArgs a) {
+  __shared__ __attribute__((aligned(16))) __bf16 row[512 * C];
+  __shared__ __attribute__((aligned(16))) __bf16 inner[kSideMaxInner];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+  const long m = blockIdx.x;
+  // the first gate rows and the first row of proj are asked for before anything else
+  constexpr int GU = C >= 8 ? 1 : C >= 4 ? 2 : 4;  // gate rows in flight together
+  bf16x8 g8[GU][C];
+  auto fetch = [&](int j0) {
+#pragma unroll
+    for (int u = 0; u < GU; ++u)
+#pragma unroll
+      for (int c = 0; c < C; ++c) {
+        const int e = (c * 64 + lane) * 8, j = j0 + u;
+        g8[u][c] = *reinterpret_cast<const bf16x8*>(a.gate_w + (long)(j < a.n ? j : 0) * a.D + (e < a.D ? e : 0));
+      }
+  };
+  fetch(wave * GU);
+  const long src = a.index[m];
+  const bool bad = src < 0 || src >= a.t_n;
+  for (int e = tid * 4; e < 512 * C; e += kSideThreads * 4) {
+    f32x4 r = {0.f, 0.f, 0.f, 0.f};
+    if (e < a.D) {
+      const bf16x4 x = *reinterpret_cast<const bf16x4*>(a.x + m * a.x_sr + e);
+      if (a.res_in != nullptr) {
+        r = *reinterpret_cast<const f32x4*>(a.res_in + m * a.D + e);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) r[j] = __builtin_fmaf(a.mult, to_f32(x[j]), r[j]);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j) r[j] = to_f32(x[j]);
+      }
+      *reinterpret_cast<f32x4*>(a.res_out + m * a.D + e) = r;
+    }
+    bf16x4 o;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) o[j] = (__bf16)r[j];
+    *reinterpret_cast<bf16x4*>(row + e) = o;  // (zeros behind the row)
+  }
+  lds_barrier();
+  for (int j0 = wave * GU; j0 < a.n; j0 += kSideWaves * GU) {
+    if (j0 != wave * GU) fetch(j0);
+    float acc[GU];
+#pragma unroll
+    for (int u = 0; u < GU; ++u) acc[u] = 0.f;
+#pragma unroll
+    for (int c = 0; c < C; ++c) {
+      float x[8];
+      load_vec<__bf16, 8>(row + (c * 64 + lane) * 8, x);
+#pragma unroll
+      for (int u = 0; u < GU; ++u)
+#pragma unroll
+        for (int i = 0; i < 8; ++i) acc[u] = __builtin_fmaf(to_f32(g8[u][c][i]), x[i], acc[u]);
+    }
+#pragma unroll
+    for (int u = 0; u < GU; ++u) {
+      float v = sum16(acc[u]);
+      v += __shfl_xor(v, 16, 64);
+      v += __shfl_xor(v, 32, 64);
+      if (lane == 0 && j0 + u < a.n) {
+        const float e = to_f32(a.table[(bad ? 0 : src) * a.t_sr + j0 + u]);
+        inner[j0 + u] = (__bf16)(bad ? __builtin_nanf("") : gelu_tanh_f(round_to<__bf16>(v)) * e);
+      }
+    }
+  }
+  lds_barrier();
+  for (int d = tid; d < a.D; d += kSideThreads) {
+    const __bf16* w = a.proj_w + (long)d * a.n;
+    float acc = 0.f;
+#pragma unroll 8
+    for (int c = 0; c < a.n; c += 8) {
+      float x[8], wv[8];
+      load_vec<__bf16, 8>(w + c, wv);
+      load_vec<__bf16, 8>(inner + c, x);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc = __builtin_fmaf(wv[i], x[i], acc);
+    }
+    a.y[m * a.D + d] = (__bf16)acc;
+  }
+}
+
 }  // namespace based
 
 extern "C" BASED_API int based_token_mix(const void* x, const void* mu, void* y, void* ring, const int32_t* pos, int64_t pos_host,
@@ -257,7 +360,7 @@ extern "C" BASED_API int based_channel_decay(const void* h, const void* w2, cons
   if (io_dtype == BASED_BF16 && R % 8 == 0 && R <= 256 && C % 4 == 0 && C * R < (1ll << 31) && h_sr % 8 == 0 &&
       aligned_to(h, 16) && aligned_to(w2, 16) && aligned_to(w0, 8) && aligned_to(y, 16)) {
     // parts of the channels: enough workgroups for short portions, few times tanh for long ones
-    const int64_t blocks = (rows + 63) / 64, parts = blocks >= 1024 ? 2 : (2048 + blocks - 1) / blocks;
+    const int64_t blocks = (rows + 63) / 64, parts = blocks >= 512 ? 2 : (1024 + blocks - 1) / blocks;
     const dim3 grid((unsigned)blocks, (unsigned)(parts < (C + 63) / 64 ? parts : (C + 63) / 64));
     const int kc = (int)((R + 31) / 32);
     if (kc <= 1)
@@ -311,4 +414,34 @@ extern "C" BASED_API int based_softcap(void* x, int64_t n, float cap, int io_dty
   else
     hipLaunchKernelGGL(softcap_kernel<float>, grid, dim3(256), 0, s, static_cast<float*>(x), (long)n, cap);
   return check_launch("softcap");
+}
+
+extern "C" BASED_API int based_token_side_step(const void* x, const float* residual_in, float* residual_out, const void* gate_w,
+                                               const void* proj_w, const void* table, const int64_t* index, void* y, int64_t M, int64_t D,
+                                               int64_t n, int64_t x_sr, int64_t table_sr, int64_t table_n, float mult, void* stream) {
+  using namespace based;
+  BASED_REQUIRE(x && residual_out && gate_w && proj_w && table && index && y, BASED_ERR_ARG, "token_side_step: null pointer argument");
+  BASED_REQUIRE(M >= 0 && D > 0 && n > 0 && table_n > 0 && M < (1ll << 31), BASED_ERR_ARG, "token_side_step: bad sizes");
+  BASED_REQUIRE(D % 8 == 0 && D <= kSideMaxDim && n % 8 == 0 && n <= kSideMaxInner, BASED_ERR_SHAPE,
+                "token_side_step: sizes %ld and %ld (multiples of 8, at most %d and %d)", (long)D, (long)n, kSideMaxDim, kSideMaxInner);
+  BASED_REQUIRE(x_sr % 4 == 0 && aligned_to(x, 8) && aligned_to(residual_in, 16) && aligned_to(residual_out, 16) && aligned_to(gate_w, 16) &&
+                    aligned_to(proj_w, 16),
+                BASED_ERR_ALIGN, "token_side_step: rows must be whole 16-byte pieces");
+  BASED_REQUIRE(residual_in != residual_out, BASED_ERR_ARG, "token_side_step: residual_out must not be residual_in");
+  if (M == 0) return BASED_OK;
+  const SideStepArgs a{static_cast<const __bf16*>(x), residual_in, residual_out, static_cast<const __bf16*>(gate_w),
+                       static_cast<const __bf16*>(proj_w), static_cast<const __bf16*>(table), index, static_cast<__bf16*>(y), (long)x_sr,
+                       (long)table_sr, (long)table_n, (int)D, (int)n, mult};
+  hipStream_t s = static_cast<hipStream_t>(stream);
+  const dim3 grid((unsigned)M), block(kSideThreads);
+  const int chunks = (int)((D + 511) / 512);
+  if (chunks <= 1)
+    hipLaunchKernelGGL((token_side_step_kernel<1>), grid, block, 0, s, a);
+  else if (chunks <= 2)
+    hipLaunchKernelGGL((token_side_step_kernel<2>), grid, block, 0, s, a);
+  else if (chunks <= 4)
+    hipLaunchKernelGGL((token_side_step_kernel<4>), grid, block, 0, s, a);
+  else
+    hipLaunchKernelGGL((token_side_step_kernel<8>), grid, block, 0, s, a);
+  return check_launch("token_side_step");
 }

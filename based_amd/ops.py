@@ -1084,6 +1084,40 @@ def gelu_mul(g, table, index) -> torch.Tensor:
     return y
 
 
+SIDE_STEP_MAX_DIM, SIDE_STEP_MAX_INNER = 4096, 512
+
+
+def token_side_step_ok(gate_w, proj_w) -> bool:
+    """Whether `token_side_step` takes these weights: bf16 (n, D) and (D, n) with whole 16-byte pieces."""
+    n, D = gate_w.shape
+    return (gate_w.is_cuda and gate_w.dtype == torch.bfloat16 and proj_w.dtype == torch.bfloat16 and gate_w.is_contiguous()
+            and proj_w.is_contiguous() and n % 8 == 0 and D % 8 == 0 and D <= SIDE_STEP_MAX_DIM and n <= SIDE_STEP_MAX_INNER)
+
+
+def token_side_step(x, residual, residual_out, gate_w, proj_w, table, index, mult: float = 1.0) -> torch.Tensor:
+    """r = residual + mult * x in fp32 (x without a residual), written to residual_out, and proj_w (gelu_tanh(gate_w r) * table[index]), for
+    single tokens in one launch: x (M, D) bf16, gate_w (n, D), proj_w (D, n), table (entries, n) with rows at any stride, index (M)."""
+    M, D = x.shape
+    n = gate_w.shape[0]
+    _require_cuda(x, residual_out, gate_w, proj_w, table, index)
+    _check_same_dtype(x, gate_w, proj_w, table)
+    if x.dtype != torch.bfloat16 or x.stride(1) != 1 or tuple(gate_w.shape) != (n, D) or tuple(proj_w.shape) != (D, n) \
+            or not gate_w.is_contiguous() or not proj_w.is_contiguous():
+        raise ValueError(f"bad shapes x{tuple(x.shape)} gate_w{tuple(gate_w.shape)} proj_w{tuple(proj_w.shape)}")
+    if table.dim() != 2 or table.shape[1] != n or table.stride(1) != 1 or index.dtype != torch.int64 or index.numel() != M \
+            or not index.is_contiguous():
+        raise ValueError(f"bad table {tuple(table.shape)} or index {tuple(index.shape)}")
+    for r in (residual, residual_out):
+        if r is not None and (r.dtype != torch.float32 or tuple(r.shape) != (M, D) or not r.is_contiguous()):
+            raise ValueError(f"residuals must be contiguous float32 ({M}, {D})")
+    y = torch.empty(M, D, dtype=x.dtype, device=x.device)
+    with _on_device(x.device):
+        _lib.check(_lib.lib().based_token_side_step(x.data_ptr(), _ptr(residual), residual_out.data_ptr(), gate_w.data_ptr(), proj_w.data_ptr(),
+                                                    table.data_ptr(), index.data_ptr(), y.data_ptr(), M, D, n, x.stride(0), table.stride(0),
+                                                    table.shape[0], float(mult), _stream_ptr(x)))
+    return y
+
+
 def softcap_(x, cap: float) -> torch.Tensor:
     """x <- cap * tanh(x / cap), in place."""
     _require_cuda(x)

@@ -407,7 +407,7 @@ class Block(nn.Module):
     def supports_decode_step(self) -> bool:
         mlp = self.mlp
         side = self.side
-        if side is not None and not (ops.decode_linear_weight_ok(side.gate.weight) and ops.decode_linear_weight_ok(side.proj.weight)):
+        if side is not None and not ops.token_side_step_ok(side.gate.weight, side.proj.weight):
             return False
         return (getattr(self.mixer, "supports_decode_step", lambda: False)()
                 and (mlp is None or (isinstance(mlp, ExpertMlp) and isinstance(self.norm2, StreamNorm) and norm_fuses(self.norm2)) or (
@@ -455,9 +455,8 @@ class Block(nn.Module):
             mid, last = last, mid
         if self.side is not None:
             side = self.side
-            g = ops.decode_linear(hidden_states, side.gate.weight, prologue=ops.PROLOGUE_STREAM, norm_kind=ops.NORM_NONE,
-                                  mult=self.norm1.mult, residual_in=mid, residual_out=last, gate=(side.table(side_table), ids))
-            hidden_states = ops.decode_linear(g, side.proj.weight)
+            hidden_states = ops.token_side_step(hidden_states, mid, last, side.gate.weight, side.proj.weight, side.table(side_table), ids,
+                                                self.norm1.mult)
             mid, last = last, mid
         return hidden_states, mid, last
 

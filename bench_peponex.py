@@ -137,11 +137,16 @@ def bench_kernels(torch, ops, B=8, L=4096, D=1024):
                      ("addends + cap", dict(addends=add, softcap=30.0))):
         pair("decode_linear 4160x1024 M=4, norm + %s" % name, _entry(time(lambda i: ops.decode_linear(x, ws[i], **more, **kw), n), ws[0].numel() * 2),
              "decode_linear (RMS norm)", like)
-    sg, st = [rnd(64, D) for _ in range(n)], rnd(1000, 64)
-    small = _entry(time(lambda i: ops.decode_linear(x, sg[i], prologue=ops.PROLOGUE_ADD_RMS_NORM, **rows), n), sg[0].numel() * 2)
-    pair("decode_linear 64x1024 M=4, sum + gate table",
-         _entry(time(lambda i: ops.decode_linear(x, sg[i], prologue=ops.PROLOGUE_STREAM, norm_kind=ops.NORM_NONE, residual_in=res, residual_out=ro,
-                                                 gate=(st, tok)), n), sg[0].numel() * 2), "decode_linear 64x1024 (RMS norm)", small)
+    sg, sp, st = [rnd(64, D) for _ in range(n)], [rnd(D, 64) for _ in range(n)], rnd(1000, 64)
+    for M in (4, 32):
+        x, res, ro, tok = rnd(M, D), torch.randn(M, D, device=dev), torch.empty(M, D, device=dev), torch.arange(M, device=dev)
+
+        def small(i):
+            ops.decode_linear(ops.decode_linear(x, sg[i], prologue=ops.PROLOGUE_ADD_RMS_NORM, residual_in=res, residual_out=ro, norm_weight=nw),
+                              sp[i])
+
+        pair("token_side_step 64 of 1024 M=%d" % M, _entry(time(lambda i: ops.token_side_step(x, res, ro, sg[i], sp[i], st, tok), n), 4 * 64 * D),
+             "decode_linear 64x1024 (RMS norm), 1024x64", _entry(time(small, n), 4 * 64 * D))
     for M in (4, 32):
         x, res, ro = rnd(M, D), torch.randn(M, D, device=dev), torch.empty(M, D, device=dev)
         f1, f2 = [rnd(4096, D) for _ in range(12)], [rnd(D, 2048) for _ in range(12)]

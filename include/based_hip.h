@@ -590,6 +590,13 @@ BASED_API int based_gelu_mul(const void* g, const void* table, const int64_t* in
 /* x <- cap * tanh(x / cap), n contiguous elements. */
 BASED_API int based_softcap(void* x, int64_t n, float cap, int io_dtype, void* stream);
 
+/* A per-layer token input for single tokens (bf16): r = residual_in + mult * x (x without one) in fp32 into residual_out, and
+ * y = proj_w (gelu_tanh(gate_w r) * table[index]); x, y (M, D), gate_w (n, D), proj_w (D, n), table rows of n elements table_sr
+ * apart.  D a multiple of 8 up to 4096, n up to 512. */
+BASED_API int based_token_side_step(const void* x, const float* residual_in, float* residual_out, const void* gate_w,
+                                    const void* proj_w, const void* table, const int64_t* index, void* y, int64_t M, int64_t D,
+                                    int64_t n, int64_t x_sr, int64_t table_sr, int64_t table_n, float mult, void* stream);
+
 /* Linear attention with decaying states over a portion; q, k (B, L, H * D), v, o (B, L, H * DV), silu on q, k
  * and v first with BASED_ACT_SILU.  channel_log2 (B, L, H * D) contiguous, the log2 of a decay w per key channel, with
  * bonus u (H, D): o_t = (S + diag(u) k v^T)^T q, S <- diag(w) S + k v^T.  Or head_decay (2, H), the log2 of constants w

@@ -476,6 +476,24 @@ def test_projection_with_gate_table_and_cap(dev, M, N, K):
     close(y, 1.5 * torch.tanh((O.rms(r, 1e-5) * nw.double()).bfloat16().double() @ w.double().T / 1.5), 2 * TOL[BF16])
 
 
+@pytest.mark.parametrize("M", [1, 5, 32])
+@pytest.mark.parametrize("n,D", [(8, 64), (24, 192), (64, 1024), (136, 1544), (16, 4096), (512, 512)])
+def test_token_input_of_single_tokens(dev, M, n, D):
+    from based_amd import ops
+
+    x, gw, pw, res = rnd(M, D, dtype=BF16), rnd(n, D, seed=1, dtype=BF16, scale=D ** -0.5), rnd(D, n, seed=2, dtype=BF16, scale=n ** -0.5), rnd(M, D, seed=3)
+    table, idx = rnd(7, 3 * n, seed=4, dtype=BF16), torch.arange(M) % 7
+    d = lambda t: t.to(dev)
+    assert ops.token_side_step_ok(d(gw), d(pw))
+    for r in (res, None):
+        out = torch.empty(M, D, device=dev)
+        y = ops.token_side_step(d(x), None if r is None else d(r), out, d(gw), d(pw), d(table)[:, n:2 * n], d(idx), 0.5)
+        total = x.double() if r is None else r.double() + 0.5 * x.double()
+        close(out, total, 1e-6)
+        g = O.gelu_tanh(total.bfloat16().double() @ gw.double().T) * table[:, n:2 * n].double()[idx]
+        close(y, g @ pw.double().T, 2 * TOL[BF16])
+
+
 def test_refusals(dev):
     from based_amd import ops
 
