@@ -8,6 +8,7 @@
 //   latent_query   one token per sequence: q~ and the rotated q of every head, and the token's cache row
 //   latent_step    scores, softmax and weighted latents, the keys of a sequence dealt to several workgroups
 //   latent_values  their partial results put together, times uv
+// The first and the last have a form on MFMA for 16 sequences at a time.
 #include "stream_common.hpp"
 
 namespace based {
@@ -115,6 +116,23 @@ __global__ __launch_bounds__(256) void latent_write_vec_kernel(const LatentArgs 
 constexpr int kQueryCols = 128;  // latent channels per workgroup of latent_query
 constexpr int kQueryRows = 4;    // sequences at a time
 
+// The cache row and the rotated queries of sequence b, by one workgroup.
+template <typename T> __device__ __forceinline__ void query_row(const LatentArgs& a, int b) {
+  const int tid = threadIdx.x, W = a.R + a.rot;
+  if (b >= a.B) return;
+  const int pos = row_pos(a.pos, a.pos_host, b);
+  if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;
+  if (tid < 64) {
+    write_row<T>(a, static_cast<const T*>(a.x) + b * a.x_sb, static_cast<T*>(a.cache) + b * a.c_sb + pos * a.c_st, pos, tid);
+  } else {
+    for (int i = tid - 64; i < a.H * a.rot; i += 192) {
+      const int h = i / a.rot, c = i % a.rot;
+      const T* q = static_cast<const T*>(a.q) + b * a.q_sb + (long)h * (a.rot + a.d);
+      a.qa[((long)b * a.H + h) * W + a.R + c] = round_to<T>(turned(q, c, pos, a));
+    }
+  }
+}
+
 // N: elements per load (8 or 1); kQueryRows sequences per workgroup.  In x, workgroups 0 .. H * ceil(R / kQueryCols) - 1 form q~, the
 // rest (one per sequence) write the cache row and rotate the queries.
 template <typename T, int N>
@@ -124,19 +142,7 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
   __shared__ float part[GROUPS][kQueryRows][kQueryCols];
   const int tid = threadIdx.x, W = a.R + a.rot, col_blocks = (a.R + kQueryCols - 1) / kQueryCols;
   if ((int)blockIdx.x >= a.H * col_blocks) {
-    const int b = blockIdx.y * kQueryRows + blockIdx.x - a.H * col_blocks;
-    if (b >= a.B) return;
-    const int pos = row_pos(a.pos, a.pos_host, b);
-    if (pos < 0 || pos >= a.S || (a.rot > 0 && pos >= a.n_pos)) return;
-    if (tid < 64) {
-      write_row<T>(a, static_cast<const T*>(a.x) + b * a.x_sb, static_cast<T*>(a.cache) + b * a.c_sb + pos * a.c_st, pos, tid);
-    } else {
-      for (int i = tid - 64; i < a.H * a.rot; i += 192) {
-        const int h = i / a.rot, c = i % a.rot;
-        const T* q = static_cast<const T*>(a.q) + b * a.q_sb + (long)h * (a.rot + a.d);
-        a.qa[((long)b * a.H + h) * W + a.R + c] = round_to<T>(turned(q, c, pos, a));
-      }
-    }
+    query_row<T>(a, blockIdx.y * kQueryRows + blockIdx.x - a.H * col_blocks);
     return;
   }
   const int h = blockIdx.x / col_blocks, r0 = (blockIdx.x % col_blocks) * kQueryCols;
@@ -186,10 +192,65 @@ __global__ __launch_bounds__(256) void latent_query_kernel(const LatentArgs a) {
   }
 }
 
+__device__ __forceinline__ f32x4 latent_mfma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+
+// The same for 16 sequences per workgroup, bf16 rows of whole 16-byte pieces: uk is turned round in LDS, 64 of a head's channels at a time.
+constexpr int kTileRows = 16;
+constexpr int kTileMinRows = 8;  // sequences from which these forms are used
+
+__global__ __launch_bounds__(256) void latent_query_mfma_kernel(const LatentArgs a) {
+  constexpr int KD = 64, KS = KD + 8;
+  __shared__ __attribute__((aligned(16))) __bf16 ut[kQueryCols * KS];  // [latent channel][channel of the head]
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4, W = a.R + a.rot;
+  const int col_blocks = (a.R + kQueryCols - 1) / kQueryCols;
+  if ((int)blockIdx.x >= a.H * col_blocks) {
+    query_row<__bf16>(a, blockIdx.y * kTileRows + blockIdx.x - a.H * col_blocks);
+    return;
+  }
+  const int h = blockIdx.x / col_blocks, r0 = (blockIdx.x % col_blocks) * kQueryCols, b0 = blockIdx.y * kTileRows;
+  const __bf16* w = static_cast<const __bf16*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot) * a.w_sr;
+  const __bf16* q = static_cast<const __bf16*>(a.q) + (long)(b0 + l16 < a.B ? b0 + l16 : b0) * a.q_sb + (long)h * (a.rot + a.d) + a.rot;
+  const int k4 = tid & 15, e = (tid >> 4) * 8;  // this thread's (4 channels of the head x 8 of the latent)
+  const int col = r0 + e < a.R ? r0 + e : 0;
+  f32x4 acc[2] = {f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+  for (int d0 = 0; d0 < a.d; d0 += KD) {
+    bf16x8 wf[4], qf[2];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = d0 + k4 * 4 + r;
+      wf[r] = *reinterpret_cast<const bf16x8*>(w + (long)(d < a.d ? d : 0) * a.w_sr + col);
+    }
+#pragma unroll
+    for (int s = 0; s < 2; ++s) {  // (channels past the end are zero here, anything in ut)
+      const int d = d0 + s * 32 + quad * 8;
+      qf[s] = *reinterpret_cast<const bf16x8*>(q + (d < a.d ? d : 0));
+      if (d >= a.d) qf[s] = bf16x8{};
+    }
+    if (d0 > 0) lds_barrier();
+#pragma unroll
+    for (int j = 0; j < 8; ++j) *reinterpret_cast<bf16x4*>(&ut[(e + j) * KS + k4 * 4]) = bf16x4{wf[0][j], wf[1][j], wf[2][j], wf[3][j]};
+    lds_barrier();
+#pragma unroll
+    for (int i = 0; i < 2; ++i)
+#pragma unroll
+      for (int s = 0; s < 2; ++s)
+        acc[i] = latent_mfma(qf[s], *reinterpret_cast<const bf16x8*>(&ut[((wave * 2 + i) * 16 + l16) * KS + s * 32 + quad * 8]), acc[i]);
+  }
+#pragma unroll
+  for (int i = 0; i < 2; ++i) {
+    const int r = r0 + (wave * 2 + i) * 16 + l16;
+#pragma unroll
+    for (int m = 0; m < 4; ++m) {
+      const int b = b0 + quad * 4 + m;
+      if (b < a.B && r < a.R) a.qa[((long)b * a.H + h) * W + r] = acc[i][m];
+    }
+  }
+}
+
 // The keys of one split: first key and their number.
 __device__ __forceinline__ void split_range(const LatentArgs& a, int pos, int split, int& k0, int& n) {
   const int lo = pos - a.window + 1 > 0 ? pos - a.window + 1 : 0, all = pos - lo + 1;
-  const int per = ((all + a.splits - 1) / a.splits + 63) / 64 * 64;
+  const int per = ((all + a.splits - 1) / a.splits + 15) / 16 * 16;
   k0 = lo + split * per;
   n = all - split * per;
   n = n < 0 ? 0 : n > per ? per : n;
@@ -259,8 +320,6 @@ __global__ __launch_bounds__(256) void latent_step_any_kernel(const LatentArgs a
     a.part_ml[2 * at + 1] = l_run;
   }
 }
-
-__device__ __forceinline__ f32x4 latent_mfma(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
 
 // bf16, MFMA: 16 heads per workgroup, 64 keys at a time; a wavefront forms the scores of 16 of them and a
 // quarter of the weighted latents.  KC: 32-channel pieces of a row (rounded up); RT: 16-channel tiles of the latent per
@@ -511,6 +570,94 @@ __global__ __launch_bounds__(256) void latent_values_kernel(const LatentArgs a) 
   }
 }
 
+// The same for 16 sequences per workgroup, bf16: KC 32-channel pieces of the latent (rounded up), 64 value channels per workgroup.
+// R a multiple of 8, part 16-byte aligned.
+template <int KC>
+__global__ __launch_bounds__(256) void latent_values_mfma_kernel(const LatentArgs a) {
+  constexpr int RS = KC * 32 + 8;
+  __shared__ __attribute__((aligned(16))) __bf16 lat[kTileRows * RS];
+  __shared__ float share[kTileRows][kMaxSplits];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, l16 = lane & 15, quad = lane >> 4;
+  const int h = blockIdx.x, b0 = blockIdx.y * kTileRows, j = blockIdx.z * 64 + wave * 16 + l16;
+  const int rows = a.B - b0 < kTileRows ? a.B - b0 : kTileRows;
+  // this lane's row of uv is asked for first
+  const __bf16* w = static_cast<const __bf16*>(a.w) + ((long)h * (a.rot + a.d + a.dv) + a.rot + a.d + (j < a.dv ? j : 0)) * a.w_sr;
+  bf16x8 wf[KC];
+#pragma unroll
+  for (int c = 0; c < KC; ++c) {
+    const int e = c * 32 + quad * 8;
+    wf[c] = *reinterpret_cast<const bf16x8*>(w + (e < a.R ? e : 0));
+  }
+  {  // what each split counts for: exp(m_s - max) / sum; 16 lanes per row
+    const int m = tid >> 4, b = b0 + (m < rows ? m : 0);
+    const int pos = row_pos(a.pos, a.pos_host, b);
+    const bool ok = m < rows && pos >= 0 && pos < a.S;
+    const float* ml = a.part_ml + 2 * ((long)b * a.splits * a.H + h);
+    constexpr int N = kMaxSplits / 16;
+    float ms[N], ls[N], mx = -INFINITY, l = 0.f;
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      const int s = i * 16 + (tid & 15);
+      const bool in = ok && s < a.splits;
+      ms[i] = in ? ml[2 * (long)s * a.H] : -INFINITY;
+      ls[i] = in ? ml[2 * (long)s * a.H + 1] : 0.f;
+      mx = fmaxf(mx, ms[i]);
+    }
+#pragma unroll
+    for (int x = 8; x >= 1; x >>= 1) mx = fmaxf(mx, __shfl_xor(mx, x, 64));
+#pragma unroll
+    for (int i = 0; i < N; ++i) {
+      ms[i] = ms[i] == -INFINITY ? 0.f : expf(ms[i] - mx);
+      l = __builtin_fmaf(ms[i], ls[i], l);
+    }
+    l = sum16(l);
+#pragma unroll
+    for (int i = 0; i < N; ++i) share[m][i * 16 + (tid & 15)] = l > 0.f ? ms[i] / l : 0.f;
+  }
+  lds_barrier();
+  // (a split without keys has left nothing in its part: it is not read)
+  const float* p0 = a.part + ((long)b0 * a.splits * a.H + h) * a.R;
+  const long p_row = (long)a.splits * a.H * a.R, p_split = (long)a.H * a.R;
+  constexpr int PIECES = KC * 8, IU = 4, SU = 2;  // 4-channel pieces of a row; pieces and splits in flight together
+  for (int i0 = tid; i0 < kTileRows * PIECES; i0 += 256 * IU) {
+    f32x4 v[IU];
+#pragma unroll
+    for (int u = 0; u < IU; ++u) v[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int s0 = 0; s0 < a.splits; s0 += SU) {
+      f32x4 x[IU][SU];
+      float f[IU][SU];
+#pragma unroll
+      for (int u = 0; u < IU; ++u)
+#pragma unroll
+        for (int s = 0; s < SU; ++s) {
+          const int m = (i0 + u * 256) / PIECES, c = (i0 + u * 256) % PIECES * 4;
+          const bool in = m < rows && c < a.R;
+          f[u][s] = in && s0 + s < a.splits ? share[m][s0 + s] : 0.f;
+          x[u][s] = *reinterpret_cast<const f32x4*>(p0 + (f[u][s] != 0.f ? m * p_row + (s0 + s) * p_split + c : 0));
+        }
+#pragma unroll
+      for (int u = 0; u < IU; ++u)
+#pragma unroll
+        for (int s = 0; s < SU; ++s)
+#pragma unroll
+          for (int k = 0; k < 4; ++k) v[u][k] = f[u][s] != 0.f ? __builtin_fmaf(f[u][s], x[u][s][k], v[u][k]) : v[u][k];
+    }
+#pragma unroll
+    for (int u = 0; u < IU; ++u) {
+      const int m = (i0 + u * 256) / PIECES, c = (i0 + u * 256) % PIECES * 4;
+      *reinterpret_cast<bf16x4*>(&lat[m * RS + c]) = bf16x4{(__bf16)v[u][0], (__bf16)v[u][1], (__bf16)v[u][2], (__bf16)v[u][3]};
+    }
+  }
+  lds_barrier();
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int c = 0; c < KC; ++c) acc = latent_mfma(*reinterpret_cast<const bf16x8*>(&lat[l16 * RS + c * 32 + quad * 8]), wf[c], acc);
+#pragma unroll
+  for (int m = 0; m < 4; ++m)
+    if (quad * 4 + m < rows && j < a.dv)
+      static_cast<__bf16*>(a.o)[(long)(b0 + quad * 4 + m) * a.o_sb + (long)h * a.dv + j] = (__bf16)(acc[m] * a.out_scale);
+}
+
 static int latent_check(const char* who, const LatentArgs& a, int64_t last, int io_dtype) {
   BASED_REQUIRE(a.x && a.norm_w && a.cache, BASED_ERR_ARG, "%s: null pointer argument", who);
   BASED_REQUIRE(a.B >= 0 && a.L >= 0 && a.S > 0 && a.R > 0 && a.rot >= 0 && a.rot % 2 == 0, BASED_ERR_ARG, "%s: bad sizes", who);
@@ -616,7 +763,11 @@ extern "C" BASED_API int based_latent_step(const void* q, const void* x, const v
   hipStream_t s = static_cast<hipStream_t>(stream);
   const int n = io_dtype == BASED_BF16 ? 8 : 4;
   const bool vec = R % n == 0 && w_sr % n == 0 && aligned_to(weight, 16);
-  if (io_dtype == BASED_BF16)
+  const bool tiles = io_dtype == BASED_BF16 && vec && B >= kTileMinRows;
+  if (tiles && D % 8 == 0 && rot % 8 == 0 && q_sb % 8 == 0 && aligned_to(q, 16))
+    hipLaunchKernelGGL(latent_query_mfma_kernel, dim3((unsigned)(H * ((R + kQueryCols - 1) / kQueryCols) + kTileRows),
+                       (unsigned)((B + kTileRows - 1) / kTileRows)), dim3(256), 0, s, a);
+  else if (io_dtype == BASED_BF16)
     launch_latent_query<__bf16>(a, vec, s);
   else
     launch_latent_query<float>(a, vec, s);
@@ -629,7 +780,12 @@ extern "C" BASED_API int based_latent_step(const void* q, const void* x, const v
     else
       hipLaunchKernelGGL(latent_step_any_kernel<float>, grid, dim3(256), 0, s, a);
   }
-  if (io_dtype == BASED_BF16)
+  const dim3 tile_grid((unsigned)H, (unsigned)((B + kTileRows - 1) / kTileRows), (unsigned)((DV + 63) / 64));
+  if (tiles && aligned_to(work_part, 16) && R <= 256)
+    hipLaunchKernelGGL(latent_values_mfma_kernel<8>, tile_grid, dim3(256), 0, s, a);
+  else if (tiles && aligned_to(work_part, 16) && R <= 512)
+    hipLaunchKernelGGL(latent_values_mfma_kernel<16>, tile_grid, dim3(256), 0, s, a);
+  else if (io_dtype == BASED_BF16)
     launch_latent_values<__bf16>(a, vec, s);
   else
     launch_latent_values<float>(a, vec, s);

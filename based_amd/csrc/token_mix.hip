@@ -7,7 +7,7 @@
 //   gelu_mul:       gelu_tanh(g) * table[index], the gate of a per-token embedding.
 //   softcap:        cap * tanh(x / cap) in place.
 //   token_side_step: a per-layer token input for single tokens, r = residual + mult * x and
-//                   proj(gelu_tanh(gate r) * table[index]) in one launch, a workgroup per token.
+//                   proj(gelu_tanh(gate r) * table[index]) in one launch, a few workgroups per token.
 #include "stream_common.hpp"
 
 namespace based {
@@ -225,21 +225,23 @@ struct SideStepArgs {
   const int64_t* index;
   __bf16* y;             // (M, D)
   long x_sr, t_sr, t_n;
-  int D, n;
+  int D, n, d_rows;
   float mult;
 };
 
 constexpr int kSideThreads = 1024, kSideWaves = kSideThreads / 64;
 constexpr int kSideMaxDim = 4096, kSideMaxInner = 512;
 
-// C: 512-channel pieces of a row a lane holds of each gate row (D <= 512 C).
+// C: 512-channel pieces of a row a lane holds of each gate row (D <= 512 C).  Several workgroups per token: each forms the whole
+// gate and d_rows rows of the product behind it; the first one writes the residual.
 template <int C>
 __global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const SideStepArgs a) {
   __shared__ __attribute__((aligned(16))) __bf16 row[512 * C];
   __shared__ __attribute__((aligned(16))) __bf16 inner[kSideMaxInner];
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const long m = blockIdx.x;
-  // the first gate rows and the first row of proj are asked for before anything else
+  const int d0 = blockIdx.y * a.d_rows, d1 = d0 + a.d_rows < a.D ? d0 + a.d_rows : a.D;
+  // the first gate rows and the first pieces of proj are asked for before anything else
   constexpr int GU = C >= 8 ? 1 : C >= 4 ? 2 : 4;  // gate rows in flight together
   bf16x8 g8[GU][C];
   auto fetch = [&](int j0) {
@@ -252,6 +254,16 @@ __global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const Sid
       }
   };
   fetch(wave * GU);
+  // rows of proj are `lpr` lanes wide where that is a power of two up to 16, else one lane walks a row
+  const int pieces = a.n / 8, lpr = pieces <= 16 && (pieces & (pieces - 1)) == 0 ? pieces : 1;
+  const int first = d0 + tid / lpr, step = kSideThreads / lpr, piece = (tid % lpr) * 8;
+  constexpr int PU = 2;  // rows of proj in flight together
+  bf16x8 p8[PU];
+#pragma unroll
+  for (int u = 0; u < PU; ++u) {
+    const int d = first + u * step;
+    p8[u] = *reinterpret_cast<const bf16x8*>(a.proj_w + (long)(d < d1 ? d : d0) * a.n + piece);
+  }
   const long src = a.index[m];
   const bool bad = src < 0 || src >= a.t_n;
   for (int e = tid * 4; e < 512 * C; e += kSideThreads * 4) {
@@ -266,7 +278,7 @@ __global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const Sid
 #pragma unroll
         for (int j = 0; j < 4; ++j) r[j] = to_f32(x[j]);
       }
-      *reinterpret_cast<f32x4*>(a.res_out + m * a.D + e) = r;
+      if (blockIdx.y == 0) *reinterpret_cast<f32x4*>(a.res_out + m * a.D + e) = r;
     }
     bf16x4 o;
 #pragma unroll
@@ -276,9 +288,12 @@ __global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const Sid
   lds_barrier();
   for (int j0 = wave * GU; j0 < a.n; j0 += kSideWaves * GU) {
     if (j0 != wave * GU) fetch(j0);
-    float acc[GU];
+    float acc[GU], e[GU];
 #pragma unroll
-    for (int u = 0; u < GU; ++u) acc[u] = 0.f;
+    for (int u = 0; u < GU; ++u) {
+      acc[u] = 0.f;
+      e[u] = to_f32(a.table[(bad ? 0 : src) * a.t_sr + (j0 + u < a.n ? j0 + u : 0)]);
+    }
 #pragma unroll
     for (int c = 0; c < C; ++c) {
       float x[8];
@@ -293,25 +308,42 @@ __global__ __launch_bounds__(kSideThreads) void token_side_step_kernel(const Sid
       float v = sum16(acc[u]);
       v += __shfl_xor(v, 16, 64);
       v += __shfl_xor(v, 32, 64);
-      if (lane == 0 && j0 + u < a.n) {
-        const float e = to_f32(a.table[(bad ? 0 : src) * a.t_sr + j0 + u]);
-        inner[j0 + u] = (__bf16)(bad ? __builtin_nanf("") : gelu_tanh_f(round_to<__bf16>(v)) * e);
-      }
+      if (lane == 0 && j0 + u < a.n) inner[j0 + u] = (__bf16)(bad ? __builtin_nanf("") : gelu_tanh_f(round_to<__bf16>(v)) * e[u]);
     }
   }
   lds_barrier();
-  for (int d = tid; d < a.D; d += kSideThreads) {
-    const __bf16* w = a.proj_w + (long)d * a.n;
-    float acc = 0.f;
-#pragma unroll 8
-    for (int c = 0; c < a.n; c += 8) {
-      float x[8], wv[8];
-      load_vec<__bf16, 8>(w + c, wv);
-      load_vec<__bf16, 8>(inner + c, x);
+  for (int t0 = d0; t0 < d1; t0 += PU * step) {  // (the same rounds for every lane: lanes of a row add up together)
+    float acc[PU];
 #pragma unroll
-      for (int i = 0; i < 8; ++i) acc = __builtin_fmaf(wv[i], x[i], acc);
+    for (int u = 0; u < PU; ++u) {
+      const int d = t0 + tid / lpr + u * step;
+      const __bf16* w = a.proj_w + (long)(d < d1 ? d : d0) * a.n;
+      if (t0 != d0) p8[u] = *reinterpret_cast<const bf16x8*>(w + piece);
+      acc[u] = 0.f;
+      float x[8];
+      load_vec<__bf16, 8>(inner + piece, x);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) acc[u] = __builtin_fmaf(to_f32(p8[u][i]), x[i], acc[u]);
+      if (lpr == 1) {
+#pragma unroll 4
+        for (int c = 8; c < a.n; c += 8) {
+          float wv[8];
+          load_vec<__bf16, 8>(w + c, wv);
+          load_vec<__bf16, 8>(inner + c, x);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) acc[u] = __builtin_fmaf(wv[i], x[i], acc[u]);
+        }
+      }
     }
-    a.y[m * a.D + d] = (__bf16)acc;
+#pragma unroll
+    for (int u = 0; u < PU; ++u) {
+      if (lpr >= 2) acc[u] = dpp_move_add<0xB1>(acc[u]);   // quad_perm [1,0,3,2]
+      if (lpr >= 4) acc[u] = dpp_move_add<0x4E>(acc[u]);   // quad_perm [2,3,0,1]
+      if (lpr >= 8) acc[u] = dpp_move_add<0x141>(acc[u]);  // row_half_mirror
+      if (lpr >= 16) acc[u] = dpp_move_add<0x140>(acc[u]); // row_mirror
+      const int d = t0 + tid / lpr + u * step;
+      if (tid % lpr == 0 && d < d1) a.y[m * a.D + d] = (__bf16)acc[u];
+    }
   }
 }
 
@@ -429,11 +461,14 @@ extern "C" BASED_API int based_token_side_step(const void* x, const float* resid
                 BASED_ERR_ALIGN, "token_side_step: rows must be whole 16-byte pieces");
   BASED_REQUIRE(residual_in != residual_out, BASED_ERR_ARG, "token_side_step: residual_out must not be residual_in");
   if (M == 0) return BASED_OK;
+  // rows of the second product per workgroup: 256 or more, and no more workgroups than compute units
+  const int most = M < 256 ? (int)(256 / M) : 1, wanted = (int)((D + 255) / 256), parts = wanted < most ? wanted : most;
+  const int d_rows = (int)((D + parts - 1) / parts);
   const SideStepArgs a{static_cast<const __bf16*>(x), residual_in, residual_out, static_cast<const __bf16*>(gate_w),
                        static_cast<const __bf16*>(proj_w), static_cast<const __bf16*>(table), index, static_cast<__bf16*>(y), (long)x_sr,
-                       (long)table_sr, (long)table_n, (int)D, (int)n, mult};
+                       (long)table_sr, (long)table_n, (int)D, (int)n, d_rows, mult};
   hipStream_t s = static_cast<hipStream_t>(stream);
-  const dim3 grid((unsigned)M), block(kSideThreads);
+  const dim3 grid((unsigned)M, (unsigned)((D + d_rows - 1) / d_rows)), block(kSideThreads);
   const int chunks = (int)((D + 511) / 512);
   if (chunks <= 1)
     hipLaunchKernelGGL((token_side_step_kernel<1>), grid, block, 0, s, a);

@@ -1270,7 +1270,7 @@ def latent_write(x, norm_weight, cache, start: int, eps: float, rope) -> None:
                                                  n_pos, half, _dtype_code(x), _stream_ptr(x)))
 
 
-LATENT_STEP_TARGET = 512  # workgroups that the keys of a step are dealt to, where there are enough
+LATENT_STEP_TARGET = 256  # workgroups that the keys of a step are dealt to, where there are enough
 LATENT_STEP_MAX_SPLITS = 64
 
 
@@ -1288,7 +1288,7 @@ def latent_step(q, x, norm_weight, weight, cache, heads: int, dim: int, window: 
             or weight.shape[1] < R:
         raise ValueError(f"bad shapes q{tuple(q.shape)} weight{tuple(weight.shape)} out{tuple(out.shape)}")
     groups = B * ((heads + 15) // 16)
-    splits = max(1, min(LATENT_STEP_TARGET // groups, (min(window, S) + 127) // 128, LATENT_STEP_MAX_SPLITS))
+    splits = max(1, min(LATENT_STEP_TARGET // groups, (min(window, S) + 63) // 64, LATENT_STEP_MAX_SPLITS))
     f32 = dict(dtype=torch.float32, device=x.device)
     work_q = torch.empty(B, heads, R + rot, **f32)
     part, part_ml = torch.empty(B, splits, heads, R, **f32), torch.empty(B, splits, heads, 2, **f32)

@@ -364,6 +364,34 @@ def test_latent_steps_of_rows_at_their_own_positions(dev, dtype):
             close(o[b, 0], want, 2 * TOL[dtype])
 
 
+@pytest.mark.parametrize("dtype", DTYPES)
+@pytest.mark.parametrize("H,d,r,dv,R,window", [(4, 24, 8, 32, 64, 30), (3, 136, 16, 96, 264, 50), (17, 64, 32, 64, 512, 90), (2, 14, 6, 10, 40, 7)])
+def test_latent_steps_of_many_rows(dev, H, d, r, dv, R, window, dtype):
+    """More rows than one tile of 16, at positions from the first one on; a row that is at no position has no say in the others."""
+    from based_amd.generation import InferenceParams
+
+    B, T = 19, 120
+    core, uk, uv, nw = latent_core(dev, dtype, H, d, r, dv, R, window)
+    q, x = rnd(B, T, H, r + d, seed=4).bfloat16(), rnd(B, T, R + r, seed=5).bfloat16()
+    at = [(37 * b) % (T - 2) for b in range(B)]
+    params = InferenceParams(max_seqlen=T, max_batch_size=B)
+    for b in range(B):
+        params.seqlen_offset, params.batch_size_offset = 0, b
+        if at[b]:
+            run_latent(core, dev, dtype, q[b:b + 1, :at[b]], x[b:b + 1, :at[b]], [at[b]], params)
+    params.batch_size_offset, params.seqlen_offset = 0, max(at)
+    idle = 5
+    for step in range(2):
+        places = [a + step for a in at]
+        params.lengths_per_sample = torch.tensor([-1 if b == idle else p for b, p in enumerate(places)], dtype=torch.int32, device=dev)
+        pick = lambda y: torch.stack([y[b, places[b]] for b in range(B)])[:, None]
+        o = run_latent(core, dev, dtype, pick(q), pick(x), [1], params)
+        for b in range(B):
+            if b != idle:
+                n = places[b] + 1
+                close(o[b, 0], latent_want(core, uk, uv, nw, q[b, :n].double(), x[b, :n].double())[-1], 2 * TOL[dtype])
+
+
 # ---- experts ----
 def expert_case(n, D, F, E, top, dtype, seed=0):
     h, router = rnd(n, D, seed=seed, dtype=dtype), rnd(E, D, seed=seed + 1, dtype=dtype, scale=2 * D ** -0.5)
