@@ -305,12 +305,19 @@ __global__ __launch_bounds__(512) void expert_route_row_kernel(const RouteRowArg
 
 constexpr long kPlanSlots = 8192;  // choices that the planning workgroup puts in order by itself
 
-__global__ __launch_bounds__(256) void expert_plan_kernel(const int32_t* counts, const int32_t* ids, const int32_t* rank, int32_t* tile_first,
-                                                          int32_t* tile_expert, int32_t* order, long slots, int E, int tile_rows) {
+constexpr int kPlanThreads = 1024;
+
+__global__ __launch_bounds__(kPlanThreads) void expert_plan_kernel(const int32_t* counts, const int32_t* __restrict__ ids,
+                                                                   const int32_t* __restrict__ rank, int32_t* tile_first,
+                                                                   int32_t* tile_expert, int32_t* __restrict__ order, long slots, int E,
+                                                                   int tile_rows) {
   __shared__ int scan[256], first_of[kMaxExperts];
   plan_tiles(counts, scan, first_of, tile_first, tile_expert, E, tile_rows);
-  if (slots <= kPlanSlots)
-    for (long i = threadIdx.x; i < slots; i += 256) order[(long)first_of[ids[i]] * tile_rows + rank[i]] = (int32_t)i;
+  if (slots <= kPlanSlots) {
+    // (the loads of the unrolled places are independent of each other)
+#pragma unroll 4
+    for (int i = threadIdx.x; i < (int)slots; i += kPlanThreads) order[(long)first_of[ids[i]] * tile_rows + rank[i]] = i;
+  }
 }
 
 __global__ __launch_bounds__(256) void expert_scatter_kernel(const int32_t* ids, const int32_t* rank, const int32_t* tile_first, int32_t* order,
@@ -724,7 +731,7 @@ extern "C" BASED_API int based_expert_grouped(const void* h, const void* router,
   const bool vec = route_vec(r);
   launch_route<__bf16>(r, vec, s);
   if (!route_is_single(r, vec)) {
-    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(256), 0, s, counts, ids, rank, tile_first, tile_expert, order, (long)slots, (int)E,
+    hipLaunchKernelGGL(expert_plan_kernel, dim3(1), dim3(kPlanThreads), 0, s, counts, ids, rank, tile_first, tile_expert, order, (long)slots, (int)E,
                        rows);
     if (slots > kPlanSlots)
       hipLaunchKernelGGL(expert_scatter_kernel, dim3((unsigned)((slots + 255) / 256)), dim3(256), 0, s, ids, rank, tile_first, order,
