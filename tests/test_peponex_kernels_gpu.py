@@ -504,8 +504,8 @@ def test_projection_with_gate_table_and_cap(dev, M, N, K):
     close(y, 1.5 * torch.tanh((O.rms(r, 1e-5) * nw.double()).bfloat16().double() @ w.double().T / 1.5), 2 * TOL[BF16])
 
 
-@pytest.mark.parametrize("M", [1, 5, 32])
-@pytest.mark.parametrize("n,D", [(8, 64), (24, 192), (64, 1024), (136, 1544), (16, 4096), (512, 512)])
+@pytest.mark.parametrize("M", [1, 5, 32, 300])
+@pytest.mark.parametrize("n,D", [(8, 64), (24, 192), (64, 1024), (136, 1544), (16, 4096), (512, 512), (32, 264), (128, 1000)])
 def test_token_input_of_single_tokens(dev, M, n, D):
     from based_amd import ops
 
